@@ -3,8 +3,10 @@ from .llama import LlamaConfig, RopeScaling, ConfigError, PRESETS
 from .mifutar import MifutarConfig
 from .bomotar import BomotarConfig
 from .golavik import GolavikConfig
+from .zemarax import ZemaraxConfig
+from .tokatar import TokatarConfig
 from .registry import register_architecture, architecture_names, config_class_for, load_config, config_from_file
 
-__all__ = ["PartSpec", "LayerSpec", "LayerCall", "ModelSpec", "LlamaConfig", "MifutarConfig", "BomotarConfig", "GolavikConfig", "RopeScaling",
+__all__ = ["PartSpec", "LayerSpec", "LayerCall", "ModelSpec", "LlamaConfig", "MifutarConfig", "BomotarConfig", "GolavikConfig", "ZemaraxConfig", "TokatarConfig", "RopeScaling",
            "ConfigError", "PRESETS", "register_architecture", "architecture_names",
            "config_class_for", "load_config", "config_from_file"]

@@ -16,6 +16,7 @@ from .mifutar import MifutarConfig
 from .bomotar import BomotarConfig
 from .golavik import GolavikConfig
 from .zemarax import ZemaraxConfig
+from .tokatar import TokatarConfig
 
 _ARCHITECTURES: Dict[str, Any] = {}
 
@@ -78,3 +79,4 @@ register_architecture("Mifutar", MifutarConfig)
 register_architecture("Bomotar", BomotarConfig)
 register_architecture("Golavik", GolavikConfig)
 register_architecture("Zemarax", ZemaraxConfig)
+register_architecture("Tokatar", TokatarConfig)

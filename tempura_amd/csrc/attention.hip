@@ -1,5 +1,5 @@
-// Attention over the paged cache, general kernel: any head size up to 512, any number
-// of heads and groups, any page size, optional window, float32 or bfloat16.
+// Attention over the paged cache, general kernel: any value size up to 512, any key size up to 4096, any number
+// of heads and groups, any page size, optional window or chunks, float32 or bfloat16.
 //
 // One wave per (query token, head).  Keys are taken 64 at a time: each lane scores one
 // key (a full dot product with the query, which sits in LDS), the tile's maximum and
@@ -9,7 +9,9 @@
 //
 // Query token t belongs to request r = token_req[t]; its position is
 // context_lens[r] - q_len_r + (t - cu_seqlens[r]) and it sees keys lo..pos with
-// lo = max(0, pos - window + 1) when window > 0, else 0.
+// lo = max(0, pos - window + 1) when window > 0, pos - pos mod chunk when chunk > 0, else 0.
+//
+// Capped scores: with softcap > 0 a scaled score s becomes softcap * tanh(s / softcap) before the softmax.
 //
 // Kept first keys: with keep_first > 0 a windowed query also sees keys 0..keep_first-1 (those of them that lie
 // before lo; they are visited first, so the order of keys stays ascending).
@@ -22,7 +24,8 @@
 
 #include "common.h"
 
-#define ATT_MAX_ACC 8  // head_dim <= 64 * ATT_MAX_ACC
+#define ATT_MAX_ACC 8      // value size <= 64 * ATT_MAX_ACC
+#define ATT_MAX_KEY 4096   // key size (the query row lies in LDS)
 
 template <typename T>
 __global__ __launch_bounds__(64) void paged_attention_kernel(
@@ -30,14 +33,14 @@ __global__ __launch_bounds__(64) void paged_attention_kernel(
     const int* __restrict__ block_tables, int table_width, const int* __restrict__ cu_seqlens,
     const int* __restrict__ context_lens, const int* __restrict__ token_req, T* __restrict__ out, int n_heads,
     int n_kv, int head_dim, int page_size, float scale, int window, const float* __restrict__ dist_bias, int bias_len,
-    int value_dim, int keep_first, const float* __restrict__ sink) {
+    int value_dim, int keep_first, const float* __restrict__ sink, int chunk, float softcap) {
   extern __shared__ float qs[];  // the query row, float32
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int r = token_req[t];
   const int q_start = cu_seqlens[r];
   const int q_len = cu_seqlens[r + 1] - q_start;
   const int pos = context_lens[r] - q_len + (t - q_start);
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = chunk > 0 ? pos / chunk * chunk : (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
   const int kvh = h / (n_heads / n_kv);
   const T* qrow = q + ((size_t)t * n_heads + h) * head_dim;
   for (int d = lane; d < head_dim; d += TP_WAVE) qs[d] = to_float(qrow[d]);
@@ -67,6 +70,7 @@ __global__ __launch_bounds__(64) void paged_attention_kernel(
       float dot = 0.f;
       for (int d = 0; d < head_dim; ++d) dot = fmaf(qs[d], to_float(kr[d]), dot);
       s = dot * scale;
+      if (softcap > 0.f) s = softcap * tanhf(s / softcap);
       if (dist_bias != nullptr) s += dist_bias[(size_t)h * bias_len + min(pos - j, bias_len - 1)];
     }
     const float m_new = fmaxf(m, wave_max(s));
@@ -112,7 +116,8 @@ int tp_paged_attention_fast(const void* q, const void* k_cache, const void* v_ca
                             int n_req, int n_heads, int n_kv, int head_dim, int page_size, float scale, int window,
                             int max_q_len, int num_single, int num_splits, float* scratch, const int* token_req,
                             int portion_splits, int portion_min_steps, float* portion_scratch, const float* dist_bias,
-                            int bias_len, int keep_first, const float* sink, hipStream_t s);
+                            int bias_len, int keep_first, const float* sink, int value_dim, int chunk, float softcap,
+                            hipStream_t s);
 
 extern "C" int tp_paged_attention(const void* q, int dt, const void* k_cache, const void* v_cache,
                                   const int* block_tables, int table_width, const int* cu_seqlens,
@@ -121,9 +126,9 @@ extern "C" int tp_paged_attention(const void* q, int dt, const void* k_cache, co
                                   int window, int max_q_len, int max_ctx, int allow_fast, int num_single,
                                   int num_splits, float* scratch, int portion_splits, int portion_min_steps,
                                   float* portion_scratch, const float* dist_bias, int bias_len, int value_dim,
-                                  int keep_first, const float* sink, hipStream_t s) {
+                                  int keep_first, const float* sink, int chunk, float softcap, hipStream_t s) {
   // value_dim: the size of a value head (0: head_dim): v_cache is [page, kv_head, value_dim, page_size] and out
-  // [n, heads * value_dim]; the matrix-core kernels take equal sizes only.
+  // [n, heads * value_dim]; the matrix-core kernels take equal sizes and a few pairs with wider keys.
   if (value_dim <= 0) value_dim = head_dim;
   // num_single: how many requests bring exactly one token (they go to the split decode kernel,
   // which, with more than one split, needs `scratch` of n_req * n_heads * num_splits * (head_dim + 2)
@@ -132,19 +137,26 @@ extern "C" int tp_paged_attention(const void* q, int dt, const void* k_cache, co
   TP_REQUIRE(n_tokens >= 0 && n_req >= 0 && n_heads > 0 && n_kv > 0 && head_dim > 0 && page_size > 0,
              "paged_attention: bad sizes");
   TP_REQUIRE(n_heads % n_kv == 0, "paged_attention: %d heads is not a multiple of %d kv heads", n_heads, n_kv);
-  TP_REQUIRE(head_dim <= TP_WAVE * ATT_MAX_ACC && value_dim <= TP_WAVE * ATT_MAX_ACC, "paged_attention: head size %d / %d exceeds %d",
-             head_dim, value_dim, TP_WAVE * ATT_MAX_ACC);
+  TP_REQUIRE(head_dim <= ATT_MAX_KEY && value_dim <= TP_WAVE * ATT_MAX_ACC, "paged_attention: head sizes %d / %d exceed %d / %d",
+             head_dim, value_dim, ATT_MAX_KEY, TP_WAVE * ATT_MAX_ACC);
   TP_REQUIRE(window >= 0, "paged_attention: window must be >= 0");
   TP_REQUIRE(keep_first >= 0, "paged_attention: keep_first must be >= 0");
+  TP_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "paged_attention: chunks and a window exclude each other");
+  TP_REQUIRE(softcap >= 0.f && (softcap == 0.f || dist_bias == nullptr), "paged_attention: a cap and a distance bias exclude each other");
+  if (chunk == 1) {   // (a chunk of one position: the query itself)
+    chunk = 0;
+    window = 1;
+  }
   if (window == 0) keep_first = 0;   // (without a window every key is seen anyway)
   TP_REQUIRE(n_heads <= 65535, "paged_attention: too many heads");
   if (n_tokens == 0) return 0;
   TP_REQUIRE(dist_bias == nullptr || bias_len > 0, "paged_attention: empty distance bias table");
-  if (dt == TP_BF16 && allow_fast && value_dim == head_dim) {
+  if (dt == TP_BF16 && allow_fast) {
     const int rc = tp_paged_attention_fast(q, k_cache, v_cache, block_tables, table_width, cu_seqlens,
                                            context_lens, out, n_tokens, n_req, n_heads, n_kv, head_dim,
                                            page_size, scale, window, max_q_len, num_single, num_splits, scratch, token_req,
-                                           portion_splits, portion_min_steps, portion_scratch, dist_bias, bias_len, keep_first, sink, s);
+                                           portion_splits, portion_min_steps, portion_scratch, dist_bias, bias_len, keep_first, sink, value_dim, chunk,
+                                           softcap, s);
     if (rc >= 0) return rc;
   }
   const dim3 grid(n_tokens, n_heads);
@@ -152,11 +164,11 @@ extern "C" int tp_paged_attention(const void* q, int dt, const void* k_cache, co
   if (dt == TP_F32)
     hipLaunchKernelGGL(paged_attention_kernel<float>, grid, dim3(64), shmem, s, (const float*)q,
                        (const float*)k_cache, (const float*)v_cache, block_tables, table_width, cu_seqlens,
-                       context_lens, token_req, (float*)out, n_heads, n_kv, head_dim, page_size, scale, window, dist_bias, bias_len, value_dim, keep_first, sink);
+                       context_lens, token_req, (float*)out, n_heads, n_kv, head_dim, page_size, scale, window, dist_bias, bias_len, value_dim, keep_first, sink, chunk, softcap);
   else if (dt == TP_BF16)
     hipLaunchKernelGGL(paged_attention_kernel<bf16_t>, grid, dim3(64), shmem, s, (const bf16_t*)q,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_tables, table_width, cu_seqlens,
-                       context_lens, token_req, (bf16_t*)out, n_heads, n_kv, head_dim, page_size, scale, window, dist_bias, bias_len, value_dim, keep_first, sink);
+                       context_lens, token_req, (bf16_t*)out, n_heads, n_kv, head_dim, page_size, scale, window, dist_bias, bias_len, value_dim, keep_first, sink, chunk, softcap);
   else
     TP_REQUIRE(false, "paged_attention: unknown dtype %d", dt);
   TP_CHECK_LAUNCH("paged_attention");

@@ -1,6 +1,8 @@
 // bfloat16 attention over the paged cache on the gfx950 matrix cores
 // (v_mfma_f32_16x16x32_bf16), for head sizes that are multiples of 32 (up to 128) and
-// page sizes that are multiples of 8.  Other shapes go to the general kernel.
+// page sizes that are multiples of 8; and for keys wider than values in the pairs of sizes (D, DV)
+// that the dispatch at the end names (a caller pads narrower keys with zeros up to one of them).
+// Other shapes go to the general kernel.
 //
 // Everything is computed transposed, so that no operand ever needs a transpose in LDS:
 //   S^T[key, query] = K[key, :] . Q[query, :]          (A = K rows, B = Q rows)
@@ -103,7 +105,27 @@ struct AttnArgs {
   // before the window's first step come first, and the masks let a key pass that is kept.  (Not in the kernels with a
   // bias by distance, and never together with portions whose keys are split over blocks: the host sees to both.)
   int keep_first;
+  // a query sees only the keys of its own aligned chunk of `chunk` positions (0: no chunks; never together with a
+  // window): its first visible key is pos - pos mod chunk.  The quotient is mulhi(pos, chunk_mul) >> chunk_shift, exact
+  // for every position below 2^31 (chunk_mul = ceil(2^(32 + chunk_shift) / chunk) with chunk >= 2).
+  int chunk, chunk_shift;
+  unsigned chunk_mul;
+  // scores capped before the mask (MODE_CAP): cap * tanh(score / cap).  cap_log2 = cap * log2(e), cap_in = what turns
+  // q . k into 2 log2(e) score / cap
+  float cap_log2, cap_in;
 };
+// what happens to a score between the product and the mask (a template parameter of the kernels)
+enum { MODE_PLAIN = 0, MODE_BIAS = 1, MODE_CAP = 2 };
+// the first key that a query at position `pos` sees (kept first keys apart); it never falls as pos grows
+__device__ inline int attn_first_key(const AttnArgs& a, int pos) {
+  if (a.chunk > 0) return (int)(__umulhi((unsigned)pos, a.chunk_mul) >> a.chunk_shift) * a.chunk;
+  return a.window > 0 ? pos - a.window + 1 : 0;
+}
+// a capped score in units of log 2: cap_log2 * tanh(x), tanh(x) = 1 - 2 / (2^(2 x log2 e) + 1), with the hardware's exp2
+// and reciprocal (an error of a few 1e-8 of the cap; both limits come out right: 2^large is infinite and its reciprocal 0)
+__device__ inline float attn_capped(const AttnArgs& a, float dot) {
+  return fmaf(-2.0f * a.cap_log2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(dot * a.cap_in) + 1.0f), a.cap_log2);
+}
 #define PART_STRIDE(D) ((D) + 4)
 // the sink's share of a denominator that is relative to the maximum m (scores and m are in units of log 2): 2^(sink *
 // log2(e) - m); a sink far above m makes the sum infinite and the row zero, which is its limit
@@ -112,10 +134,10 @@ __device__ inline float sink_term(const float* sink, int head, float m) {
 }
 
 // The keys and values of one step of 32 keys, as MFMA operand fragments.
-template <int D>
+template <int D, int DV>
 struct KvFrags {
   bf16x8_t k[2][D / 32];
-  bf16x8_t v[D / 16];
+  bf16x8_t v[DV / 16];
 };
 
 // A lane's value fragment holds eight consecutive key places of one element.  Places past the last key that
@@ -134,9 +156,9 @@ __device__ inline u32x4_t attn_existing_keys(int n) {
 
 // Fetch the fragments of the step starting at key j0 (kvh: kv head; ctx: keys that exist; keys
 // past the end are clamped to the last one and masked later, values past the end are cleared).
-template <int D>
+template <int D, int DV>
 __device__ inline void attn_load(const AttnArgs& a, const int* __restrict__ table, int kvh, int ctx, int j0,
-                                 KvFrags<D>& f) {
+                                 KvFrags<D, DV>& f) {
   const int lane = threadIdx.x & 63;
   const int g = lane >> 4, c = lane & 15;
   const int ps = a.page_size;
@@ -151,15 +173,15 @@ __device__ inline void attn_load(const AttnArgs& a, const int* __restrict__ tabl
   // values: eight consecutive keys of element d per lane
   const int kb = min(j0 + 8 * g, (ctx - 1) & ~7);
   const int vpage = table[kb / ps];
-  const bf16_t* vr = a.v_cache + ((size_t)(vpage * a.n_kv + kvh) * D + c) * ps + kb % ps;
+  const bf16_t* vr = a.v_cache + ((size_t)(vpage * a.n_kv + kvh) * DV + c) * ps + kb % ps;
   if (j0 + 32 > ctx) {   // the step that holds the last key
     const u32x4_t keep = attn_existing_keys(ctx - (j0 + 8 * g));
 #pragma unroll
-    for (int dt = 0; dt < D / 16; ++dt) f.v[dt] = frag_of(ATTN_KV_LOAD((const u32x4_t*)(vr + (size_t)dt * 16 * ps)) & keep);
+    for (int dt = 0; dt < DV / 16; ++dt) f.v[dt] = frag_of(ATTN_KV_LOAD((const u32x4_t*)(vr + (size_t)dt * 16 * ps)) & keep);
     return;
   }
 #pragma unroll
-  for (int dt = 0; dt < D / 16; ++dt) f.v[dt] = frag_of(ATTN_KV_LOAD((const u32x4_t*)(vr + (size_t)dt * 16 * ps)));
+  for (int dt = 0; dt < DV / 16; ++dt) f.v[dt] = frag_of(ATTN_KV_LOAD((const u32x4_t*)(vr + (size_t)dt * 16 * ps)));
 }
 
 // One step of 32 keys starting at j0 for NQ query tiles, on fetched fragments.  qpos[nq] is the
@@ -184,13 +206,15 @@ __device__ inline void attn_scores(const bf16x8_t (&k)[2][D / 32], const bf16x8_
 
 // Softmax of one step's scores: probabilities as the next product's operand (pf), and the factor by
 // which the running sums shrink (alpha; `moved` false when no maximum of the wave moved: alpha is 1).
-// BIAS: bias_row is this lane's row of the distance table (the row of its query column's head); the values
+// MODE_BIAS: bias_row is this lane's row of the distance table (the row of its query column's head); the values
 // that are compared and exponentiated are then score * scale_log2 + bias * log2(e), formed before the maximum.
+// MODE_CAP: they are the capped scores (attn_capped), likewise formed before the maximum.
 // (BP: a pointer to global memory, or to LDS where a kernel keeps its heads' rows there)
-template <int NQ, bool MASK, bool BIAS = false, typename BP = const float*>
+template <int NQ, bool MASK, int MODE = MODE_PLAIN, typename BP = const float*>
 __device__ inline void attn_softmax(const AttnArgs& a, int j0, const f32x4_t (&s)[NQ][2], const int (&qpos)[NQ],
                                     float (&m)[NQ], float (&l)[NQ], bf16x8_t (&pf)[NQ], float (&alpha)[NQ], bool (&moved)[NQ],
                                     BP bias_row = nullptr) {
+  constexpr bool BIAS = MODE == MODE_BIAS, CAP = MODE == MODE_CAP, DONE = BIAS || CAP;   // (DONE: v is in units of log 2 already)
   const int lane = threadIdx.x & 63;
   const int g = lane >> 4;
 #pragma unroll
@@ -200,7 +224,7 @@ __device__ inline void attn_softmax(const AttnArgs& a, int j0, const f32x4_t (&s
     float mx = -INFINITY;
     if (BIAS) {
       const int hi = qpos[nq];
-      const int lo = a.window > 0 ? hi - a.window + 1 : 0;
+      const int lo = attn_first_key(a, hi);
       float b[8];
 #pragma unroll
       for (int i = 0; i < 8; ++i) {   // (all eight loads in flight; keys above the query read entry 0 and are masked)
@@ -216,29 +240,29 @@ __device__ inline void attn_softmax(const AttnArgs& a, int j0, const f32x4_t (&s
         }
     } else if (MASK) {
       const int hi = qpos[nq];
-      const int lo = a.window > 0 ? hi - a.window + 1 : 0;
+      const int lo = attn_first_key(a, hi);
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int key = j0 + 8 * g + 4 * t + r;
-          v[t * 4 + r] = (key <= hi && (key >= lo || key < a.keep_first)) ? s[nq][t][r] : -INFINITY;
+          v[t * 4 + r] = (key <= hi && (key >= lo || key < a.keep_first)) ? (CAP ? attn_capped(a, s[nq][t][r]) : s[nq][t][r]) : -INFINITY;
         }
     } else {
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[t * 4 + r] = s[nq][t][r];
+        for (int r = 0; r < 4; ++r) v[t * 4 + r] = CAP ? attn_capped(a, s[nq][t][r]) : s[nq][t][r];
     }
 #pragma unroll
     for (int i = 0; i < 8; ++i) mx = fmaxf(mx, v[i]);
     mx = quad_rows_max(mx);
-    const float m_new = fmaxf(m[nq], BIAS ? mx : mx * a.scale_log2);    // the scale is positive
+    const float m_new = fmaxf(m[nq], DONE ? mx : mx * a.scale_log2);    // the scale is positive
     const float m_use = (m_new == -INFINITY) ? 0.f : m_new;  // a column with nothing visible yet
     float sum = 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      v[i] = __builtin_amdgcn_exp2f(BIAS ? v[i] - m_use : fmaf(v[i], a.scale_log2, -m_use));
+      v[i] = __builtin_amdgcn_exp2f(DONE ? v[i] - m_use : fmaf(v[i], a.scale_log2, -m_use));
       sum += v[i];
     }
     u32x4_t pk;
@@ -264,7 +288,7 @@ __device__ inline void attn_softmax(const AttnArgs& a, int j0, const f32x4_t (&s
 // masked values and the new maximum of every column; it runs while the next step's key fragments travel from LDS.
 // The second half is the exponentials and the sums: alpha is computed always and chosen afterwards; where no
 // maximum moved it is exactly 1 and l * 1 + sum is l + sum.
-template <int NQ, bool MASK>
+template <int NQ, bool MASK, bool CAP = false>
 __device__ inline void attn_softmax_max(const AttnArgs& a, int j0, const f32x4_t (&s)[NQ][2], const int (&qpos)[NQ],
                                         const float (&m)[NQ], float (&v)[NQ][8], float (&m_new)[NQ]) {
   const int lane = threadIdx.x & 63;
@@ -274,28 +298,28 @@ __device__ inline void attn_softmax_max(const AttnArgs& a, int j0, const f32x4_t
     float mx = -INFINITY;
     if (MASK) {
       const int hi = qpos[nq];
-      const int lo = a.window > 0 ? hi - a.window + 1 : 0;
+      const int lo = attn_first_key(a, hi);
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int key = j0 + 8 * g + 4 * t + r;
-          v[nq][t * 4 + r] = (key <= hi && (key >= lo || key < a.keep_first)) ? s[nq][t][r] : -INFINITY;
+          v[nq][t * 4 + r] = (key <= hi && (key >= lo || key < a.keep_first)) ? (CAP ? attn_capped(a, s[nq][t][r]) : s[nq][t][r]) : -INFINITY;
         }
     } else {
 #pragma unroll
       for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[nq][t * 4 + r] = s[nq][t][r];
+        for (int r = 0; r < 4; ++r) v[nq][t * 4 + r] = CAP ? attn_capped(a, s[nq][t][r]) : s[nq][t][r];
     }
 #pragma unroll
     for (int i = 0; i < 8; ++i) mx = fmaxf(mx, v[nq][i]);
     mx = quad_rows_max(mx);
-    m_new[nq] = fmaxf(m[nq], mx * a.scale_log2);
+    m_new[nq] = fmaxf(m[nq], CAP ? mx : mx * a.scale_log2);
   }
 }
 
-template <int NQ>
+template <int NQ, bool CAP = false>
 __device__ inline void attn_softmax_exp(const AttnArgs& a, float (&v)[NQ][8], const float (&m_new)[NQ], float (&m)[NQ],
                                         float (&l)[NQ], bf16x8_t (&pf)[NQ], float (&alpha)[NQ], bool (&moved)[NQ]) {
 #pragma unroll
@@ -304,7 +328,7 @@ __device__ inline void attn_softmax_exp(const AttnArgs& a, float (&v)[NQ][8], co
     float sum = 0.f;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      v[nq][i] = __builtin_amdgcn_exp2f(fmaf(v[nq][i], a.scale_log2, -m_use));
+      v[nq][i] = __builtin_amdgcn_exp2f(CAP ? v[nq][i] - m_use : fmaf(v[nq][i], a.scale_log2, -m_use));
       sum += v[nq][i];
     }
     u32x4_t pk;
@@ -321,14 +345,14 @@ __device__ inline void attn_softmax_exp(const AttnArgs& a, float (&v)[NQ][8], co
   }
 }
 
-template <int D, int NQ>
-__device__ inline void attn_pv(const bf16x8_t (&vf)[D / 16], const bf16x8_t (&pf)[NQ], const float (&alpha)[NQ],
-                               const bool (&moved)[NQ], f32x4_t (&o)[NQ][D / 16]) {
+template <int DV, int NQ>
+__device__ inline void attn_pv(const bf16x8_t (&vf)[DV / 16], const bf16x8_t (&pf)[NQ], const float (&alpha)[NQ],
+                               const bool (&moved)[NQ], f32x4_t (&o)[NQ][DV / 16]) {
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
     if (moved[nq]) {
 #pragma unroll
-      for (int dt = 0; dt < D / 16; ++dt) {
+      for (int dt = 0; dt < DV / 16; ++dt) {
         o[nq][dt][0] *= alpha[nq];
         o[nq][dt][1] *= alpha[nq];
         o[nq][dt][2] *= alpha[nq];
@@ -336,42 +360,42 @@ __device__ inline void attn_pv(const bf16x8_t (&vf)[D / 16], const bf16x8_t (&pf
       }
     }
 #pragma unroll
-    for (int dt = 0; dt < D / 16; ++dt) o[nq][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[dt], pf[nq], o[nq][dt], 0, 0, 0);
+    for (int dt = 0; dt < DV / 16; ++dt) o[nq][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[dt], pf[nq], o[nq][dt], 0, 0, 0);
   }
 }
 
-template <int D, int NQ, bool MASK, bool BIAS = false>
-__device__ inline void attn_softmax_pv(const AttnArgs& a, int j0, const f32x4_t (&s)[NQ][2], const bf16x8_t (&vf)[D / 16],
-                                       const int (&qpos)[NQ], float (&m)[NQ], float (&l)[NQ], f32x4_t (&o)[NQ][D / 16],
+template <int DV, int NQ, bool MASK, int MODE = MODE_PLAIN>
+__device__ inline void attn_softmax_pv(const AttnArgs& a, int j0, const f32x4_t (&s)[NQ][2], const bf16x8_t (&vf)[DV / 16],
+                                       const int (&qpos)[NQ], float (&m)[NQ], float (&l)[NQ], f32x4_t (&o)[NQ][DV / 16],
                                        const float* __restrict__ bias_row = nullptr) {
   bf16x8_t pf[NQ];
   float alpha[NQ];
   bool moved[NQ];
-  attn_softmax<NQ, MASK, BIAS>(a, j0, s, qpos, m, l, pf, alpha, moved, bias_row);
-  attn_pv<D, NQ>(vf, pf, alpha, moved, o);
+  attn_softmax<NQ, MASK, MODE>(a, j0, s, qpos, m, l, pf, alpha, moved, bias_row);
+  attn_pv<DV, NQ>(vf, pf, alpha, moved, o);
 }
 
-template <int D, int NQ, bool MASK = true, bool BIAS = false>
-__device__ inline void attn_compute(const AttnArgs& a, int j0, const KvFrags<D>& f, const bf16x8_t (&qf)[NQ][D / 32],
-                                    const int (&qpos)[NQ], float (&m)[NQ], float (&l)[NQ], f32x4_t (&o)[NQ][D / 16],
+template <int D, int DV, int NQ, bool MASK = true, int MODE = MODE_PLAIN>
+__device__ inline void attn_compute(const AttnArgs& a, int j0, const KvFrags<D, DV>& f, const bf16x8_t (&qf)[NQ][D / 32],
+                                    const int (&qpos)[NQ], float (&m)[NQ], float (&l)[NQ], f32x4_t (&o)[NQ][DV / 16],
                                     const float* __restrict__ bias_row = nullptr) {
   f32x4_t s[NQ][2];
   attn_scores<D, NQ>(f.k, qf, s);
-  attn_softmax_pv<D, NQ, MASK, BIAS>(a, j0, s, f.v, qpos, m, l, o, bias_row);
+  attn_softmax_pv<DV, NQ, MASK, MODE>(a, j0, s, f.v, qpos, m, l, o, bias_row);
 }
 
-template <int D, int NQ, bool BIAS = false>
+template <int D, int DV, int NQ, int MODE = MODE_PLAIN>
 __device__ inline void attn_step(const AttnArgs& a, const int* __restrict__ table, int kvh, int ctx, int j0,
                                  const bf16x8_t (&qf)[NQ][D / 32], const int (&qpos)[NQ], float (&m)[NQ],
-                                 float (&l)[NQ], f32x4_t (&o)[NQ][D / 16], const float* __restrict__ bias_row = nullptr) {
-  KvFrags<D> f;
-  attn_load<D>(a, table, kvh, ctx, j0, f);
-  attn_compute<D, NQ, true, BIAS>(a, j0, f, qf, qpos, m, l, o, bias_row);
+                                 float (&l)[NQ], f32x4_t (&o)[NQ][DV / 16], const float* __restrict__ bias_row = nullptr) {
+  KvFrags<D, DV> f;
+  attn_load<D, DV>(a, table, kvh, ctx, j0, f);
+  attn_compute<D, DV, NQ, true, MODE>(a, j0, f, qf, qpos, m, l, o, bias_row);
 }
 
 // ---- prefill ----------------------------------------------------------------------------
 // grid: (query blocks of 16*NQ rows, kv_heads * ceil(group / 4), requests); block: 4 waves.
-template <int D, int NQ, bool BIAS = false>
+template <int D, int DV, int NQ, int MODE = MODE_PLAIN>
 __global__ __launch_bounds__(256) void attn_prefill_kernel(AttnArgs a, int skip_single) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int g = lane >> 4, c = lane & 15;
@@ -394,7 +418,7 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(AttnArgs a, int skip_
   bf16x8_t qf[NQ][D / 32];
   int qpos[NQ];
   float m[NQ], l[NQ];
-  f32x4_t o[NQ][D / 16];
+  f32x4_t o[NQ][DV / 16];
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
     const int qi = min(q0 + nq * 16 + c, q_len - 1);  // rows past the end repeat the last one, never written
@@ -405,16 +429,15 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(AttnArgs a, int skip_
     m[nq] = -INFINITY;
     l[nq] = 0.f;
 #pragma unroll
-    for (int dt = 0; dt < D / 16; ++dt) o[nq][dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    for (int dt = 0; dt < DV / 16; ++dt) o[nq][dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
   }
   const int last_pos = pos0 + min(q0 + 16 * NQ, q_len) - 1;
-  int first = 0;
-  if (a.window > 0) first = max(0, pos0 + q0 - a.window + 1) & ~31;
-  const float* bias_row = BIAS ? a.dist_bias + (size_t)head * a.bias_len : nullptr;
+  const int first = max(0, attn_first_key(a, pos0 + q0)) & ~31;
+  const float* bias_row = MODE == MODE_BIAS ? a.dist_bias + (size_t)head * a.bias_len : nullptr;
   // the kept first keys that lie before the window's first step (keys are visited in ascending order either way)
   const int kept_end = min(first, (a.keep_first + 31) & ~31);
-  for (int j0 = 0; j0 < kept_end; j0 += 32) attn_step<D, NQ, BIAS>(a, table, kvh, ctx, j0, qf, qpos, m, l, o, bias_row);
-  for (int j0 = first; j0 <= last_pos; j0 += 32) attn_step<D, NQ, BIAS>(a, table, kvh, ctx, j0, qf, qpos, m, l, o, bias_row);
+  for (int j0 = 0; j0 < kept_end; j0 += 32) attn_step<D, DV, NQ, MODE>(a, table, kvh, ctx, j0, qf, qpos, m, l, o, bias_row);
+  for (int j0 = first; j0 <= last_pos; j0 += 32) attn_step<D, DV, NQ, MODE>(a, table, kvh, ctx, j0, qf, qpos, m, l, o, bias_row);
 
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
@@ -424,9 +447,9 @@ __global__ __launch_bounds__(256) void attn_prefill_kernel(AttnArgs a, int skip_
     const float inv = 1.0f / (lt + sink_term(a.sink, head, m[nq]));
     const int qi = q0 + nq * 16 + c;
     if (qi < q_len) {
-      bf16_t* orow = a.out + ((size_t)(q_start + qi) * a.n_heads + head) * D;
+      bf16_t* orow = a.out + ((size_t)(q_start + qi) * a.n_heads + head) * DV;
 #pragma unroll
-      for (int dt = 0; dt < D / 16; ++dt) {
+      for (int dt = 0; dt < DV / 16; ++dt) {
         // O^T tile: rows d = dt*16 + 4g + r
         uint2 w;
         w.x = pack_bf16(o[nq][dt][0] * inv, o[nq][dt][1] * inv);
@@ -466,18 +489,21 @@ __device__ __host__ inline int portion_parts(int steps, int max_parts, int min_s
 }
 
 #define ATTN_BIAS_LDS 1024   // the longest distance table a wave keeps in LDS
-template <int D, int NQ, int NS = 4, int OCC = 2, bool BIAS = false>
+template <int D, int DV, int NQ, int NS = 4, int OCC = 2, int MODE = MODE_PLAIN>
 __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, int skip_single) {
+  constexpr bool BIAS = MODE == MODE_BIAS, CAP = MODE == MODE_CAP;
   static_assert(!BIAS || NQ == 1, "the distance bias is in the variant of one query tile a wave");
   // (each wave's head has its row of the distance table in LDS: a load from global memory inside the loop would
   // have to wait for every copy into LDS that is in flight)
   __shared__ float bias_lds[BIAS ? 4 * ATTN_BIAS_LDS : 1];
   constexpr int C = D / 8;             // 16-byte chunks per key row
-  constexpr int SH = C == 16 ? 0 : (C == 8 ? 1 : 2);
-  constexpr int KI = D / 16;           // 1 KB loads per key tile (32 rows of 2 D bytes), and per value tile
-  constexpr int LP = 2 * KI / 4;       // loads per wave and step
-  constexpr int STAGE = 2 * KI * 1024;
-  static_assert(D == 32 || D == 64 || D == 128, "head size");
+  constexpr int SH = C == 16 ? 0 : (C == 8 || C == 24 ? 1 : 2);   // (by the row's length modulo the 64 banks)
+  constexpr int KI = D / 16;           // 1 KB loads per key tile (32 rows of 2 D bytes)
+  constexpr int VI = DV / 16;          // and per value tile
+  constexpr int LP = (KI + VI) / 4;    // loads per wave and step
+  constexpr int STAGE = (KI + VI) * 1024;
+  static_assert(D == 32 || D == 64 || D == 128 || D == 192, "head size");
+  static_assert((KI + VI) % 4 == 0 && VI <= 8, "every wave issues the same number of loads");
   __shared__ __attribute__((aligned(1024))) unsigned char stages[NS * STAGE];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int g = lane >> 4, c = lane & 15;
@@ -511,7 +537,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
   bf16x8_t qf[NQ][D / 32];
   int qpos[NQ];
   float m[NQ], l[NQ];
-  f32x4_t o[NQ][D / 16];
+  f32x4_t o[NQ][DV / 16];
 #pragma unroll
   for (int nq = 0; nq < NQ; ++nq) {
     const int qi = min(q0 + nq * 16 + c, q_len - 1);
@@ -522,13 +548,12 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
     m[nq] = -INFINITY;
     l[nq] = 0.f;
 #pragma unroll
-    for (int dt = 0; dt < D / 16; ++dt) o[nq][dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    for (int dt = 0; dt < DV / 16; ++dt) o[nq][dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
   }
   // the block walks the keys that any of its rows sees; a wave masks what its own rows do not see
   const int last_pos = pos0 + min(qb0 + rows_b, q_len) - 1;
   const int last_mine = pos0 + min(q0 + 16 * NQ, q_len) - 1;   // the last query of this wave
-  int first = 0;
-  if (a.window > 0) first = max(0, pos0 + qb0 - a.window + 1) & ~31;
+  int first = max(0, attn_first_key(a, pos0 + qb0)) & ~31;
   int nsteps = (last_pos - first) / 32 + 1;
   const int my_parts = portion_parts(nsteps, a.portion_splits, a.portion_min_steps);
   if (part >= my_parts) return;
@@ -542,6 +567,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
   nsteps += kept_steps;
   auto key0 = [&](int step) { return step < kept_steps ? step * 32 : first + (step - kept_steps) * 32; };
   const int qpos_min = pos0 + min(q0, q_len - 1);   // the earliest query of this wave
+  const int seen_by_all = attn_first_key(a, last_mine);   // from this key on every query of this wave sees what is behind it
   if constexpr (BIAS) {
     for (int i = lane; i < a.bias_len; i += 64) bias_lds[wave * ATTN_BIAS_LDS + i] = a.dist_bias[(size_t)head * a.bias_len + i];
     __syncthreads();
@@ -565,7 +591,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
   auto key_byte = [&](int t) {
     const int row = (64 * t + lane) / C, pc = (64 * t + lane) % C;
     const int f = ((((row >> 3) << 2) | (row & 3)) >> SH);
-    return ((pc - f) & (C - 1)) * 16;
+    return ((pc - f + C) % C) * 16;
   };
   auto value_row = [&](int t) { return 32 * ((t - KI) >> 1) + (lane & 31); };
   unsigned lane_off[LP];   // byte offset of this lane's 16 bytes from the uniform part of a load's address
@@ -585,9 +611,10 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
       row8[i] = 0;
     }
   }
-  const unsigned page_bytes = (unsigned)(a.n_kv * D * ps * 2);   // of a key page, and of a value page
+  const unsigned page_bytes = (unsigned)(a.n_kv * D * ps * 2);      // of a key page
+  const unsigned vpage_bytes = (unsigned)(a.n_kv * DV * ps * 2);    // of a value page
   const unsigned char* kbase = (const unsigned char*)a.k_cache + (size_t)kvh * ps * D * 2;
-  const unsigned char* vbase = (const unsigned char*)a.v_cache + (size_t)kvh * D * ps * 2;
+  const unsigned char* vbase = (const unsigned char*)a.v_cache + (size_t)kvh * DV * ps * 2;
   // the pages of the two halves of the step that is issued next (the second clamped to the last key that exists)
   int pp0 = 0, pp1 = 0;
   auto pages_of = [&](int step) {
@@ -595,7 +622,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
     pp0 = ctab[j0 >> psh];
     pp1 = ctab[min(j0 + 16, (ctx - 1) & ~7) >> psh];
   };
-  auto issue = [&](int step, int stage) {
+  auto issue = [&](int step, int stage) __attribute__((always_inline)) {
     const int j0 = key0(step);
     unsigned char* buf = stages + stage * STAGE;
     if (j0 + 32 <= ctx) {   // all 32 keys exist
@@ -607,7 +634,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
         if (t < KI)
           src = kbase + (size_t)page * page_bytes + (unsigned)(((j0 + row8[i]) & pmask) * D * 2);
         else
-          src = vbase + (size_t)page * page_bytes + (unsigned)(((j0 + (second[i] ? 16 : 0)) & pmask) * 2);
+          src = vbase + (size_t)page * vpage_bytes + (unsigned)(((j0 + (second[i] ? 16 : 0)) & pmask) * 2);
         __builtin_amdgcn_global_load_lds(GPTR(src + lane_off[i]), LPTR(buf + t * 1024), 16, 0, 0);
       }
       return;
@@ -625,7 +652,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
       } else {
         const int kb = min(j0 + (second[i] ? 16 : 0) + 8 * (lane >> 5), (ctx - 1) & ~7);
         const int page = second[i] ? pp1 : pp0;
-        src = (const unsigned char*)(a.v_cache + ((size_t)(page * a.n_kv + kvh) * D + value_row(t)) * ps + (kb & pmask));
+        src = (const unsigned char*)(a.v_cache + ((size_t)(page * a.n_kv + kvh) * DV + value_row(t)) * ps + (kb & pmask));
       }
       __builtin_amdgcn_global_load_lds(GPTR(src), LPTR(buf + t * 1024), 16, 0, 0);
     }
@@ -637,7 +664,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
   for (int t2 = 0; t2 < 2; ++t2) {
     const int row = 8 * (c >> 2) + 4 * t2 + (c & 3);
 #pragma unroll
-    for (int dk = 0; dk < D / 32; ++dk) kaddr[t2][dk] = (row * C + ((dk * 4 + g + (c >> SH)) & (C - 1))) * 16;
+    for (int dk = 0; dk < D / 32; ++dk) kaddr[t2][dk] = (row * C + (dk * 4 + g + (c >> SH)) % C) * 16;
   }
   // value fragment dt of lane (g, c): element 16 dt + c, keys 8 g..: load 2 (dt / 2) + g / 2, place 32 (g % 2) + 16 (dt % 2) + c;
   // eight neighbouring lanes read 128 contiguous bytes
@@ -653,7 +680,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
   // The scores of step s + 1 are multiplied while the softmax of step s runs on the vector ALU (two
   // independent instruction streams for the scheduler to interleave); so step s reads the values of
   // stage s and the keys of stage s + 1, and a stage is free again one step later than it would be.
-  auto read_keys = [&](unsigned base, bf16x8_t (&kf)[2][D / 32]) {
+  auto read_keys = [&](unsigned base, bf16x8_t (&kf)[2][D / 32]) __attribute__((always_inline)) {
     u32x4_t kk[2][D / 32];
 #pragma unroll
     for (int t2 = 0; t2 < 2; ++t2)
@@ -680,7 +707,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
   int stage = 0;
   // one step: `cur` holds this step's scores, the next step's go to `nxt` (the loop below runs two steps per
   // turn with the two sets swapping roles, so that no register is copied)
-  auto step = [&](int s, f32x4_t (&cur)[NQ][2], f32x4_t (&nxt)[NQ][2]) {
+  auto step = [&](int s, f32x4_t (&cur)[NQ][2], f32x4_t (&nxt)[NQ][2]) __attribute__((always_inline)) {
     const int nstage = stage + 1 == NS ? 0 : stage + 1;
     // step s + 1 has landed for this wave (later steps may stay in flight), then for all; every wave
     // is done with the stage of step s - 1
@@ -700,10 +727,10 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
     bf16x8_t pf[NQ];
     float alpha[NQ];
     bool moved[NQ];
-    u32x4_t vv[D / 16];
+    u32x4_t vv[DV / 16];
     const int j0 = key0(s);
-    const bool plain_step = j0 + 31 <= qpos_min && (a.window <= 0 || j0 >= last_mine - a.window + 1);
-#define ATTN_RV(dt) if constexpr (dt < D / 16) vv[dt] = attn_lds_read<(dt >> 1) * 2048 + (dt & 1) * 256>(base + vaddr)
+    const bool plain_step = j0 + 31 <= qpos_min && j0 >= seen_by_all;
+#define ATTN_RV(dt) if constexpr (dt < DV / 16) vv[dt] = attn_lds_read<(dt >> 1) * 2048 + (dt & 1) * 256>(base + vaddr)
 #define ATTN_BODY(NEXT, MASK)                                                                          \
   {                                                                                                    \
     u32x4_t kk[2][D / 32];                                                                             \
@@ -714,13 +741,13 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
     }                                                                                                  \
     ATTN_RV(0); ATTN_RV(1); ATTN_RV(2); ATTN_RV(3); ATTN_RV(4); ATTN_RV(5); ATTN_RV(6); ATTN_RV(7);    \
     float v[NQ][8], m_new[NQ];                                                                         \
-    attn_softmax_max<NQ, MASK>(a, j0, cur, qpos, m, v, m_new);                                         \
+    attn_softmax_max<NQ, MASK, CAP>(a, j0, cur, qpos, m, v, m_new);                                         \
     __builtin_amdgcn_sched_barrier(0);                                                                 \
     if (NEXT) {                                                                                        \
-      /* the key fragments have arrived (the D / 16 value fragments behind them need not) */           \
-      static_assert(D / 16 <= 8, "value fragments of a step");                                         \
-      if constexpr (D == 128) asm volatile("s_waitcnt lgkmcnt(8)" ::: "memory");                       \
-      else if constexpr (D == 64) asm volatile("s_waitcnt lgkmcnt(4)" ::: "memory");                   \
+      /* the key fragments have arrived (the DV / 16 value fragments behind them need not) */           \
+      static_assert(DV / 16 <= 8, "value fragments of a step");                                         \
+      if constexpr (DV == 128) asm volatile("s_waitcnt lgkmcnt(8)" ::: "memory");                       \
+      else if constexpr (DV == 64) asm volatile("s_waitcnt lgkmcnt(4)" ::: "memory");                   \
       else asm volatile("s_waitcnt lgkmcnt(2)" ::: "memory");                                          \
       bf16x8_t kf[2][D / 32];                                                                          \
       _Pragma("unroll") for (int t2 = 0; t2 < 2; ++t2)                                                 \
@@ -730,7 +757,7 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
         }                                                                                              \
       attn_scores<D, NQ>(kf, qf, nxt);                                                                 \
     }                                                                                                  \
-    attn_softmax_exp<NQ>(a, v, m_new, m, l, pf, alpha, moved);                                         \
+    attn_softmax_exp<NQ, CAP>(a, v, m_new, m, l, pf, alpha, moved);                                         \
     if (NEXT) {                                                                                        \
       _Pragma("unroll") for (int i = 0; i < 4 * NQ * (D / 32); ++i) {                                  \
         __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);                                             \
@@ -749,11 +776,11 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
       }
       ATTN_RV(0); ATTN_RV(1); ATTN_RV(2); ATTN_RV(3); ATTN_RV(4); ATTN_RV(5); ATTN_RV(6); ATTN_RV(7);
       if constexpr (BIAS)
-        attn_softmax<NQ, true, true, lds_row_t>(a, j0, cur, qpos, m, l, pf, alpha, moved, bias_row);
+        attn_softmax<NQ, true, MODE_BIAS, lds_row_t>(a, j0, cur, qpos, m, l, pf, alpha, moved, bias_row);
       else if (plain_step)
-        attn_softmax<NQ, false>(a, j0, cur, qpos, m, l, pf, alpha, moved);
+        attn_softmax<NQ, false, MODE>(a, j0, cur, qpos, m, l, pf, alpha, moved);
       else
-        attn_softmax<NQ, true>(a, j0, cur, qpos, m, l, pf, alpha, moved);
+        attn_softmax<NQ, true, MODE>(a, j0, cur, qpos, m, l, pf, alpha, moved);
     } else if (s + 1 < nsteps) {
       if (plain_step) ATTN_BODY(true, false) else ATTN_BODY(true, true)
     } else {
@@ -762,18 +789,18 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
 #undef ATTN_BODY
 #undef ATTN_RV
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    bf16x8_t vf[D / 16];
+    bf16x8_t vf[DV / 16];
 #pragma unroll
-    for (int dt = 0; dt < D / 16; ++dt) {
+    for (int dt = 0; dt < DV / 16; ++dt) {
       asm volatile("" : "+v"(vv[dt]));
       vf[dt] = frag_of(vv[dt]);
     }
     if (j0 + 32 > ctx) {   // the step that holds the last key: places past it are cleared (see attn_existing_keys)
       const u32x4_t keep = attn_existing_keys(ctx - (j0 + 8 * g));
 #pragma unroll
-      for (int dt = 0; dt < D / 16; ++dt) vf[dt] = frag_of(vv[dt] & keep);
+      for (int dt = 0; dt < DV / 16; ++dt) vf[dt] = frag_of(vv[dt] & keep);
     }
-    attn_pv<D, NQ>(vf, pf, alpha, moved, o);
+    attn_pv<DV, NQ>(vf, pf, alpha, moved, o);
     stage = nstage;
   };
   f32x4_t sd[NQ][2];
@@ -790,17 +817,17 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
     const float inv = 1.0f / (lt + sink_term(a.sink, head, m[nq]));   // (used by rows this block writes itself)
     const int qi = q0 + nq * 16 + c;
     if (qi < q_len && my_parts > 1) {
-      float* pr = a.portion_scratch + (((size_t)(q_start + qi) * a.n_heads + head) * a.portion_splits + part) * PART_STRIDE(D);
+      float* pr = a.portion_scratch + (((size_t)(q_start + qi) * a.n_heads + head) * a.portion_splits + part) * PART_STRIDE(DV);
 #pragma unroll
-      for (int dt = 0; dt < D / 16; ++dt) *(f32x4_t*)(pr + dt * 16 + 4 * g) = o[nq][dt];
+      for (int dt = 0; dt < DV / 16; ++dt) *(f32x4_t*)(pr + dt * 16 + 4 * g) = o[nq][dt];
       if (g == 0) {
-        pr[D] = m[nq];
-        pr[D + 1] = lt;
+        pr[DV] = m[nq];
+        pr[DV + 1] = lt;
       }
     } else if (qi < q_len) {
-      bf16_t* orow = a.out + ((size_t)(q_start + qi) * a.n_heads + head) * D;
+      bf16_t* orow = a.out + ((size_t)(q_start + qi) * a.n_heads + head) * DV;
 #pragma unroll
-      for (int dt = 0; dt < D / 16; ++dt) {
+      for (int dt = 0; dt < DV / 16; ++dt) {
         uint2 w;
         w.x = pack_bf16(o[nq][dt][0] * inv, o[nq][dt][1] * inv);
         w.y = pack_bf16(o[nq][dt][2] * inv, o[nq][dt][3] * inv);
@@ -813,15 +840,15 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
 
 // ---- decode -----------------------------------------------------------------------------
 // grid: (kv_heads * ceil(group / 16), requests, splits); block: 4 waves.  Handles requests
-// with exactly one new token.  Scratch per (request, head, split): D floats of O, then max, sum.
+// with exactly one new token.  Scratch per (request, head, split): DV floats of O, then max, sum.
 // (The kv heads run fastest: consecutive blocks go to the eight XCDs in turn, so the heads of every request are
 // spread over all of them and each XCD reads about the same number of bytes however the contexts differ.  With
 // the requests fastest, 60 requests of 128 to 2,304 keys took 77 us where 60 of their mean took 54: the XCD
 // with the longest requests set the time, and more splits changed nothing, since the splits of a (request, head)
 // pair fell to the same XCD.)
-template <int D, bool BIAS = false>
+template <int D, int DV, int MODE = MODE_PLAIN>
 __global__ __launch_bounds__(256) void attn_decode_kernel(AttnArgs a) {
-  __shared__ float red_o[4][D][16];
+  __shared__ float red_o[4][DV][16];
   __shared__ float red_m[4][16], red_l[4][16];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int g = lane >> 4, c = lane & 15;
@@ -841,15 +868,14 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(AttnArgs a) {
   bf16x8_t qf[1][D / 32];
   int qpos[1] = {pos};
   float m[1] = {-INFINITY}, l[1] = {0.f};
-  f32x4_t o[1][D / 16];
+  f32x4_t o[1][DV / 16];
   const bf16_t* qr = a.q + ((size_t)q_start * a.n_heads + head) * D + g * 8;
 #pragma unroll
   for (int dk = 0; dk < D / 32; ++dk) qf[0][dk] = frag_of(*(const u32x4_t*)(qr + dk * 32));
 #pragma unroll
-  for (int dt = 0; dt < D / 16; ++dt) o[0][dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+  for (int dt = 0; dt < DV / 16; ++dt) o[0][dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 
-  int first = 0;
-  if (a.window > 0) first = max(0, pos - a.window + 1) & ~31;
+  const int first = max(0, attn_first_key(a, pos)) & ~31;
   // steps of 32 keys: those of the kept first keys that lie before the window's first step, then the window's
   const int kept_steps = min(first, (a.keep_first + 31) & ~31) / 32;
   const int steps = kept_steps + (ctx - first + 31) / 32;
@@ -857,9 +883,9 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(AttnArgs a) {
   const int s_begin = blockIdx.z * per_split, s_end = min(steps, s_begin + per_split);
   // (Fetching the next step's fragments while this one is computed was measured: the doubled
   // fragment registers halve the occupancy and the kernel gets slower, not faster.)
-  const float* bias_row = BIAS ? a.dist_bias + (size_t)head * a.bias_len : nullptr;   // (a column is a head)
+  const float* bias_row = MODE == MODE_BIAS ? a.dist_bias + (size_t)head * a.bias_len : nullptr;   // (a column is a head)
   for (int s = s_begin + wave; s < s_end; s += 4)
-    attn_step<D, 1, BIAS>(a, table, kvh, ctx, s < kept_steps ? s * 32 : first + (s - kept_steps) * 32, qf, qpos, m, l, o, bias_row);
+    attn_step<D, DV, 1, MODE>(a, table, kvh, ctx, s < kept_steps ? s * 32 : first + (s - kept_steps) * 32, qf, qpos, m, l, o, bias_row);
 
   // merge the four waves (fixed order), then write this split's partial
   float lt = l[0];
@@ -870,11 +896,11 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(AttnArgs a) {
     red_l[wave][c] = lt;
   }
 #pragma unroll
-  for (int dt = 0; dt < D / 16; ++dt)
+  for (int dt = 0; dt < DV / 16; ++dt)
 #pragma unroll
     for (int rr = 0; rr < 4; ++rr) red_o[wave][dt * 16 + 4 * g + rr][c] = o[0][dt][rr];
   __syncthreads();
-  for (int e = threadIdx.x; e < D * 16; e += 256) {
+  for (int e = threadIdx.x; e < DV * 16; e += 256) {
     const int d = e / 16, col = e % 16;
     if (col >= ncols) continue;
     float mg = red_m[0][col];
@@ -890,14 +916,14 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(AttnArgs a) {
     }
     if (a.num_splits == 1) {  // nothing to combine: this is the answer
       lsum += sink_term(a.sink, kvh * group + h0 + col, mu);
-      a.out[((size_t)q_start * a.n_heads + (kvh * group + h0 + col)) * D + d] = float_to_bf16(acc / lsum);
+      a.out[((size_t)q_start * a.n_heads + (kvh * group + h0 + col)) * DV + d] = float_to_bf16(acc / lsum);
       continue;
     }
-    float* part = a.scratch + (((size_t)r * a.n_heads + (kvh * group + h0 + col)) * a.num_splits + blockIdx.z) * (D + 2);
+    float* part = a.scratch + (((size_t)r * a.n_heads + (kvh * group + h0 + col)) * a.num_splits + blockIdx.z) * (DV + 2);
     part[d] = acc;
     if (d == 0) {
-      part[D] = mg;
-      part[D + 1] = lsum;
+      part[DV] = mg;
+      part[DV + 1] = lsum;
     }
   }
 }
@@ -952,7 +978,7 @@ __global__ __launch_bounds__(64) void attn_combine_rows_kernel(const float* __re
                                                                const int* __restrict__ context_lens,
                                                                const int* __restrict__ token_req,
                                                                bf16_t* __restrict__ out, int n_heads, int D,
-                                                               int max_parts, int min_steps, int window, int skip_single,
+                                                               int max_parts, int min_steps, int window, int chunk, int skip_single,
                                                                const float* __restrict__ sink) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int r = token_req[t];
@@ -961,7 +987,8 @@ __global__ __launch_bounds__(64) void attn_combine_rows_kernel(const float* __re
   const int pos0 = context_lens[r] - q_len;
   const int q0 = ((t - q_start) / 32) * 32;
   const int last_pos = pos0 + min(q0 + 32, q_len) - 1;
-  const int first = window > 0 ? (max(0, pos0 + q0 - window + 1) & ~31) : 0;
+  const int seen = chunk > 0 ? (pos0 + q0) / chunk * chunk : (window > 0 ? pos0 + q0 - window + 1 : 0);
+  const int first = max(0, seen) & ~31;
   const int parts = portion_parts((last_pos - first) / 32 + 1, max_parts, min_steps);
   if (parts == 1) return;
   const int stride = PART_STRIDE(D);
@@ -987,20 +1014,29 @@ __global__ __launch_bounds__(64) void attn_combine_rows_kernel(const float* __re
 static int g_attn_tune = 0;   // 1: portions take the kernel that loads keys and values per wave; 2 / 3: 32 / 16 query rows per wave
 extern "C" void tp_attention_tune(int v) { g_attn_tune = v; }
 
-template <int D>
+// MODE: MODE_PLAIN, or MODE_CAP where the scores are capped; a bias by distance (square sizes only) is chosen inside.
+template <int D, int DV, int MODE>
 static int launch_all(AttnArgs a, int n_tokens, int n_req, int max_q_len, int num_single, hipStream_t s) {
   const int group = a.n_heads / a.n_kv;
   const bool has_multi = num_single < n_req;
   const bool bias = a.dist_bias != nullptr;
+  // sizes the kernel through LDS is built for
+  constexpr bool LDS = (D == 32 || D == 64 || D == 128 || D == 192) && (D + DV) % 64 == 0;
+  constexpr bool WITH_BIAS = MODE == MODE_PLAIN && D == DV;
+  // (keys of 192: 32 query rows a wave need more registers than two blocks a CU leave, so only portions whose keys are
+  // split take them, one block a CU; everything else takes 16 rows a wave, two blocks a CU of three 20 KB stages)
+  constexpr bool WIDE = D + DV > 256;
+  constexpr int OCC2 = WIDE ? 1 : 2;     // 32 query rows a wave
+  constexpr int OCC1 = WIDE ? 2 : 3;     // 16 query rows a wave
   if (num_single > 0) {
     const dim3 grid(a.n_kv * ((group + 15) / 16), n_req, a.num_splits);
-    if (bias)
-      hipLaunchKernelGGL((attn_decode_kernel<D, true>), grid, dim3(256), 0, s, a);
-    else
-      hipLaunchKernelGGL(attn_decode_kernel<D>, grid, dim3(256), 0, s, a);
+    if constexpr (WITH_BIAS) {
+      if (bias) hipLaunchKernelGGL((attn_decode_kernel<D, DV, MODE_BIAS>), grid, dim3(256), 0, s, a);
+    }
+    if (!bias) hipLaunchKernelGGL((attn_decode_kernel<D, DV, MODE>), grid, dim3(256), 0, s, a);
     if (a.num_splits > 1) {
       const dim3 cgrid(n_req, a.n_heads);
-      hipLaunchKernelGGL(attn_combine_kernel, cgrid, dim3(64), 0, s, a.scratch, a.cu_seqlens, a.out, a.n_heads, D,
+      hipLaunchKernelGGL(attn_combine_kernel, cgrid, dim3(64), 0, s, a.scratch, a.cu_seqlens, a.out, a.n_heads, DV,
                          a.num_splits, a.sink);
     }
   }
@@ -1015,71 +1051,89 @@ static int launch_all(AttnArgs a, int n_tokens, int n_req, int max_q_len, int nu
     // (blocks of 32 rows that have work: from the rows of the portions, not from the grid, which spans the longest
     // portion for every request; single tokens take the decode kernel)
     const long blocks2 = (long)((n_tokens - num_single + 31) / 32 + (n_req - num_single - 1)) * kv_groups;
-    const bool two = g_attn_tune == 2 || (g_attn_tune != 3 && blocks2 >= 768);
+    const bool two = g_attn_tune == 2 || (g_attn_tune != 3 && blocks2 >= 768 && !WIDE);
     const int rows = two ? 32 : 16;
     const int skip = num_single > 0 ? 1 : 0;
-    if (bias) {
-      // (only the kernel whose waves load their own keys and values has the bias; it never splits a portion's keys)
-      a.portion_splits = 1;
-      if constexpr (D == 32 || D == 64 || D == 128) {
-        // keys and values through LDS, one query tile a wave, the heads' rows of the table in LDS
-        if (g_attn_tune != 1 && a.page_shift >= 4 && a.page_size >= 512 / D && a.bias_len <= ATTN_BIAS_LDS) {
-          const dim3 lgrid((max_q_len + 15) / 16, kv_groups, n_req);
-          hipLaunchKernelGGL((attn_prefill_lds_kernel<D, 1, 3, 3, true>), lgrid, dim3(256), 0, s, a, skip);
-          return 0;
+    const bool lds_pages = g_attn_tune != 1 && a.page_shift >= 4 && a.page_size >= 512 / D;   // (a key load covers 512 / D rows, which must lie in one page)
+    if constexpr (WITH_BIAS) {
+      if (bias) {
+        // (only the kernel whose waves load their own keys and values has the bias; it never splits a portion's keys)
+        a.portion_splits = 1;
+        if constexpr (LDS) {
+          // keys and values through LDS, one query tile a wave, the heads' rows of the table in LDS
+          if (lds_pages && a.bias_len <= ATTN_BIAS_LDS) {
+            const dim3 lgrid((max_q_len + 15) / 16, kv_groups, n_req);
+            hipLaunchKernelGGL((attn_prefill_lds_kernel<D, DV, 1, 3, 3, MODE_BIAS>), lgrid, dim3(256), 0, s, a, skip);
+            return 0;
+          }
         }
+        const dim3 grid((max_q_len + rows - 1) / rows, kv_groups, n_req);
+        if (two)
+          hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 2, MODE_BIAS>), grid, dim3(256), 0, s, a, skip);
+        else
+          hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 1, MODE_BIAS>), grid, dim3(256), 0, s, a, skip);
+        return 0;
       }
-      const dim3 grid((max_q_len + rows - 1) / rows, kv_groups, n_req);
-      if (two)
-        hipLaunchKernelGGL((attn_prefill_kernel<D, 2, true>), grid, dim3(256), 0, s, a, skip);
-      else
-        hipLaunchKernelGGL((attn_prefill_kernel<D, 1, true>), grid, dim3(256), 0, s, a, skip);
-      return 0;
     }
-    if constexpr (D == 32 || D == 64 || D == 128) {
-      if (a.portion_splits > 1 && g_attn_tune != 1 && a.keep_first == 0 && a.page_shift >= 4 && a.page_size >= 512 / D) {
+    if constexpr (LDS) {
+      if (a.portion_splits > 1 && lds_pages && a.keep_first == 0) {
         // few query blocks under a long context: the keys of each are split over blocks (of 32 query rows)
         const dim3 sgrid((max_q_len + 31) / 32, kv_groups, n_req * a.portion_splits);
-        hipLaunchKernelGGL((attn_prefill_lds_kernel<D, 2>), sgrid, dim3(256), 0, s, a, skip);
+        hipLaunchKernelGGL((attn_prefill_lds_kernel<D, DV, 2, 4, OCC2, MODE>), sgrid, dim3(256), 0, s, a, skip);
         hipLaunchKernelGGL(attn_combine_rows_kernel, dim3(n_tokens, a.n_heads), dim3(64), 0, s, a.portion_scratch,
-                           a.cu_seqlens, a.context_lens, a.token_req, a.out, a.n_heads, D, a.portion_splits,
-                           a.portion_min_steps, a.window, skip, a.sink);
+                           a.cu_seqlens, a.context_lens, a.token_req, a.out, a.n_heads, DV, a.portion_splits,
+                           a.portion_min_steps, a.window, a.chunk, skip, a.sink);
         return 0;
       }
     }
     a.portion_splits = 1;   // (the kernels below do not split)
     const dim3 grid((max_q_len + rows - 1) / rows, kv_groups, n_req);
-    if constexpr (D == 32 || D == 64 || D == 128) {
-      // (a key load covers 512 / D rows, which must lie in one page)
-      if (g_attn_tune != 1 && a.page_shift >= 4 && a.page_size >= 512 / D) {
+    if constexpr (LDS) {
+      if (lds_pages) {
         if (group <= 2) {
           // one or two heads a key group: a block takes them all and 4 / group query tiles of each (its four waves
           // share the keys and values of 64 or 128 rows instead of three or two of them idling)
           a.heads_per_block = group;
           const int tiles = 4 / group;
           const long wide2 = (long)((n_tokens - num_single + 32 * tiles - 1) / (32 * tiles) + (n_req - num_single - 1)) * a.n_kv;
-          const bool two_w = g_attn_tune == 2 || (g_attn_tune != 3 && wide2 >= 768);
+          const bool two_w = g_attn_tune == 2 || (g_attn_tune != 3 && wide2 >= 768 && !WIDE);
           const int rows_w = (two_w ? 32 : 16) * tiles;
           const dim3 wgrid((max_q_len + rows_w - 1) / rows_w, a.n_kv, n_req);
           if (two_w)
-            hipLaunchKernelGGL((attn_prefill_lds_kernel<D, 2>), wgrid, dim3(256), 0, s, a, skip);
+            hipLaunchKernelGGL((attn_prefill_lds_kernel<D, DV, 2, 4, OCC2, MODE>), wgrid, dim3(256), 0, s, a, skip);
           else
-            hipLaunchKernelGGL((attn_prefill_lds_kernel<D, 1, 3, 3>), wgrid, dim3(256), 0, s, a, skip);
+            hipLaunchKernelGGL((attn_prefill_lds_kernel<D, DV, 1, 3, OCC1, MODE>), wgrid, dim3(256), 0, s, a, skip);
           return 0;
         }
         if (two)
-          hipLaunchKernelGGL((attn_prefill_lds_kernel<D, 2>), grid, dim3(256), 0, s, a, skip);
+          hipLaunchKernelGGL((attn_prefill_lds_kernel<D, DV, 2, 4, OCC2, MODE>), grid, dim3(256), 0, s, a, skip);
         else
-          hipLaunchKernelGGL((attn_prefill_lds_kernel<D, 1, 3, 3>), grid, dim3(256), 0, s, a, skip);
+          hipLaunchKernelGGL((attn_prefill_lds_kernel<D, DV, 1, 3, OCC1, MODE>), grid, dim3(256), 0, s, a, skip);
         return 0;
       }
     }
     if (two)
-      hipLaunchKernelGGL((attn_prefill_kernel<D, 2>), grid, dim3(256), 0, s, a, skip);
+      hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 2, MODE>), grid, dim3(256), 0, s, a, skip);
     else
-      hipLaunchKernelGGL((attn_prefill_kernel<D, 1>), grid, dim3(256), 0, s, a, skip);
+      hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 1, MODE>), grid, dim3(256), 0, s, a, skip);
   }
   return 0;
+}
+
+// the pairs (key size, value size) that the kernels are built for; ops.FAST_PAIRS names the same ones
+template <int MODE>
+static int launch_sizes(const AttnArgs& a, int d, int dv, int n_tokens, int n_req, int max_q_len, int num_single, hipStream_t s) {
+  switch (d * 1000 + dv) {
+    case 32032: return launch_all<32, 32, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 64064: return launch_all<64, 64, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 96096: return launch_all<96, 96, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 128128: return launch_all<128, 128, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 64032: return launch_all<64, 32, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 128064: return launch_all<128, 64, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 160096: return launch_all<160, 96, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 192128: return launch_all<192, 128, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    default: return -1;
+  }
 }
 
 int tp_paged_attention_fast(const void* q, const void* k_cache, const void* v_cache, const int* block_tables,
@@ -1087,8 +1141,11 @@ int tp_paged_attention_fast(const void* q, const void* k_cache, const void* v_ca
                             int n_req, int n_heads, int n_kv, int head_dim, int page_size, float scale, int window,
                             int max_q_len, int num_single, int num_splits, float* scratch, const int* token_req,
                             int portion_splits, int portion_min_steps, float* portion_scratch, const float* dist_bias,
-                            int bias_len, int keep_first, const float* sink, hipStream_t s) {
-  if (head_dim % 32 != 0 || head_dim > 128 || page_size % 8 != 0) return -1;
+                            int bias_len, int keep_first, const float* sink, int value_dim, int chunk, float softcap,
+                            hipStream_t s) {
+  if (head_dim % 32 != 0 || page_size % 8 != 0) return -1;
+  if (dist_bias != nullptr && (value_dim != head_dim || softcap > 0.f)) return -1;
+  if (chunk < 0 || chunk == 1 || (chunk > 0 && (window > 0 || keep_first > 0))) return -1;
   if (keep_first > 0 && (dist_bias != nullptr || window <= 0)) return -1;
   if (portion_min_steps < 1) return -1;
   if (portion_splits < 1 || portion_splits > 64 || (portion_splits > 1 && (portion_scratch == nullptr || token_req == nullptr))) return -1;
@@ -1125,13 +1182,18 @@ int tp_paged_attention_fast(const void* q, const void* k_cache, const void* v_ca
   a.keep_first = window > 0 ? keep_first : 0;
   if (dist_bias != nullptr && bias_len <= 0) return -1;
   a.scale_log2 = scale * 1.4426950408889634f;
-  switch (head_dim) {
-    case 32: launch_all<32>(a, n_tokens, n_req, max_q_len, num_single, s); break;
-    case 64: launch_all<64>(a, n_tokens, n_req, max_q_len, num_single, s); break;
-    case 96: launch_all<96>(a, n_tokens, n_req, max_q_len, num_single, s); break;
-    case 128: launch_all<128>(a, n_tokens, n_req, max_q_len, num_single, s); break;
-    default: return -1;
+  a.chunk = chunk;
+  a.chunk_shift = 0;
+  a.chunk_mul = 0;
+  if (chunk > 0) {
+    while ((2u << a.chunk_shift) < (unsigned)chunk) ++a.chunk_shift;      // ceil(log2(chunk)) - 1
+    a.chunk_mul = (unsigned)((((unsigned long long)1 << (32 + a.chunk_shift)) + (unsigned)chunk - 1) / (unsigned)chunk);
   }
+  a.cap_log2 = softcap * 1.4426950408889634f;
+  a.cap_in = softcap > 0.f ? 2.0f * 1.4426950408889634f * scale / softcap : 0.f;
+  const int rc = softcap > 0.f ? launch_sizes<MODE_CAP>(a, head_dim, value_dim, n_tokens, n_req, max_q_len, num_single, s)
+                               : launch_sizes<MODE_PLAIN>(a, head_dim, value_dim, n_tokens, n_req, max_q_len, num_single, s);
+  if (rc != 0) return rc;
   TP_CHECK_LAUNCH("paged_attention (mfma)");
   return 0;
 }

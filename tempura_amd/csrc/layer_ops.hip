@@ -72,24 +72,25 @@ extern "C" int tp_embed_bigram(const int* tokens, const int* positions, const in
 }
 
 // ---- gate on a mixer's output -----------------------------------------------------------------
-// out[t, out_col0 + c] = a[t, c] * sigmoid(proj[t, gate_col0 + c]) * scale (no gate: a * scale); the product is
-// formed in float32 and rounded once.
+// out[t, out_col0 + c] = a[t, c] * sigmoid(proj[t, gate_col0 + c / per]) * scale (no gate: a * scale; per 1: a gate per
+// column, per = head size: one per head); the product is formed in float32 and rounded once.
 template <typename T>
 __global__ void sigmoid_gate_kernel(const T* __restrict__ a, const float* __restrict__ proj, int proj_stride, int gate_col0,
-                                    float scale, T* __restrict__ out, int out_stride, int out_col0, int width, size_t total) {
+                                    float scale, T* __restrict__ out, int out_stride, int out_col0, int width, size_t total, int per) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= total) return;
   const size_t t = i / width;
   const int c = (int)(i % width);
   float v = to_float(a[i]);
-  if (proj != nullptr) v *= l_sigmoid(proj[t * proj_stride + gate_col0 + c]);
+  if (proj != nullptr) v *= l_sigmoid(proj[t * proj_stride + gate_col0 + c / per]);
   from_float(out + t * out_stride + out_col0 + c, v * scale);
 }
 
-// the same, four neighbouring columns a thread (every width, stride and first column a multiple of four)
+// the same, four neighbouring columns a thread (every width, stride and first column a multiple of four; per 1 or a
+// multiple of four)
 template <typename T>
 __global__ void sigmoid_gate4_kernel(const T* __restrict__ a, const float* __restrict__ proj, int proj_stride, int gate_col0,
-                                     float scale, T* __restrict__ out, int out_stride, int out_col0, int width, size_t total4) {
+                                     float scale, T* __restrict__ out, int out_stride, int out_col0, int width, size_t total4, int per) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= total4) return;
   const int w4 = width / 4;
@@ -104,7 +105,10 @@ __global__ void sigmoid_gate4_kernel(const T* __restrict__ a, const float* __res
     const float4 raw = *(const float4*)(a + t * width + c);
     v[0] = raw.x; v[1] = raw.y; v[2] = raw.z; v[3] = raw.w;
   }
-  if (proj != nullptr) {
+  if (proj != nullptr && per != 1) {
+    const float g = l_sigmoid(proj[t * proj_stride + gate_col0 + c / per]);
+    v[0] *= g; v[1] *= g; v[2] *= g; v[3] *= g;
+  } else if (proj != nullptr) {
     const float4 g = *(const float4*)(proj + t * proj_stride + gate_col0 + c);
     v[0] *= l_sigmoid(g.x); v[1] *= l_sigmoid(g.y); v[2] *= l_sigmoid(g.z); v[3] *= l_sigmoid(g.w);
   }
@@ -112,32 +116,34 @@ __global__ void sigmoid_gate4_kernel(const T* __restrict__ a, const float* __res
 }
 
 extern "C" int tp_sigmoid_gate(const void* a, int dt, const float* proj, int proj_stride, int gate_col0, float scale, void* out,
-                               int out_stride, int out_col0, int n, int width, hipStream_t s) {
+                               int out_stride, int out_col0, int n, int width, int per, hipStream_t s) {
   TP_REQUIRE(n >= 0 && width > 0 && out_col0 >= 0 && out_stride >= out_col0 + width, "sigmoid_gate: bad sizes");
-  TP_REQUIRE(proj == nullptr || (gate_col0 >= 0 && proj_stride >= gate_col0 + width), "sigmoid_gate: gate rows too short");
+  TP_REQUIRE(per >= 1 && width % per == 0, "sigmoid_gate: %d columns are not runs of %d", width, per);
+  TP_REQUIRE(proj == nullptr || (gate_col0 >= 0 && proj_stride >= gate_col0 + width / per), "sigmoid_gate: gate rows too short");
   TP_REQUIRE(dt == TP_F32 || dt == TP_BF16, "sigmoid_gate: unknown dtype %d", dt);
   if (n == 0) return 0;
   const size_t esz = dt == TP_F32 ? 4 : 2;
-  const bool four = width % 4 == 0 && out_stride % 4 == 0 && out_col0 % 4 == 0 && (proj == nullptr || (proj_stride % 4 == 0 && gate_col0 % 4 == 0)) &&
-                    (uintptr_t)a % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)proj % 16 == 0 && esz * 4 <= 16;
+  const bool four = width % 4 == 0 && out_stride % 4 == 0 && out_col0 % 4 == 0 &&
+                    (proj == nullptr || (per == 1 ? proj_stride % 4 == 0 && gate_col0 % 4 == 0 && (uintptr_t)proj % 16 == 0 : per % 4 == 0)) &&
+                    (uintptr_t)a % 16 == 0 && (uintptr_t)out % 16 == 0 && esz * 4 <= 16;
   if (four) {
     const size_t total4 = (size_t)n * (width / 4);
     const dim3 grid((unsigned)((total4 + 255) / 256));
     if (dt == TP_F32)
       hipLaunchKernelGGL(sigmoid_gate4_kernel<float>, grid, dim3(256), 0, s, (const float*)a, proj, proj_stride, gate_col0, scale,
-                         (float*)out, out_stride, out_col0, width, total4);
+                         (float*)out, out_stride, out_col0, width, total4, per);
     else
       hipLaunchKernelGGL(sigmoid_gate4_kernel<bf16_t>, grid, dim3(256), 0, s, (const bf16_t*)a, proj, proj_stride, gate_col0, scale,
-                         (bf16_t*)out, out_stride, out_col0, width, total4);
+                         (bf16_t*)out, out_stride, out_col0, width, total4, per);
   } else {
     const size_t total = (size_t)n * width;
     const dim3 grid((unsigned)((total + 255) / 256));
     if (dt == TP_F32)
       hipLaunchKernelGGL(sigmoid_gate_kernel<float>, grid, dim3(256), 0, s, (const float*)a, proj, proj_stride, gate_col0, scale,
-                         (float*)out, out_stride, out_col0, width, total);
+                         (float*)out, out_stride, out_col0, width, total, per);
     else
       hipLaunchKernelGGL(sigmoid_gate_kernel<bf16_t>, grid, dim3(256), 0, s, (const bf16_t*)a, proj, proj_stride, gate_col0, scale,
-                         (bf16_t*)out, out_stride, out_col0, width, total);
+                         (bf16_t*)out, out_stride, out_col0, width, total, per);
   }
   TP_CHECK_LAUNCH("sigmoid_gate");
   return 0;
@@ -146,20 +152,36 @@ extern "C" int tp_sigmoid_gate(const void* a, int dt, const float* proj, int pro
 // ---- a sublayer's output, normed, into the residual stream ------------------------------------
 // h[t] += y[t] / sqrt(mean(y[t]^2) + eps) * w; then, with w_next, the next sublayer's input
 // x[t] = h[t] / sqrt(mean(h[t]^2) + eps_next) * w_next as TO.  One block per row.
+// With gate rows, y stands for y[t, c] * sigmoid(gate.rows[t, gate.col0 + c] + gate.bias[c]).
+struct InputGate {
+  const float* rows;   // float32 [n, stride], or nullptr: no gate
+  const float* bias;   // [width], or nullptr
+  size_t stride;
+  int col0;
+};
+
 template <typename TO>
 __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ h, const float* __restrict__ y,
                                                        const float* __restrict__ w, float eps,
                                                        const float* __restrict__ w_next, float eps_next,
-                                                       TO* __restrict__ x, int width) {
+                                                       TO* __restrict__ x, int width, InputGate gate) {
   __shared__ float scratch[32];
   const size_t base = (size_t)blockIdx.x * width;
+  const float* gr = gate.rows != nullptr ? gate.rows + (size_t)blockIdx.x * gate.stride + gate.col0 : nullptr;
+  auto value = [&](int c) {
+    const float v = y[base + c];
+    return gr != nullptr ? v * l_sigmoid(gr[c] + (gate.bias != nullptr ? gate.bias[c] : 0.f)) : v;
+  };
   float ss = 0.f;
-  for (int c = threadIdx.x; c < width; c += blockDim.x) ss = fmaf(y[base + c], y[base + c], ss);
+  for (int c = threadIdx.x; c < width; c += blockDim.x) {
+    const float v = value(c);
+    ss = fmaf(v, v, ss);
+  }
   ss = block_sum(ss, scratch);
   const float rstd = 1.0f / sqrtf(ss / (float)width + eps);
   float ss2 = 0.f;
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
-    const float v = h[base + c] + y[base + c] * rstd * w[c];
+    const float v = h[base + c] + value(c) * rstd * w[c];
     h[base + c] = v;
     ss2 = fmaf(v, v, ss2);
   }
@@ -173,11 +195,11 @@ __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ h, co
 // The same with the row in registers: every value is read once, sixteen bytes a load, all loads of a pass in flight
 // together (width a multiple of four, at most 256 * 4 * NV).  The sums are formed in the generic kernel's order of
 // a thread's own elements only where the widths agree; a row's result never depends on other rows either way.
-template <typename TO, int NV>
+template <typename TO, int NV, bool GATE>
 __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h, const float* __restrict__ y,
                                                            const float* __restrict__ w, float eps,
                                                            const float* __restrict__ w_next, float eps_next,
-                                                           TO* __restrict__ x, int width) {
+                                                           TO* __restrict__ x, int width, InputGate gate) {
   __shared__ float scratch[32];
   const size_t base = (size_t)blockIdx.x * width;
   const int w4 = width / 4;
@@ -190,6 +212,26 @@ __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h
       hv[k] = *(const float4*)(h + base + 4 * c);
       wv[k] = *(const float4*)(w + 4 * c);
     }
+  }
+  if constexpr (GATE) {
+    const float* gr = gate.rows + (size_t)blockIdx.x * gate.stride + gate.col0;
+    float4 gv[NV], bv[NV];
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+      const int c = k * 256 + threadIdx.x;
+      if (c < w4) {
+        gv[k] = *(const float4*)(gr + 4 * c);
+        bv[k] = gate.bias != nullptr ? *(const float4*)(gate.bias + 4 * c) : make_float4(0.f, 0.f, 0.f, 0.f);
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < NV; ++k)
+      if (k * 256 + threadIdx.x < w4) {
+        yv[k].x *= l_sigmoid(gv[k].x + bv[k].x);
+        yv[k].y *= l_sigmoid(gv[k].y + bv[k].y);
+        yv[k].z *= l_sigmoid(gv[k].z + bv[k].z);
+        yv[k].w *= l_sigmoid(gv[k].w + bv[k].w);
+      }
   }
   float ss = 0.f;
 #pragma unroll
@@ -234,34 +276,44 @@ __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h
 }
 
 extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, const float* w_next, float eps_next, void* x,
-                           int x_dt, int n, int width, hipStream_t s) {
+                           int x_dt, int n, int width, const float* gate_rows, size_t gate_stride, int gate_col0,
+                           const float* gate_bias, hipStream_t s) {
   TP_REQUIRE(n >= 0 && width > 0, "norm_add: bad sizes");
+  TP_REQUIRE(gate_rows == nullptr || (gate_col0 >= 0 && gate_stride >= (size_t)gate_col0 + width), "norm_add: gate rows too short");
+  const InputGate gate{gate_rows, gate_bias, gate_stride, gate_col0};
   TP_REQUIRE(w_next == nullptr || x != nullptr, "norm_add: no place for the next rows");
   if (n == 0) return 0;
   TP_REQUIRE(w_next == nullptr || x_dt == TP_F32 || x_dt == TP_BF16, "norm_add: unknown dtype %d", x_dt);
   const bool aligned = ((uintptr_t)h % 16) == 0 && ((uintptr_t)y % 16) == 0 && ((uintptr_t)w % 16) == 0 && ((uintptr_t)w_next % 16) == 0 &&
-                       ((uintptr_t)x % 16) == 0;
+                       ((uintptr_t)x % 16) == 0 &&
+                       (gate_rows == nullptr || (((uintptr_t)gate_rows | (uintptr_t)gate_bias) % 16 == 0 && gate_stride % 4 == 0 && gate_col0 % 4 == 0));
   if (width % 4 == 0 && width >= 1024 && width <= 256 * 4 * 8 && aligned) {
     const bool bf = w_next != nullptr && x_dt == TP_BF16;
-#define NA(NV)                                                                                                                   \
-  do {                                                                                                                           \
-    if (bf)                                                                                                                      \
-      hipLaunchKernelGGL((norm_add_reg_kernel<bf16_t, NV>), dim3(n), dim3(256), 0, s, h, y, w, eps, w_next, eps_next, (bf16_t*)x, width); \
-    else                                                                                                                         \
-      hipLaunchKernelGGL((norm_add_reg_kernel<float, NV>), dim3(n), dim3(256), 0, s, h, y, w, eps, w_next, eps_next, (float*)x, width);   \
+#define NA1(TO, NV, G) \
+  hipLaunchKernelGGL((norm_add_reg_kernel<TO, NV, G>), dim3(n), dim3(256), 0, s, h, y, w, eps, w_next, eps_next, (TO*)x, width, gate)
+#define NA(NV)                                    \
+  do {                                            \
+    if (gate_rows != nullptr) {                   \
+      if (bf) NA1(bf16_t, NV, true);              \
+      else NA1(float, NV, true);                  \
+    } else {                                      \
+      if (bf) NA1(bf16_t, NV, false);             \
+      else NA1(float, NV, false);                 \
+    }                                             \
   } while (0)
     if (width <= 2048) NA(2);
     else if (width <= 4096) NA(4);
     else NA(8);
 #undef NA
+#undef NA1
     TP_CHECK_LAUNCH("norm_add");
     return 0;
   }
   const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
   if (w_next == nullptr || x_dt == TP_F32)
-    hipLaunchKernelGGL(norm_add_kernel<float>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (float*)x, width);
+    hipLaunchKernelGGL(norm_add_kernel<float>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (float*)x, width, gate);
   else if (x_dt == TP_BF16)
-    hipLaunchKernelGGL(norm_add_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (bf16_t*)x, width);
+    hipLaunchKernelGGL(norm_add_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (bf16_t*)x, width, gate);
   else
     TP_REQUIRE(false, "norm_add: unknown dtype %d", x_dt);
   TP_CHECK_LAUNCH("norm_add");
@@ -270,10 +322,14 @@ extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, 
 
 // ---- a plain activation -----------------------------------------------------------------------
 // kind 0: the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))); kind 1: SiLU; kind 2: the exact
-// GELU, 0.5 z (1 + erf(z / sqrt(2))).
+// GELU, 0.5 z (1 + erf(z / sqrt(2))); kind 3: the square of ReLU, max(z, 0)^2.
 __device__ inline float act_f(float z, int kind) {
   if (kind == 0) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
   if (kind == 2) return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
+  if (kind == 3) {
+    const float r = fmaxf(z, 0.f);
+    return r * r;
+  }
   return z * l_sigmoid(z);
 }
 
@@ -292,12 +348,35 @@ __global__ void activation_rows_kernel(const float* __restrict__ in, size_t in_s
   from_float(out + i, v);
 }
 
+// the same without a gate, four neighbouring columns a thread (every width, stride and first column a multiple of four)
+template <typename TO>
+__global__ void activation_rows4_kernel(const float* __restrict__ in, size_t in_stride, int col0, int width, TO* __restrict__ out,
+                                        size_t total4, int kind) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= total4) return;
+  const int w4 = width / 4;
+  const size_t t = i / w4;
+  const float4 z = *(const float4*)(in + t * in_stride + col0 + 4 * (int)(i % w4));
+  from_float4(out + 4 * i, act_f(z.x, kind), act_f(z.y, kind), act_f(z.z, kind), act_f(z.w, kind));
+}
+
 extern "C" int tp_activation_rows(const float* in, size_t in_stride, int col0, int width, int gate_col, void* out, int out_dt, int n,
                                   int kind, hipStream_t s) {
-  TP_REQUIRE(kind >= 0 && kind <= 2, "activation: unknown kind %d", kind);
+  TP_REQUIRE(kind >= 0 && kind <= 3, "activation: unknown kind %d", kind);
   TP_REQUIRE(n >= 0 && width > 0 && col0 >= 0 && (size_t)(col0 + width) <= in_stride && gate_col < (long)in_stride, "activation: bad rows");
   const size_t total = (size_t)n * width;
   if (total == 0) return 0;
+  if (gate_col < 0 && width % 4 == 0 && in_stride % 4 == 0 && col0 % 4 == 0 && (uintptr_t)in % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+      (out_dt == TP_F32 || out_dt == TP_BF16)) {
+    const size_t total4 = total / 4;
+    const dim3 grid4((unsigned)((total4 + 255) / 256));
+    if (out_dt == TP_F32)
+      hipLaunchKernelGGL(activation_rows4_kernel<float>, grid4, dim3(256), 0, s, in, in_stride, col0, width, (float*)out, total4, kind);
+    else
+      hipLaunchKernelGGL(activation_rows4_kernel<bf16_t>, grid4, dim3(256), 0, s, in, in_stride, col0, width, (bf16_t*)out, total4, kind);
+    TP_CHECK_LAUNCH("activation_rows");
+    return 0;
+  }
   const dim3 grid((unsigned)((total + 255) / 256));
   if (out_dt == TP_F32)
     hipLaunchKernelGGL(activation_rows_kernel<float>, grid, dim3(256), 0, s, in, in_stride, col0, width, gate_col, (float*)out, total, kind);
@@ -326,7 +405,7 @@ __global__ void activation4_kernel(const float* __restrict__ in, TO* __restrict_
 }
 
 extern "C" int tp_activation(const void* in, int in_dt, void* out, int out_dt, size_t total, int kind, hipStream_t s) {
-  TP_REQUIRE(kind >= 0 && kind <= 2, "activation: unknown kind %d", kind);
+  TP_REQUIRE(kind >= 0 && kind <= 3, "activation: unknown kind %d", kind);
   if (total == 0) return 0;
   if (in_dt == TP_F32 && total % 4 == 0 && (uintptr_t)in % 16 == 0 && (uintptr_t)out % 16 == 0 && (out_dt == TP_F32 || out_dt == TP_BF16)) {
     const size_t total4 = total / 4;

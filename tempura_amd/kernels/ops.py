@@ -839,6 +839,17 @@ portion_min_keys = 1024
 portion_scratch_limit = 256 << 20
 
 
+#: the pairs (key size, value size) the matrix-core attention kernels are built for
+FAST_PAIRS = ((32, 32), (64, 64), (96, 96), (128, 128), (64, 32), (128, 64), (160, 96), (192, 128))
+
+
+def fast_pair(key_dim: int, value_dim: int, exact_values: bool = True):
+    """The smallest pair of ``FAST_PAIRS`` whose key size is at least ``key_dim`` and whose value size is ``value_dim``
+    (``exact_values`` False: at least ``value_dim``), or None.  A part pads its keys (values) with zeros up to it."""
+    fit = [p for p in FAST_PAIRS if p[0] >= key_dim and (p[1] == value_dim if exact_values else p[1] >= value_dim)]
+    return min(fit, key=lambda p: (p[0] + p[1], p)) if fit else None
+
+
 def fast_attention_takes(has_sink: bool, keep_first: int) -> bool:
     """Whether the matrix-core attention kernels take a softmax with a sink and kept first keys (else the general
     kernel runs, and no splits or partial results are prepared for them): both (kept first keys by the kernels that
@@ -850,15 +861,21 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     cu_seqlens: torch.Tensor, context_lens: torch.Tensor, token_req: torch.Tensor,
                     scale: float, window: int, max_q_len: int, max_context_len: int,
                     num_single: Optional[int] = None, dist_bias: Optional[torch.Tensor] = None,
-                    sink: Optional[torch.Tensor] = None, keep_first: int = 0) -> torch.Tensor:
+                    sink: Optional[torch.Tensor] = None, keep_first: int = 0, chunk: int = 0, softcap: float = 0.0) -> torch.Tensor:
     """q [n, heads, head_dim] over k [pages, kv_heads, page_size, head_dim] and transposed
     v [pages, kv_heads, value_dim, page_size] -> [n, heads * value_dim] (value_dim is the value cache's own; the
-    matrix-core kernels take value_dim == head_dim, other sizes run the general kernel).
+    matrix-core kernels take the pairs of sizes in ``FAST_PAIRS``, other sizes run the general kernel).
     ``dist_bias`` (float32 [heads, L]): added to the scaled score of a query at position p and a key at j as
     dist_bias[head, min(p - j, L - 1)].
     ``sink`` (float32 [heads]): the softmax's denominator holds one more term, exp(sink[head]), without key or value.
-    ``keep_first``: under a window, the request's first ``keep_first`` keys stay visible as well."""
+    ``keep_first``: under a window, the request's first ``keep_first`` keys stay visible as well.
+    ``chunk`` (instead of a window): a query sees the keys of its own aligned chunk of that many positions only.
+    ``softcap`` > 0: a scaled score s becomes softcap * tanh(s / softcap) before the softmax (no distance bias then)."""
     if _backend is not None:
+        if chunk or softcap:
+            return _backend.paged_attention(q, k_cache, v_cache, block_tables, cu_seqlens, context_lens,
+                                            token_req, scale, window, max_q_len, max_context_len, dist_bias=dist_bias,
+                                            sink=sink, keep_first=keep_first, chunk=chunk, softcap=softcap)
         if sink is not None or keep_first:
             return _backend.paged_attention(q, k_cache, v_cache, block_tables, cu_seqlens, context_lens,
                                             token_req, scale, window, max_q_len, max_context_len, dist_bias=dist_bias,
@@ -897,9 +914,14 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         _dev_ok(sink)
         _need(sink.dtype == torch.float32 and sink.numel() == heads, "paged_attention: sink must be float32 [heads]")
     _need(keep_first >= 0, "paged_attention: keep_first must be >= 0")
+    _need(chunk >= 0 and not (chunk and window), "paged_attention: chunks and a window exclude each other")
+    _need(softcap >= 0 and not (softcap and dist_bias is not None), "paged_attention: a cap and a distance bias exclude each other")
+    if chunk == 1:      # (a chunk of one position: the query itself)
+        chunk, window = 0, 1
     if not window:
         keep_first = 0
-    fast = allow_fast_attention and q.dtype == torch.bfloat16 and d % 32 == 0 and d <= 128 and page_size % 8 == 0 and vd == d
+    fast = allow_fast_attention and q.dtype == torch.bfloat16 and (d, vd) in FAST_PAIRS and page_size % 8 == 0
+    fast = fast and (dist_bias is None or d == vd)
     fast = fast and fast_attention_takes(sink is not None, keep_first) and not (keep_first and dist_bias is not None)
     splits, scratch = 1, None
     if fast and num_single > 0:
@@ -931,10 +953,10 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
             bound *= 2
         splits = max(1, min(64, want, bound // 128))
         if splits > 1:
-            scratch = torch.empty((r * heads * splits * (d + 2),), dtype=torch.float32, device=q.device)
+            scratch = torch.empty((r * heads * splits * (vd + 2),), dtype=torch.float32, device=q.device)
     parts, part_scratch = 1, None
     # (the kernel with a distance bias does not split a portion's keys)
-    if fast and dist_bias is None and not keep_first and num_single < r and d in (32, 64, 128) and page_size & (page_size - 1) == 0 and page_size >= max(8, 512 // d):
+    if fast and dist_bias is None and not keep_first and num_single < r and d in (32, 64, 128, 192) and (d + vd) % 64 == 0 and page_size & (page_size - 1) == 0 and page_size >= max(8, 512 // d):
         # Few query blocks under a long context (a portion of a prompt behind a long cached prefix): the keys of
         # every portion are split over blocks until the chip is full (T = 512 behind 7,680 keys: 219 -> 137 us).
         q_blocks = -(-(n - num_single) // 32) + (r - num_single)
@@ -942,15 +964,16 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
         # (a query block is split into at most as many parts as it has portion_min_keys keys: the short blocks
         # of a prompt from an empty cache stay whole)
         parts = max(1, min(16, portion_target_blocks // blocks, max_context_len // portion_min_keys, 65535 // r))
-        if parts > 1 and n * heads * parts * (d + 4) * 4 > portion_scratch_limit:
+        if parts > 1 and n * heads * parts * (vd + 4) * 4 > portion_scratch_limit:
             parts = 1
         if parts > 1:
-            part_scratch = torch.empty((n * heads * parts * (d + 4),), dtype=torch.float32, device=q.device)
+            part_scratch = torch.empty((n * heads * parts * (vd + 4),), dtype=torch.float32, device=q.device)
     _call("tp_paged_attention", _ptr(q), _dt(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables), width,
           _ptr(cu_seqlens), _ptr(context_lens), _ptr(token_req), _ptr(out), n, r, heads, kvh, d, page_size,
           ctypes.c_float(scale), int(window), int(max_q_len), int(max_context_len), int(fast),
           int(num_single), int(splits), _ptr(scratch), int(parts), max(1, portion_min_keys // 32), _ptr(part_scratch),
-          _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1], int(vd), int(keep_first), _ptr(sink), _stream())
+          _ptr(dist_bias), 0 if dist_bias is None else dist_bias.shape[1], int(vd), int(keep_first), _ptr(sink), int(chunk),
+          ctypes.c_float(softcap), _stream())
     return out
 
 
@@ -1252,49 +1275,174 @@ def embed_bigram(tokens: torch.Tensor, table: torch.Tensor, bigram: Optional[tor
     return out
 
 
-def sigmoid_gate(a: torch.Tensor, proj: Optional[torch.Tensor], gate_col0: int, scale: float, out: torch.Tensor, out_col0: int) -> None:
-    """out[:, out_col0 + c] = a[:, c] * sigmoid(proj[:, gate_col0 + c]) * scale (``proj`` float32 rows; None: no
-    gate); ``a`` and ``out`` are of one type, ``out`` [n, wider]."""
+def sigmoid_gate(a: torch.Tensor, proj: Optional[torch.Tensor], gate_col0: int, scale: float, out: torch.Tensor, out_col0: int,
+                 per: int = 1) -> None:
+    """out[:, out_col0 + c] = a[:, c] * sigmoid(proj[:, gate_col0 + c // per]) * scale (``proj`` float32 rows; None: no
+    gate; ``per`` columns in a row share a gate); ``a`` and ``out`` are of one type, ``out`` [n, wider]."""
     if _backend is not None:
+        if per != 1:
+            return _backend.sigmoid_gate(a, proj, gate_col0, scale, out, out_col0, per)
         return _backend.sigmoid_gate(a, proj, gate_col0, scale, out, out_col0)
     _dev_ok(a, proj, out)
     _need(a.dim() == 2 and out.dim() == 2 and a.dtype == out.dtype and a.shape[0] == out.shape[0], "sigmoid_gate: bad operands")
     n, width = a.shape
     _need(0 <= out_col0 and out_col0 + width <= out.shape[1], "sigmoid_gate: output rows too short")
+    _need(per >= 1 and width % per == 0, "sigmoid_gate: columns are no whole runs of per")
     if proj is not None:
-        _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.shape[0] == n and 0 <= gate_col0 and gate_col0 + width <= proj.shape[1],
+        _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.shape[0] == n and 0 <= gate_col0 and gate_col0 + width // per <= proj.shape[1],
               "sigmoid_gate: bad gate rows")
     _call("tp_sigmoid_gate", _ptr(a), _dt(a), _ptr(proj), 0 if proj is None else proj.shape[1], int(gate_col0), ctypes.c_float(scale),
-          _ptr(out), out.shape[1], int(out_col0), n, width, _stream())
+          _ptr(out), out.shape[1], int(out_col0), n, width, int(per), _stream())
+
+
+def turn_gate(a: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor, dim: int, gate: Optional[torch.Tensor] = None,
+              gate_col0: int = 0, cos_sin: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """a [n, heads * dim] with every head's pairs of neighbours (2 m, 2 m + 1) turned by -positions * inv_freq[m], times
+    sigmoid(gate[:, gate_col0 + c]) when ``gate`` (float32 rows) is given; same type.  ``inv_freq`` float64 [dim / 2];
+    ``cos_sin``: this step's table of its angles (``rope_table``)."""
+    if _backend is not None:
+        return _backend.turn_gate(a, positions, inv_freq, dim, gate, gate_col0)
+    _dev_ok(a, positions, inv_freq, gate, cos_sin)
+    _need(a.dim() == 2 and dim > 0 and dim % 2 == 0 and a.shape[1] % dim == 0, "turn_gate: rows must be whole heads of an even size")
+    n, width = a.shape
+    _i32(positions, n, "positions") if n else None
+    _need(inv_freq.dtype == torch.float64 and inv_freq.numel() == dim // 2, "turn_gate: inv_freq must be float64 [dim / 2]")
+    if gate is not None:
+        _need(gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == n and 0 <= gate_col0 and gate_col0 + width <= gate.shape[1],
+              "turn_gate: bad gate rows")
+    if cos_sin is not None:
+        _need(cos_sin.dtype == torch.float32 and tuple(cos_sin.shape) == (n, dim // 2, 2), "turn_gate: table must be float32 [n, dim / 2, 2]")
+    out = torch.empty_like(a)
+    _call("tp_turn_gate", _ptr(a), _dt(a), _ptr(positions), _ptr(inv_freq), _ptr(cos_sin), _ptr(gate),
+          ctypes.c_size_t(0 if gate is None else gate.shape[1]), int(gate_col0), _ptr(out), n, width // dim, int(dim), _stream())
+    return out
+
+
+def _cache_pair(k_cache, v_cache, kv_heads, key_dim, value_dim, what):
+    _need(k_cache.dim() == 4 and v_cache.dim() == 4 and k_cache.shape[1] == kv_heads and k_cache.shape[3] == key_dim
+          and tuple(v_cache.shape) == (k_cache.shape[0], kv_heads, value_dim, k_cache.shape[2]) and v_cache.dtype == k_cache.dtype,
+          f"{what}: caches must be k [pages, {kv_heads}, page_size, {key_dim}], v [pages, {kv_heads}, {value_dim}, page_size] of one type")
+
+
+def _rotation(inv_freq, pairs, cos_sin, n, what):
+    if pairs:
+        _need(inv_freq is not None and inv_freq.dtype == torch.float64 and inv_freq.numel() == pairs, f"{what}: frequencies must be float64 [{pairs}]")
+    if cos_sin is not None:
+        _need(cos_sin.dtype == torch.float32 and tuple(cos_sin.shape) == (n, pairs, 2), f"{what}: table must be float32 [n, {pairs}, 2]")
+
+
+def qkv_rows(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
+             value_dim: int, k_cache: torch.Tensor, v_cache: torch.Tensor, inv_freq: Optional[torch.Tensor] = None, rotary_dim: int = 0,
+             factor: float = 1.0, cos_sin: Optional[torch.Tensor] = None, biases=(None, None, None), norms=None, eps: float = 0.0,
+             value_inv_freq: Optional[torch.Tensor] = None, value_cos_sin: Optional[torch.Tensor] = None,
+             pad_dim: Optional[int] = None) -> torch.Tensor:
+    """Float32 rows [n, q | k | v | any more columns] of a projection, step by step: ``biases`` (float32 per column of q, k,
+    v; each may be None) are added; with ``norms`` (q weight, k weight: float32, one value a column) q and k are divided
+    by the root mean square of the WHOLE projection (all heads together, ``eps`` inside the root) and multiplied by the
+    weight; the pairs of neighbours of the first ``rotary_dim`` elements of q and k heads turn by position *
+    ``inv_freq``; with ``value_inv_freq`` (float64 [value_dim / 2]) the pairs of a value head turn likewise; k and v go
+    to the cache rows ``slots``.  Returns q in the caches' type as [n, heads, pad_dim or head_dim] (keys are stored as
+    wide; zeros behind a head's own elements)."""
+    od = head_dim if pad_dim is None else int(pad_dim)
+    if _backend is not None:
+        return _backend.qkv_rows(rows, positions, slots, num_heads, num_kv_heads, head_dim, value_dim, k_cache, v_cache, inv_freq,
+                                 rotary_dim, factor, biases, norms, eps, value_inv_freq, od)
+    qb, kb, vb = biases
+    qn, kn = norms if norms is not None else (None, None)
+    _dev_ok(rows, positions, slots, k_cache, v_cache, inv_freq, cos_sin, qb, kb, vb, qn, kn, value_inv_freq, value_cos_sin)
+    n = rows.shape[0]
+    widths = (num_heads * head_dim, num_kv_heads * head_dim, num_kv_heads * value_dim)
+    _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.shape[1] >= sum(widths) and rows.shape[1] % 2 == 0,
+          "qkv_rows: rows must be float32 [n, an even width of at least q | k | v]")
+    for b, size, what in ((qb, widths[0], "q bias"), (kb, widths[1], "k bias"), (vb, widths[2], "v bias"), (qn, widths[0], "q norm"),
+                          (kn, widths[1], "k norm")):
+        _need(b is None or (b.dtype == torch.float32 and b.numel() == size), f"qkv_rows: {what} must be float32 with {size} elements")
+    _need((qn is None) == (kn is None), "qkv_rows: the norms of q and k come together")
+    if n:
+        _i32(positions, n, "positions")
+        _i32(slots, n, "slots")
+    _need(head_dim % 2 == 0 and value_dim % 2 == 0 and od >= head_dim and od % 2 == 0, "qkv_rows: head sizes must be even")
+    _need(0 <= rotary_dim <= head_dim and rotary_dim % 2 == 0, "qkv_rows: bad rotary_dim")
+    _cache_pair(k_cache, v_cache, num_kv_heads, od, value_dim, "qkv_rows")
+    _rotation(inv_freq, rotary_dim // 2, cos_sin, n, "qkv_rows")
+    if value_inv_freq is not None:
+        _rotation(value_inv_freq, value_dim // 2, value_cos_sin, n, "qkv_rows: values")
+    q = torch.empty((n, num_heads, od), dtype=k_cache.dtype, device=rows.device)
+    _call("tp_qkv_rows", _ptr(rows), ctypes.c_size_t(rows.shape[1]), _ptr(qb), _ptr(kb), _ptr(vb), _ptr(qn), _ptr(kn), ctypes.c_float(eps),
+          _ptr(positions), _ptr(slots), _ptr(inv_freq), _ptr(cos_sin), int(rotary_dim), ctypes.c_float(factor), _ptr(value_inv_freq),
+          _ptr(value_cos_sin), n, int(num_heads), int(num_kv_heads), int(head_dim), int(value_dim), od, _ptr(q), _ptr(k_cache),
+          _ptr(v_cache), _dt(k_cache), k_cache.shape[2], _stream())
+    return q
+
+
+def latent_rows_write(rows: torch.Tensor, q_col0: int, d_col0: int, weight: torch.Tensor, eps: float, positions: torch.Tensor,
+                      slots: torch.Tensor, inv_freq: Optional[torch.Tensor], factor: float, num_heads: int, rotary_dim: int,
+                      latent_dim: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
+                      cos_sin: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Float32 rows [n, width]: queries at ``q_col0``, per head [rotary_dim | latent_dim] elements, and at ``d_col0`` a latent
+    before its norm [latent_dim] followed by one shared rotated key part [rotary_dim].  The latent is RMS-normed
+    (``weight``, ``eps``), the rotary elements of the queries and of the key part turn (pairs of neighbours, position *
+    ``inv_freq``); the cache rows ``slots`` get keys [rotated | latent | zeros] (one head) and, transposed, values
+    [latent | zeros]; the sizes of both are the caches' own.  Returns q [n, heads, key size], laid out like the keys."""
+    if _backend is not None:
+        return _backend.latent_rows_write(rows, q_col0, d_col0, weight, eps, positions, slots, inv_freq, factor, num_heads, rotary_dim,
+                                          latent_dim, k_cache, v_cache)
+    _dev_ok(rows, weight, positions, slots, inv_freq, k_cache, v_cache, cos_sin)
+    n, key = rows.shape[0], rotary_dim + latent_dim
+    _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.shape[1] % 2 == 0 and q_col0 >= 0 and q_col0 % 2 == 0 and d_col0 >= 0
+          and q_col0 + num_heads * key <= rows.shape[1] and d_col0 + key <= rows.shape[1], "latent_rows_write: bad rows")
+    _need(weight.dtype == torch.float32 and weight.numel() == latent_dim, "latent_rows_write: weight must be float32 [latent_dim]")
+    _need(k_cache.dim() == 4 and v_cache.dim() == 4, "latent_rows_write: bad caches")
+    od, vd = k_cache.shape[3], v_cache.shape[2]
+    _need(rotary_dim % 2 == 0 and key % 2 == 0 and od >= key and od % 2 == 0 and vd >= latent_dim, "latent_rows_write: bad head sizes")
+    _cache_pair(k_cache, v_cache, 1, od, vd, "latent_rows_write")
+    _rotation(inv_freq, rotary_dim // 2, cos_sin, n, "latent_rows_write")
+    if n:
+        _i32(positions, n, "positions")
+        _i32(slots, n, "slots")
+    q = torch.empty((n, num_heads, od), dtype=k_cache.dtype, device=rows.device)
+    _call("tp_latent_rows_write", _ptr(rows), ctypes.c_size_t(rows.shape[1]), int(q_col0), int(d_col0), _ptr(weight), ctypes.c_float(eps),
+          _ptr(positions), _ptr(slots), _ptr(inv_freq), _ptr(cos_sin), ctypes.c_float(factor), n, int(num_heads), int(rotary_dim),
+          int(latent_dim), od, vd, _ptr(q), _ptr(k_cache), _ptr(v_cache), _dt(k_cache), k_cache.shape[2], _stream())
+    return q
 
 
 def norm_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, next_weight: Optional[torch.Tensor] = None,
-             next_eps: float = 0.0, out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
+             next_eps: float = 0.0, out_dtype: Optional[torch.dtype] = None, gate: Optional[torch.Tensor] = None, gate_col0: int = 0,
+             gate_bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """h += y / sqrt(mean(y^2) + eps) * weight, per row, in place (float32 [n, width]).  With ``next_weight`` the
-    rows of the new h normed with it (and ``next_eps``) come back as ``out_dtype``."""
+    rows of the new h normed with it (and ``next_eps``) come back as ``out_dtype``.  With ``gate`` (float32 rows [n,
+    wider]) y is first multiplied by sigmoid(gate[:, gate_col0 + c] + gate_bias[c])."""
     if _backend is not None:
+        if gate is not None:
+            return _backend.norm_add(h, y, weight, eps, next_weight, next_eps, out_dtype, gate, gate_col0, gate_bias)
         return _backend.norm_add(h, y, weight, eps, next_weight, next_eps, out_dtype)
-    _dev_ok(h, y, weight, next_weight)
+    _dev_ok(h, y, weight, next_weight, gate, gate_bias)
     _need(h.dtype == torch.float32 and h.dim() == 2 and y.dtype == torch.float32 and tuple(y.shape) == tuple(h.shape),
           "norm_add: h and y must be float32 [n, width]")
     n, width = h.shape
     _need(weight.dtype == torch.float32 and weight.numel() == width, "norm_add: weight must be float32 [width]")
+    if gate is not None:
+        _need(gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == n and 0 <= gate_col0 and gate_col0 + width <= gate.shape[1],
+              "norm_add: bad gate rows")
+        _need(gate_bias is None or (gate_bias.dtype == torch.float32 and gate_bias.numel() == width), "norm_add: gate bias must be float32 [width]")
     x = None
     if next_weight is not None:
         _need(next_weight.dtype == torch.float32 and next_weight.numel() == width and out_dtype is not None, "norm_add: bad next norm")
         x = torch.empty((n, width), dtype=out_dtype, device=h.device)
     _call("tp_norm_add", _ptr(h), _ptr(y), _ptr(weight), ctypes.c_float(eps), _ptr(next_weight), ctypes.c_float(next_eps), _ptr(x),
-          _dtcode(out_dtype) if x is not None else _F32, n, width, _stream())
+          _dtcode(out_dtype) if x is not None else _F32, n, width, _ptr(gate), ctypes.c_size_t(0 if gate is None else gate.shape[1]),
+          int(gate_col0), _ptr(gate_bias), _stream())
     return x
 
 
-ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "gelu_erf": 2}
+ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "gelu_erf": 2, "relu2": 3}
 
 
 def activation(u: torch.Tensor, kind: str, out_dtype: torch.dtype, col0: int = 0, width: Optional[int] = None,
                gate_col: Optional[int] = None) -> torch.Tensor:
     """Element by element: ``gelu_tanh`` (0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))), ``gelu_erf``
-    (0.5 z (1 + erf(z / sqrt(2)))) or ``silu``, formed in float32, as ``out_dtype``.
+    (0.5 z (1 + erf(z / sqrt(2)))), ``relu2`` (max(z, 0)^2) or ``silu``, formed in float32, as ``out_dtype``.
     With ``width`` (``u`` float32 rows [n, wider]): the columns col0 .. col0 + width of every row, and with ``gate_col``
     each row's results times the sigmoid of that column of the row."""
     _need(kind in ACTIVATIONS, f"activation: {kind!r} unknown (known: {sorted(ACTIVATIONS)})")

@@ -22,8 +22,20 @@ The first two need a position encoding that does not rotate (``"none"``).
 * ``value_dim``: the values of a head have another size than its keys;
 * ``sink`` (tensor ``sink`` [heads]): the softmax's denominator holds one more term exp(sink[head]) that has no key
   and no value;
+  A number instead of True: every head's sink has that score, and there is no tensor;
 * ``keep_first``: under a ``window`` a query also sees the request's first ``keep_first`` keys (their pages stay held).
-The last four run without projection biases, own values, and a rows-in-float32 projection (no split norm).
+The last four run with own values and a rows-in-float32 projection (no split norm).
+* ``chunk`` (instead of ``window``): a query sees the keys of its own aligned chunk of that many positions, counted from
+  the request's start; pages of finished chunks go back to the pool;
+* ``softcap``: a scaled score s becomes softcap * tanh(s / softcap);
+* ``gate``: the concatenated heads are multiplied by sigmoid(W_g x) (tensor ``gate``) before the output projection.
+Between the projection and the cache, in this order (``bias``, this form of ``qk_norm`` and ``value_position`` select one
+kernel that does all of it on the projection's float32 rows, ``ops.qkv_rows``):
+* ``bias`` with values of their own: q, k and v have biases (tensors ``q_bias``, ``k_bias``, ``v_bias``);
+* ``qk_norm`` with ``over: "projection"``: q is divided by the root mean square of the whole q projection, all heads
+  together, and multiplied by its weight (one value per row of the projection); k likewise;
+* ``value_position``: a rotary position part over ``value_dim`` elements that turns the values by their own positions
+  before they are cached; every head's output is turned back by the query's position (in front of the gate).
 """
 from __future__ import annotations
 
@@ -33,7 +45,8 @@ from dataclasses import dataclass
 import torch
 
 from ..kernels import ops
-from .base import BranchMixer, CacheSpec, Mixer, WeightInfo, build_part, part_class, register_part
+from .base import BranchMixer, CacheSpec, Mixer, WeightInfo, build_part, pad_rows, part_class, register_part
+from .rope import paired_order, reorder_heads
 
 
 def log_bucket(n: int, buckets: int, max_distance: int) -> int:
@@ -65,6 +78,7 @@ class PagedAttention(Mixer):
     preferred_portion_align = 8
     split_norm = True      # takes rows whose norm its first product finishes; prepares the next norm in its last
     returns_output = True  # with ``residual`` None the output comes back instead of being added
+    takes_side_rows = True  # (behind the gate's rows, or behind q | k | v where one kernel reads the projection's rows)
 
     def __init__(self, spec, hidden_size, dtype, device):
         super().__init__(spec, hidden_size, dtype, device)
@@ -87,32 +101,55 @@ class PagedAttention(Mixer):
         self.distance_bias = p.get("distance_bias")
         if self.distance_bias is not None and self.distance_bias.get("kind") != "log_buckets":
             raise ValueError(f"attention: distance bias {self.distance_bias.get('kind')!r} unknown (known: log_buckets)")
-        if (self.has_bias or self.values_are_keys) and self.position.rotary() is not None:
-            raise ValueError("attention: projection biases and values that are the keys need a position encoding that does not rotate")
-        if self.has_bias and not self.values_are_keys:
-            raise ValueError("attention: projection biases are supported together with values that are the keys")
+        if self.values_are_keys and self.position.rotary() is not None:
+            raise ValueError("attention: values that are the keys need a position encoding that does not rotate")
         #: q and k come straight from the projection (biases added, keys stored as keys and as values): no rotation kernel
         self.plain_qk = self.values_are_keys
         self.qk_norm = p.get("qk_norm")
         self.value_dim = int(p.get("value_dim") or self.head_dim)
-        self.has_sink = bool(p.get("sink", False))
+        sink = p.get("sink", False)
+        self.has_sink = sink is not None and sink is not False
+        #: the score of every head's sink when it is a constant (None: a tensor holds the scores)
+        self.sink_score = float(sink) if self.has_sink and sink is not True else None
         self.keep_first = int(p.get("keep_first") or 0)
         if self.keep_first < 0 or (self.keep_first and self.window is None):
             raise ValueError("attention: keep_first needs a window and must not be negative")
+        self.chunk = int(p.get("chunk") or 0)
+        self.softcap = float(p.get("softcap") or 0.0)
+        if self.chunk < 0 or self.softcap < 0 or (self.chunk and self.window is not None):
+            raise ValueError("attention: chunks exclude a window; chunk and softcap must not be negative")
+        if self.softcap and self.distance_bias is not None:
+            raise ValueError("attention: a softcap and a distance bias do not combine")
+        self.gate = bool(p.get("gate", False))
+        over = self.qk_norm.get("over", "head") if self.qk_norm is not None else "head"
+        if over not in ("head", "projection"):
+            raise ValueError(f"attention: qk_norm over {over!r} unknown (known: head, projection)")
+        vp = p.get("value_position")
+        self.value_position = None if vp is None else build_part("position", vp, hidden_size, dtype, device)
+        if vp is not None and (self.value_position.rotary() is None or self.value_position.rotary()[1] != self.value_dim
+                               or self.value_position.factor != 1.0):
+            raise ValueError("attention: value_position must turn all value_dim elements, without a factor")
+        #: biases, the norm over the whole projection and turned values are one kernel on the projection's rows
+        self.rows_path = (self.has_bias and not self.values_are_keys) or over == "projection" or vp is not None
+        if self.rows_path and self.qk_norm is not None and over == "head":
+            raise ValueError("attention: a norm per head does not combine with biases on own values or turned values")
         #: the options that take the projection's float32 rows through kernels of their own
-        self.extended = self.qk_norm is not None or self.value_dim != self.head_dim or self.has_sink or self.keep_first > 0
-        if self.extended and (self.plain_qk or self.has_bias or self.distance_bias is not None):
-            raise ValueError("attention: qk_norm, value_dim, sink and keep_first do not combine with biases, values that are the keys "
-                             "or a distance bias")
+        self.extended = self.rows_path or self.qk_norm is not None or self.value_dim != self.head_dim or self.has_sink or self.keep_first > 0
+        if self.extended and (self.plain_qk or self.distance_bias is not None):
+            raise ValueError("attention: qk_norm, value_dim, sink, keep_first, biases on own values and turned values do not combine with "
+                             "values that are the keys or a distance bias")
         self.v_dim = self.num_kv_heads * self.value_dim
-        # values wider than keys, of a size the matrix-core attention kernels take: q and the cached keys get zeros
-        # behind their own elements up to the values' size (no score changes), so that those kernels serve
+        # sizes the matrix-core attention kernels take once q and the cached keys have zeros behind their own elements
+        # (no score changes): keys narrower than values, or than the key size of a pair that the kernels are built for
         self.key_dim = self.head_dim
-        if (dtype == torch.bfloat16 and self.head_dim < self.value_dim <= 128 and self.value_dim % 32 == 0 and self.head_dim % 2 == 0
+        pair = ops.fast_pair(self.head_dim, self.value_dim)
+        if (self.extended and dtype == torch.bfloat16 and pair is not None and self.head_dim % 2 == 0
                 and ops.fast_attention_takes(self.has_sink, self.keep_first)):
-            self.key_dim = self.value_dim
+            self.key_dim = pair[0]
         self.split_norm = not self.plain_qk and not self.extended      # (these projections take finished rows only)
         self.q_norm_w = self.k_norm_w = self.sink_w = None
+        self.v_bias = None
+        self.w_gates = None        # rows of the gate and side rows, where they are no part of wqkv
         self.wqkv = None
         self.wo = None
         self.q_bias = self.k_bias = self.dist_table = None
@@ -132,13 +169,18 @@ class PagedAttention(Mixer):
             out[w["v"]] = WeightInfo((p["num_kv_heads"] * vd, hidden_size))
         out[w["o"]] = WeightInfo((hidden_size, p["num_heads"] * vd))
         if p.get("qk_norm") is not None:
-            out[w["q_norm"]] = WeightInfo((p["head_dim"],), "ones")
-            out[w["k_norm"]] = WeightInfo((p["head_dim"],), "ones")
-        if p.get("sink", False):
+            whole = p["qk_norm"].get("over", "head") == "projection"
+            out[w["q_norm"]] = WeightInfo((q_dim if whole else p["head_dim"],), "ones")
+            out[w["k_norm"]] = WeightInfo((kv_dim if whole else p["head_dim"],), "ones")
+        if p.get("sink", False) is True:
             out[w["sink"]] = WeightInfo((p["num_heads"],))
         if p.get("bias", False):
             out[w["q_bias"]] = WeightInfo((q_dim,))
             out[w["k_bias"]] = WeightInfo((kv_dim,))
+            if p.get("values", "own") != "keys":
+                out[w["v_bias"]] = WeightInfo((p["num_kv_heads"] * vd,))
+        if p.get("gate", False):
+            out[w["gate"]] = WeightInfo((p["num_heads"] * vd, hidden_size))
         if p.get("distance_bias") is not None:
             # (the number of rows is the tensor's own; a configuration may name it for random weights)
             out[w["distance_bias"]] = WeightInfo((p["distance_bias"].get("buckets"), p["num_heads"]))
@@ -153,49 +195,76 @@ class PagedAttention(Mixer):
         product's epilogue can rotate what it holds).  q and k are permuted alike, which leaves every score
         as it was; the cache then holds keys in this order."""
         rot = self.position.rotary()
-        if rot is None or rot[1] == 0:
+        if rot is None:
             return t
-        rd, half, d = rot[1], rot[1] // 2, self.head_dim
-        order = torch.arange(d)
-        order[0:rd:2] = torch.arange(half)
-        order[1:rd:2] = torch.arange(half) + half
-        heads = t.shape[0] // d
-        return t.view(heads, d, -1)[:, order.to(t.device), :].reshape(t.shape)
+        return reorder_heads(t, self.head_dim, paired_order(self.head_dim, rot[1], getattr(self.position, "layout", "halves")))
+
+    def _paired_values(self, t: torch.Tensor) -> torch.Tensor:
+        """The rows of a value projection (its bias, the gate's rows) with every head's elements in the order in which
+        turned values are kept."""
+        if self.value_position is None:
+            return t
+        return reorder_heads(t, self.value_dim, paired_order(self.value_dim, self.value_dim, self.value_position.layout))
 
     def load_weights(self, get):
         w = self.spec.weights
         if self.has_bias:
-            self.q_bias = self._to_device(get(w["q_bias"]), torch.float32)
-            self.k_bias = self._to_device(get(w["k_bias"]), torch.float32)
+            self.q_bias = self._to_device(self._paired(get(w["q_bias"])), torch.float32)
+            self.k_bias = self._to_device(self._paired(get(w["k_bias"])), torch.float32)
+            if not self.values_are_keys:
+                self.v_bias = self._to_device(self._paired_values(get(w["v_bias"])), torch.float32)
         if self.distance_bias is not None:
             self.dist_table = self._to_device(distance_table(get(w["distance_bias"]), int(self.distance_bias["max_distance"]),
                                                              self.window), torch.float32)
         # One [q_dim + 2 kv_dim, hidden] matrix: one product instead of three.
         parts = [self._paired(get(w["q"])), self._paired(get(w["k"]))]
         if not self.values_are_keys:
-            parts.append(get(w["v"]))
+            parts.append(self._paired_values(get(w["v"])))
+        # what else reads the same input: the gate's rows, then the side rows.  Where one kernel takes the projection's
+        # rows anyway they are columns of the same product; else (the projection may rotate and store in its epilogue)
+        # they are a product of their own.
+        beside = [self._paired_values(get(w["gate"]))] if self.gate else []
+        if self.side_rows is not None:
+            beside.append(self.side_rows)
+            self.side_rows = True
+        self.gate_col0 = self.q_dim + self.kv_dim + self.v_dim if self.rows_path else 0
+        self.side_col0 = self.gate_col0 + (self.num_heads * self.value_dim if self.gate else 0)
+        if self.rows_path:
+            parts, beside = parts + beside, []
+        rows = torch.cat([self._to_device(t) for t in parts], dim=0).contiguous()
         # (stored tiled where the sizes allow: the products then read whole cache lines)
-        self.wqkv = ops.tile_weight(torch.cat([self._to_device(t) for t in parts], dim=0).contiguous())
-        self.wo = ops.tile_weight(self._to_device(get(w["o"])))
+        self.wqkv = ops.tile_weight(pad_rows(rows, 16) if self.rows_path else rows)
+        if beside:
+            self.w_gates = ops.tile_weight(pad_rows(torch.cat([self._to_device(t) for t in beside], dim=0), 16))
+        wo = get(w["o"])
+        if self.value_position is not None:
+            wo = self._paired_values(wo.t()).t()
+        self.wo = ops.tile_weight(self._to_device(wo))
         if self.qk_norm is not None:
-            self.q_norm_w = self._to_device(get(w["q_norm"]), torch.float32)
-            self.k_norm_w = self._to_device(get(w["k_norm"]), torch.float32)
-        if self.has_sink:
+            whole = self.rows_path
+            self.q_norm_w = self._to_device(self._paired(get(w["q_norm"])) if whole else get(w["q_norm"]), torch.float32)
+            self.k_norm_w = self._to_device(self._paired(get(w["k_norm"])) if whole else get(w["k_norm"]), torch.float32)
+        if self.sink_score is not None:
+            self.sink_w = torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=self.device)
+        elif self.has_sink:
             self.sink_w = self._to_device(get(w["sink"]), torch.float32)
         self.position.load_weights(get)
 
     def cache_spec(self):
-        kind = "window" if self.window is not None else "full"
+        kind, span = ("window", self.window) if self.window is not None else ("chunk", self.chunk) if self.chunk else ("full", None)
         if self.keep_first:
             return SizedValueCacheSpec("window_keep_first", self.num_kv_heads, self.key_dim, self.window, self.value_dim, self.keep_first)
         if self.value_dim != self.key_dim:
-            return SizedValueCacheSpec(kind, self.num_kv_heads, self.key_dim, self.window, self.value_dim)
-        return CacheSpec(kind, self.num_kv_heads, self.key_dim, self.window)
+            return SizedValueCacheSpec(kind, self.num_kv_heads, self.key_dim, span, self.value_dim)
+        return CacheSpec(kind, self.num_kv_heads, self.key_dim, span)
 
     def forward(self, x, ctx, cache, residual, next_norm=None):
         rot = self.position.rotary()
         q = None
-        if self.plain_qk:
+        gates = None       # float32 rows that hold the gate's and the side rows' columns
+        if self.rows_path:
+            q, gates = self._project_rows(x, ctx, cache, rot)
+        elif self.plain_qk:
             q = self._project_plain(x, ctx, cache)
         elif rot is not None and cache.writes and not self.extended:
             rows = x.x if isinstance(x, ops.Prenormed) else x
@@ -207,11 +276,13 @@ class PagedAttention(Mixer):
                                        self.num_heads, self.num_kv_heads, self.head_dim, cache.k, cache.v, table)
         if q is None:
             q = self._project_and_rotate(x, ctx, cache, rot)
-        if self.extended:
+        if self.w_gates is not None:
+            gates = ops.linear(x, self.w_gates, torch.float32)
+        if self.extended or self.chunk or self.softcap:
             a = ops.paged_attention(
                 q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.cu_seqlens, ctx.context_lens,
                 ctx.token_req, self.scale, int(self.window or 0), ctx.max_q_len, ctx.max_context_len,
-                ctx.num_single, sink=self.sink_w, keep_first=self.keep_first)
+                ctx.num_single, sink=self.sink_w, keep_first=self.keep_first, chunk=self.chunk, softcap=self.softcap)
         elif self.dist_table is not None:
             a = ops.paged_attention(
                 q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.cu_seqlens, ctx.context_lens,
@@ -222,12 +293,38 @@ class PagedAttention(Mixer):
                 q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.cu_seqlens, ctx.context_lens,
                 ctx.token_req, self.scale, int(self.window or 0), ctx.max_q_len, ctx.max_context_len,
                 ctx.num_single)
+        if self.value_position is not None:
+            vp = self.value_position
+            a = ops.turn_gate(a, ctx.positions, vp.inv_freq, self.value_dim, gates if self.gate else None, self.gate_col0, vp.table(ctx))
+        elif self.gate:
+            gated = torch.empty_like(a)
+            ops.sigmoid_gate(a, gates, self.gate_col0, 1.0, gated, 0)
+            a = gated
+        if self.side_rows is not None:
+            if residual is not None:
+                raise ValueError("attention: with side rows the output comes back, it is not added")
+            return ops.linear(a, self.wo, torch.float32), (gates, self.side_col0)
         if residual is None:
             return ops.linear(a, self.wo, torch.float32)
         if next_norm is None:
             ops.linear(a, self.wo, torch.float32, residual=residual)
             return None
         return ops.linear(a, self.wo, torch.float32, residual=residual, next_norm=next_norm)[1]
+
+    def _project_rows(self, x, ctx, cache, rot):
+        """(q, the product's float32 rows): biases, the norm over the whole projection, rotation of q, k and v and the
+        cache write are one kernel behind one product, whose columns behind q | k | v are the gate's and the side rows'."""
+        if not cache.writes:
+            raise ValueError("attention: a projection with biases, a norm over all heads or turned values writes its own cache")
+        rows = ops.linear(x, self.wqkv, torch.float32)
+        inv_freq, rotary_dim, factor = rot if rot is not None else (None, 0, 1.0)
+        vp = self.value_position
+        q = ops.qkv_rows(rows, ctx.positions, ctx.slot_mapping[cache.group], self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
+                         cache.k, cache.v, inv_freq, rotary_dim, factor, self.position.table(ctx) if rot is not None else None,
+                         (self.q_bias, self.k_bias, self.v_bias), None if self.qk_norm is None else (self.q_norm_w, self.k_norm_w),
+                         0.0 if self.qk_norm is None else float(self.qk_norm["eps"]), None if vp is None else vp.inv_freq,
+                         None if vp is None else vp.table(ctx), self.key_dim)
+        return q, rows
 
     def _project_plain(self, x, ctx, cache):
         """q ([n, heads, head_dim]) of a projection without rotation: biases added, k stored as keys and, when the
@@ -599,3 +696,105 @@ class LatentCacheAttention(BranchMixer):
 
 
 register_part("mixer", "latent_cache_attention", LatentCacheAttention)
+
+
+class RotaryLatentAttention(BranchMixer):
+    """Softmax attention over one cached latent a token (as ``LatentCacheAttention``) beside a rotated key part that all
+    heads share.  With H = ``num_heads``, per head D = ``head_dim`` unrotated and R = ``rotary_dim`` rotated query/key
+    elements, values of Dv = ``value_dim`` and a latent of L = ``latent_dim``:
+
+        q = W_q x, per head [D unrotated | R rotated]      (no latent of the queries' own)
+        W_dkv x has L + R rows: c = rmsnorm(first L) * w_dkv, the last R (not normed) are the shared rotated key part
+        k_h = W_uk[h] c    v_h = W_uv[h] c    score = (q_plain . k_h + q_rot . k_rot) * ``scale``
+
+    causal, or under a ``window``; ``gate: "head"`` multiplies head h's output by sigmoid(W_g x)_h; then W_o on the
+    concatenated heads.  The position part turns the R rotated elements.
+
+    Only c and the rotated part are cached: keys [R rotated | L latent] of one head, values [L latent], both with zeros
+    behind up to a pair of sizes that the matrix-core attention kernels take (bfloat16).  W_uk and W_uv are folded into the
+    ends, formed once at load in float64: the queries' rows W_uk[h]^T W_q[h, :D] (L a head, beside the R rotated ones) and
+    the output's columns W_o[:, h] W_uv[h].  A head's gate is one number, so it may multiply the sum over the latents.
+
+    The columns of its input product are [q | latent | rotated key part | gate]; it keeps no per-request state."""
+
+    def __init__(self, spec, hidden_size, dtype, device):
+        super().__init__(spec, hidden_size, dtype, device)
+        p = spec.params
+        self.num_heads = int(p["num_heads"])
+        self.head_dim = int(p["head_dim"])
+        self.rotary_dim = int(p["rotary_dim"])
+        self.value_dim = int(p["value_dim"])
+        self.latent_dim = int(p["latent_dim"])
+        self.scale = float(p["scale"])
+        self.norm_eps = float(p["norm_eps"])
+        self.window = p.get("window")
+        gate = p.get("gate")
+        if gate not in (None, "head"):
+            raise ValueError(f"rotary_latent_attention: gate {gate!r} unknown (known: head)")
+        self.gate = gate == "head"
+        self.position = build_part("position", p["position"], hidden_size, dtype, device)
+        rot = self.position.rotary()
+        if (rot[1] if rot is not None else 0) != self.rotary_dim:
+            raise ValueError("rotary_latent_attention: the position part must turn exactly the rotated elements")
+        if self.rotary_dim <= 0 or self.rotary_dim % 2 != 0 or self.latent_dim % 2 != 0:
+            raise ValueError("rotary_latent_attention: rotary_dim and latent_dim must be positive and even")
+        key = self.rotary_dim + self.latent_dim
+        pair = ops.fast_pair(key, self.latent_dim, exact_values=False) if dtype == torch.bfloat16 else None
+        #: sizes of a cached key and of a cached value
+        self.cached_key, self.cached_value = pair if pair is not None else (key, self.latent_dim)
+        self.q_cols = self.num_heads * key
+        self.inner = self.num_heads * self.cached_value
+
+    @classmethod
+    def expected_weights(cls, spec, hidden_size):
+        p, w = spec.params, spec.weights
+        H, D, R, Dv, L = (int(p[k]) for k in ("num_heads", "head_dim", "rotary_dim", "value_dim", "latent_dim"))
+        out = {w["q"]: WeightInfo((H * (D + R), hidden_size)), w["dkv"]: WeightInfo((L + R, hidden_size)), w["dkv_norm"]: WeightInfo((L,), "ones"),
+               w["uk"]: WeightInfo((H * D, L)), w["uv"]: WeightInfo((H * Dv, L)), w["o"]: WeightInfo((hidden_size, H * Dv))}
+        if p.get("gate") is not None:
+            out[w["gate"]] = WeightInfo((H, hidden_size))
+        out.update(part_class("position", p["position"].kind).expected_weights(p["position"], hidden_size))
+        return out
+
+    def cache_spec(self):
+        kind = "window" if self.window is not None else "full"
+        if self.cached_value == self.cached_key:
+            return CacheSpec(kind, 1, self.cached_key, self.window)
+        return SizedValueCacheSpec(kind, 1, self.cached_key, self.window, self.cached_value)
+
+    def load_branch(self, get):
+        w = self.spec.weights
+        H, D, R, Dv, L = self.num_heads, self.head_dim, self.rotary_dim, self.value_dim, self.latent_dim
+        f64 = lambda name: get(w[name]).to(torch.float64)
+        q, uk, uv, o = f64("q").view(H, D + R, -1), f64("uk").view(H, D, L), f64("uv").view(H, Dv, L), f64("o").view(-1, H, Dv)
+        order = paired_order(R, R, getattr(self.position, "layout", "halves"))
+        latent_q = torch.matmul(uk.transpose(1, 2).contiguous(), q[:, :D].contiguous())
+        rot_q = reorder_heads(q[:, D:].reshape(H * R, -1), R, order).view(H, R, -1)
+        rows = [self._to_device(torch.cat([rot_q, latent_q], dim=1).reshape(H * (R + L), -1))]
+        dkv = get(w["dkv"])
+        rows.append(self._to_device(torch.cat([dkv[:L], reorder_heads(dkv[L:], R, order)], dim=0)))
+        if self.gate:
+            rows.append(self._to_device(get(w["gate"])))
+        # columns h V .. (h + 1) V, V the cached values' size: W_o[:, h] W_uv[h], zeros for the padding
+        out = torch.matmul(o.transpose(0, 1).contiguous(), uv)                      # [H, hidden, L]
+        out = torch.nn.functional.pad(out, (0, self.cached_value - L)).transpose(0, 1).reshape(-1, self.inner)
+        self.latent_norm_w = self._to_device(get(w["dkv_norm"]), torch.float32)
+        self.position.load_weights(get)
+        return torch.cat(rows, dim=0).contiguous(), self._to_device(out)
+
+    def run(self, proj, col0, ctx, cache, out, out_col0, scale):
+        if not cache.writes:
+            raise ValueError("rotary_latent_attention: a call that reads another call's cache is not supported")
+        rot = self.position.rotary()
+        inv_freq, _, factor = rot if rot is not None else (None, 0, 1.0)
+        table = self.position.table(ctx) if hasattr(self.position, "table") else None
+        d_col0 = col0 + self.q_cols
+        q = ops.latent_rows_write(proj, col0, d_col0, self.latent_norm_w, self.norm_eps, ctx.positions, ctx.slot_mapping[cache.group],
+                                  inv_freq, factor, self.num_heads, self.rotary_dim, self.latent_dim, cache.k, cache.v, table)
+        a = ops.paged_attention(q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.cu_seqlens, ctx.context_lens, ctx.token_req,
+                                self.scale, int(self.window or 0), ctx.max_q_len, ctx.max_context_len, ctx.num_single)
+        ops.sigmoid_gate(a, proj if self.gate else None, d_col0 + self.latent_dim + self.rotary_dim, scale, out, out_col0,
+                         self.cached_value if self.gate else 1)
+
+
+register_part("mixer", "rotary_latent_attention", RotaryLatentAttention)

@@ -93,6 +93,16 @@ class Part:
     def load_weights(self, get: Callable[[str], torch.Tensor]) -> None:
         """Fetch tensors by checkpoint name (``get`` returns them on the host as stored)."""
 
+    #: True: ``take_side_rows`` may hand the part rows of another weight that reads the same input (a gate on the part's
+    #: result, say); they ride along in one of the part's own input products
+    takes_side_rows = False
+    side_rows = None
+
+    def take_side_rows(self, rows: torch.Tensor) -> None:
+        """Called before ``load_weights`` with rows [r, hidden].  ``forward`` (with ``residual`` None) then returns the pair
+        (output, (float32 rows, first column)): the r products of these rows with the input, from that column on."""
+        self.side_rows = rows
+
     def _to_device(self, t: torch.Tensor, dtype: Optional[torch.dtype] = None) -> torch.Tensor:
         return t.to(device=self.device, dtype=dtype or self.dtype).contiguous()
 
@@ -132,6 +142,7 @@ class BranchMixer(Mixer):
 
     graph_safe = True
     returns_output = True      # with ``residual`` None the output comes back instead of being added
+    takes_side_rows = True     # (behind the branch's own columns of the input product)
     inner = 0
     state_off = 0
 
@@ -151,6 +162,9 @@ class BranchMixer(Mixer):
     def load_weights(self, get):
         from ..kernels import ops
         w_in, w_out = self.load_branch(get)
+        self.side_col0 = w_in.shape[0]
+        if self.side_rows is not None:
+            w_in, self.side_rows = torch.cat([w_in, self.side_rows], dim=0), True
         self.w_in = ops.tile_weight(pad_rows(w_in, 16))
         self.w_out = ops.tile_weight(w_out)
 
@@ -159,7 +173,8 @@ class BranchMixer(Mixer):
         proj = ops.linear(x, self.w_in, torch.float32)
         act = torch.empty((proj.shape[0], self.inner), dtype=self.dtype, device=proj.device)
         self.run(proj, 0, ctx, cache, act, 0, 1.0)
-        return ops.linear(act, self.w_out, torch.float32, residual=residual)
+        y = ops.linear(act, self.w_out, torch.float32, residual=residual)
+        return y if self.side_rows is None else (y, (proj, self.side_col0))
 
 
 def pad_rows(w: torch.Tensor, multiple: int) -> torch.Tensor:

@@ -214,21 +214,75 @@ class HyperBlock(ArrangedBlock):
 register_part("block", "hyper", HyperBlock)
 
 
+class InputGate(Part):
+    """What multiplies a sublayer's result y element by element: sigmoid(W x + b), x being the sublayer's input.  The
+    rows of W ride along in the sublayer's own input product where its part takes them (``Part.take_side_rows``), else
+    they are a product of their own; bias, sigmoid and multiplication are the closing kernel's."""
+    category = "gate"
+    graph_safe = True
+
+    @classmethod
+    def expected_weights(cls, spec, hidden_size):
+        w = spec.weights
+        return {w["weight"]: WeightInfo((hidden_size, hidden_size)), w["bias"]: WeightInfo((hidden_size,))}
+
+    def load_for(self, part, get):
+        """Load the tensors and hand the rows to ``part`` if it takes them (before ``part`` loads its own)."""
+        w = self.spec.weights
+        rows = self._to_device(get(w["weight"]))
+        self.bias = self._to_device(get(w["bias"]), torch.float32)
+        self.weight = None
+        if getattr(part, "takes_side_rows", False):
+            part.take_side_rows(rows)
+        else:
+            self.weight = ops.tile_weight(rows)
+
+    def split(self, x, result):
+        """(the sublayer's output, float32 rows of the gate before bias and sigmoid, their first column)."""
+        if self.weight is None:
+            y, (rows, col0) = result
+            return y, rows, col0
+        return result, ops.linear(x, self.weight, torch.float32), 0
+
+
+class LayerScale(Part):
+    """A vector that multiplies what a sublayer adds to the stream, element by element."""
+    category = "scale"
+    graph_safe = True
+
+    @classmethod
+    def expected_weights(cls, spec, hidden_size):
+        return {spec.weights["weight"]: WeightInfo((hidden_size,), "ones")}
+
+    def load_weights(self, get):
+        self.weight = self._to_device(get(self.spec.weights["weight"]), torch.float32)
+
+
+register_part("gate", "input_sigmoid", InputGate)
+register_part("scale", "vector", LayerScale)
+
+
 class SandwichBlock(ArrangedBlock):
     """A norm before and a norm behind each sublayer: ``h += post(mixer(pre(h)))``, then, when the layer has a
     feed-forward, ``h += post(ffn(pre(h)))``.  A constant that multiplies what enters the stream is the ``scale`` of
     the norm behind the sublayer.  The norms behind the sublayers are RMS norms; one kernel norms a sublayer's
     output, adds it into the stream and norms the stream for the next sublayer, also across layers (``entry_norm``
-    says what the block before needs for that)."""
-    ROLES = {"mixer_norm": "norm", "mixer": "mixer", "mixer_post_norm": "norm",
-             "ffn_norm": "norm", "ffn": "ffn", "ffn_post_norm": "norm"}
-    OPTIONAL = frozenset({"ffn_norm", "ffn", "ffn_post_norm"})
+    says what the block before needs for that).
+
+    Each sublayer may have a gate (``InputGate``: its result times a sigmoid of its input, in front of the norm behind
+    it) and a layer scale (a vector behind that norm, multiplied into the norm's weight once, when they are loaded):
+    ``h += scale * post(gate(pre(h)) * mixer(pre(h)))``.  Both belong to the same kernel."""
+    ROLES = {"mixer_norm": "norm", "mixer": "mixer", "mixer_post_norm": "norm", "mixer_gate": "gate", "mixer_scale": "scale",
+             "ffn_norm": "norm", "ffn": "ffn", "ffn_post_norm": "norm", "ffn_gate": "gate", "ffn_scale": "scale"}
+    OPTIONAL = frozenset({"ffn_norm", "ffn", "ffn_post_norm", "mixer_gate", "mixer_scale", "ffn_gate", "ffn_scale"})
     handoff = "sandwich"
 
     def __init__(self, layer_spec, hidden_size, dtype, device):
         super().__init__(layer_spec, hidden_size, dtype, device)
         if len({self.ffn is None, self.ffn_norm is None, self.ffn_post_norm is None}) != 1:
             raise ValueError("block 'sandwich': a feed-forward and its two norms come together")
+        if self.ffn is None and (self.ffn_gate is not None or self.ffn_scale is not None):
+            raise ValueError("block 'sandwich': a gate or a scale without a feed-forward")
         for post in (self.mixer_post_norm, self.ffn_post_norm):
             if post is not None and (type(post).__name__ != "RMSNorm" or getattr(post, "groups", 1) != 1):
                 raise ValueError("block 'sandwich': the norm behind a sublayer must be an RMS norm")
@@ -254,13 +308,28 @@ class SandwichBlock(ArrangedBlock):
         part.forward(*args, y)
         return y
 
-    def _close(self, h, y, post, opening):
-        """Norm ``y``, add it into the stream; with ``opening`` (weight, eps) also return the stream normed for the
-        next sublayer."""
-        if opening is None:
-            ops.norm_add(h, y, post.weight, post.eps)
-            return None
-        return ops.norm_add(h, y, post.weight, post.eps, opening[0], opening[1], self.dtype)
+    def load_weights(self, get):
+        for name in ("mixer", "ffn"):
+            gate = getattr(self, name + "_gate")
+            if gate is not None:
+                gate.load_for(getattr(self, name), get)
+        super().load_weights(get)
+        #: what multiplies a sublayer's normed result, by sublayer: the norm's weight times the layer scale
+        self.closing = {}
+        for name in ("mixer", "ffn"):
+            post, scale = getattr(self, name + "_post_norm"), getattr(self, name + "_scale")
+            if post is not None:
+                self.closing[name] = post.weight if scale is None else (post.weight.double() * scale.weight.double()).to(torch.float32)
+
+    def _close(self, h, x, result, name, opening):
+        """Gate and norm the result of sublayer ``name`` (``x`` its input), add it into the stream; with ``opening``
+        (weight, eps) also return the stream normed for the next sublayer."""
+        gate, weight, eps = getattr(self, name + "_gate"), self.closing[name], getattr(self, name + "_post_norm").eps
+        after = (None, 0.0, None) if opening is None else (opening[0], opening[1], self.dtype)
+        if gate is not None:
+            y, rows, col0 = gate.split(x, result)
+            return ops.norm_add(h, y, weight, eps, *after, gate=rows, gate_col0=col0, gate_bias=gate.bias)
+        return ops.norm_add(h, result, weight, eps, *after)
 
     def forward(self, h, ctx, cache, x=None, next_norm=None):
         n = h.shape[0]
@@ -269,12 +338,12 @@ class SandwichBlock(ArrangedBlock):
         y = self._run(self.mixer, x, ctx, cache, n, h.device)
         after = next_norm if isinstance(next_norm, tuple) else None
         if self.ffn is None:
-            return self._close(h, y, self.mixer_post_norm, after)
-        x2 = self._close(h, y, self.mixer_post_norm, self._rms(self.ffn_norm))
+            return self._close(h, x, y, "mixer", after)
+        x2 = self._close(h, x, y, "mixer", self._rms(self.ffn_norm))
         if x2 is None:
             x2 = self.ffn_norm.forward(h)
         y2 = self._run(self.ffn, x2, ctx, None, n, h.device)
-        return self._close(h, y2, self.ffn_post_norm, after)
+        return self._close(h, x2, y2, "ffn", after)
 
 
 register_part("block", "sandwich", SandwichBlock)

@@ -106,9 +106,10 @@ class GatedFFN(FeedForward):
 
 
 class DenseMLP(FeedForward):
-    """``down(act(up(x)))`` without a gate; ``activation`` names the function (``gelu_tanh``, ``silu``), which reads
-    the float32 sums of the up product."""
+    """``down(act(up(x)))`` without a gate; ``activation`` names the function (``ops.ACTIVATIONS``: ``gelu_tanh``, ``silu``,
+    ``relu2``, ..), which reads the float32 sums of the up product."""
     graph_safe = True
+    takes_side_rows = True     # (behind the up product's own columns)
     returns_output = True      # with ``residual`` None the output comes back instead of being added
 
     def __init__(self, spec, hidden_size, dtype, device):
@@ -126,11 +127,18 @@ class DenseMLP(FeedForward):
 
     def load_weights(self, get):
         w = self.spec.weights
-        self.w_up = ops.tile_weight(self._to_device(get(w["up"])))
+        up = self._to_device(get(w["up"]))
+        if self.side_rows is not None:
+            from .base import pad_rows
+            up, self.side_rows = pad_rows(torch.cat([up, self.side_rows], dim=0), 16), True
+        self.w_up = ops.tile_weight(up)
         self.w_down = ops.tile_weight(self._to_device(get(w["down"])))
 
     def forward(self, x, ctx, residual=None):
         u = ops.linear(x, self.w_up, torch.float32)
+        if self.side_rows is not None:
+            a = ops.activation(u, self.activation, self.dtype, 0, self.intermediate_size)
+            return ops.linear(a, self.w_down, torch.float32, residual=residual), (u, self.intermediate_size)
         a = ops.activation(u, self.activation, self.dtype)
         return ops.linear(a, self.w_down, torch.float32, residual=residual)
 

@@ -5,6 +5,7 @@ mean square; the weight spans the whole row.
 
 ``weight_offset`` (default 0) serves checkpoints that store the weight around zero: with 1.0 the stored tensor is
 the deviation from one.  The offset is added once, in float32, when the weight is loaded.
+``scalar`` (default False): the stored weight is ONE number, the same for every element of the row.
 ``scale`` (default 1) multiplies the result: a norm behind a sublayer whose output enters the residual stream
 times a constant carries the constant here (the weight is multiplied once, when it is loaded).
 
@@ -37,11 +38,14 @@ class RMSNorm(Norm):
     def expected_weights(cls, spec, hidden_size):
         # (a weight stored around zero is drawn like any other tensor, one stored around one as ones)
         init = "normal" if float(spec.params.get("weight_offset", 0.0)) != 0.0 else "ones"
-        return {spec.weights["weight"]: WeightInfo((hidden_size,), init)}
+        return {spec.weights["weight"]: WeightInfo(() if spec.params.get("scalar", False) else (hidden_size,), init)}
 
     def load_weights(self, get):
         # Norm weights are tiny and multiply in float32: keep them in float32.
-        self.weight = self._to_device(get(self.spec.weights["weight"]), torch.float32)
+        w = get(self.spec.weights["weight"])
+        if self.spec.params.get("scalar", False):
+            w = w.reshape(1).expand(self.hidden_size)      # (the kernels read a weight per element)
+        self.weight = self._to_device(w, torch.float32)
         if self.weight_offset != 0.0:
             self.weight = (self.weight.double() + self.weight_offset).to(torch.float32)
         if self.scale != 1.0:

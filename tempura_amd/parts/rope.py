@@ -8,7 +8,10 @@ float64 on the host.  The YaRN rule (``type: "yarn"`` with ``factor``, ``origina
 each frequency f_i with f_i / factor by a ramp over the pair index: with
 c(t) = D ln(original / (2 pi t)) / (2 ln theta), lo = max(floor(c(fast)), 0), hi = min(ceil(c(slow)), D - 1) and
 ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1) the frequency is f_i / factor * ramp_i + f_i (1 - ramp_i); what
-multiplies cosine and sine is the part's ``attn_factor``.  Kernels form the angle from the integer position in 64-bit
+multiplies cosine and sine is the part's ``attn_factor``.
+``layout`` says which elements of a checkpoint's heads form pair i: ``"halves"`` (the default; i and i + D/2) or
+``"neighbours"`` (2 i and 2 i + 1).  The kernels turn neighbours; ``paired_order`` is the order of a head's elements that
+brings a checkpoint's pairs side by side.  Kernels form the angle from the integer position in 64-bit
 and take sine and cosine of it, so no precision is lost at large positions.
 """
 from __future__ import annotations
@@ -63,6 +66,29 @@ def rotary_inv_freq(head_dim: int, theta: float, scaling=None, rotary_dim=None) 
     return out
 
 
+LAYOUTS = ("halves", "neighbours")
+
+
+def paired_order(size: int, rotary_dim: int, layout: str = "halves"):
+    """int64 [size]: element i of a head as the kernels keep it is element order[i] of the checkpoint's, so that the two
+    elements that turn together are neighbours; None when the checkpoint has them so already."""
+    if rotary_dim == 0 or layout == "neighbours":
+        return None
+    half = rotary_dim // 2
+    order = torch.arange(size)
+    order[0:rotary_dim:2] = torch.arange(half)
+    order[1:rotary_dim:2] = torch.arange(half) + half
+    return order
+
+
+def reorder_heads(t: torch.Tensor, size: int, order):
+    """Rows [heads * size, ...] with every head's ``size`` rows in ``order`` (None: as they are)."""
+    if order is None:
+        return t
+    heads = t.shape[0] // size
+    return t.reshape(heads, size, -1)[:, order.to(t.device), :].reshape(t.shape)
+
+
 class RotaryPosition(PositionEncoding):
     def __init__(self, spec, hidden_size, dtype, device):
         super().__init__(spec, hidden_size, dtype, device)
@@ -70,6 +96,9 @@ class RotaryPosition(PositionEncoding):
         self.head_dim = int(p["head_dim"])
         self.rotary_dim = int(p.get("rotary_dim") or self.head_dim)
         self.factor = float(p.get("attn_factor", 1.0))
+        self.layout = str(p.get("layout", "halves"))
+        if self.layout not in LAYOUTS:
+            raise ValueError(f"rope: layout {self.layout!r} unknown (known: {', '.join(LAYOUTS)})")
         inv_freq = rotary_inv_freq(self.head_dim, float(p["theta"]), p.get("scaling"), self.rotary_dim)
         self.inv_freq = inv_freq.to(device)
         # layers whose rotations have the same frequencies share one table per step

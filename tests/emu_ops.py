@@ -257,7 +257,8 @@ class EmuOps:
         return q
 
     def paged_attention(self, q, k_cache, v_cache, block_tables, cu_seqlens, context_lens, token_req, scale,
-                        window, max_q_len, max_context_len, num_single=None, dist_bias=None, sink=None, keep_first=0):
+                        window, max_q_len, max_context_len, num_single=None, dist_bias=None, sink=None, keep_first=0, chunk=0,
+                        softcap=0.0):
         n, heads, d = q.shape
         kvh, ps = k_cache.shape[1], k_cache.shape[2]
         group = heads // kvh
@@ -274,11 +275,13 @@ class EmuOps:
             V = v_cache[rows_page, :, :, rows_off].double()      # [ctx, kvh, d]
             for t in range(qs, qe):
                 pos = ctx - (qe - qs) + (t - qs)
-                lo = max(0, pos - window + 1) if window > 0 else 0
+                lo = max(0, pos - window + 1) if window > 0 else (pos // chunk * chunk if chunk > 0 else 0)
                 # (the keys a query sees: the window, and under a window the request's first keep_first keys)
                 seen = torch.cat([torch.arange(0, min(keep_first, lo) if window > 0 else 0), torch.arange(lo, pos + 1)])
                 for h in range(heads):
                     sc = (K[seen, h // group] @ q[t, h].double()) * scale
+                    if softcap:
+                        sc = softcap * torch.tanh(sc / softcap)
                     if dist_bias is not None:
                         dist = torch.clamp(pos - seen, max=dist_bias.shape[1] - 1)
                         sc = sc + dist_bias[h].double()[dist]
@@ -311,14 +314,75 @@ class EmuOps:
                 prev_state[slot] = int(tokens[cu[r + 1] - 1])
         return out.to(torch.float32)
 
-    def sigmoid_gate(self, a, proj, gate_col0, scale, out, out_col0):
+    def sigmoid_gate(self, a, proj, gate_col0, scale, out, out_col0, per=1):
         v = a.double()
         if proj is not None:
-            v = v * torch.sigmoid(proj.double()[:, gate_col0: gate_col0 + a.shape[1]])
+            v = v * torch.sigmoid(proj.double()[:, gate_col0: gate_col0 + a.shape[1] // per]).repeat_interleave(per, dim=1)
         out[:, out_col0: out_col0 + a.shape[1]] = (v * scale).to(out.dtype)
 
-    def norm_add(self, h, y, weight, eps, next_weight=None, next_eps=0.0, out_dtype=None):
+    @staticmethod
+    def _turned(x, positions, inv_freq, dims, sign=1.0):
+        """x [n, heads, d]: pairs of neighbours of the first ``dims`` elements turned by sign * position * inv_freq."""
+        x = x.clone()
+        if dims:
+            ang = sign * positions.double()[:, None, None] * inv_freq.double()[None, None, :]
+            a, b = x[..., 0:dims:2].clone(), x[..., 1:dims:2].clone()
+            x[..., 0:dims:2] = a * torch.cos(ang) - b * torch.sin(ang)
+            x[..., 1:dims:2] = a * torch.sin(ang) + b * torch.cos(ang)
+        return x
+
+    def turn_gate(self, a, positions, inv_freq, dim, gate=None, gate_col0=0):
+        n, width = a.shape
+        v = self._turned(a.double().reshape(n, width // dim, dim), positions, inv_freq, dim, -1.0).reshape(n, width)
+        if gate is not None:
+            v = v * torch.sigmoid(gate.double()[:, gate_col0: gate_col0 + width])
+        return v.to(a.dtype)
+
+    def qkv_rows(self, rows, positions, slots, num_heads, num_kv_heads, head_dim, value_dim, k_cache, v_cache, inv_freq, rotary_dim,
+                 factor, biases, norms, eps, value_inv_freq, pad_dim):
+        n = rows.shape[0]
+        widths = [num_heads * head_dim, num_kv_heads * head_dim, num_kv_heads * value_dim]
+        q, k, v = rows.double()[:, : sum(widths)].split(widths, dim=1)
+        q, k, v = (x if b is None else x + b.double() for x, b in zip((q, k, v), biases))
+        if norms is not None:
+            q, k = (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w.double() for x, w in zip((q, k), norms))
+        q = q.reshape(n, num_heads, head_dim)
+        k = k.reshape(n, num_kv_heads, head_dim)
+        v = v.reshape(n, num_kv_heads, value_dim)
+        q, k = self._turned(q, positions, inv_freq, rotary_dim), self._turned(k, positions, inv_freq, rotary_dim)
+        q[..., :rotary_dim] *= factor
+        k[..., :rotary_dim] *= factor
+        if value_inv_freq is not None:
+            v = self._turned(v, positions, value_inv_freq, value_dim)
+        pad = (0, pad_dim - head_dim)
+        ps = k_cache.shape[2]
+        page, off = slots.long() // ps, slots.long() % ps
+        k_cache[page, :, off] = torch.nn.functional.pad(k, pad).to(k_cache.dtype)
+        v_cache[page, :, :, off] = v.to(v_cache.dtype)
+        return torch.nn.functional.pad(q, pad).to(k_cache.dtype).contiguous()
+
+    def latent_rows_write(self, rows, q_col0, d_col0, weight, eps, positions, slots, inv_freq, factor, num_heads, rotary_dim, latent_dim,
+                          k_cache, v_cache):
+        n, key = rows.shape[0], rotary_dim + latent_dim
+        q = rows.double()[:, q_col0: q_col0 + num_heads * key].reshape(n, num_heads, key)
+        x = rows.double()[:, d_col0: d_col0 + key]
+        c = x[:, :latent_dim]
+        c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * weight.double()
+        k = torch.cat([x[:, latent_dim:], c], dim=1)[:, None, :]
+        q, k = self._turned(q, positions, inv_freq, rotary_dim), self._turned(k, positions, inv_freq, rotary_dim)
+        q[..., :rotary_dim] *= factor
+        k[..., :rotary_dim] *= factor
+        ps, od, vd = k_cache.shape[2], k_cache.shape[3], v_cache.shape[2]
+        page, off = slots.long() // ps, slots.long() % ps
+        k_cache[page, :, off] = torch.nn.functional.pad(k, (0, od - key)).to(k_cache.dtype)
+        v_cache[page, 0, :, off] = torch.nn.functional.pad(c, (0, vd - latent_dim)).to(v_cache.dtype)
+        return torch.nn.functional.pad(q, (0, od - key)).to(k_cache.dtype).contiguous()
+
+    def norm_add(self, h, y, weight, eps, next_weight=None, next_eps=0.0, out_dtype=None, gate=None, gate_col0=0, gate_bias=None):
         yd = y.double()
+        if gate is not None:
+            z = gate.double()[:, gate_col0: gate_col0 + y.shape[1]]
+            yd = yd * torch.sigmoid(z if gate_bias is None else z + gate_bias.double())
         h.copy_((h.double() + yd / torch.sqrt((yd * yd).mean(-1, keepdim=True) + eps) * weight.double()).to(torch.float32))
         if next_weight is None:
             return None
@@ -330,6 +394,8 @@ class EmuOps:
             v = 0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))
         elif kind == "gelu_erf":
             v = 0.5 * z * (1.0 + torch.erf(z * 0.7071067811865476))
+        elif kind == "relu2":
+            v = torch.clamp(z, min=0.0) ** 2
         else:
             v = z * torch.sigmoid(z)
         if gate_col is not None:
