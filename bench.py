@@ -58,7 +58,7 @@ def parse_args():
     ap.add_argument("--mixed-chunk", type=int, default=512)
     ap.add_argument("--mixed-temperature", type=float, default=0.0, help="0: greedy; above: seeded sampling with top-k 50")
     ap.add_argument("--decode-target-blocks", type=int, default=None, help="tuning: blocks the split decode attention aims at")
-    ap.add_argument("--design", default=None, choices=["mifutar", "bomotar", "golavik", "zemarax"],
+    ap.add_argument("--design", default=None, choices=["mifutar", "bomotar", "golavik", "zemarax", "tokatar"],
                     help="instead of the headline: prefill and decode throughput of this design at layer sizes of real models, "
                          "beside Llama layers of equal size, with the time of every kernel entry point")
     ap.add_argument("--design-sizes", default="2048,4096", help="model widths of --design (comma separated)")
@@ -89,11 +89,16 @@ def design_bench(args) -> int:
     heads with a norm per head (window 1,024 keeping the first 64 tokens) and a latent attention that reads the second
     layer's latents, every attention with a sink; feed-forwards alternate between a dense one and eight ungated experts
     of a quarter of its width, two a token, with a shared expert; it stands beside the Bomotar model (the closest: norms
-    around every sublayer, a matrix recurrence, a bigram embedding, routed experts) and the Llama layers.
+    around every sublayer, a matrix recurrence, a bigram embedding, routed experts) and the Llama layers.  A Tokatar model
+    here has layers of an attention of the Llama layer's heads (chunks of 1,024, scores capped at 30, llama3-scaled
+    rotation, gated heads), the same with biases, a norm over the projections, turned values and one added to the
+    denominator, a latent attention of the Llama layer's heads (a latent of 128 beside a rotated part of half a head) and
+    the first kind again, each with a gate on both sublayers and an ungated feed-forward of the Llama layer's width; it
+    stands beside the Zemarax model (the closest: norms around every sublayer, attention over cached latents) and the
+    Llama layers.
     Prints one JSON line."""
     import torch
-    from tempura_amd.config import BomotarConfig, GolavikConfig, LlamaConfig, MifutarConfig
-    from tempura_amd.config.zemarax import ZemaraxConfig
+    from tempura_amd.config import BomotarConfig, GolavikConfig, LlamaConfig, MifutarConfig, TokatarConfig, ZemaraxConfig
     from tempura_amd.engine import Engine
     from tempura_amd.engine.loading import random_model
     from tempura_amd.engine.runner import StepEntry
@@ -155,6 +160,19 @@ def design_bench(args) -> int:
         return ZemaraxConfig.from_dict({"architecture": "Zemarax", "vocab": vocab, "width": width, "max_positions": 8192, "logit_scale": 1.0,
                                         "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0, "bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 7}},
                                         "layers": ls})
+
+    def tokatar_config(width, ff, heads, dim, kv, layers):
+        scaling = {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}
+        attn = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": window}, "softcap": 30.0,
+                "rot": {"dims": dim, "base": 500000.0, "scaling": scaling}}
+        attn_2 = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": window},
+                  "rot": {"dims": dim, "base": 500000.0}}
+        latent = {"heads": heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "kv_rank": 128, "scale": (dim + dim // 2) ** -0.5,
+                  "rot": {"dims": dim // 2, "base": 500000.0}}
+        kinds = [("attention", attn), ("attention_2", attn_2), ("latent_attention", latent), ("attention", attn)]
+        ls = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": ff}} for i in range(layers)]
+        return TokatarConfig.from_dict({"architecture": "Tokatar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+                                        "embedding": {"scale": 1.0}, "layers": ls, "max_positions": 8192})
 
     def llama_config(width, ff, heads, dim, kv, layers):
         return LlamaConfig(width, ff, layers, heads, kv, dim, vocab, 8192, 1e-5, 500000.0, None, False,
@@ -218,6 +236,9 @@ def design_bench(args) -> int:
         if design == "zemarax":
             models = [("zemarax", zemarax_config(width, ff, heads, dim, kv, args.design_layers)),
                       ("bomotar", bomotar_config(width, ff, heads, dim, kv, args.design_layers)), models[1]]
+        if design == "tokatar":
+            models = [("tokatar", tokatar_config(width, ff, heads, dim, kv, args.design_layers)),
+                      ("zemarax", zemarax_config(width, ff, heads, dim, kv, args.design_layers)), models[1]]
         chosen = [m for m in args.design_models.split(",") if m]
         for name, cfg in [m for m in models if not chosen or m[0] in chosen]:
             say(f"{name} width {width}: building")
@@ -234,7 +255,8 @@ def design_bench(args) -> int:
                       "config": {"design": {"mifutar": "Mifutar beside Llama layers of equal size",
                                             "bomotar": "Bomotar beside Mifutar and Llama layers of equal size",
                                             "golavik": "Golavik beside Bomotar and Llama layers of equal size",
-                                            "zemarax": "Zemarax beside Bomotar and Llama layers of equal size"}[design],
+                                            "zemarax": "Zemarax beside Bomotar and Llama layers of equal size",
+                                            "tokatar": "Tokatar beside Zemarax and Llama layers of equal size"}[design],
                                  "layers": args.design_layers, "prompt": T, "decode_batch": batch,
                                  "window": window if design == "mifutar" else None}, "points": points}))
     return 0
