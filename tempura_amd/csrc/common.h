@@ -74,6 +74,10 @@ __device__ inline void rope_cos_sin(int pos, double inv_freq, float factor, floa
 // (SwiGLU), bit for bit as without these constants; a kernel gets them by value.
 struct GateAct {
   float extra_slope, limit, offset;
+  // mode OUT_SPLIT (below): how many of the launch's columns are activated (a multiple of 128), the row stride of the
+  // activated output, and where the other columns go
+  int act_cols, act_ld, side_ld;
+  float* side;
 };
 
 struct RopeOut {
@@ -90,6 +94,14 @@ struct RopeOut {
   GateAct gate;              // (mode OUT_SWIGLU of the same kernels: the activation's constants)
 };
 enum { OUT_ROPE = 4 };
+// OUT_SPLIT: an ungated feed-forward's up product that leaves activated.  The first act_cols columns become max(v, 0)^2 as
+// bfloat16 in `out` (rows of act_ld); the columns behind them (rows of another weight with the same input) leave as they
+// are, float32, in `side` (rows of side_ld).  A wave's result tile lies on one side (act_cols is a multiple of 128).
+enum { OUT_SPLIT = 5 };
+__device__ inline float relu_squared(float v) {
+  const float r = fmaxf(v, 0.f);
+  return r * r;
+}
 
 // g * sigmoid(slope g) * (u + offset) with the hardware's exp2 and reciprocal (one ulp each; the result is rounded to
 // bfloat16), the same arithmetic in every bfloat16 product, whatever the number of rows

@@ -187,6 +187,10 @@ extern "C" int tp_linear_rope(const void* x, const void* w, int w_tiled, int M, 
 // block of rows 16 i.. and columns 32 j.. as 1,024 contiguous bytes, element (r, c) of the block at
 // ((c / 8) * 16 + r) * 8 + c % 8 (the matrix cores' operand order), blocks of a row group side by side.
 //
+// accumulate == 3 (bfloat16, K % 64 == 0): the first act_cols columns (a multiple of 128) become max(v, 0)^2, bfloat16
+// [M, act_cols] in `out` (bit 1 of `layout`, at most 16 rows: k-blocked [act_cols / 8, M, 8]), the others float32
+// [M, N - act_cols] in `side`.
+//
 // `defer_reduce` (products of more than 16 rows whose K is split over blocks): the partial sums stay in `scratch`
 // as [*splits_out, M, N] float32 and `out` is not touched; the caller's next kernel adds them (ascending).
 // *splits_out == 1 means that the product wrote `out` itself.
@@ -194,12 +198,12 @@ extern "C" int tp_linear_fused(const void* x, const void* w, int in_dt, void* ou
                                int N, int K, int allow_mfma, float* scratch, size_t scratch_floats,
                                const float* pre_ss, int pre_count, float pre_eps, const void* post_w, void* post_xg,
                                float* post_ss, int layout, int defer_reduce, int* splits_out, float gate_slope,
-                               float gate_limit, float gate_offset, hipStream_t s) {
+                               float gate_limit, float gate_offset, int act_cols, float* side, hipStream_t s) {
   if (splits_out) *splits_out = 1;
   TP_REQUIRE(M >= 0 && N > 0 && K > 0, "linear: bad sizes M=%d N=%d K=%d", M, N, K);
   TP_REQUIRE(accumulate != 1 || out_dt == TP_F32, "linear: accumulating output must be float32");
   const bool split_norm = pre_ss != nullptr || post_w != nullptr || (layout & 3) != 0;
-  TP_REQUIRE((layout & ~15) == 0 && (!(layout & 2) || accumulate == 2) && (!(layout & 8) || post_w != nullptr),
+  TP_REQUIRE((layout & ~15) == 0 && (!(layout & 2) || accumulate == 2 || accumulate == 3) && (!(layout & 8) || post_w != nullptr),
              "linear: bad layout flags %d", layout);
   TP_REQUIRE(!(layout & 4) || (in_dt == TP_BF16 && allow_mfma && N % 16 == 0 && K % 64 == 0),
              "linear: tiled weights are bfloat16 with N %% 16 == 0 and K %% 64 == 0 (N=%d K=%d)", N, K);
@@ -217,6 +221,20 @@ extern "C" int tp_linear_fused(const void* x, const void* w, int in_dt, void* ou
     const int r = tp_linear_mfma(x, w, out, out_dt, 2, M, N, K, scratch, scratch_floats, pre_ss, pre_count, pre_eps,
                                  nullptr, nullptr, nullptr, layout, 0, nullptr, gate, s);
     TP_REQUIRE(r >= 0, "linear: sizes M=%d N=%d K=%d do not fit the gated epilogue", M, N, K);
+    return r;
+  }
+  if (accumulate == 3) {
+    TP_REQUIRE(in_dt == TP_BF16 && allow_mfma && act_cols > 0 && act_cols <= N && (act_cols == N || side != nullptr),
+               "linear: the epilogue with side columns needs bfloat16 operands and a place for the side columns");
+    GateAct gate = {};
+    gate.act_cols = act_cols;
+    gate.act_ld = act_cols;
+    gate.side = side;
+    gate.side_ld = N - act_cols;
+    if (M == 0) return 0;
+    const int r = tp_linear_mfma(x, w, out, out_dt, 3, M, N, K, scratch, scratch_floats, pre_ss, pre_count, pre_eps, nullptr, nullptr,
+                                 nullptr, layout, 0, nullptr, gate, s);
+    TP_REQUIRE(r >= 0, "linear: sizes M=%d N=%d K=%d, %d of the columns activated, do not fit the epilogue with side columns", M, N, K, act_cols);
     return r;
   }
   TP_REQUIRE((size_t)M * N < ((size_t)1 << 40), "linear: output too large");

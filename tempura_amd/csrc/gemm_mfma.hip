@@ -67,6 +67,14 @@ __device__ inline void store_out(void* out, int mode, size_t idx, float v) {
     ((float*)out)[idx] += v;
 }
 
+// mode OUT_SPLIT (see GateAct); layout OUT_KBLOCKED: the activated columns k-blocked
+__device__ inline void store_split(void* out, int layout, const GateAct& ga, int M, int m, int n, float v) {
+  if (n < ga.act_cols)
+    store_gated(out, layout, M, ga.act_ld, m, n, relu_squared(v));
+  else
+    ga.side[(size_t)m * ga.side_ld + n - ga.act_cols] = v;
+}
+
 // v: this lane's sum of column n of row m; other: the sum of column n ^ 1 (the partner of a rotary pair)
 __device__ inline void rope_store(const RopeOut& rp, int m, int n, float v, float other) {
   const int h = n / rp.head_dim, d = n % rp.head_dim;
@@ -272,6 +280,8 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_mfma_kernel(const bf16
     } else if (mode == OUT_ROPE) {
       const float other = __shfl_xor(v, 1, 64);   // r and r ^ 1 are neighbouring lanes
       if (n < N && m < M) rope_store(rp, m, n, v, other);
+    } else if (mode == OUT_SPLIT) {
+      if (n < N && m < M) store_split(out, layout, rp.gate, M, m, n, v);
     } else if (n < N && m < M) {
       store_out(out, mode, (size_t)m * N + n, v);
     }
@@ -428,6 +438,8 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_lds_kernel(const bf16_
     } else if (mode == OUT_ROPE) {
       const float other = __shfl_xor(v, 1, 64);
       if (n < N && m < M) rope_store(rp, m, n, v, other);
+    } else if (mode == OUT_SPLIT) {
+      if (n < N && m < M) store_split(out, layout, rp.gate, M, m, n, v);
     } else if (n < N && m < M) {
       store_out(out, mode, (size_t)m * N + n, v);
     }
@@ -589,6 +601,10 @@ __global__ void gemm_splitk_reduce_kernel(const float* __restrict__ partial, voi
   if (idx >= total) return;
   float v = 0.f;
   for (int s = 0; s < splits; ++s) v += partial[(size_t)s * total + idx];
+  if (mode == OUT_SPLIT) {
+    store_split(out, 0, ga, M, (int)(idx / N), (int)(idx % N), v);
+    return;
+  }
   store_out(out, mode, idx, v);
 }
 
@@ -798,7 +814,8 @@ int tp_linear_rope_mfma(const void* x, const void* w, int w_tiled, int M, int N,
   return 0;
 }
 
-// accumulate: 0 store, 1 add into the float32 output, 2 gated-SiLU epilogue (see OUT_SWIGLU).
+// accumulate: 0 store, 1 add into the float32 output, 2 gated-SiLU epilogue (see OUT_SWIGLU), 3 the squared-ReLU epilogue
+// with side columns (see OUT_SPLIT; gate.act_cols, act_ld, side and side_ld are set).
 // pre_ss / post_w: the split norm (RowScale / NormPrep above), at most 16 rows; nullptr without.
 int tp_linear_mfma(const void* x, const void* w, void* out, int out_dt, int accumulate, int M, int N, int K,
                    float* scratch, size_t scratch_floats, const float* pre_ss, int pre_count, float pre_eps,
@@ -810,14 +827,15 @@ int tp_linear_mfma(const void* x, const void* w, void* out, int out_dt, int accu
   if (w_tiled && (N % 16 != 0 || K % 64 != 0)) return -1;
   if ((layout & (X_KBLOCKED | OUT_KBLOCKED | XG_KBLOCKED)) != 0 && M > 16) return -1;
   if ((layout & XG_KBLOCKED) && (post_w == nullptr || N % 8 != 0)) return -1;
-  if ((layout & OUT_KBLOCKED) && accumulate != 2) return -1;
+  if ((layout & OUT_KBLOCKED) && accumulate != 2 && accumulate != 3) return -1;
+  if (accumulate == 3 && (K % 64 != 0 || gate.act_cols % 128 != 0 || gate.act_cols <= 0 || gate.act_cols > N || out_dt != TP_BF16)) return -1;
   if ((pre_ss != nullptr || post_w != nullptr) && M > 16) return -1;
   if (post_w != nullptr && accumulate != 1) return -1;
   const RowScale pre = {pre_ss, pre_count, 1.0f / (float)K, pre_eps};
   const NormPrep post = {(const float*)post_w, (bf16_t*)post_xg, post_ss};
   if (((uintptr_t)x & 15) || ((uintptr_t)w & 15)) return -1;
   if (accumulate == 2 && (N % 16 != 0 || out_dt != TP_BF16)) return -1;
-  const int mode = accumulate == 2 ? OUT_SWIGLU : (accumulate ? OUT_ACC_F32 : (out_dt == TP_F32 ? OUT_F32 : OUT_BF16));
+  const int mode = accumulate == 3 ? OUT_SPLIT : accumulate == 2 ? OUT_SWIGLU : (accumulate ? OUT_ACC_F32 : (out_dt == TP_F32 ? OUT_F32 : OUT_BF16));
   const bf16_t* xb = (const bf16_t*)x;
   const bf16_t* wb = (const bf16_t*)w;
   const bool mid_ok = scratch != nullptr && g_tune_mid != 1;
@@ -847,8 +865,8 @@ int tp_linear_mfma(const void* x, const void* w, void* out, int out_dt, int accu
     } else if (pipe64 && tp_linear_pipe64(xb, wb, w_tiled, out, mode, M, N, K, scratch, scratch_floats, g_tune_splits,
                                           defer_reduce, splits_out, gate, s) == 0) {
       // taken by the 64-row pipelined kernel
-    } else if (w_tiled) {
-      return -1;   // the kernels below read row-major weights only
+    } else if (w_tiled || mode == OUT_SPLIT) {
+      return -1;   // the kernels below read row-major weights only, and have no columns that go elsewhere
     } else if (M > 128 || scratch == nullptr) {
       dim3 grid((N + 127) / 128, (M + 127) / 128);
       if (grid.y > 65535) return -1;

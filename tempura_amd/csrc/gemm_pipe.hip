@@ -201,7 +201,7 @@ __device__ inline void emit_tile_fast(const float* ct, int lane, int mrow0, int 
     }
     return;
   }
-  if (mode == OUT_BF16) {
+  if (mode == OUT_BF16 || mode == OUT_SPLIT) {   // (OUT_SPLIT here: the activated columns)
     constexpr int LPR = COLS / 8, RPP = 64 / LPR, PASSES = ROWS / RPP, B = PASSES < 4 ? PASSES : 4;
     const int col = (lane % LPR) * 8, rr = lane / LPR;
     const float* src = ct + rr * LD + col;
@@ -214,6 +214,15 @@ __device__ inline void emit_tile_fast(const float* ct, int lane, int mrow0, int 
       for (int u = 0; u < B; ++u) {
         a[u] = *(const f32x4_t*)(src + (p0 + u) * RPP * LD);
         b[u] = *(const f32x4_t*)(src + (p0 + u) * RPP * LD + 4);
+      }
+      if (mode == OUT_SPLIT) {
+#pragma unroll
+        for (int u = 0; u < B; ++u)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            a[u][e] = relu_squared(a[u][e]);
+            b[u][e] = relu_squared(b[u][e]);
+          }
       }
 #pragma unroll
       for (int u = 0; u < B; ++u) {
@@ -413,6 +422,17 @@ __device__ inline void emit_tile_rope(const float* ct, int lane, int mrow0, int 
 template <int ROWS, int COLS, int LD>
 __device__ inline void emit_tile(const float* ct, int lane, int mrow0, int ncol0, void* out, int mode, int M, int N, int ldo,
                                  const GateAct& ga) {
+  if (mode == OUT_SPLIT) {
+    if (ncol0 < ga.act_cols) {
+      ldo = ga.act_ld;
+    } else {   // the columns behind the activated ones
+      mode = OUT_F32;
+      out = ga.side;
+      ncol0 -= ga.act_cols;
+      N -= ga.act_cols;
+      ldo = ga.side_ld;
+    }
+  }
   if (mrow0 + ROWS <= M && ncol0 + COLS <= N && ldo % 8 == 0 && ((uintptr_t)out & 15) == 0) {
     emit_tile_fast<ROWS, COLS, LD>(ct, lane, mrow0, ncol0, out, mode, ldo, ga);
     return;
@@ -467,7 +487,11 @@ __device__ inline void emit_tile(const float* ct, int lane, int mrow0, int ncol0
         const int m = mrow0 + (p0 + u) * RPP + rr;
         if (m >= M) continue;
         const size_t idx = (size_t)m * ldo + ncol0 + col;
-        if (mode == OUT_BF16) {
+        if (mode == OUT_SPLIT) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[u][e] = relu_squared(v[u][e]);
+        }
+        if (mode == OUT_BF16 || mode == OUT_SPLIT) {
           u32x2_t pk;
           pk[0] = pack_bf16(v[u][0], v[u][1]);
           pk[1] = pack_bf16(v[u][2], v[u][3]);
@@ -489,7 +513,9 @@ __device__ inline void emit_tile(const float* ct, int lane, int mrow0, int ncol0
     for (int e = 0; e < 4; ++e) {
       if (ncol0 + col + e >= N) break;
       const float v = ct[row * LD + col + e];
-      if (mode == OUT_BF16)
+      if (mode == OUT_SPLIT)
+        ((bf16_t*)out)[idx + e] = float_to_bf16(relu_squared(v));
+      else if (mode == OUT_BF16)
         ((bf16_t*)out)[idx + e] = float_to_bf16(v);
       else if (mode == OUT_F32)
         ((float*)out)[idx + e] = v;
@@ -1400,7 +1426,7 @@ static int tp_linear_pipe128(const bf16_t* x, const bf16_t* w, int w_tiled, void
   if (8 * per_xcd > 0x7fffffffL) return -1;
   hipLaunchKernelGGL(gemm_pipe128_kernel, dim3((unsigned)(8 * per_xcd)), dim3(256), 0, s, x, w, out,
                      splits > 1 ? scratch : nullptr, mode, M, N, K, ldo, rp, w_tiled, splits);
-  if (splits > 1 && defer && splits_out != nullptr && mode != OUT_SWIGLU) {
+  if (splits > 1 && defer && splits_out != nullptr && mode != OUT_SWIGLU && mode != OUT_SPLIT) {
     *splits_out = splits;   // the parts stay unadded for the caller's next kernel
   } else if (splits > 1) {
     const size_t n_out = mode == OUT_SWIGLU ? (size_t)M * (N / 2) : (size_t)M * N;
@@ -1473,7 +1499,7 @@ int tp_linear_pipe(const bf16_t* x, const bf16_t* w, int w_tiled, void* out, int
     // Tiles of 256 x 192 where N is a multiple of 192 and that many more tiles fill whole rounds: priced at 1.35
     // small tiles (the q/k/v projection of 2,048 rows, N = 6,144: 256 tiles in one round instead of 192 of 256 x 256
     // on three quarters of the CUs, 109 -> 8x us).
-    if (N % 192 == 0 && mode != OUT_SWIGLU && g_pipe_big != 4 && (rope == nullptr || rope->head_dim == 128)) {
+    if (N % 192 == 0 && mode != OUT_SWIGLU && mode != OUT_SPLIT && g_pipe_big != 4 && (rope == nullptr || rope->head_dim == 128)) {
       const long t192 = (long)MB * (N / 192);
       if (1.35 * (double)((t192 + 255) / 256) < best - 1e-9 || g_pipe_big == 3) {
         const long blocks3 = blocks_for(N / 192);
@@ -1493,16 +1519,17 @@ int tp_linear_pipe(const bf16_t* x, const bf16_t* w, int w_tiled, void* out, int
     const int N2 = N - n_done;
     const int NBr = (N2 + BN - 1) / BN;
     const long blocksr = blocks_for(NBr);
-    const size_t esz = mode == OUT_BF16 || mode == OUT_SWIGLU ? 2 : 4;
+    const size_t esz = mode == OUT_BF16 || mode == OUT_SWIGLU || mode == OUT_SPLIT ? 2 : 4;
     void* out2 = out == nullptr ? nullptr : (char*)out + (size_t)(mode == OUT_SWIGLU ? n_done / 2 : n_done) * esz;
     rp.col0 = n_done;
+    rp.gate.act_cols -= n_done;   // (counted from the launch's first column; not above zero: none of them is activated)
     hipLaunchKernelGGL(gemm_pipe_kernel, dim3((unsigned)blocksr, 1), dim3(256), 0, s, x, w + (size_t)n_done * K, out2, scratch,
                        mode, M, N2, K, pm, ldo, rp, w_tiled);
     return 0;
   }
   hipLaunchKernelGGL(gemm_pipe_kernel, dim3((unsigned)blocks, splits), dim3(256), 0, s, x, w, out, scratch, mode, M, N, K,
                      pm, ldo, rp, w_tiled);
-  if (splits > 1 && defer && splits_out != nullptr && mode != OUT_SWIGLU) {
+  if (splits > 1 && defer && splits_out != nullptr && mode != OUT_SWIGLU && mode != OUT_SPLIT) {
     *splits_out = splits;   // the parts stay unadded for the caller's next kernel
   } else if (splits > 1) {
     const size_t n_out = mode == OUT_SWIGLU ? (size_t)M * (N / 2) : (size_t)M * N;
@@ -1552,7 +1579,7 @@ int tp_linear_pipe64(const bf16_t* x, const bf16_t* w, int w_tiled, void* out, i
     tiles = tiles_narrow;
     splits = splits_narrow;
   }
-  const bool leave = defer && splits > 1 && splits_out != nullptr && mode != OUT_SWIGLU;
+  const bool leave = defer && splits > 1 && splits_out != nullptr && mode != OUT_SWIGLU && mode != OUT_SPLIT;
   if (narrow)
     hipLaunchKernelGGL(gemm_pipe64_kernel<2>, dim3((unsigned)tiles, splits), dim3(256), 0, s, x, w, out,
                        splits > 1 ? scratch : nullptr, mode, M, N, K, w_tiled, gate);

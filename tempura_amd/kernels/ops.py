@@ -587,8 +587,38 @@ def linear_swiglu(x, w: torch.Tensor, blocked_out: bool = False, slope: float = 
     scratch, nscratch = _splitk_scratch(x, m, n)
     _call("tp_linear_fused", _ptr(x), _ptr(wd), _BF16, _ptr(out.data if blocked_out else out), _BF16, 2, m, n, k, 1,
           _ptr(scratch), ctypes.c_size_t(nscratch), *pre, _ptr(None), _ptr(None), _ptr(None), (2 if blocked_out else 0) | wl | xl,
-          0, _ptr(None), ctypes.c_float(slope), ctypes.c_float(limit), ctypes.c_float(up_offset), _stream(), tag=(m, n, k))
+          0, _ptr(None), ctypes.c_float(slope), ctypes.c_float(limit), ctypes.c_float(up_offset), 0, _ptr(None), _stream(), tag=(m, n, k))
     return out
+
+
+def linear_relu2_ok(act_cols: int, k: int, dtype: torch.dtype) -> bool:
+    """Whether ``linear_relu2`` takes a weight of k columns whose first ``act_cols`` rows are the activated ones."""
+    return allow_mfma and dtype == torch.bfloat16 and k % 64 == 0 and act_cols % 128 == 0
+
+
+def linear_relu2(x: torch.Tensor, w, act_cols: int, blocked_out: bool = False):
+    """bfloat16 x [m, k], weight [n, k] -> (bfloat16 [m, act_cols] = max(x w^T, 0)^2 of the first ``act_cols`` columns, the
+    activation applied to the float32 accumulators; float32 [m, n - act_cols], the other columns as they are).  With
+    ``blocked_out`` the first comes as ``KBlocked`` when there are at most 16 rows.  Sizes: ``linear_relu2_ok``."""
+    if _backend is not None:
+        return _backend.linear_relu2(x, w, act_cols, blocked_out)
+    wd, wl = _w_args(w)
+    _dev_ok(x, wd)
+    _need(x.dim() == 2 and w.dim() == 2 and x.shape[1] == w.shape[1], f"linear_relu2: shapes {tuple(x.shape)} x {tuple(w.shape)}")
+    _need(x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and linear_relu2_ok(act_cols, x.shape[1], x.dtype)
+          and 0 < act_cols <= w.shape[0], "linear_relu2: needs bfloat16 operands, k % 64 == 0 and a multiple of 128 activated columns")
+    (m, k), n = x.shape, w.shape[0]
+    blocked_out = blocked_out and 0 < m <= 16
+    if blocked_out:
+        out = KBlocked(torch.empty((act_cols // 8, m, 8), dtype=torch.bfloat16, device=x.device), m, act_cols)
+    else:
+        out = torch.empty((m, act_cols), dtype=torch.bfloat16, device=x.device)
+    side = torch.empty((m, n - act_cols), dtype=torch.float32, device=x.device)
+    scratch, nscratch = _splitk_scratch(x, m, n)
+    _call("tp_linear_fused", _ptr(x), _ptr(wd), _BF16, _ptr(out.data if blocked_out else out), _BF16, 3, m, n, k, 1, _ptr(scratch),
+          ctypes.c_size_t(nscratch), _ptr(None), 0, ctypes.c_float(0.0), _ptr(None), _ptr(None), _ptr(None), (2 if blocked_out else 0) | wl,
+          0, _ptr(None), ctypes.c_float(1.0), ctypes.c_float(0.0), ctypes.c_float(0.0), int(act_cols), _ptr(side), _stream(), tag=(m, n, k))
+    return out, side
 
 
 def _splitk_scratch(x: torch.Tensor, m: int, n: int):
@@ -667,7 +697,7 @@ def linear(x, w: torch.Tensor, out_dtype: torch.dtype, residual: Optional[torch.
     splits = ctypes.c_int(1)
     _call("tp_linear_fused", _ptr(x), _ptr(wd), _dt(x), _ptr(out), _dt(out), acc, m, n, k, int(allow_mfma), _ptr(scratch),
           ctypes.c_size_t(nscratch), *pre, *post, layout, int(defer), ctypes.byref(splits), ctypes.c_float(1.0),
-          ctypes.c_float(0.0), ctypes.c_float(0.0), _stream(), tag=(m, n, k))
+          ctypes.c_float(0.0), ctypes.c_float(0.0), 0, _ptr(None), _stream(), tag=(m, n, k))
     if defer and splits.value > 1:
         if next_norm is None:
             return Partials(scratch[: splits.value * m * n].view(splits.value, m, n))

@@ -107,7 +107,8 @@ class GatedFFN(FeedForward):
 
 class DenseMLP(FeedForward):
     """``down(act(up(x)))`` without a gate; ``activation`` names the function (``ops.ACTIVATIONS``: ``gelu_tanh``, ``silu``,
-    ``relu2``, ..), which reads the float32 sums of the up product."""
+    ``relu2``, ..), which reads the float32 sums of the up product: in the product's own epilogue for ``relu2`` in bfloat16
+    (sizes ``ops.linear_relu2_ok``), else as a kernel of its own."""
     graph_safe = True
     takes_side_rows = True     # (behind the up product's own columns)
     returns_output = True      # with ``residual`` None the output comes back instead of being added
@@ -118,6 +119,7 @@ class DenseMLP(FeedForward):
         self.activation = str(spec.params.get("activation", "gelu_tanh"))
         if self.activation not in ops.ACTIVATIONS:
             raise ValueError(f"mlp: activation {self.activation!r} unknown (known: {sorted(ops.ACTIVATIONS)})")
+        self.fused = self.activation == "relu2" and ops.linear_relu2_ok(self.intermediate_size, hidden_size, dtype)
         self.w_up = self.w_down = None
 
     @classmethod
@@ -135,6 +137,11 @@ class DenseMLP(FeedForward):
         self.w_down = ops.tile_weight(self._to_device(get(w["down"])))
 
     def forward(self, x, ctx, residual=None):
+        if self.fused:
+            # (a few rows go to the down product k-blocked: it reads them straight from global memory)
+            a, side = ops.linear_relu2(x, self.w_up, self.intermediate_size, blocked_out=True)
+            y = ops.linear(a, self.w_down, torch.float32, residual=residual)
+            return y if self.side_rows is None else (y, (side, 0))
         u = ops.linear(x, self.w_up, torch.float32)
         if self.side_rows is not None:
             a = ops.activation(u, self.activation, self.dtype, 0, self.intermediate_size)

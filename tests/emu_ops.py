@@ -230,6 +230,15 @@ class EmuOps:
             return KBlocked(out.reshape(m, i // 8, 8).permute(1, 0, 2).contiguous(), m, i)
         return out
 
+    def linear_relu2(self, x, w, act_cols, blocked_out=False):
+        from tempura_amd.kernels.ops import KBlocked
+        y = x.double() @ w.double().T
+        out = (torch.clamp(y[:, :act_cols], min=0.0) ** 2).to(torch.bfloat16)
+        m = out.shape[0]
+        if blocked_out and 0 < m <= 16:
+            out = KBlocked(out.reshape(m, act_cols // 8, 8).permute(1, 0, 2).contiguous(), m, act_cols)
+        return out, y[:, act_cols:].to(torch.float32)
+
     def rope_kv_write(self, qkv, positions, slots, inv_freq, rotary_dim, factor, num_heads, num_kv_heads,
                       head_dim, k_cache, v_cache, q_dtype, value_dim=None, pad_dim=None):
         n = qkv.shape[0]

@@ -527,3 +527,26 @@ def test_replay_program_on_a_model_folder(dirs, tmp_path):
     a = torch.from_numpy(np.fromfile(out / "0.f32", dtype="<f4").reshape(-1, vocab))
     c = torch.from_numpy(np.fromfile(out / "2.f32", dtype="<f4").reshape(-1, vocab))
     assert plain.logit_error(torch.cat([a, c]), torch.stack([ref[0], ref[10], ref[29], ref[3]])) < TOL["float32"]
+
+
+@pytest.mark.parametrize("m", [1, 2, 8, 16, 17, 40, 64, 65, 100, 128, 129, 200, 300, 700, 2049])
+@pytest.mark.parametrize("n,act,k", [(384, 128, 128), (384, 384, 192), (640, 512, 256), (2576, 1536, 2048), (1168, 1024, 64), (4608, 3584, 512)])
+def test_up_product_that_leaves_squared_relu_beside_plain_columns(m, n, act, k):
+    """Every product kernel that a number of rows selects, weights tiled and row-major: the activated columns in bfloat16
+    (a few rows also k-blocked), the side columns in float32."""
+    ops = _ops()
+    g = torch.Generator().manual_seed(n + k)
+    w = (torch.randn(n, k, generator=g) * k ** -0.5).to(torch.bfloat16).to(DEV)
+    x = torch.randn(m, k, generator=torch.Generator().manual_seed(m)).to(torch.bfloat16).to(DEV)
+    y = x.float() @ w.float().T
+    want = torch.clamp(y[:, :act], min=0.0) ** 2
+    for weight in (w, ops.tile_weight(w)):
+        out, side = ops.linear_relu2(x, weight, act)
+        assert out.dtype == torch.bfloat16 and side.shape == (m, n - act)
+        _close(out, want, 6e-3)
+        if n > act:
+            _close(side, y[:, act:], 3e-5)
+        blocked, side2 = ops.linear_relu2(x, weight, act, blocked_out=True)
+        if m <= 16:
+            assert isinstance(blocked, ops.KBlocked) and torch.equal(blocked.row_major(), out)
+        assert torch.equal(side2, side)
