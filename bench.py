@@ -92,7 +92,7 @@ def design_bench(args) -> int:
     around every sublayer, a matrix recurrence, a bigram embedding, routed experts) and the Llama layers.  A Tokatar model
     here has layers of an attention of the Llama layer's heads (chunks of 1,024, scores capped at 30, llama3-scaled
     rotation, gated heads), the same with biases, a norm over the projections, turned values and one added to the
-    denominator, a latent attention of the Llama layer's heads (a latent of 128 beside a rotated part of half a head) and
+    denominator, a latent attention of the Llama layer's heads (a latent of four heads beside a rotated part of half a head) and
     the first kind again, each with a gate on both sublayers and an ungated feed-forward of the Llama layer's width; it
     stands beside the Zemarax model (the closest: norms around every sublayer, attention over cached latents) and the
     Llama layers.
@@ -167,7 +167,7 @@ def design_bench(args) -> int:
                 "rot": {"dims": dim, "base": 500000.0, "scaling": scaling}}
         attn_2 = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": window},
                   "rot": {"dims": dim, "base": 500000.0}}
-        latent = {"heads": heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "kv_rank": 128, "scale": (dim + dim // 2) ** -0.5,
+        latent = {"heads": heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "kv_rank": 4 * dim, "scale": (dim + dim // 2) ** -0.5,
                   "rot": {"dims": dim // 2, "base": 500000.0}}
         kinds = [("attention", attn), ("attention_2", attn_2), ("latent_attention", latent), ("attention", attn)]
         ls = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": ff}} for i in range(layers)]

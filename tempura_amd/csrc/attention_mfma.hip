@@ -384,10 +384,57 @@ __device__ inline void attn_compute(const AttnArgs& a, int j0, const KvFrags<D, 
   attn_softmax_pv<DV, NQ, MASK, MODE>(a, j0, s, f.v, qpos, m, l, o, bias_row);
 }
 
+// The same step for keys of more than 192 (latents of a few hundred with a rotated part): the fragments of a whole step
+// would not fit beside the running output, so keys and values are fetched as they are multiplied.  One query tile.
+template <int D, int DV, int MODE>
+__device__ inline void attn_step_wide(const AttnArgs& a, const int* __restrict__ table, int kvh, int ctx, int j0,
+                                      const bf16x8_t (&qf)[1][D / 32], const int (&qpos)[1], float (&m)[1], float (&l)[1],
+                                      f32x4_t (&o)[1][DV / 16]) {
+  const int lane = threadIdx.x & 63;
+  const int g = lane >> 4, c = lane & 15;
+  const int ps = a.page_size;
+  const bf16_t* kr[2];
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    const int key = min(j0 + 8 * (c >> 2) + 4 * t + (c & 3), ctx - 1);
+    kr[t] = a.k_cache + ((size_t)(table[key / ps] * a.n_kv + kvh) * ps + key % ps) * D + g * 8;
+  }
+  const int kb = min(j0 + 8 * g, (ctx - 1) & ~7);
+  const bf16_t* vr = a.v_cache + ((size_t)(table[kb / ps] * a.n_kv + kvh) * DV + c) * ps + kb % ps;
+  const u32x4_t keep = attn_existing_keys(ctx - (j0 + 8 * g));
+  f32x4_t s[1][2];
+  s[0][0] = s[0][1] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int dk = 0; dk < D / 32; ++dk)
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+      s[0][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag_of(*(const u32x4_t*)(kr[t] + dk * 32)), qf[0][dk], s[0][t], 0, 0, 0);
+  bf16x8_t pf[1];
+  float alpha[1];
+  bool moved[1];
+  attn_softmax<1, true, MODE>(a, j0, s, qpos, m, l, pf, alpha, moved);
+#pragma unroll
+  for (int dt = 0; dt < DV / 16; ++dt) {
+    const bf16x8_t vf = frag_of(*(const u32x4_t*)(vr + (size_t)dt * 16 * ps) & keep);
+    if (moved[0]) {
+      o[0][dt][0] *= alpha[0];
+      o[0][dt][1] *= alpha[0];
+      o[0][dt][2] *= alpha[0];
+      o[0][dt][3] *= alpha[0];
+    }
+    o[0][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[0], o[0][dt], 0, 0, 0);
+  }
+}
+
 template <int D, int DV, int NQ, int MODE = MODE_PLAIN>
 __device__ inline void attn_step(const AttnArgs& a, const int* __restrict__ table, int kvh, int ctx, int j0,
                                  const bf16x8_t (&qf)[NQ][D / 32], const int (&qpos)[NQ], float (&m)[NQ],
                                  float (&l)[NQ], f32x4_t (&o)[NQ][DV / 16], const float* __restrict__ bias_row = nullptr) {
+  if constexpr (D > 192) {
+    static_assert(NQ == 1 && MODE != MODE_BIAS, "one query tile, no bias by distance");
+    attn_step_wide<D, DV, MODE>(a, table, kvh, ctx, j0, qf, qpos, m, l, o);
+    return;
+  }
   KvFrags<D, DV> f;
   attn_load<D, DV>(a, table, kvh, ctx, j0, f);
   attn_compute<D, DV, NQ, true, MODE>(a, j0, f, qf, qpos, m, l, o, bias_row);
@@ -1051,7 +1098,7 @@ static int launch_all(AttnArgs a, int n_tokens, int n_req, int max_q_len, int nu
     // (blocks of 32 rows that have work: from the rows of the portions, not from the grid, which spans the longest
     // portion for every request; single tokens take the decode kernel)
     const long blocks2 = (long)((n_tokens - num_single + 31) / 32 + (n_req - num_single - 1)) * kv_groups;
-    const bool two = g_attn_tune == 2 || (g_attn_tune != 3 && blocks2 >= 768 && !WIDE);
+    const bool two = D <= 192 && (g_attn_tune == 2 || (g_attn_tune != 3 && blocks2 >= 768 && !WIDE));
     const int rows = two ? 32 : 16;
     const int skip = num_single > 0 ? 1 : 0;
     const bool lds_pages = g_attn_tune != 1 && a.page_shift >= 4 && a.page_size >= 512 / D;   // (a key load covers 512 / D rows, which must lie in one page)
@@ -1112,10 +1159,13 @@ static int launch_all(AttnArgs a, int n_tokens, int n_req, int max_q_len, int nu
         return 0;
       }
     }
-    if (two)
-      hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 2, MODE>), grid, dim3(256), 0, s, a, skip);
-    else
-      hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 1, MODE>), grid, dim3(256), 0, s, a, skip);
+    if constexpr (D <= 192) {
+      if (two) {
+        hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 2, MODE>), grid, dim3(256), 0, s, a, skip);
+        return 0;
+      }
+    }
+    hipLaunchKernelGGL((attn_prefill_kernel<D, DV, 1, MODE>), grid, dim3(256), 0, s, a, skip);
   }
   return 0;
 }
@@ -1132,6 +1182,9 @@ static int launch_sizes(const AttnArgs& a, int d, int dv, int n_tokens, int n_re
     case 128064: return launch_all<128, 64, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
     case 160096: return launch_all<160, 96, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
     case 192128: return launch_all<192, 128, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 288256: return launch_all<288, 256, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 320256: return launch_all<320, 256, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
+    case 576512: return launch_all<576, 512, MODE>(a, n_tokens, n_req, max_q_len, num_single, s);
     default: return -1;
   }
 }

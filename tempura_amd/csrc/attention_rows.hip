@@ -264,7 +264,8 @@ extern "C" int tp_qkv_rows(const float* rows, size_t stride, const float* q_bias
 }
 
 // ---- queries in a latent's space, one latent and one rotated key part a token --------------------
-// rows float32 [n, stride]: at q_col0 the queries, per head [rot rotated | latent unrotated] elements; at d_col0 the
+// rows float32 [n, stride]: at q_col0 the queries, q_head elements a head, whose rot rotated elements start at q_rot; the
+// latent elements follow them, or (latent_follows 0) somebody else writes the latent part of q_out.  At d_col0 the
 // latent before its norm [latent] and the shared rotated key part [rot].  The latent becomes c = x / sqrt(mean(x^2) +
 // eps) * w.  Written: q_out [n, heads, out_dim] and keys [page, 1, page_size, out_dim] as [rotated | latent | zeros],
 // values [page, 1, value_dim, page_size] as [latent | zeros], transposed.
@@ -275,7 +276,8 @@ __global__ __launch_bounds__(256) void latent_rows_write_kernel(const float* __r
                                                                 const int* __restrict__ slots, const double* __restrict__ inv_freq,
                                                                 const float2* __restrict__ table, float factor, int heads, int rot, int latent,
                                                                 int out_dim, int value_dim, T* __restrict__ q_out, T* __restrict__ k_cache,
-                                                                T* __restrict__ v_cache, int page_size, int per_slice) {
+                                                                T* __restrict__ v_cache, int page_size, int per_slice, int q_head, int q_rot,
+                                                                int latent_follows) {
   __shared__ float scratch[32];
   const int t = blockIdx.x, pos = positions[t];
   const float* row = rows + (size_t)t * stride;
@@ -310,7 +312,8 @@ __global__ __launch_bounds__(256) void latent_rows_write_kernel(const float* __r
     const int h = g * V / out_dim, i = g * V % out_dim;
     Elems<V> r;
     if (i < key) {
-      r = load_elems<V>(row + q_col0 + (size_t)h * key + i);
+      if (i >= rot && !latent_follows) continue;
+      r = load_elems<V>(row + q_col0 + (size_t)h * q_head + q_rot + i);
       turn_pairs<V>(r, i, rot / 2, t, pos, inv_freq, table, factor, 1.0f);
     } else {
 #pragma unroll
@@ -323,16 +326,18 @@ __global__ __launch_bounds__(256) void latent_rows_write_kernel(const float* __r
 extern "C" int tp_latent_rows_write(const float* rows, size_t stride, int q_col0, int d_col0, const float* w, float eps,
                                     const int* positions, const int* slots, const double* inv_freq, const float* table, float factor,
                                     int n, int heads, int rot, int latent, int out_dim, int value_dim, void* q_out, void* k_cache,
-                                    void* v_cache, int dt, int page_size, hipStream_t s) {
+                                    void* v_cache, int dt, int page_size, int q_head, int q_rot, int latent_follows, hipStream_t s) {
   TP_REQUIRE(n >= 0 && heads > 0 && rot >= 0 && latent > 0 && q_col0 >= 0 && d_col0 >= 0 && page_size > 0, "latent_rows_write: bad sizes");
   const int key = rot + latent;
   TP_REQUIRE(rot % 2 == 0 && key % 2 == 0 && out_dim % 2 == 0 && out_dim >= key && value_dim >= latent, "latent_rows_write: head sizes must be even");
-  TP_REQUIRE(stride % 2 == 0 && q_col0 % 2 == 0 && stride >= (size_t)q_col0 + (size_t)heads * key && stride >= (size_t)d_col0 + key,
+  TP_REQUIRE(stride % 2 == 0 && q_col0 % 2 == 0 && q_head % 2 == 0 && q_rot % 2 == 0 && q_rot >= 0 &&
+                 q_head >= q_rot + rot + (latent_follows ? latent : 0) && stride >= (size_t)q_col0 + (size_t)heads * q_head &&
+                 stride >= (size_t)d_col0 + key,
              "latent_rows_write: rows too short or odd");
   TP_REQUIRE(rot == 0 || inv_freq != nullptr, "latent_rows_write: no frequency table");
   TP_REQUIRE(dt == TP_F32 || dt == TP_BF16, "latent_rows_write: unknown dtype %d", dt);
   if (n == 0) return 0;
-  const bool four = key % 4 == 0 && out_dim % 4 == 0 && stride % 4 == 0 && q_col0 % 4 == 0 && ((uintptr_t)rows & 15) == 0;
+  const bool four = key % 4 == 0 && rot % 4 == 0 && q_head % 4 == 0 && q_rot % 4 == 0 && out_dim % 4 == 0 && stride % 4 == 0 && q_col0 % 4 == 0 && ((uintptr_t)rows & 15) == 0;
   const int V = four ? 4 : 2;
   const int per_slice = n >= 256 ? 1024 : 256;
   const dim3 grid(n, 1 + (heads * out_dim / V + per_slice - 1) / per_slice);
@@ -340,7 +345,7 @@ extern "C" int tp_latent_rows_write(const float* rows, size_t stride, int q_col0
 #define LAT(T, VV)                                                                                                            \
   hipLaunchKernelGGL((latent_rows_write_kernel<T, VV>), grid, dim3(256), 0, s, rows, stride, q_col0, d_col0, w, eps, positions, slots, \
                      inv_freq, (const float2*)table, factor, heads, rot, latent, out_dim, value_dim, (T*)q_out, (T*)k_cache,  \
-                     (T*)v_cache, page_size, per_slice)
+                     (T*)v_cache, page_size, per_slice, q_head, q_rot, latent_follows)
   if (dt == TP_F32) {
     if (four) LAT(float, 4); else LAT(float, 2);
   } else {

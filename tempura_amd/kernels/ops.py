@@ -870,7 +870,7 @@ portion_scratch_limit = 256 << 20
 
 
 #: the pairs (key size, value size) the matrix-core attention kernels are built for
-FAST_PAIRS = ((32, 32), (64, 64), (96, 96), (128, 128), (64, 32), (128, 64), (160, 96), (192, 128))
+FAST_PAIRS = ((32, 32), (64, 64), (96, 96), (128, 128), (64, 32), (128, 64), (160, 96), (192, 128), (288, 256), (320, 256), (576, 512))
 
 
 def fast_pair(key_dim: int, value_dim: int, exact_values: bool = True):
@@ -1408,19 +1408,21 @@ def qkv_rows(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, n
 def latent_rows_write(rows: torch.Tensor, q_col0: int, d_col0: int, weight: torch.Tensor, eps: float, positions: torch.Tensor,
                       slots: torch.Tensor, inv_freq: Optional[torch.Tensor], factor: float, num_heads: int, rotary_dim: int,
                       latent_dim: int, k_cache: torch.Tensor, v_cache: torch.Tensor,
-                      cos_sin: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """Float32 rows [n, width]: queries at ``q_col0``, per head [rotary_dim | latent_dim] elements, and at ``d_col0`` a latent
-    before its norm [latent_dim] followed by one shared rotated key part [rotary_dim].  The latent is RMS-normed
+                      cos_sin: Optional[torch.Tensor] = None, plain_dim: Optional[int] = None) -> torch.Tensor:
+    """Float32 rows [n, width]: queries at ``q_col0``, per head [rotary_dim | latent_dim] elements (``plain_dim`` given: per
+    head [plain_dim | rotary_dim] elements of which only the rotary ones are taken; the latent part of the result is left
+    for the caller to fill), and at ``d_col0`` a latent before its norm [latent_dim] followed by one shared rotated key part [rotary_dim].  The latent is RMS-normed
     (``weight``, ``eps``), the rotary elements of the queries and of the key part turn (pairs of neighbours, position *
     ``inv_freq``); the cache rows ``slots`` get keys [rotated | latent | zeros] (one head) and, transposed, values
     [latent | zeros]; the sizes of both are the caches' own.  Returns q [n, heads, key size], laid out like the keys."""
     if _backend is not None:
         return _backend.latent_rows_write(rows, q_col0, d_col0, weight, eps, positions, slots, inv_freq, factor, num_heads, rotary_dim,
-                                          latent_dim, k_cache, v_cache)
+                                          latent_dim, k_cache, v_cache, plain_dim)
     _dev_ok(rows, weight, positions, slots, inv_freq, k_cache, v_cache, cos_sin)
     n, key = rows.shape[0], rotary_dim + latent_dim
+    q_head, q_rot = (key, 0) if plain_dim is None else (int(plain_dim) + rotary_dim, int(plain_dim))
     _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.shape[1] % 2 == 0 and q_col0 >= 0 and q_col0 % 2 == 0 and d_col0 >= 0
-          and q_col0 + num_heads * key <= rows.shape[1] and d_col0 + key <= rows.shape[1], "latent_rows_write: bad rows")
+          and q_head % 2 == 0 and q_rot % 2 == 0 and q_col0 + num_heads * q_head <= rows.shape[1] and d_col0 + key <= rows.shape[1], "latent_rows_write: bad rows")
     _need(weight.dtype == torch.float32 and weight.numel() == latent_dim, "latent_rows_write: weight must be float32 [latent_dim]")
     _need(k_cache.dim() == 4 and v_cache.dim() == 4, "latent_rows_write: bad caches")
     od, vd = k_cache.shape[3], v_cache.shape[2]
@@ -1433,8 +1435,37 @@ def latent_rows_write(rows: torch.Tensor, q_col0: int, d_col0: int, weight: torc
     q = torch.empty((n, num_heads, od), dtype=k_cache.dtype, device=rows.device)
     _call("tp_latent_rows_write", _ptr(rows), ctypes.c_size_t(rows.shape[1]), int(q_col0), int(d_col0), _ptr(weight), ctypes.c_float(eps),
           _ptr(positions), _ptr(slots), _ptr(inv_freq), _ptr(cos_sin), ctypes.c_float(factor), n, int(num_heads), int(rotary_dim),
-          int(latent_dim), od, vd, _ptr(q), _ptr(k_cache), _ptr(v_cache), _dt(k_cache), k_cache.shape[2], _stream())
+          int(latent_dim), od, vd, _ptr(q), _ptr(k_cache), _ptr(v_cache), _dt(k_cache), k_cache.shape[2], q_head, q_rot,
+          int(plain_dim is None), _stream())
     return q
+
+
+def head_linear_ok(n: int, k: int, dtype: torch.dtype) -> bool:
+    """Whether ``head_linear`` takes weights [heads, n, k]."""
+    return allow_mfma and dtype == torch.bfloat16 and k % 32 == 0 and n % 16 == 0
+
+
+def head_linear(x: torch.Tensor, x_col0: int, x_head: int, w: torch.Tensor, out: torch.Tensor, out_col0: int, out_head: int,
+                gate: Optional[torch.Tensor] = None, gate_col0: int = 0, scale: float = 1.0) -> None:
+    """A product per head: out[m, out_col0 + h * out_head + n] = scale * sigmoid(gate[m, gate_col0 + h]) * sum_k w[h, n, k] *
+    x[m, x_col0 + h * x_head + k], for bfloat16 weights [heads, n, k], rows ``x`` (float32 or bfloat16; float32 is rounded to
+    bfloat16) and bfloat16 rows ``out``; ``gate`` float32 rows or None.  Sizes: ``head_linear_ok``."""
+    if _backend is not None:
+        return _backend.head_linear(x, x_col0, x_head, w, out, out_col0, out_head, gate, gate_col0, scale)
+    _dev_ok(x, w, out, gate)
+    _need(w.dim() == 3 and w.dtype == torch.bfloat16 and head_linear_ok(w.shape[1], w.shape[2], w.dtype), "head_linear: bad weights")
+    H, N, K = w.shape
+    _need(x.dim() == 2 and out.dim() == 2 and out.dtype == torch.bfloat16 and x.shape[0] == out.shape[0], "head_linear: bad rows")
+    _need(0 <= x_col0 and x_col0 + (H - 1) * x_head + K <= x.shape[1] and x_head >= K, "head_linear: input rows too short")
+    _need(0 <= out_col0 and out_col0 + (H - 1) * out_head + N <= out.shape[1] and out_head >= N, "head_linear: output rows too short")
+    m = x.shape[0]
+    if gate is not None:
+        _need(gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape[0] == m and 0 <= gate_col0 and gate_col0 + H <= gate.shape[1],
+              "head_linear: bad gate rows")
+    at = lambda t, col: ctypes.c_void_p(t.data_ptr() + col * t.element_size())
+    _call("tp_head_linear", at(x, x_col0), _dt(x), ctypes.c_size_t(x.shape[1]), int(x_head), _ptr(w), at(out, out_col0),
+          ctypes.c_size_t(out.shape[1]), int(out_head), _ptr(None) if gate is None else at(gate, gate_col0),
+          ctypes.c_size_t(0 if gate is None else gate.shape[1]), ctypes.c_float(scale), m, H, N, K, _stream(), tag=(m, H, N, K))
 
 
 def norm_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, next_weight: Optional[torch.Tensor] = None,

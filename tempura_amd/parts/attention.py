@@ -711,9 +711,19 @@ class RotaryLatentAttention(BranchMixer):
     concatenated heads.  The position part turns the R rotated elements.
 
     Only c and the rotated part are cached: keys [R rotated | L latent] of one head, values [L latent], both with zeros
-    behind up to a pair of sizes that the matrix-core attention kernels take (bfloat16).  W_uk and W_uv are folded into the
-    ends, formed once at load in float64: the queries' rows W_uk[h]^T W_q[h, :D] (L a head, beside the R rotated ones) and
-    the output's columns W_o[:, h] W_uv[h].  A head's gate is one number, so it may multiply the sum over the latents.
+    behind up to a pair of sizes that the matrix-core attention kernels take (bfloat16).  The attention itself is one shared
+    key/value head over the latents, q_plain . (W_uk[h] c) = (W_uk[h]^T q_plain) . c and sum_j p_j W_uv[h] c_j =
+    W_uv[h] sum_j p_j c_j, so a step expands nothing of what it reads.  The two maps run in one of two ways:
+
+    * ``folded`` into the ends, formed once at load in float64: the queries' rows are W_uk[h]^T W_q[h, :D] (L a head,
+      beside the R rotated ones), the output's columns W_o[:, h] W_uv[h].  No more launches; a head's gate is one number,
+      so it may multiply the sum over the latents;
+    * as a product per head each (``ops.head_linear``, bfloat16): W_uk[h]^T on the projection's plain queries, straight
+      into the attention's rows, and W_uv[h] with the gate on the attention's outputs.  With latents wider than the heads
+      this is less arithmetic and far fewer weight bytes: per token H L (D + Dv) + H (D + Dv) hidden multiply-adds against
+      2 H L hidden.
+
+    The part takes whichever has fewer multiply-adds among those whose sizes fit (float32: folded).
 
     The columns of its input product are [q | latent | rotated key part | gate]; it keeps no per-request state."""
 
@@ -742,8 +752,11 @@ class RotaryLatentAttention(BranchMixer):
         pair = ops.fast_pair(key, self.latent_dim, exact_values=False) if dtype == torch.bfloat16 else None
         #: sizes of a cached key and of a cached value
         self.cached_key, self.cached_value = pair if pair is not None else (key, self.latent_dim)
-        self.q_cols = self.num_heads * key
-        self.inner = self.num_heads * self.cached_value
+        H, D, Dv, L = self.num_heads, self.head_dim, self.value_dim, self.latent_dim
+        self.folded = not (ops.head_linear_ok(L, D, dtype) and ops.head_linear_ok(Dv, self.cached_value, dtype) and self.rotary_dim % 4 == 0
+                           and L * (D + Dv) + (D + Dv) * hidden_size < 2 * L * hidden_size)
+        self.q_cols = H * (key if self.folded else D + self.rotary_dim)
+        self.inner = H * (self.cached_value if self.folded else Dv)
 
     @classmethod
     def expected_weights(cls, spec, hidden_size):
@@ -766,18 +779,27 @@ class RotaryLatentAttention(BranchMixer):
         w = self.spec.weights
         H, D, R, Dv, L = self.num_heads, self.head_dim, self.rotary_dim, self.value_dim, self.latent_dim
         f64 = lambda name: get(w[name]).to(torch.float64)
-        q, uk, uv, o = f64("q").view(H, D + R, -1), f64("uk").view(H, D, L), f64("uv").view(H, Dv, L), f64("o").view(-1, H, Dv)
         order = paired_order(R, R, getattr(self.position, "layout", "halves"))
-        latent_q = torch.matmul(uk.transpose(1, 2).contiguous(), q[:, :D].contiguous())
-        rot_q = reorder_heads(q[:, D:].reshape(H * R, -1), R, order).view(H, R, -1)
-        rows = [self._to_device(torch.cat([rot_q, latent_q], dim=1).reshape(H * (R + L), -1))]
+        pad = (0, self.cached_value - L)
+        if self.folded:
+            q, uk, uv, o = f64("q").view(H, D + R, -1), f64("uk").view(H, D, L), f64("uv").view(H, Dv, L), f64("o").view(-1, H, Dv)
+            latent_q = torch.matmul(uk.transpose(1, 2).contiguous(), q[:, :D].contiguous())
+            rot_q = reorder_heads(q[:, D:].reshape(H * R, -1), R, order).view(H, R, -1)
+            rows = [self._to_device(torch.cat([rot_q, latent_q], dim=1).reshape(H * (R + L), -1))]
+            # columns h V .. (h + 1) V, V the cached values' size: W_o[:, h] W_uv[h], zeros for the padding
+            out = torch.matmul(o.transpose(0, 1).contiguous(), uv)                      # [H, hidden, L]
+            out = torch.nn.functional.pad(out, pad).transpose(0, 1).reshape(-1, self.inner)
+        else:
+            q = get(w["q"]).view(H, D + R, -1)
+            rot_q = reorder_heads(q[:, D:].reshape(H * R, -1), R, order).view(H, R, -1)
+            rows = [self._to_device(torch.cat([q[:, :D], rot_q], dim=1).reshape(H * (D + R), -1))]
+            self.w_uk = self._to_device(get(w["uk"]).view(H, D, L).transpose(1, 2))               # [H, L, D]
+            self.w_uv = self._to_device(torch.nn.functional.pad(get(w["uv"]).view(H, Dv, L), pad))     # [H, Dv, V]
+            out = get(w["o"])
         dkv = get(w["dkv"])
         rows.append(self._to_device(torch.cat([dkv[:L], reorder_heads(dkv[L:], R, order)], dim=0)))
         if self.gate:
             rows.append(self._to_device(get(w["gate"])))
-        # columns h V .. (h + 1) V, V the cached values' size: W_o[:, h] W_uv[h], zeros for the padding
-        out = torch.matmul(o.transpose(0, 1).contiguous(), uv)                      # [H, hidden, L]
-        out = torch.nn.functional.pad(out, (0, self.cached_value - L)).transpose(0, 1).reshape(-1, self.inner)
         self.latent_norm_w = self._to_device(get(w["dkv_norm"]), torch.float32)
         self.position.load_weights(get)
         return torch.cat(rows, dim=0).contiguous(), self._to_device(out)
@@ -790,11 +812,17 @@ class RotaryLatentAttention(BranchMixer):
         table = self.position.table(ctx) if hasattr(self.position, "table") else None
         d_col0 = col0 + self.q_cols
         q = ops.latent_rows_write(proj, col0, d_col0, self.latent_norm_w, self.norm_eps, ctx.positions, ctx.slot_mapping[cache.group],
-                                  inv_freq, factor, self.num_heads, self.rotary_dim, self.latent_dim, cache.k, cache.v, table)
+                                  inv_freq, factor, self.num_heads, self.rotary_dim, self.latent_dim, cache.k, cache.v, table,
+                                  None if self.folded else self.head_dim)
+        n, gate_col0 = proj.shape[0], d_col0 + self.latent_dim + self.rotary_dim
+        if not self.folded:
+            ops.head_linear(proj, col0, self.head_dim + self.rotary_dim, self.w_uk, q.view(n, -1), self.rotary_dim, self.cached_key)
         a = ops.paged_attention(q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.cu_seqlens, ctx.context_lens, ctx.token_req,
                                 self.scale, int(self.window or 0), ctx.max_q_len, ctx.max_context_len, ctx.num_single)
-        ops.sigmoid_gate(a, proj if self.gate else None, d_col0 + self.latent_dim + self.rotary_dim, scale, out, out_col0,
-                         self.cached_value if self.gate else 1)
+        if not self.folded:
+            ops.head_linear(a, 0, self.cached_value, self.w_uv, out, out_col0, self.value_dim, proj if self.gate else None, gate_col0, scale)
+            return
+        ops.sigmoid_gate(a, proj if self.gate else None, gate_col0, scale, out, out_col0, self.cached_value if self.gate else 1)
 
 
 register_part("mixer", "rotary_latent_attention", RotaryLatentAttention)

@@ -371,9 +371,14 @@ class EmuOps:
         return torch.nn.functional.pad(q, pad).to(k_cache.dtype).contiguous()
 
     def latent_rows_write(self, rows, q_col0, d_col0, weight, eps, positions, slots, inv_freq, factor, num_heads, rotary_dim, latent_dim,
-                          k_cache, v_cache):
+                          k_cache, v_cache, plain_dim=None):
         n, key = rows.shape[0], rotary_dim + latent_dim
-        q = rows.double()[:, q_col0: q_col0 + num_heads * key].reshape(n, num_heads, key)
+        if plain_dim is None:
+            q = rows.double()[:, q_col0: q_col0 + num_heads * key].reshape(n, num_heads, key)
+        else:      # (the latent part is the caller's)
+            per = plain_dim + rotary_dim
+            q = rows.double()[:, q_col0: q_col0 + num_heads * per].reshape(n, num_heads, per)[..., plain_dim:]
+            q = torch.nn.functional.pad(q, (0, latent_dim))
         x = rows.double()[:, d_col0: d_col0 + key]
         c = x[:, :latent_dim]
         c = c / torch.sqrt((c * c).mean(-1, keepdim=True) + eps) * weight.double()
@@ -386,6 +391,14 @@ class EmuOps:
         k_cache[page, :, off] = torch.nn.functional.pad(k, (0, od - key)).to(k_cache.dtype)
         v_cache[page, 0, :, off] = torch.nn.functional.pad(c, (0, vd - latent_dim)).to(v_cache.dtype)
         return torch.nn.functional.pad(q, (0, od - key)).to(k_cache.dtype).contiguous()
+
+    def head_linear(self, x, x_col0, x_head, w, out, out_col0, out_head, gate, gate_col0, scale):
+        for h in range(w.shape[0]):
+            xs = x[:, x_col0 + h * x_head: x_col0 + h * x_head + w.shape[2]].to(w.dtype).double()
+            y = xs @ w[h].double().T * scale
+            if gate is not None:
+                y = y * torch.sigmoid(gate.double()[:, gate_col0 + h: gate_col0 + h + 1])
+            out[:, out_col0 + h * out_head: out_col0 + h * out_head + w.shape[1]] = y.to(out.dtype)
 
     def norm_add(self, h, y, weight, eps, next_weight=None, next_eps=0.0, out_dtype=None, gate=None, gate_col0=0, gate_bias=None):
         yd = y.double()

@@ -162,6 +162,23 @@ def test_each_part_alone_matches_its_plain_function(dirs, name):
     tokatar_mechanisms.check(dirs[name], name, "cpu", TOL)
 
 
+@pytest.mark.parametrize("name", ["wide", "deep"])
+def test_each_part_alone_in_bfloat16(dirs, name):
+    """The parts as the bfloat16 engine builds them: padded cache sizes, the activation in the product's epilogue, the
+    latent's maps as products per head (and folded where that is cheaper)."""
+    import tokatar_mechanisms
+    tokatar_mechanisms.check(dirs[name], name, "cpu", 6e-2, dtype="bfloat16")
+
+
+def test_the_latent_maps_are_folded_where_that_is_cheaper(dirs):
+    from tempura_amd.engine.loading import load_model
+    kinds = lambda name, dtype: [b.mixer.folded for b in load_model(dirs[name], dtype, "cpu").layers if hasattr(b.mixer, "folded")]
+    assert kinds("deep", "bfloat16") == [False] * 3 and kinds("deep", "float32") == [True] * 3
+    assert kinds("mix", "bfloat16") == [True, True]      # (heads of ten and eight elements: no product per head)
+    model = load_model(dirs["deep"], "bfloat16", "cpu")
+    assert [(g.head_dim, g.value_dim) for g in model.cache_groups] == [(288, 256), (320, 256), (576, 512)]
+
+
 def test_every_mechanism_matters_to_the_logits(monkeypatch):
     """The premise of every comparison of logits here: with any one mechanism left out or done otherwise, the plain
     implementation's own logits change far beyond the bounds."""

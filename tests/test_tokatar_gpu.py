@@ -141,6 +141,54 @@ def test_latent_rows_into_queries_and_cache(H, R, L, key, value, col0, n, dtype)
         _close(vd, v, tol)
 
 
+@pytest.mark.parametrize("n", [1, 30, 258])
+def test_rotated_queries_whose_latent_part_comes_from_elsewhere(n):
+    """The queries' rows hold [plain | rotated]: only the rotated part and the padding are written."""
+    ops = _ops()
+    g = torch.Generator().manual_seed(n)
+    for H, D, R, L, key, value in ((4, 32, 32, 256, 288, 256), (3, 48, 8, 20, 32, 32), (2, 10, 6, 10, 16, 10)):
+        rows = torch.randn(n, H * (D + R) + L + R + 6, generator=g)
+        w = torch.randn(L, generator=g)
+        pages = (n + 15) // 16 + 2
+        slots = _places(n, pages, 16, g)
+        positions = torch.randint(0, 3000, (n,), generator=g).to(torch.int32)
+        f = torch.pow(torch.tensor(900.0, dtype=torch.float64), -2.0 * torch.arange(R // 2, dtype=torch.float64) / R)
+        k, v = torch.zeros(pages, 1, 16, key, dtype=torch.bfloat16), torch.zeros(pages, 1, value, 16, dtype=torch.bfloat16)
+        kd, vd = _dev(k, v)
+        d_col0 = H * (D + R)
+        want = emu.latent_rows_write(rows, 0, d_col0, w, 1e-5, positions, slots, f, 1.0, H, R, L, k, v, D)
+        rd, wd, pd, sd, fd = _dev(rows, w, positions, slots, f)
+        got = ops.latent_rows_write(rd, 0, d_col0, wd, 1e-5, pd, sd, fd, 1.0, H, R, L, kd, vd, None, D)
+        _close(got[..., :R], want[..., :R], 8e-3)
+        assert key == R + L or float(got[..., R + L:].abs().max()) == 0.0
+        _close(kd, k, 8e-3)
+        _close(vd, v, 8e-3)
+
+
+@pytest.mark.parametrize("m", [1, 8, 17, 64, 65, 300, 1000])
+@pytest.mark.parametrize("H,N,K", [(3, 16, 32), (4, 256, 32), (18, 512, 64), (5, 48, 256), (8, 128, 512), (2, 80, 96)])
+def test_product_per_head(m, H, N, K):
+    """Strided float32 and bfloat16 rows in, pieces of wider bfloat16 rows out, with and without a gate per head; nothing
+    beside the pieces is touched."""
+    ops = _ops()
+    g = torch.Generator().manual_seed(H * N + K + m)
+    w = (torch.randn(H, N, K, generator=g) * K ** -0.5).to(torch.bfloat16)
+    x_head, out_head = K + 8, N + 4
+    x = torch.randn(m, 8 + H * x_head + 8, generator=g)
+    gate = torch.randn(m, 3 + H + 2, generator=g)
+    for xt in (x, x.to(torch.bfloat16)):
+        for gt in (None, gate):
+            out = torch.full((m, 4 + H * out_head + 4), 7.0, dtype=torch.bfloat16)
+            dev = out.to(DEV)
+            emu.head_linear(xt, 8, x_head, w, out, 4, out_head, gt, 3, 1.5)
+            ops.head_linear(xt.to(DEV), 8, x_head, w.to(DEV), dev, 4, out_head, None if gt is None else gt.to(DEV), 3, 1.5)
+            _close(dev, out, 8e-3)
+            same = torch.ones(out.shape[1], dtype=torch.bool)
+            for h in range(H):
+                same[4 + h * out_head: 4 + h * out_head + N] = False
+            assert bool((dev.cpu()[:, same] == 7.0).all())
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_outputs_turned_back_and_gated(dtype):
     ops = _ops()
@@ -252,7 +300,8 @@ def _attend(q, k, v, bt, cu, cl, scale, chunk, cap, sink, ps):
 @pytest.mark.parametrize("heads,kvh,d,vd,chunk,cap", [(4, 2, 12, 10, 9, 2.0), (1, 1, 20, 28, 16, 0.0), (3, 3, 6, 6, 1, 5.0), (4, 2, 64, 64, 50, 6.0),
                                                      (8, 1, 32, 32, 33, 0.0), (4, 4, 64, 32, 72, 3.0), (4, 4, 64, 32, 0, 0.0), (16, 1, 128, 128, 100, 4.0),
                                                      (4, 1, 128, 64, 0, 8.0), (2, 2, 128, 64, 64, 0.0), (5, 1, 160, 96, 0, 0.0), (4, 1, 192, 128, 0, 0.0),
-                                                     (32, 1, 192, 128, 90, 7.0), (2, 1, 96, 96, 48, 2.5), (6, 2, 32, 32, 32, 9.0)])
+                                                     (32, 1, 192, 128, 90, 7.0), (4, 1, 288, 256, 0, 0.0), (18, 1, 576, 512, 0, 0.0),
+                                                     (3, 1, 320, 256, 40, 4.0), (33, 1, 576, 512, 77, 3.0), (2, 1, 96, 96, 48, 2.5), (6, 2, 32, 32, 32, 9.0)])
 def test_attention_with_chunks_and_capped_scores(dtype, heads, kvh, d, vd, chunk, cap):
     """Portions behind cached prefixes and single tokens in one batch, every pair of sizes the matrix-core kernels take and
     some that they do not; with and without a sink of a constant score."""
@@ -283,7 +332,7 @@ def test_attention_with_chunks_and_capped_scores(dtype, heads, kvh, d, vd, chunk
         _close(got, want, tol)
 
 
-@pytest.mark.parametrize("heads,kvh,d,vd,chunk,cap", [(4, 1, 192, 128, 0, 0.0), (4, 2, 128, 128, 1500, 5.0), (2, 1, 128, 64, 0, 4.0), (8, 2, 64, 64, 700, 0.0)])
+@pytest.mark.parametrize("heads,kvh,d,vd,chunk,cap", [(4, 1, 192, 128, 0, 0.0), (20, 1, 576, 512, 0, 0.0), (4, 2, 128, 128, 1500, 5.0), (2, 1, 128, 64, 0, 4.0), (8, 2, 64, 64, 700, 0.0)])
 def test_long_contexts_in_parts_and_tiles(heads, kvh, d, vd, chunk, cap):
     """bfloat16, a portion behind 2,400 cached keys whose keys are split over blocks, a prompt beside it, and the kernels
     of 16 and of 32 query rows a wave and of per-wave loads forced in turn."""
@@ -374,7 +423,7 @@ def _ref(name, rid):
     return _REFS[(name, rid)]
 
 
-@pytest.mark.parametrize("name", ["mix", "one", "wide"])
+@pytest.mark.parametrize("name", ["mix", "one", "wide", "deep"])
 @pytest.mark.parametrize("dtype,tol", [("float32", 3e-5), ("bfloat16", 6e-2)])
 def test_each_part_alone_matches_its_plain_function(dirs, name, dtype, tol):
     import tokatar_mechanisms
@@ -382,7 +431,7 @@ def test_each_part_alone_matches_its_plain_function(dirs, name, dtype, tol):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["mix", "one", "wide"])
+@pytest.mark.parametrize("name", ["mix", "one", "wide", "deep"])
 @pytest.mark.parametrize("mode", ["whole", "bulk_tail", "portions", "mixed"])
 def test_every_cutting_matches_plain(dirs, name, mode, dtype):
     reqs = cases.requests(name)
@@ -469,14 +518,14 @@ def test_a_far_latent_decides_on_the_gpu(tmp_path):
     assert plain.logit_error(torch.cat(rows), ref) < SHARP_TOL
 
 
-@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_long_decoding_through_a_captured_step(dirs, dtype):
+@pytest.mark.parametrize("name,dtype", [("wide", "float32"), ("wide", "bfloat16"), ("deep", "bfloat16")])
+def test_long_decoding_through_a_captured_step(dirs, name, dtype):
     """Two requests decoded token by token for 150 steps through the graph path: pages, latents and chunks move along."""
     from tempura_amd.engine.runner import StepEntry
-    cfg, W = cases.config_json("wide"), cases.make_weights("wide")
-    runner = _runner(dirs["wide"], dtype, 512, use_graph=True)
+    cfg, W = cases.config_json(name), cases.make_weights(name)
+    runner = _runner(dirs[name], dtype, 512, use_graph=True)
     assert runner.use_graph, "every part of the design may be captured"
-    seqs = {"p": cases.tokens("wide", 170, 41), "q": cases.tokens("wide", 158, 42)}
+    seqs = {"p": cases.tokens(name, 170, 41), "q": cases.tokens(name, 158, 42)}
     start = {"p": 20, "q": 8}
     got = {rid: [] for rid in seqs}
     for rid in seqs:
@@ -488,7 +537,7 @@ def test_long_decoding_through_a_captured_step(dirs, dtype):
             got[rid].append(logits[k: k + 1].clone())
     assert runner.graph_steps >= 149
     for rid in seqs:
-        _assert_logits(torch.cat(got[rid]), plain.forward(cfg, W, seqs[rid]), dtype, f"captured {dtype} {rid}")
+        _assert_logits(torch.cat(got[rid]), plain.forward(cfg, W, seqs[rid]), dtype, f"captured {name} {dtype} {rid}")
 
 
 @pytest.mark.parametrize("name", ["mix", "wide"])

@@ -68,6 +68,10 @@ CASES: Dict[str, dict] = {
                             _layer(_attention(8, 1, 32, 32, 0.2, _rot(16, 3000.0), chunk=33), None),
                             _layer(_latent(2, 64, 64, 32, 128, 0.09, 8000.0), 64),
                             _layer(_attention_2(2, 1, 128, 128, 0.09, _rot(128, 20000.0)), 128)], 1e-5, 1.75),
+    # latents much wider than the heads: the matrix-core kernels for keys of several hundred, maps as products per head
+    "deep": _case(70, 64, [_layer(_latent(4, 32, 32, 32, 256, 0.125, 1000.0), 64),
+                           _layer(_latent(3, 32, 64, 48, 256, 0.1, 3000.0), None),
+                           _layer(_latent(18, 64, 64, 32, 512, 0.09, 8000.0), 128)], 1e-5, 2.0),
 }
 
 
@@ -148,7 +152,8 @@ def tokens(name: str, n: int, seed: int) -> List[int]:
 #: request lengths per case: one token, a few, around pages' and chunks' edges, long
 LENGTHS = {"mix": {"m0": 1, "m1": 6, "m2": 23, "m3": 49, "m4": 33, "m5": 16},
            "one": {"o0": 2, "o1": 31, "o2": 17, "o3": 1, "o4": 40},
-           "wide": {"w0": 5, "w1": 74, "w2": 33, "w3": 160, "w4": 50}}
+           "wide": {"w0": 5, "w1": 74, "w2": 33, "w3": 160, "w4": 50},
+           "deep": {"d0": 3, "d1": 90, "d2": 17, "d3": 140, "d4": 64}}
 
 
 def requests(name: str) -> Dict[str, List[int]]:
