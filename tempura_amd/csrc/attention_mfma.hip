@@ -885,6 +885,347 @@ __global__ __launch_bounds__(256, OCC) void attn_prefill_lds_kernel(AttnArgs a, 
   }
 }
 
+// ---- prefill, keys of several hundred (latents) -----------------------------------------------
+// A block owns 64 query rows, rows being (token, head) pairs of one key group in memory order (so any number of heads
+// fills them), and walks the keys 64 at a time.  Its four waves split the work twice: for the scores by keys (wave w
+// multiplies keys 16 w.. of the step with all 64 rows, whose q lies in its registers), for the sums over the values by
+// elements (wave w owns the w-th quarter of the value elements of all rows).  So every key and value fragment is needed
+// by ONE wave: each wave copies its own into its own part of LDS by direct global-to-LDS loads and waits for them alone,
+// the next step's keys behind the score product, the next step's values behind the value product.  What the waves
+// exchange is small: the maxima of their keys and the probabilities, two barriers a step.
+// Pages of at least 16 keys (a power of two): the 16 keys of a wave lie in one page.
+// LDS per wave: 16 key rows of D elements, chunk c (16 bytes) of row r at (c + f(r)) mod (D / 8) with f chosen so that
+// eight neighbouring rows fall into different banks; the values in pieces of 1 KB, one per (32 elements, 16 keys), the
+// eight keys 8 e.. of element d at place 32 e + d % 32.
+__device__ inline void attn_lds_write8(unsigned addr, unsigned a, unsigned b) {
+  typedef unsigned int u32x2 __attribute__((ext_vector_type(2)));
+  const u32x2 v = {a, b};
+  asm volatile("ds_write_b64 %0, %1" ::"v"(addr), "v"(v) : "memory");
+}
+__device__ inline void attn_lds_write4(unsigned addr, float v) { asm volatile("ds_write_b32 %0, %1" ::"v"(addr), "v"(v) : "memory"); }
+template <int N>
+__device__ inline void attn_wait_lds() {
+  asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(N) : "memory");
+}
+
+// o += values x probabilities with the running sum in VECTOR registers, where the softmax rescales it: the builtin would put
+// it into the accumulation registers and copy all of it there and back in every step.  (Nothing here waits for the
+// product or for what its operands wait for: the operands come from LDS reads that have returned, o is rescaled before a
+// barrier and read by the next step's softmax, a whole score product later.)
+__device__ inline void attn_pv_in_place(f32x4_t& o, const bf16x8_t& v, const bf16x8_t& p) {
+  asm volatile("v_mfma_f32_16x16x32_bf16 %0, %1, %2, %0" : "+v"(o) : "v"(v), "v"(p));
+}
+// f(integral_constant<I>) for I = B .. E - 1
+template <int I>
+struct attn_int {
+  static constexpr int value = I;
+};
+template <int B, int E, typename F>
+__device__ __attribute__((always_inline)) inline void attn_for(F&& f) {
+  if constexpr (B < E) {
+    f(attn_int<B>{});
+    attn_for<B + 1, E>(f);
+  }
+}
+// one direct load of 16 bytes a lane from base + off (the lane's) + uniform into LDS, as a buffer load: neither part needs
+// a 64-bit address per lane
+__device__ inline void attn_copy16(const unsigned char* base, unsigned off, unsigned uniform, unsigned char* lds) {
+  const __amdgpu_buffer_rsrc_t rsrc = __builtin_amdgcn_make_buffer_rsrc((void*)base, 0, 0x7fffffff, 0x00020000);
+  __builtin_amdgcn_raw_ptr_buffer_load_lds(rsrc, LPTR(lds), 16, off, uniform, 0, 0);
+}
+
+template <int D, int DV, int MODE>
+__global__ __launch_bounds__(256, 1) void attn_prefill_latent_kernel(AttnArgs a, int skip_single) {
+  constexpr bool CAP = MODE == MODE_CAP;
+  constexpr int C = D / 8;                       // 16-byte chunks of a key row
+  constexpr int NK = D / 32;                     // key fragments, and 1 KB loads, of a wave's 16 keys
+  constexpr int NT = DV / 64;                    // tiles of 16 value elements a wave owns
+  constexpr int NV = DV / 128 * 4;               // 1 KB loads of a wave's values: (32 elements, 16 keys) each
+  constexpr int PER = C % 8 == 0 ? C / 8 : C / 4;   // loads after which the pattern of the key rows repeats (eight or sixteen rows)
+  constexpr int DW = (D / 2) % 64;
+  constexpr int SH = DW == 32 ? 1 : 2;           // f(r) = (r % 8) >> SH
+  static_assert(DW == 32 || DW == 16 || DW == 48, "the rotation of the key rows is worked out for these row lengths");
+  static_assert(D % 32 == 0 && DV % 128 == 0 && 16 * C == NK * 64, "sizes");
+  constexpr int PIN = 15;                        // fragments of q (of all four row tiles) in accumulation registers
+  constexpr int QL = NK > PIN + 1 ? NK - PIN - 1 : 0;   // and in LDS (the last ones); at most one in vector registers
+  constexpr int PLD = 144;                       // bytes of a row of probabilities (64 keys, padded)
+  constexpr int KB = NK * 1024, VB = NV * 1024;
+  __shared__ __attribute__((aligned(1024))) unsigned char kv_lds[4 * (KB + VB)];
+  __shared__ __attribute__((aligned(16))) unsigned char p_lds[64 * PLD];
+  __shared__ __attribute__((aligned(16))) float m_lds[64 * 4];
+  __shared__ u32x4_t q_lds[QL > 0 ? QL * 4 * 64 : 1];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int g = lane >> 4, c = lane & 15;
+  const int r = blockIdx.z, kvh = blockIdx.y;
+  const int q_start = a.cu_seqlens[r];
+  const int q_len = a.cu_seqlens[r + 1] - q_start;
+  if (q_len <= 0 || (skip_single && q_len == 1)) return;
+  const int group = a.n_heads / a.n_kv;
+  const int rows = q_len * group;
+  const int nb = (rows + 63) / 64;
+  if ((int)blockIdx.x >= nb) return;
+  const int row0 = (nb - 1 - (int)blockIdx.x) * 64;      // (the longest blocks first)
+  const int ctx = a.context_lens[r];
+  const int pos0 = ctx - q_len;
+  const int ps = a.page_size, psh = a.page_shift, pmask = ps - 1;
+  const __attribute__((address_space(4))) int* ctab =
+      (const __attribute__((address_space(4))) int*)(uintptr_t)(a.block_tables + (size_t)r * a.table_width);
+
+  bf16x8_t qf[4][NK - QL];
+  int qpos[4];
+  float m[4], l[4];
+  f32x4_t o[4][NT];
+#pragma unroll
+  for (int nq = 0; nq < 4; ++nq) {
+    const int row = min(row0 + nq * 16 + c, rows - 1);     // (rows past the end repeat the last one, never written)
+    const int t = row / group;
+    qpos[nq] = pos0 + t;
+    const bf16_t* qr = a.q + ((size_t)(q_start + t) * a.n_heads + kvh * group + row % group) * D + g * 8;
+#pragma unroll
+    for (int dk = 0; dk < NK - QL; ++dk) qf[nq][dk] = frag_of(*(const u32x4_t*)(qr + dk * 32));
+    if (QL > 0 && wave == nq) {
+#pragma unroll
+      for (int e = 0; e < QL; ++e) q_lds[(e * 4 + nq) * 64 + lane] = *(const u32x4_t*)(qr + (NK - QL + e) * 32);
+    }
+    // (as much of q as fits beside the scores goes to the accumulation registers)
+#pragma unroll
+    for (int dk = 0; dk < NK - QL && dk < PIN; ++dk) asm volatile("" : "+a"(qf[nq][dk]));
+    asm volatile("" ::: "memory");
+    m[nq] = -INFINITY;
+    l[nq] = 0.f;
+#pragma unroll
+    for (int dt = 0; dt < NT; ++dt) o[nq][dt] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+  }
+  const int first_pos = pos0 + row0 / group, last_pos = pos0 + min(row0 + 63, rows - 1) / group;
+  const int first = max(0, attn_first_key(a, first_pos)) & ~63;
+  const int seen_by_all = attn_first_key(a, last_pos);
+  const int nsteps = (last_pos - first) / 64 + 1;
+
+  // ---- loads
+  const unsigned kpage_bytes = (unsigned)(a.n_kv * D * ps * 2), vpage_bytes = (unsigned)(a.n_kv * DV * ps * 2);
+  const unsigned char* kbase = (const unsigned char*)a.k_cache + (size_t)kvh * ps * D * 2;
+  const unsigned char* vbase = (const unsigned char*)a.v_cache + ((size_t)kvh * DV + wave * (DV / 4)) * ps * 2;
+  unsigned char* kbuf = kv_lds + wave * KB;
+  unsigned char* vbuf = kv_lds + 4 * KB + wave * VB;
+  unsigned koff[PER];      // where slot 64 t + lane of the key rows comes from
+#pragma unroll
+  for (int t = 0; t < PER; ++t) {
+    const int row = (64 * t + lane) / C, f = (row & 7) >> SH;
+    koff[t] = (unsigned)(row * D * 2 + (((64 * t + lane) % C - f + C) % C) * 16);
+  }
+  const unsigned voff = (unsigned)(((lane & 31) * ps + 8 * (lane >> 5)) * 2);
+  auto issue_keys = [&](int j0) __attribute__((always_inline)) {
+    const int k0 = min(j0 + 16 * wave, (ctx - 1) & ~15);    // (a quarter past the last key: that key's, masked below)
+    const unsigned char* base = kbase + (size_t)(unsigned)ctab[k0 >> psh] * kpage_bytes + (unsigned)((k0 & pmask) * D * 2);
+    // (places past the last key hold anything: their scores are masked)
+#pragma unroll
+    for (int t = 0; t < NK; ++t) attn_copy16(base, koff[t % PER], (unsigned)(t / PER * 8 * D * 2), kbuf + t * 1024);
+  };
+  auto issue_values = [&](int j0) __attribute__((always_inline)) {
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int k0 = min(j0 + 16 * q, (ctx - 1) & ~15);
+      const unsigned char* base = vbase + (size_t)(unsigned)ctab[k0 >> psh] * vpage_bytes + (unsigned)((k0 & pmask) * 2);
+#pragma unroll
+      for (int b = 0; b < DV / 128; ++b)
+        attn_copy16(base, voff, (unsigned)(b * 32 * ps * 2), vbuf + (b * 4 + q) * 1024);
+    }
+  };
+  // ---- this lane's LDS addresses
+  const unsigned lds0 = (unsigned)(size_t)(__attribute__((address_space(3))) const unsigned char*)&kv_lds[0];
+  const unsigned plds = (unsigned)(size_t)(__attribute__((address_space(3))) const unsigned char*)&p_lds[0];
+  const unsigned mlds = (unsigned)(size_t)(__attribute__((address_space(3))) const unsigned char*)(const __attribute__((address_space(3))) float*)&m_lds[0];
+  // key fragment dk: row c, chunk 4 dk + g, rotated; only the last fragment's chunk can wrap to the row's start
+  static_assert(4 * (NK - 2) + 3 + (7 >> SH) < C, "only the last fragment wraps");
+  const int kf = g + ((c & 7) >> SH), klast = 4 * (NK - 1) + kf;
+  const unsigned krow = lds0 + wave * KB + c * D * 2 + kf * 16;
+  const unsigned kwrap = lds0 + wave * KB + c * D * 2 + (klast >= C ? klast - C : klast) * 16;
+  const unsigned vaddr = lds0 + 4 * KB + wave * VB + (g >> 1) * 1024 + (g & 1) * 512 + c * 16;
+  const unsigned pwrite = plds + c * PLD + (16 * wave + 4 * g) * 2;
+  const unsigned pread = plds + c * PLD + g * 16;
+  const unsigned mwrite = mlds + (unsigned)((lane * 4 + wave) * 4), mread = mlds + c * 16;
+
+  const unsigned qaddr = (unsigned)(size_t)(__attribute__((address_space(3))) const unsigned char*)(const __attribute__((address_space(3))) u32x4_t*)&q_lds[0] + lane * 16;
+  if (QL > 0) __syncthreads();
+  issue_keys(first);
+  issue_values(first);
+  for (int s = 0; s < nsteps; ++s) {
+    const int j0 = first + s * 64;
+    // this step's keys have landed (its values, issued behind them, may still travel)
+    ATTN_WAIT_VM(NV);
+    f32x4_t sc[4];
+#pragma unroll
+    for (int nq = 0; nq < 4; ++nq) sc[nq] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+    u32x4_t kk[NK];
+    auto read_key = [&](auto i) __attribute__((always_inline)) {
+      constexpr int dk = decltype(i)::value;
+      if constexpr (dk < NK - 1) kk[dk] = attn_lds_read<dk * 64>(krow);
+      else if constexpr (dk == NK - 1) kk[dk] = attn_lds_read<0>(kwrap);
+    };
+    constexpr int AHEAD = 3;
+    attn_for<0, AHEAD>(read_key);
+    static_assert(QL < AHEAD, "the keys of the fragments whose q lies in LDS are read ahead");
+    attn_for<0, NK - QL>([&](auto i) __attribute__((always_inline)) {
+      constexpr int dk = decltype(i)::value;
+      read_key(attn_int<dk + AHEAD>{});
+      attn_wait_lds<(NK - 1 - dk < AHEAD ? NK - 1 - dk : AHEAD)>();
+      asm volatile("" : "+v"(kk[dk]));
+#pragma unroll
+      for (int nq = 0; nq < 4; ++nq) sc[nq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag_of(kk[dk]), qf[nq][dk], sc[nq], 0, 0, 0);
+    });
+    attn_for<NK - QL, NK>([&](auto i) __attribute__((always_inline)) {
+      constexpr int dk = decltype(i)::value;
+      u32x4_t qq[4];
+      qq[0] = attn_lds_read<(dk - NK + QL) * 4096>(qaddr);
+      qq[1] = attn_lds_read<(dk - NK + QL) * 4096 + 1024>(qaddr);
+      qq[2] = attn_lds_read<(dk - NK + QL) * 4096 + 2048>(qaddr);
+      qq[3] = attn_lds_read<(dk - NK + QL) * 4096 + 3072>(qaddr);
+      attn_wait_lds<0>();
+      asm volatile("" : "+v"(kk[dk]));
+#pragma unroll
+      for (int nq = 0; nq < 4; ++nq) {
+        asm volatile("" : "+v"(qq[nq]));
+        sc[nq] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag_of(kk[dk]), frag_of(qq[nq]), sc[nq], 0, 0, 0);
+      }
+    });
+    if (s + 1 < nsteps) issue_keys(j0 + 64);      // (every read of the keys has returned)
+    // ---- softmax: this lane holds keys j0 + 16 wave + 4 g + 0..3 of row 16 nq + c
+    float v[4][4], mine = -INFINITY;
+    const bool all_seen = j0 + 63 <= first_pos && j0 >= seen_by_all;
+    const int key0 = j0 + 16 * wave + 4 * g;
+#pragma unroll
+    for (int nq = 0; nq < 4; ++nq) {
+      const int hi = qpos[nq], lo = all_seen ? 0 : attn_first_key(a, hi);
+      float mx = -INFINITY;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float x = CAP ? attn_capped(a, sc[nq][e]) : sc[nq][e];
+        const int key = key0 + e;
+        v[nq][e] = (all_seen | ((key <= hi) & (key >= lo))) ? x : -INFINITY;
+        mx = fmaxf(mx, v[nq][e]);
+      }
+      mx = quad_rows_max(mx);
+      mine = g == nq ? mx : mine;                 // (lane (g, c) hands over tile g's maximum of row c)
+    }
+    attn_lds_write4(mwrite, mine);
+    attn_wait_lds<0>();
+    __builtin_amdgcn_s_barrier();
+    u32x4_t mm[4];      // (the other waves' maxima of a row, one tile ahead)
+    mm[0] = attn_lds_read<0>(mread);
+    float alpha[4];
+    bool moved[4];
+#pragma unroll
+    for (int nq = 0; nq < 4; ++nq) {
+      attn_wait_lds<0>();
+      asm volatile("" : "+v"(mm[nq]));
+      if (nq == 0) mm[1] = attn_lds_read<256>(mread);
+      if (nq == 1) mm[2] = attn_lds_read<512>(mread);
+      if (nq == 2) mm[3] = attn_lds_read<768>(mread);
+      const f32x4_t w4 = __builtin_bit_cast(f32x4_t, mm[nq]);
+      const float mx = fmaxf(fmaxf(w4[0], w4[1]), fmaxf(w4[2], w4[3]));
+      const float m_new = fmaxf(m[nq], CAP ? mx : mx * a.scale_log2);
+      const float m_use = m_new == -INFINITY ? 0.f : m_new;
+      float sum = 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        v[nq][e] = __builtin_amdgcn_exp2f(CAP ? v[nq][e] - m_use : fmaf(v[nq][e], a.scale_log2, -m_use));
+        sum += v[nq][e];
+      }
+      moved[nq] = __builtin_amdgcn_ballot_w64(m_new != m[nq]) != 0;
+      const float shrink = __builtin_amdgcn_exp2f(m[nq] - m_use);
+      alpha[nq] = moved[nq] ? shrink : 1.0f;
+      l[nq] = fmaf(l[nq], alpha[nq], sum);        // (this lane's keys; lanes and waves are added at the end)
+      m[nq] = m_new;
+      attn_lds_write8(pwrite + nq * 16 * PLD, pack_bf16(v[nq][0], v[nq][1]), pack_bf16(v[nq][2], v[nq][3]));
+    }
+#pragma unroll
+    for (int nq = 0; nq < 4; ++nq)
+      if (moved[nq]) {
+#pragma unroll
+        for (int dt = 0; dt < NT; ++dt) {
+          o[nq][dt][0] *= alpha[nq];
+          o[nq][dt][1] *= alpha[nq];
+          o[nq][dt][2] *= alpha[nq];
+          o[nq][dt][3] *= alpha[nq];
+        }
+      }
+    attn_wait_lds<0>();
+    __builtin_amdgcn_s_barrier();
+    // ---- values: landed once only the next step's keys may be in flight
+    if (s + 1 < nsteps) ATTN_WAIT_VM(NK); else ATTN_WAIT_VM(0);
+    const bool partial = j0 + 64 > ctx;           // (places past the last key hold anything: cleared)
+#pragma unroll
+    for (int s2 = 0; s2 < 2; ++s2) {
+      u32x4_t pp[4], vv[NT];
+#pragma unroll
+      for (int nq = 0; nq < 4; ++nq) pp[nq] = attn_lds_read<0>(pread + nq * 16 * PLD + s2 * 64);
+#define LAT_RV(dt) if constexpr ((dt) < NT) vv[dt] = attn_lds_read<((dt) >> 1) * 4 * 1024 + ((dt) & 1) * 256>(vaddr + s2 * 2048)
+#define LAT_PV(dt)                                                                                                     \
+  if constexpr ((dt) < NT) {                                                                                           \
+    LAT_RV(dt + 2);                                                                                                    \
+    attn_wait_lds<(NT - 1 - (dt) < 2 ? NT - 1 - (dt) : 2)>();                                                          \
+    asm volatile("" : "+v"(vv[dt]));                                                                                   \
+    if (partial) {                                                                                                     \
+      vv[dt] &= keep;                                                                                                  \
+      asm volatile("s_nop 3" : "+v"(vv[dt]));   /* (a vector write in front of a matrix product that reads it) */      \
+    }                                                                                                                  \
+    _Pragma("unroll") for (int nq = 0; nq < 4; ++nq) attn_pv_in_place(o[nq][dt], frag_of(vv[dt]), pf[nq]);             \
+  }
+      LAT_RV(0); LAT_RV(1);
+      static_assert(NT <= 8, "value tiles of a wave");
+      const u32x4_t keep = attn_existing_keys(ctx - (j0 + 32 * s2 + 8 * g));
+      bf16x8_t pf[4];
+      attn_wait_lds<2>();
+#pragma unroll
+      for (int nq = 0; nq < 4; ++nq) {
+        asm volatile("" : "+v"(pp[nq]));
+        pf[nq] = frag_of(pp[nq]);
+      }
+      LAT_PV(0) LAT_PV(1) LAT_PV(2) LAT_PV(3) LAT_PV(4) LAT_PV(5) LAT_PV(6) LAT_PV(7)
+#undef LAT_PV
+#undef LAT_RV
+    }
+    if (s + 1 < nsteps) issue_values(j0 + 64);    // (every read of the values has returned)
+  }
+  // ---- the waves' sums, then the rows
+  asm volatile("s_nop 15\n\ts_nop 15" ::: "memory");      // (the last products have written the running sums)
+#pragma unroll
+  for (int nq = 0; nq < 4; ++nq)
+#pragma unroll
+    for (int dt = 0; dt < NT; ++dt) asm volatile("" : "+v"(o[nq][dt]));
+#pragma unroll
+  for (int nq = 0; nq < 4; ++nq) {
+    l[nq] += __shfl_xor(l[nq], 16, 64);
+    l[nq] += __shfl_xor(l[nq], 32, 64);
+  }
+  // (the maxima's reads of the last step lie before its second barrier: their place is free)
+  attn_lds_write4(mwrite, g == 0 ? l[0] : g == 1 ? l[1] : g == 2 ? l[2] : l[3]);
+  attn_wait_lds<0>();
+  __builtin_amdgcn_s_barrier();
+  int ce = c;
+  asm volatile("" : "+v"(ce));      // (the rows' tokens and heads are worked out anew: nothing of them is kept over the loop)
+#pragma unroll
+  for (int nq = 0; nq < 4; ++nq) {
+    u32x4_t lw = attn_lds_read<0>(mread + nq * 256);
+    attn_wait_lds<0>();
+    asm volatile("" : "+v"(lw));
+    const f32x4_t l4 = __builtin_bit_cast(f32x4_t, lw);
+    const int row = row0 + nq * 16 + ce;
+    if (row < rows) {
+      const int t = row / group, head = kvh * group + row % group;
+      const float inv = 1.0f / (((l4[0] + l4[1]) + (l4[2] + l4[3])) + sink_term(a.sink, head, m[nq]));
+      bf16_t* orow = a.out + ((size_t)(q_start + t) * a.n_heads + head) * DV + wave * (DV / 4);
+#pragma unroll
+      for (int dt = 0; dt < NT; ++dt) {
+        uint2 w;
+        w.x = pack_bf16(o[nq][dt][0] * inv, o[nq][dt][1] * inv);
+        w.y = pack_bf16(o[nq][dt][2] * inv, o[nq][dt][3] * inv);
+        *(uint2*)(orow + dt * 16 + 4 * g) = w;
+      }
+    }
+  }
+}
+
 // ---- decode -----------------------------------------------------------------------------
 // grid: (kv_heads * ceil(group / 16), requests, splits); block: 4 waves.  Handles requests
 // with exactly one new token.  Scratch per (request, head, split): DV floats of O, then max, sum.
@@ -1134,6 +1475,13 @@ static int launch_all(AttnArgs a, int n_tokens, int n_req, int max_q_len, int nu
       }
     }
     a.portion_splits = 1;   // (the kernels below do not split)
+    if constexpr (D > 192) {
+      if (g_attn_tune != 1 && a.page_shift >= 4 && a.keep_first == 0) {
+        const dim3 lgrid((unsigned)(((long)max_q_len * group + 63) / 64), a.n_kv, n_req);
+        hipLaunchKernelGGL((attn_prefill_latent_kernel<D, DV, MODE>), lgrid, dim3(256), 0, s, a, skip);
+        return 0;
+      }
+    }
     const dim3 grid((max_q_len + rows - 1) / rows, kv_groups, n_req);
     if constexpr (LDS) {
       if (lds_pages) {
