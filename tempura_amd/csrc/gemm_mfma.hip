@@ -169,7 +169,8 @@ __device__ inline void row_scale_finish(const RowScale& pre, const RowScaleLoads
 // MT: 16-row tiles of activations; NT: 16-row tiles of weights per block; WAVES: waves that
 // split K.  A wave takes K in runs of four consecutive 32-wide steps (256 contiguous bytes of
 // each weight row), run r going to wave r % WAVES.
-template <int MT, int NT, int WAVES, int DEPTH, bool WT>
+// SPLIT: mode OUT_SPLIT, in kernels of its own (its branch in the others' epilogue costs every short product half a microsecond)
+template <int MT, int NT, int WAVES, int DEPTH, bool WT, bool SPLIT>
 __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_mfma_kernel(const bf16_t* __restrict__ x,
                                                                       const bf16_t* __restrict__ w,
                                                                       void* __restrict__ out, int mode, int M,
@@ -255,7 +256,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_mfma_kernel(const bf16
     const int n = n0 + j * 16 + (l >> 4) * 4 + r;   // weight row = output column
     const int m = t * 16 + (l & 15);
     if (MT == 1) v *= rstd[l & 15];
-    if (mode == OUT_SWIGLU) {
+    if constexpr (SPLIT) {
+      if (n < N && m < M) store_split(out, layout, rp.gate, M, m, n, v);
+    } else if (mode == OUT_SWIGLU) {
       if ((l >> 4) < 2 && n + 8 < N && m < M) {       // a gate row: its up row is eight further on
         float u = 0.f;
 #pragma unroll
@@ -280,8 +283,6 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_mfma_kernel(const bf16
     } else if (mode == OUT_ROPE) {
       const float other = __shfl_xor(v, 1, 64);   // r and r ^ 1 are neighbouring lanes
       if (n < N && m < M) rope_store(rp, m, n, v, other);
-    } else if (mode == OUT_SPLIT) {
-      if (n < N && m < M) store_split(out, layout, rp.gate, M, m, n, v);
     } else if (n < N && m < M) {
       store_out(out, mode, (size_t)m * N + n, v);
     }
@@ -313,7 +314,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_mfma_kernel(const bf16
 // before anything is multiplied, and again as soon as their registers are free, always in the order in
 // which they are consumed (loads return in order): a block has 256 bytes per lane in flight from its
 // first cycle.  (Measured against one chunk of prefetch: 5-10 % faster at 8 and 16 rows.)
-template <int NT, int WAVES, bool WT>
+template <int NT, int WAVES, bool WT, bool SPLIT>
 __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_lds_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                                                                void* __restrict__ out, int mode, int M, int N, int K,
                                                                int layout, RowScale pre, NormPrep post, RopeOut rp) {
@@ -414,7 +415,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_lds_kernel(const bf16_
     const int n = nt0 + (l >> 4) * 4 + r;
     const int m = l & 15;
     v *= rstd[m];
-    if (mode == OUT_SWIGLU) {
+    if constexpr (SPLIT) {
+      if (n < N && m < M) store_split(out, layout, rp.gate, M, m, n, v);
+    } else if (mode == OUT_SWIGLU) {
       if ((l >> 4) < 2 && n + 8 < N && m < M) {
         float u = 0.f;
 #pragma unroll
@@ -438,8 +441,6 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_lds_kernel(const bf16_
     } else if (mode == OUT_ROPE) {
       const float other = __shfl_xor(v, 1, 64);
       if (n < N && m < M) rope_store(rp, m, n, v, other);
-    } else if (mode == OUT_SPLIT) {
-      if (n < N && m < M) store_split(out, layout, rp.gate, M, m, n, v);
     } else if (n < N && m < M) {
       store_out(out, mode, (size_t)m * N + n, v);
     }
@@ -716,12 +717,18 @@ template <int MT, int NT, int WAVES, int DEPTH>
 static void launch_skinny4(const bf16_t* x, const bf16_t* w, void* out, int mode, int M, int N, int K, int layout,
                            RowScale pre, NormPrep post, const RopeOut& rp, hipStream_t s) {
   const int blocks = (N + 16 * NT - 1) / (16 * NT);
-  if (layout & W_TILED)
-    hipLaunchKernelGGL((gemm_skinny_mfma_kernel<MT, NT, WAVES, DEPTH, true>), dim3(blocks), dim3(WAVES * 64), 0, s, x, w, out,
-                       mode, M, N, K, layout, pre, post, rp);
-  else
-    hipLaunchKernelGGL((gemm_skinny_mfma_kernel<MT, NT, WAVES, DEPTH, false>), dim3(blocks), dim3(WAVES * 64), 0, s, x, w, out,
-                       mode, M, N, K, layout, pre, post, rp);
+#define SKINNY(WT_, SPLIT_)                                                                                                              \
+  hipLaunchKernelGGL((gemm_skinny_mfma_kernel<MT, NT, WAVES, DEPTH, WT_, SPLIT_>), dim3(blocks), dim3(WAVES * 64), 0, s, x, w, out, mode, \
+                     M, N, K, layout, pre, post, rp)
+  if (mode == OUT_SPLIT) {
+    if (layout & W_TILED) SKINNY(true, true);
+    else SKINNY(false, true);
+  } else if (layout & W_TILED) {
+    SKINNY(true, false);
+  } else {
+    SKINNY(false, false);
+  }
+#undef SKINNY
 }
 
 template <int MT>
@@ -748,12 +755,15 @@ static void launch_skinny(const bf16_t* x, const bf16_t* w, void* out, int mode,
       if (nt > 2) nt = 2;
       const int blocks = (N + 16 * nt - 1) / (16 * nt);
       const bool wt = (layout & W_TILED) != 0;
-#define LDS_CASE(NT_, WT_) \
-  hipLaunchKernelGGL((gemm_skinny_lds_kernel<NT_, 8, WT_>), dim3(blocks), dim3(512), 0, s, x, w, out, mode, M, N, K, layout, pre, post, rp)
-      if (nt == 2 && wt) LDS_CASE(2, true);
-      else if (nt == 2) LDS_CASE(2, false);
-      else if (wt) LDS_CASE(1, true);
-      else LDS_CASE(1, false);
+#define LDS_CASE(NT_, WT_)                                                                                                                     \
+  do {                                                                                                                                         \
+    if (mode == OUT_SPLIT)                                                                                                                     \
+      hipLaunchKernelGGL((gemm_skinny_lds_kernel<NT_, 8, WT_, true>), dim3(blocks), dim3(512), 0, s, x, w, out, mode, M, N, K, layout, pre,    \
+                         post, rp);                                                                                                            \
+    else                                                                                                                                       \
+      hipLaunchKernelGGL((gemm_skinny_lds_kernel<NT_, 8, WT_, false>), dim3(blocks), dim3(512), 0, s, x, w, out, mode, M, N, K, layout, pre,   \
+                         post, rp);                                                                                                            \
+  } while (0)
 #undef LDS_CASE
       return;
     }
