@@ -764,6 +764,10 @@ static void launch_skinny(const bf16_t* x, const bf16_t* w, void* out, int mode,
       hipLaunchKernelGGL((gemm_skinny_lds_kernel<NT_, 8, WT_, false>), dim3(blocks), dim3(512), 0, s, x, w, out, mode, M, N, K, layout, pre,   \
                          post, rp);                                                                                                            \
   } while (0)
+      if (nt == 2 && wt) LDS_CASE(2, true);
+      else if (nt == 2) LDS_CASE(2, false);
+      else if (wt) LDS_CASE(1, true);
+      else LDS_CASE(1, false);
 #undef LDS_CASE
       return;
     }
