@@ -306,13 +306,13 @@ __global__ __launch_bounds__(256) void latent_rows_write_kernel(const float* __r
     }
     return;
   }
-  const int key = rot + latent;
-  const int end = min(heads * out_dim / V, (int)blockIdx.y * per_slice);
+  // a head's elements that this kernel writes: all of them, or all but the latent part
+  const int key = rot + latent, skip = latent_follows ? 0 : latent, span = out_dim - skip;
+  const int end = min(heads * span / V, (int)blockIdx.y * per_slice);
   for (int g = ((int)blockIdx.y - 1) * per_slice + threadIdx.x; g < end; g += blockDim.x) {
-    const int h = g * V / out_dim, i = g * V % out_dim;
+    const int h = g * V / span, j = g * V % span, i = j < rot ? j : j + skip;
     Elems<V> r;
     if (i < key) {
-      if (i >= rot && !latent_follows) continue;
       r = load_elems<V>(row + q_col0 + (size_t)h * q_head + q_rot + i);
       turn_pairs<V>(r, i, rot / 2, t, pos, inv_freq, table, factor, 1.0f);
     } else {
@@ -337,10 +337,11 @@ extern "C" int tp_latent_rows_write(const float* rows, size_t stride, int q_col0
   TP_REQUIRE(rot == 0 || inv_freq != nullptr, "latent_rows_write: no frequency table");
   TP_REQUIRE(dt == TP_F32 || dt == TP_BF16, "latent_rows_write: unknown dtype %d", dt);
   if (n == 0) return 0;
-  const bool four = key % 4 == 0 && rot % 4 == 0 && q_head % 4 == 0 && q_rot % 4 == 0 && out_dim % 4 == 0 && stride % 4 == 0 && q_col0 % 4 == 0 && ((uintptr_t)rows & 15) == 0;
+  const bool four = key % 4 == 0 && rot % 4 == 0 && (latent_follows || latent % 4 == 0) && q_head % 4 == 0 && q_rot % 4 == 0 && out_dim % 4 == 0 && stride % 4 == 0 && q_col0 % 4 == 0 && ((uintptr_t)rows & 15) == 0;
   const int V = four ? 4 : 2;
   const int per_slice = n >= 256 ? 1024 : 256;
-  const dim3 grid(n, 1 + (heads * out_dim / V + per_slice - 1) / per_slice);
+  const int span = latent_follows ? out_dim : out_dim - latent;
+  const dim3 grid(n, 1 + (heads * span / V + per_slice - 1) / per_slice);
   TP_REQUIRE(grid.y <= 65535, "latent_rows_write: too many heads");
 #define LAT(T, VV)                                                                                                            \
   hipLaunchKernelGGL((latent_rows_write_kernel<T, VV>), grid, dim3(256), 0, s, rows, stride, q_col0, d_col0, w, eps, positions, slots, \
