@@ -704,7 +704,7 @@ class RotaryLatentAttention(BranchMixer):
     elements, values of Dv = ``value_dim`` and a latent of L = ``latent_dim``:
 
         q = W_q x, per head [D unrotated | R rotated]      (no latent of the queries' own)
-        W_dkv x has L + R rows: c = rmsnorm(first L) * w_dkv, the last R (not normed) are the shared rotated key part
+        W_dkv x has L + R rows: c = rmsnorm(rows 0 .. L - 1) * w_dkv; rows L .. L + R - 1 stay unnormed and, turned, end every head's key
         k_h = W_uk[h] c    v_h = W_uv[h] c    score = (q_plain . k_h + q_rot . k_rot) * ``scale``
 
     causal, or under a ``window``; ``gate: "head"`` multiplies head h's output by sigmoid(W_g x)_h; then W_o on the
