@@ -5,8 +5,9 @@ from .bomotar import BomotarConfig
 from .golavik import GolavikConfig
 from .zemarax import ZemaraxConfig
 from .tokatar import TokatarConfig
+from .makisun import MakisunConfig
 from .registry import register_architecture, architecture_names, config_class_for, load_config, config_from_file
 
-__all__ = ["PartSpec", "LayerSpec", "LayerCall", "ModelSpec", "LlamaConfig", "MifutarConfig", "BomotarConfig", "GolavikConfig", "ZemaraxConfig", "TokatarConfig", "RopeScaling",
+__all__ = ["PartSpec", "LayerSpec", "LayerCall", "ModelSpec", "LlamaConfig", "MifutarConfig", "BomotarConfig", "GolavikConfig", "ZemaraxConfig", "TokatarConfig", "MakisunConfig", "RopeScaling",
            "ConfigError", "PRESETS", "register_architecture", "architecture_names",
            "config_class_for", "load_config", "config_from_file"]

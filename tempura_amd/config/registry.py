@@ -17,6 +17,7 @@ from .bomotar import BomotarConfig
 from .golavik import GolavikConfig
 from .zemarax import ZemaraxConfig
 from .tokatar import TokatarConfig
+from .makisun import MakisunConfig
 
 _ARCHITECTURES: Dict[str, Any] = {}
 
@@ -80,3 +81,4 @@ register_architecture("Bomotar", BomotarConfig)
 register_architecture("Golavik", GolavikConfig)
 register_architecture("Zemarax", ZemaraxConfig)
 register_architecture("Tokatar", TokatarConfig)
+register_architecture("Makisun", MakisunConfig)

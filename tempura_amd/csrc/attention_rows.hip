@@ -1,7 +1,7 @@
 // What lies between an attention's float32 projection rows and its cache, and between its heads' outputs and the
 // output product, for attentions that need more than a rotation there:
-//  * qkv_rows: biases on q, k and v, an RMS norm over the whole q and the whole k projection, rotation of q and k,
-//    rotation of the values by their own positions, cache write;
+//  * qkv_rows: biases on q, k and v, an RMS norm over the whole q and the whole k projection or over each of their heads,
+//    rotation of q and k, rotation of the values by their own positions, cache write;
 //  * latent_rows_write: queries into a latent's space beside one normed latent and one rotated key part a token;
 //  * turn_gate: outputs turned back by the query's position and multiplied by a sigmoid gate.
 // All pairs that turn together are neighbouring elements (2 i, 2 i + 1) of a head.  Float32 arithmetic throughout; a row's
@@ -148,6 +148,75 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(QkvRows a, T* __restrict_
   }
 }
 
+// The same with a norm over every head by itself (weights q_norm and k_norm [dim], shared by the heads; nullptr: no norm): a
+// wave takes one head of one token.  units: tokens times per_token, the heads of a token that this launch takes (q, k and,
+// in short steps, v).
+template <typename T, int V>
+__global__ __launch_bounds__(256) void qkv_heads_kernel(QkvRows a, long units, int per_token, T* __restrict__ q_out, T* __restrict__ k_cache,
+                                                        T* __restrict__ v_cache) {
+  const long unit = (long)blockIdx.x * 4 + threadIdx.x / TP_WAVE;
+  const int lane = threadIdx.x % TP_WAVE;
+  if (unit >= units) return;
+  const int t = (int)(unit / per_token), hh = (int)(unit % per_token);
+  const int sec = hh < a.heads ? 0 : hh < a.heads + a.kv ? 1 : 2;
+  const int h = sec == 0 ? hh : sec == 1 ? hh - a.heads : hh - a.heads - a.kv;
+  const int hdim = sec == 2 ? a.vdim : a.dim;
+  const int qd = a.heads * a.dim, kd = a.kv * a.dim;
+  const float* row = a.rows + (size_t)t * a.stride + (sec == 0 ? 0 : sec == 1 ? qd : qd + kd) + (size_t)h * hdim;
+  const float* bias = sec == 0 ? a.q_bias : sec == 1 ? a.k_bias : a.v_bias;
+  if (bias != nullptr) bias += (size_t)h * hdim;
+  const float* w = sec == 0 ? a.q_norm : sec == 1 ? a.k_norm : nullptr;
+  auto load = [&](int i) {
+    Elems<V> x = load_elems<V>(row + i);
+    if (bias != nullptr) {
+      const Elems<V> b = load_elems<V>(bias + i);
+#pragma unroll
+      for (int e = 0; e < V; ++e) x.x[e] += b.x[e];
+    }
+    return x;
+  };
+  float rstd = 1.f;
+  if (w != nullptr) {   // (uniform over the wave)
+    float ss = 0.f;
+    for (int i = lane * V; i < hdim; i += TP_WAVE * V) {
+      const Elems<V> x = load(i);
+#pragma unroll
+      for (int e = 0; e < V; ++e) ss = fmaf(x.x[e], x.x[e], ss);
+    }
+    ss = wave_sum(ss);
+    rstd = 1.0f / sqrtf(ss / (float)hdim + a.eps);
+  }
+  const int pos = a.positions[t], slot = a.slots[t];
+  const size_t page = (size_t)(slot / a.page_size), off = (size_t)(slot % a.page_size);
+  if (sec == 2) {
+    T* o = v_cache + ((page * a.kv + h) * a.vdim) * a.page_size + off;
+    for (int i = lane * V; i < hdim; i += TP_WAVE * V) {
+      Elems<V> x = load(i);
+      if (a.v_inv_freq != nullptr) turn_pairs<V>(x, i, a.vdim / 2, t, pos, a.v_inv_freq, a.v_table, 1.0f, 1.0f);
+#pragma unroll
+      for (int e = 0; e < V; ++e) from_float(o + (size_t)(i + e) * a.page_size, x.x[e]);
+    }
+    return;
+  }
+  T* o = sec == 0 ? q_out + ((size_t)t * a.heads + h) * a.out_dim : k_cache + ((page * a.kv + h) * a.page_size + off) * a.out_dim;
+  for (int i = lane * V; i < a.out_dim; i += TP_WAVE * V) {
+    Elems<V> x;
+    if (i < hdim) {
+      x = load(i);
+      if (w != nullptr) {
+        const Elems<V> wv = load_elems<V>(w + i);
+#pragma unroll
+        for (int e = 0; e < V; ++e) x.x[e] = x.x[e] * rstd * wv.x[e];
+      }
+      turn_pairs<V>(x, i, a.rotary_dim / 2, t, pos, a.inv_freq, a.table, a.factor, 1.0f);
+    } else {   // (zeros behind the head's own elements)
+#pragma unroll
+      for (int e = 0; e < V; ++e) x.x[e] = 0.f;
+    }
+    store_elems<V>(o + i, x);
+  }
+}
+
 // The values of long steps: a thread takes one element of one head for sixteen consecutive tokens and stores each run
 // of eight places that starts at a multiple of eight as one piece of the transposed layout.
 // grid: (ceil(n / 16), kv heads); block: vdim threads rounded up to whole waves (a pair's two elements are neighbours
@@ -208,19 +277,20 @@ static inline bool all_aligned16(const void* a, const void* b, const void* c, co
   return (((uintptr_t)a | (uintptr_t)b | (uintptr_t)c | (uintptr_t)d | (uintptr_t)e | (uintptr_t)f) & 15) == 0;
 }
 
-// rows float32 [n, stride] with q | k | v from column 0 on.  q_norm and k_norm come together.  out_dim >= dim: q_out
+// rows float32 [n, stride] with q | k | v from column 0 on (`width`: how many columns of a row lie behind that one).  q_norm
+// and k_norm come together; per_head: they have dim elements and norm every head by itself.  out_dim >= dim: q_out
 // [n, heads, out_dim], keys [page, kv, page_size, out_dim] with zeros behind a head's own elements; values transposed
 // [page, kv, vdim, page_size].  dt: the type of q_out and of both caches.
-extern "C" int tp_qkv_rows(const float* rows, size_t stride, const float* q_bias, const float* k_bias, const float* v_bias,
+extern "C" int tp_qkv_rows(const float* rows, size_t stride, size_t width, const float* q_bias, const float* k_bias, const float* v_bias,
                            const float* q_norm, const float* k_norm, float eps, const int* positions, const int* slots,
                            const double* inv_freq, const float* table, int rotary_dim, float factor, const double* v_inv_freq,
                            const float* v_table, int n, int heads, int kv, int dim, int vdim, int out_dim, void* q_out,
-                           void* k_cache, void* v_cache, int dt, int page_size, hipStream_t s) {
+                           void* k_cache, void* v_cache, int dt, int page_size, int per_head, hipStream_t s) {
   TP_REQUIRE(n >= 0 && heads > 0 && kv > 0 && dim > 0 && vdim > 0 && page_size > 0, "qkv_rows: bad sizes");
   TP_REQUIRE(dim % 2 == 0 && vdim % 2 == 0 && out_dim >= dim && out_dim % 2 == 0 && stride % 2 == 0, "qkv_rows: head sizes and row length must be even");
   TP_REQUIRE(vdim <= 1024 && kv <= 65535, "qkv_rows: value size %d or %d key heads too large", vdim, kv);
   TP_REQUIRE(rotary_dim >= 0 && rotary_dim % 2 == 0 && rotary_dim <= dim && (rotary_dim == 0 || inv_freq != nullptr), "qkv_rows: bad rotation");
-  TP_REQUIRE(stride >= (size_t)(heads + kv) * dim + (size_t)kv * vdim, "qkv_rows: rows too short");
+  TP_REQUIRE(width <= stride && width >= (size_t)(heads + kv) * dim + (size_t)kv * vdim, "qkv_rows: rows too short");
   TP_REQUIRE((q_norm == nullptr) == (k_norm == nullptr), "qkv_rows: the norms of q and k come together");
   TP_REQUIRE(dt == TP_F32 || dt == TP_BF16, "qkv_rows: unknown dtype %d", dt);
   if (n == 0) return 0;
@@ -237,6 +307,28 @@ extern "C" int tp_qkv_rows(const float* rows, size_t stride, const float* q_bias
   // a few rows: many blocks a token, so that a decode step fills more than a handful of CUs; long steps: one block per
   // token and section, values sixteen tokens at a time
   const bool lng = n >= 256;
+  if (per_head) {
+    const int per_token = heads + kv + (lng ? 0 : kv);
+    const long units = (long)n * per_token;
+    TP_REQUIRE((units + 3) / 4 < 0x7fffffffL, "qkv_rows: too many rows");
+    const dim3 grid((unsigned)((units + 3) / 4));
+#define QKV_HEADS(T)                                                                                                                 \
+  do {                                                                                                                               \
+    if (four)                                                                                                                        \
+      hipLaunchKernelGGL((qkv_heads_kernel<T, 4>), grid, dim3(256), 0, s, a, units, per_token, (T*)q_out, (T*)k_cache, (T*)v_cache); \
+    else                                                                                                                             \
+      hipLaunchKernelGGL((qkv_heads_kernel<T, 2>), grid, dim3(256), 0, s, a, units, per_token, (T*)q_out, (T*)k_cache, (T*)v_cache); \
+    if (lng)                                                                                                                         \
+      hipLaunchKernelGGL(qkv_values_kernel<T>, dim3((n + 15) / 16, kv), dim3((vdim + 63) / 64 * 64), 0, s, a, n, (T*)v_cache);       \
+  } while (0)
+    if (dt == TP_F32)
+      QKV_HEADS(float);
+    else
+      QKV_HEADS(bf16_t);
+#undef QKV_HEADS
+    TP_CHECK_LAUNCH("qkv_rows");
+    return 0;
+  }
   const int widest = heads * dim > kv * vdim ? heads * dim : kv * vdim;
   a.per_slice = lng ? (widest > kv * dim ? widest : kv * dim) / V : 256;
   auto slices = [&](int width) { return (width / V + a.per_slice - 1) / a.per_slice; };

@@ -291,7 +291,8 @@ extern "C" int tp_delta_scan(float* qkv, int row_stride, const float* decay, con
 // out[t, c] = f(sum_i x[t, col0 + i] * wt[i, c]) for a small inner size `rank`; x are float32 rows (the first
 // product's sums), wt float32 [rank, n_out] (the weight transposed, so that neighbouring lanes read neighbouring
 // values).  f: 0 the sum itself; 1 its sigmoid; 2 a decay, exp(-exp(a_log[c / per_head]) * softplus(sum + bias[c]));
-// 3 a decay between exp(-rate) and 1, exp(-rate * sigmoid(sum + bias[c])).  in_act 1: tanh of every x first.
+// 3 a decay between exp(-rate) and 1, exp(-rate * sigmoid(sum + bias[c])); 4 a decay exp(-exp(sum + bias[c])); 5 a power of
+// a sigmoid, sigmoid(sum + bias[c])^rate, formed from its logarithm.  in_act 1: tanh of every x first.
 // A block takes eight rows and 256 columns; a row's sum has the same order of additions wherever the row stands.
 #define LR_ROWS 8
 
@@ -333,7 +334,7 @@ __global__ __launch_bounds__(256) void lowrank_up_kernel(const float* __restrict
     rate = expf(a_log[c / per_head]);
     b = bias[c];
   }
-  if (mode == 3) {
+  if (mode >= 3) {
     rate = rate_const;
     b = bias[c];
   }
@@ -344,6 +345,8 @@ __global__ __launch_bounds__(256) void lowrank_up_kernel(const float* __restrict
     if (mode == 1) v = d_sigmoid(v);
     if (mode == 2) v = expf(-rate * d_softplus(v + b));
     if (mode == 3) v = expf(-rate * d_sigmoid(v + b));
+    if (mode == 4) v = expf(-expf(v + b));
+    if (mode == 5) v = expf(-rate * d_softplus(-(v + b)));
     out[(size_t)(t0 + t) * n_out + c] = v;
   }
 }
@@ -352,8 +355,8 @@ extern "C" int tp_lowrank_up(const float* x, int x_stride, int col0, int rank, c
                              int mode, const float* a_log, const float* bias, int per_head, int in_act, float rate, hipStream_t s) {
   TP_REQUIRE(n >= 0 && rank > 0 && n_out > 0 && col0 >= 0 && x_stride >= col0 + rank, "lowrank_up: bad sizes");
   TP_REQUIRE(rank <= 1024, "lowrank_up: inner size %d exceeds 1024", rank);
-  TP_REQUIRE(mode >= 0 && mode <= 3 && (in_act == 0 || in_act == 1), "lowrank_up: unknown epilogue %d or input function %d", mode, in_act);
-  TP_REQUIRE(mode != 3 || bias, "lowrank_up: the decay needs its biases");
+  TP_REQUIRE(mode >= 0 && mode <= 5 && (in_act == 0 || in_act == 1), "lowrank_up: unknown epilogue %d or input function %d", mode, in_act);
+  TP_REQUIRE(mode < 3 || bias, "lowrank_up: the decay needs its biases");
   TP_REQUIRE(mode != 2 || (a_log && bias && per_head > 0), "lowrank_up: the decay needs its rates and biases");
   if (n == 0) return 0;
   // (a few rows: blocks of one wave, so that the columns are spread over many CUs)
@@ -369,7 +372,8 @@ extern "C" int tp_lowrank_up(const float* x, int x_stride, int col0, int rank, c
 // ---- norm per head with a gate ----------------------------------------------------------------
 // out[t, out_col0 + h * vdim + d] = o[t, h, d] / sqrt(mean_d o^2 + eps) * w[d] * gate[t, h * vdim + d] * scale;
 // gate (float32, already between 0 and 1) may be missing.  w_stride vdim: every head has its own weight [heads, vdim]
-// (0: one weight [vdim] for all).  gate_raw: the gate is sigmoid(gate[t * gate_stride + h * vdim + d]) of raw rows.
+// (0: one weight [vdim] for all).  gate_raw: the gate is sigmoid(gate[t * gate_stride + h * vdim + d]) of raw rows (2: their
+// SiLU).
 // One wave per (token, head).
 template <typename TO>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w,
@@ -391,7 +395,7 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   const float* gr = gate != nullptr ? gate + (size_t)t * gate_stride + (size_t)h * vdim : nullptr;
   for (int d = lane; d < vdim; d += TP_WAVE) {
     float v = row[d] * rstd * wh[d];
-    if (gr != nullptr) v *= gate_raw ? d_sigmoid(gr[d]) : gr[d];
+    if (gr != nullptr) v *= gate_raw == 2 ? gr[d] * d_sigmoid(gr[d]) : gate_raw ? d_sigmoid(gr[d]) : gr[d];
     from_float(dst + d, v * scale);
   }
 }

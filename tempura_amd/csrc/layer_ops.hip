@@ -152,7 +152,7 @@ extern "C" int tp_sigmoid_gate(const void* a, int dt, const float* proj, int pro
 // ---- a sublayer's output, normed, into the residual stream ------------------------------------
 // h[t] += y[t] / sqrt(mean(y[t]^2) + eps) * w; then, with w_next, the next sublayer's input
 // x[t] = h[t] / sqrt(mean(h[t]^2) + eps_next) * w_next as TO.  One block per row.
-// With gate rows, y stands for y[t, c] * sigmoid(gate.rows[t, gate.col0 + c] + gate.bias[c]).
+// With gate rows, y stands for y[t, c] * sigmoid(gate.rows[t, gate.col0 + c] + gate.bias[c]).  Not normed: h[t] += y[t] * w.
 struct InputGate {
   const float* rows;   // float32 [n, stride], or nullptr: no gate
   const float* bias;   // [width], or nullptr
@@ -164,7 +164,7 @@ template <typename TO>
 __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ h, const float* __restrict__ y,
                                                        const float* __restrict__ w, float eps,
                                                        const float* __restrict__ w_next, float eps_next,
-                                                       TO* __restrict__ x, int width, InputGate gate) {
+                                                       TO* __restrict__ x, int width, InputGate gate, int normed) {
   __shared__ float scratch[32];
   const size_t base = (size_t)blockIdx.x * width;
   const float* gr = gate.rows != nullptr ? gate.rows + (size_t)blockIdx.x * gate.stride + gate.col0 : nullptr;
@@ -172,13 +172,16 @@ __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ h, co
     const float v = y[base + c];
     return gr != nullptr ? v * l_sigmoid(gr[c] + (gate.bias != nullptr ? gate.bias[c] : 0.f)) : v;
   };
-  float ss = 0.f;
-  for (int c = threadIdx.x; c < width; c += blockDim.x) {
-    const float v = value(c);
-    ss = fmaf(v, v, ss);
+  float rstd = 1.0f;
+  if (normed) {   // (uniform)
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < width; c += blockDim.x) {
+      const float v = value(c);
+      ss = fmaf(v, v, ss);
+    }
+    ss = block_sum(ss, scratch);
+    rstd = 1.0f / sqrtf(ss / (float)width + eps);
   }
-  ss = block_sum(ss, scratch);
-  const float rstd = 1.0f / sqrtf(ss / (float)width + eps);
   float ss2 = 0.f;
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
     const float v = h[base + c] + value(c) * rstd * w[c];
@@ -199,7 +202,7 @@ template <typename TO, int NV, bool GATE>
 __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h, const float* __restrict__ y,
                                                            const float* __restrict__ w, float eps,
                                                            const float* __restrict__ w_next, float eps_next,
-                                                           TO* __restrict__ x, int width, InputGate gate) {
+                                                           TO* __restrict__ x, int width, InputGate gate, int normed) {
   __shared__ float scratch[32];
   const size_t base = (size_t)blockIdx.x * width;
   const int w4 = width / 4;
@@ -233,17 +236,20 @@ __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h
         yv[k].w *= l_sigmoid(gv[k].w + bv[k].w);
       }
   }
-  float ss = 0.f;
+  float rstd = 1.0f;
+  if (normed) {
+    float ss = 0.f;
 #pragma unroll
-  for (int k = 0; k < NV; ++k)
-    if (k * 256 + threadIdx.x < w4) {
-      ss = fmaf(yv[k].x, yv[k].x, ss);
-      ss = fmaf(yv[k].y, yv[k].y, ss);
-      ss = fmaf(yv[k].z, yv[k].z, ss);
-      ss = fmaf(yv[k].w, yv[k].w, ss);
-    }
-  ss = block_sum(ss, scratch);
-  const float rstd = 1.0f / sqrtf(ss / (float)width + eps);
+    for (int k = 0; k < NV; ++k)
+      if (k * 256 + threadIdx.x < w4) {
+        ss = fmaf(yv[k].x, yv[k].x, ss);
+        ss = fmaf(yv[k].y, yv[k].y, ss);
+        ss = fmaf(yv[k].z, yv[k].z, ss);
+        ss = fmaf(yv[k].w, yv[k].w, ss);
+      }
+    ss = block_sum(ss, scratch);
+    rstd = 1.0f / sqrtf(ss / (float)width + eps);
+  }
   float ss2 = 0.f;
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
@@ -277,7 +283,7 @@ __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h
 
 extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, const float* w_next, float eps_next, void* x,
                            int x_dt, int n, int width, const float* gate_rows, size_t gate_stride, int gate_col0,
-                           const float* gate_bias, hipStream_t s) {
+                           const float* gate_bias, int normed, hipStream_t s) {
   TP_REQUIRE(n >= 0 && width > 0, "norm_add: bad sizes");
   TP_REQUIRE(gate_rows == nullptr || (gate_col0 >= 0 && gate_stride >= (size_t)gate_col0 + width), "norm_add: gate rows too short");
   const InputGate gate{gate_rows, gate_bias, gate_stride, gate_col0};
@@ -290,7 +296,7 @@ extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, 
   if (width % 4 == 0 && width >= 1024 && width <= 256 * 4 * 8 && aligned) {
     const bool bf = w_next != nullptr && x_dt == TP_BF16;
 #define NA1(TO, NV, G) \
-  hipLaunchKernelGGL((norm_add_reg_kernel<TO, NV, G>), dim3(n), dim3(256), 0, s, h, y, w, eps, w_next, eps_next, (TO*)x, width, gate)
+  hipLaunchKernelGGL((norm_add_reg_kernel<TO, NV, G>), dim3(n), dim3(256), 0, s, h, y, w, eps, w_next, eps_next, (TO*)x, width, gate, normed)
 #define NA(NV)                                    \
   do {                                            \
     if (gate_rows != nullptr) {                   \
@@ -311,9 +317,9 @@ extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, 
   }
   const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
   if (w_next == nullptr || x_dt == TP_F32)
-    hipLaunchKernelGGL(norm_add_kernel<float>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (float*)x, width, gate);
+    hipLaunchKernelGGL(norm_add_kernel<float>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (float*)x, width, gate, normed);
   else if (x_dt == TP_BF16)
-    hipLaunchKernelGGL(norm_add_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (bf16_t*)x, width, gate);
+    hipLaunchKernelGGL(norm_add_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (bf16_t*)x, width, gate, normed);
   else
     TP_REQUIRE(false, "norm_add: unknown dtype %d", x_dt);
   TP_CHECK_LAUNCH("norm_add");

@@ -1365,16 +1365,22 @@ def qkv_rows(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, n
              value_dim: int, k_cache: torch.Tensor, v_cache: torch.Tensor, inv_freq: Optional[torch.Tensor] = None, rotary_dim: int = 0,
              factor: float = 1.0, cos_sin: Optional[torch.Tensor] = None, biases=(None, None, None), norms=None, eps: float = 0.0,
              value_inv_freq: Optional[torch.Tensor] = None, value_cos_sin: Optional[torch.Tensor] = None,
-             pad_dim: Optional[int] = None) -> torch.Tensor:
+             pad_dim: Optional[int] = None, col0: int = 0, norm_over: str = "projection") -> torch.Tensor:
     """Float32 rows [n, q | k | v | any more columns] of a projection, step by step: ``biases`` (float32 per column of q, k,
     v; each may be None) are added; with ``norms`` (q weight, k weight: float32, one value a column) q and k are divided
     by the root mean square of the WHOLE projection (all heads together, ``eps`` inside the root) and multiplied by the
-    weight; the pairs of neighbours of the first ``rotary_dim`` elements of q and k heads turn by position *
+    weight (``norm_over`` ``"head"``: every head by its own root mean square, the weights [head_dim] shared by the heads); the
+    pairs of neighbours of the first ``rotary_dim`` elements of q and k heads turn by position *
     ``inv_freq``; with ``value_inv_freq`` (float64 [value_dim / 2]) the pairs of a value head turn likewise; k and v go
     to the cache rows ``slots``.  Returns q in the caches' type as [n, heads, pad_dim or head_dim] (keys are stored as
-    wide; zeros behind a head's own elements)."""
+    wide; zeros behind a head's own elements).  ``col0``: the column at which q | k | v start."""
     od = head_dim if pad_dim is None else int(pad_dim)
+    _need(norm_over in ("projection", "head"), f"qkv_rows: norm over {norm_over!r} unknown")
+    per_head = norm_over == "head"
     if _backend is not None:
+        if col0 or per_head:
+            return _backend.qkv_rows(rows, positions, slots, num_heads, num_kv_heads, head_dim, value_dim, k_cache, v_cache, inv_freq,
+                                     rotary_dim, factor, biases, norms, eps, value_inv_freq, od, col0, norm_over)
         return _backend.qkv_rows(rows, positions, slots, num_heads, num_kv_heads, head_dim, value_dim, k_cache, v_cache, inv_freq,
                                  rotary_dim, factor, biases, norms, eps, value_inv_freq, od)
     qb, kb, vb = biases
@@ -1382,10 +1388,10 @@ def qkv_rows(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, n
     _dev_ok(rows, positions, slots, k_cache, v_cache, inv_freq, cos_sin, qb, kb, vb, qn, kn, value_inv_freq, value_cos_sin)
     n = rows.shape[0]
     widths = (num_heads * head_dim, num_kv_heads * head_dim, num_kv_heads * value_dim)
-    _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.shape[1] >= sum(widths) and rows.shape[1] % 2 == 0,
+    _need(rows.dtype == torch.float32 and rows.dim() == 2 and col0 >= 0 and rows.shape[1] >= col0 + sum(widths) and rows.shape[1] % 2 == 0,
           "qkv_rows: rows must be float32 [n, an even width of at least q | k | v]")
-    for b, size, what in ((qb, widths[0], "q bias"), (kb, widths[1], "k bias"), (vb, widths[2], "v bias"), (qn, widths[0], "q norm"),
-                          (kn, widths[1], "k norm")):
+    for b, size, what in ((qb, widths[0], "q bias"), (kb, widths[1], "k bias"), (vb, widths[2], "v bias"),
+                          (qn, head_dim if per_head else widths[0], "q norm"), (kn, head_dim if per_head else widths[1], "k norm")):
         _need(b is None or (b.dtype == torch.float32 and b.numel() == size), f"qkv_rows: {what} must be float32 with {size} elements")
     _need((qn is None) == (kn is None), "qkv_rows: the norms of q and k come together")
     if n:
@@ -1398,10 +1404,11 @@ def qkv_rows(rows: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, n
     if value_inv_freq is not None:
         _rotation(value_inv_freq, value_dim // 2, value_cos_sin, n, "qkv_rows: values")
     q = torch.empty((n, num_heads, od), dtype=k_cache.dtype, device=rows.device)
-    _call("tp_qkv_rows", _ptr(rows), ctypes.c_size_t(rows.shape[1]), _ptr(qb), _ptr(kb), _ptr(vb), _ptr(qn), _ptr(kn), ctypes.c_float(eps),
+    _call("tp_qkv_rows", ctypes.c_void_p(rows.data_ptr() + 4 * int(col0)), ctypes.c_size_t(rows.shape[1]), ctypes.c_size_t(rows.shape[1] - int(col0)),
+          _ptr(qb), _ptr(kb), _ptr(vb), _ptr(qn), _ptr(kn), ctypes.c_float(eps),
           _ptr(positions), _ptr(slots), _ptr(inv_freq), _ptr(cos_sin), int(rotary_dim), ctypes.c_float(factor), _ptr(value_inv_freq),
           _ptr(value_cos_sin), n, int(num_heads), int(num_kv_heads), int(head_dim), int(value_dim), od, _ptr(q), _ptr(k_cache),
-          _ptr(v_cache), _dt(k_cache), k_cache.shape[2], _stream())
+          _ptr(v_cache), _dt(k_cache), k_cache.shape[2], int(per_head), _stream())
     return q
 
 
@@ -1470,8 +1477,8 @@ def head_linear(x: torch.Tensor, x_col0: int, x_head: int, w: torch.Tensor, out:
 
 def norm_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, next_weight: Optional[torch.Tensor] = None,
              next_eps: float = 0.0, out_dtype: Optional[torch.dtype] = None, gate: Optional[torch.Tensor] = None, gate_col0: int = 0,
-             gate_bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
-    """h += y / sqrt(mean(y^2) + eps) * weight, per row, in place (float32 [n, width]).  With ``next_weight`` the
+             gate_bias: Optional[torch.Tensor] = None, normed: bool = True) -> Optional[torch.Tensor]:
+    """h += y / sqrt(mean(y^2) + eps) * weight (not ``normed``: h += y * weight), per row, in place (float32 [n, width]).  With ``next_weight`` the
     rows of the new h normed with it (and ``next_eps``) come back as ``out_dtype``.  With ``gate`` (float32 rows [n,
     wider]) y is first multiplied by sigmoid(gate[:, gate_col0 + c] + gate_bias[c])."""
     if _backend is not None:
@@ -1493,8 +1500,18 @@ def norm_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float,
         x = torch.empty((n, width), dtype=out_dtype, device=h.device)
     _call("tp_norm_add", _ptr(h), _ptr(y), _ptr(weight), ctypes.c_float(eps), _ptr(next_weight), ctypes.c_float(next_eps), _ptr(x),
           _dtcode(out_dtype) if x is not None else _F32, n, width, _ptr(gate), ctypes.c_size_t(0 if gate is None else gate.shape[1]),
-          int(gate_col0), _ptr(gate_bias), _stream())
+          int(gate_col0), _ptr(gate_bias), int(normed), _stream())
     return x
+
+
+def scale_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, next_weight: Optional[torch.Tensor] = None, next_eps: float = 0.0,
+              out_dtype: Optional[torch.dtype] = None, gate: Optional[torch.Tensor] = None, gate_col0: int = 0,
+              gate_bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """``norm_add`` without the norm on y: h += y * weight, per row, in place (``weight`` a vector of scales), and with
+    ``next_weight`` the rows of the new h normed with it come back."""
+    if _backend is not None:
+        return _backend.scale_add(h, y, weight, next_weight, next_eps, out_dtype, gate, gate_col0, gate_bias)
+    return norm_add(h, y, weight, 0.0, next_weight, next_eps, out_dtype, gate, gate_col0, gate_bias, normed=False)
 
 
 ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "gelu_erf": 2, "relu2": 3}
@@ -1561,18 +1578,19 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], experts:
     return dense, ids, weights
 
 
-LOWRANK_MODES = {"plain": 0, "sigmoid": 1, "decay": 2, "rate_sigmoid": 3}
+LOWRANK_MODES = {"plain": 0, "sigmoid": 1, "decay": 2, "rate_sigmoid": 3, "exp_exp": 4, "root_sigmoid": 5}
 
 
 def lowrank_up(x: torch.Tensor, col0: int, weight_t: torch.Tensor, mode: str = "plain", a_log: Optional[torch.Tensor] = None,
                bias: Optional[torch.Tensor] = None, per_head: int = 0, rate: float = 0.0, in_act: Optional[str] = None) -> torch.Tensor:
     """The second product of a low-rank projection: float32 [n, N] = f(g(x[:, col0: col0 + r]) @ weight_t), ``x`` float32
     rows (the first product's sums), ``weight_t`` float32 [r, N].  f: ``plain``; ``sigmoid``; ``decay``:
-    exp(-exp(a_log[c // per_head]) * softplus(sum + bias[c])); ``rate_sigmoid``: exp(-rate * sigmoid(sum + bias[c])).
+    exp(-exp(a_log[c // per_head]) * softplus(sum + bias[c])); ``rate_sigmoid``: exp(-rate * sigmoid(sum + bias[c]));
+    ``exp_exp``: exp(-exp(sum + bias[c])); ``root_sigmoid``: sigmoid(sum + bias[c])^rate.
     g: the identity, or tanh with ``in_act`` ``"tanh"``."""
     _need(in_act in (None, "tanh"), f"lowrank_up: input function {in_act!r} unknown")
     if _backend is not None:
-        if mode == "rate_sigmoid" or in_act is not None:
+        if mode in ("rate_sigmoid", "exp_exp", "root_sigmoid") or in_act is not None:
             return _backend.lowrank_up(x, col0, weight_t, mode, a_log, bias, per_head, rate, in_act)
         return _backend.lowrank_up(x, col0, weight_t, mode, a_log, bias, per_head)
     _dev_ok(x, weight_t, a_log, bias)
@@ -1583,7 +1601,7 @@ def lowrank_up(x: torch.Tensor, col0: int, weight_t: torch.Tensor, mode: str = "
     if mode == "decay":
         _need(a_log is not None and bias is not None and per_head > 0 and n_out % per_head == 0 and a_log.dtype == torch.float32
               and bias.dtype == torch.float32 and a_log.numel() == n_out // per_head and bias.numel() == n_out, "lowrank_up: bad decay constants")
-    if mode == "rate_sigmoid":
+    if mode in ("rate_sigmoid", "exp_exp", "root_sigmoid"):
         _need(bias is not None and bias.dtype == torch.float32 and bias.numel() == n_out, "lowrank_up: bad decay biases")
     out = torch.empty((x.shape[0], n_out), dtype=torch.float32, device=x.device)
     _call("tp_lowrank_up", _ptr(x), x.shape[1], int(col0), r, _ptr(weight_t), _ptr(out), x.shape[0], n_out, LOWRANK_MODES[mode],
@@ -1621,13 +1639,20 @@ def delta_scan(qkv: torch.Tensor, decay: torch.Tensor, proj: torch.Tensor, beta_
     return y
 
 
+GATE_ACTS = {"sigmoid": 1, "silu": 2}
+
+
 def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate: Optional[torch.Tensor], eps: float, scale: float, heads: int,
-                   out: torch.Tensor, out_col0: int, gate_rows: Optional[torch.Tensor] = None, gate_col0: int = 0) -> None:
+                   out: torch.Tensor, out_col0: int, gate_rows: Optional[torch.Tensor] = None, gate_col0: int = 0,
+                   gate_act: str = "sigmoid") -> None:
     """out[:, out_col0 + h * vdim + d] = o[:, h, d] / sqrt(mean_d o^2 + eps) * weight[d] * gate[:, h * vdim + d] * scale:
     ``o`` float32 [n, heads * vdim]; ``weight`` float32 [vdim] shared by the heads, or [heads * vdim], every head its own;
     ``gate`` float32 like ``o`` or None.  ``gate_rows`` (float32 rows [n, wider], instead of ``gate``): the gate is the
-    sigmoid of their columns gate_col0 .. gate_col0 + heads * vdim."""
+    sigmoid (``gate_act`` ``"silu"``: the SiLU) of their columns gate_col0 .. gate_col0 + heads * vdim."""
+    _need(gate_act in GATE_ACTS, f"head_norm_gate: gate function {gate_act!r} unknown (known: {sorted(GATE_ACTS)})")
     if _backend is not None:
+        if gate_act != "sigmoid":
+            return _backend.head_norm_gate(o, weight, gate, eps, scale, heads, out, out_col0, gate_rows, gate_col0, gate_act)
         if gate_rows is not None:
             return _backend.head_norm_gate(o, weight, gate, eps, scale, heads, out, out_col0, gate_rows, gate_col0)
         return _backend.head_norm_gate(o, weight, gate, eps, scale, heads, out, out_col0)
@@ -1644,7 +1669,7 @@ def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate: Optional[torch.T
     if gate_rows is not None:
         _need(gate_rows.dtype == torch.float32 and gate_rows.dim() == 2 and gate_rows.shape[0] == n and 0 <= gate_col0
               and gate_col0 + o.shape[1] <= gate_rows.shape[1], "head_norm_gate: bad gate rows")
-        gate_ptr, gate_stride, raw = ctypes.c_void_p(gate_rows.data_ptr() + 4 * int(gate_col0)), gate_rows.shape[1], 1
+        gate_ptr, gate_stride, raw = ctypes.c_void_p(gate_rows.data_ptr() + 4 * int(gate_col0)), gate_rows.shape[1], GATE_ACTS[gate_act]
     _call("tp_head_norm_gate", _ptr(o), _ptr(weight), gate_ptr, ctypes.c_float(eps), ctypes.c_float(scale), _ptr(out), _dt(out),
           out.shape[1], int(out_col0), n, int(heads), vdim, per_head, ctypes.c_size_t(gate_stride), raw, _stream())
 
@@ -1875,3 +1900,79 @@ def mlstm_scan(proj: torch.Tensor, col0: int, i_bias: torch.Tensor, f_bias: torc
           _ptr(state), ctypes.c_size_t(state.shape[1]), ctypes.c_size_t(state_off), _ptr(cu_seqlens), _ptr(state_slots), _ptr(scratch),
           _ptr(norm_weight), ctypes.c_float(eps), ctypes.c_float(scale), _ptr(out), _dt(out), out.shape[1], int(out_col0), n,
           int(num_requests), int(heads), int(dim), int(vdim), _stream())
+
+
+# ---------------------------------------------------------------------------------
+# Operations of mixers around a linear recurrence: mixes of a row and the row before it, and the recurrence.
+
+def token_shift(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, state_off: int, cu_seqlens: torch.Tensor, token_req: torch.Tensor,
+                state_slots: torch.Tensor, num_requests: int, out_dtype: torch.dtype, max_run: Optional[int] = None):
+    """Mixes of float32 rows ``x`` [n, width] with the rows before them in their requests: for each of the ``mu`` [mixes,
+    width] x + (x' - x) * mu, as ``out_dtype``; a list of tensors [n, width].  x' of a run's first token is what the request's
+    state holds (``state`` float32 [slots, row], ``width`` numbers from ``state_off`` on); the run's last row is left there.
+    ``max_run``: the longest run of the step (None: unknown)."""
+    if _backend is not None:
+        return _backend.token_shift(x, mu, state, state_off, cu_seqlens, token_req, state_slots, num_requests, out_dtype)
+    _dev_ok(x, mu, state, cu_seqlens, token_req, state_slots)
+    _need(x.dtype == torch.float32 and x.dim() == 2, "token_shift: rows must be float32 [n, width]")
+    n, width = x.shape
+    _need(mu.dtype == torch.float32 and mu.dim() == 2 and mu.shape[1] == width, "token_shift: mu must be float32 [mixes, width]")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state_off >= 0 and state.shape[1] >= state_off + width, "token_shift: state rows too short")
+    _i32(cu_seqlens, num_requests + 1, "cu_seqlens")
+    _i32(state_slots, num_requests, "state_slots")
+    _i32(token_req, n, "token_req") if n else None
+    mixes = mu.shape[0]
+    out = torch.empty((mixes, n, width), dtype=out_dtype, device=x.device)
+    _call("tp_token_shift", _ptr(x), _ptr(mu), _ptr(state), ctypes.c_size_t(state.shape[1]), ctypes.c_size_t(state_off), _ptr(cu_seqlens),
+          _ptr(token_req), _ptr(state_slots), _ptr(out), _dtcode(out_dtype), n, int(num_requests), width, mixes, int(max_run == 1), _stream())
+    return list(out.unbind(0))
+
+
+#: runs longer than a piece are cut into pieces that run side by side; a piece has at least this many tokens
+scan_min_piece = 64
+#: and is lengthened while the pieces of a step make more blocks than this
+scan_target_blocks = 1024
+
+
+def scan_piece(n: int, max_run: int, heads: int, dim: int, vdim: int) -> int:
+    """Tokens of a piece of ``linear_scan`` (0: runs are not cut)."""
+    blocks = heads * max(1, vdim // 64)
+    piece = max(scan_min_piece, -(-n * blocks // scan_target_blocks))
+    piece = -(-piece // 16) * 16
+    return 0 if max_run <= piece else piece
+
+
+def linear_scan(q, k, v, decay: torch.Tensor, state: torch.Tensor, state_off: int, cu_seqlens: torch.Tensor, state_slots: torch.Tensor,
+                num_requests: int, heads: int, dim: int, vdim: int, bonus: Optional[torch.Tensor] = None, q_scale: float = 1.0,
+                max_run: Optional[int] = None) -> torch.Tensor:
+    """The recurrence S <- diag(decay) S + k v^T per head over each request's run of tokens.  ``q``, ``k`` and ``v`` are pairs
+    (float32 rows [n, wider], first column) of heads * dim, heads * dim and heads * vdim columns; ``decay`` float32 [n,
+    heads * dim].  Without ``bonus`` a token reads behind its update, o = S^T (q * q_scale); with it (float32 [heads *
+    dim]) in front of it, o = (S + diag(bonus) k v^T)^T (q * q_scale).  S [dim, vdim] per head lies at ``state[slot,
+    state_off:]`` column by column, [heads, vdim, dim], and is left as the run leaves it.  ``max_run``: the longest run of the
+    step (None: the step's tokens).  Returns o float32 [n, heads * vdim]."""
+    if _backend is not None:
+        return _backend.linear_scan(q, k, v, decay, state, state_off, cu_seqlens, state_slots, num_requests, heads, dim, vdim, bonus, q_scale)
+    n = decay.shape[0]
+    _dev_ok(q[0], k[0], v[0], decay, state, cu_seqlens, state_slots, bonus)
+    for (rows, col), width, what in ((q, heads * dim, "q"), (k, heads * dim, "k"), (v, heads * vdim, "v")):
+        _need(rows.dtype == torch.float32 and rows.dim() == 2 and rows.shape[0] == n and 0 <= col and col + width <= rows.shape[1],
+              f"linear_scan: bad {what} rows")
+    _need(decay.dtype == torch.float32 and tuple(decay.shape) == (n, heads * dim), "linear_scan: decay must be float32 [n, heads * dim]")
+    _need(bonus is None or (bonus.dtype == torch.float32 and bonus.numel() == heads * dim), "linear_scan: bonus must be float32 [heads * dim]")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state_off >= 0 and state.shape[1] >= state_off + heads * dim * vdim,
+          "linear_scan: state rows too short")
+    _i32(cu_seqlens, num_requests + 1, "cu_seqlens")
+    _i32(state_slots, num_requests, "state_slots")
+    max_run = n if max_run is None else int(max_run)
+    y = torch.empty((n, heads * vdim), dtype=torch.float32, device=decay.device)
+    piece, scratch, pieces = scan_piece(n, max_run, heads, dim, vdim), None, 0
+    if piece:
+        # (a request's pieces start at place cu_seqlens[r] // piece + r of the scratch)
+        pieces = n // piece + num_requests
+        scratch = torch.empty((pieces * heads * dim * (vdim + 1),), dtype=torch.float32, device=decay.device)
+    at = lambda rows: ctypes.c_void_p(rows[0].data_ptr() + 4 * int(rows[1]))
+    _call("tp_linear_scan", at(q), q[0].shape[1], at(k), k[0].shape[1], at(v), v[0].shape[1], _ptr(decay), _ptr(bonus), ctypes.c_float(q_scale),
+          _ptr(state), ctypes.c_size_t(state.shape[1]), ctypes.c_size_t(state_off), _ptr(cu_seqlens), _ptr(state_slots), _ptr(y), n,
+          int(num_requests), int(heads), int(dim), int(vdim), max_run, piece, pieces, _ptr(scratch), _stream())
+    return y

@@ -241,9 +241,9 @@ class PagedAttention(Mixer):
             wo = self._paired_values(wo.t()).t()
         self.wo = ops.tile_weight(self._to_device(wo))
         if self.qk_norm is not None:
-            whole = self.rows_path
-            self.q_norm_w = self._to_device(self._paired(get(w["q_norm"])) if whole else get(w["q_norm"]), torch.float32)
-            self.k_norm_w = self._to_device(self._paired(get(w["k_norm"])) if whole else get(w["k_norm"]), torch.float32)
+            # (a weight per head is the same for all heads: it is ordered like one of them)
+            self.q_norm_w = self._to_device(self._paired(get(w["q_norm"])), torch.float32)
+            self.k_norm_w = self._to_device(self._paired(get(w["k_norm"])), torch.float32)
         if self.sink_score is not None:
             self.sink_w = torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=self.device)
         elif self.has_sink:
@@ -402,10 +402,14 @@ class SizedValueCacheSpec(CacheSpec):
 
 
 class ConvAttention(BranchMixer):
-    """Grouped-query softmax attention over the paged cache whose q, k and v pass a short causal convolution per
+    """Grouped-query softmax attention over the paged cache as a branch (``branch_attention``; ``conv_attention`` where the
+    convolution below is part of the design).  q, k and v may pass a short causal convolution per
     channel right behind their projections (``conv_taps`` taps, no bias, no activation, zeros before a request's
-    start; before any rotation), whose values may have another size than its keys (``value_dim``), and whose
-    concatenated heads are multiplied by sigmoid(W_g x) before the output projection (``gate``).  The position
+    start; before any norm and rotation; 0 or left out: no convolution), the values may have another size than the keys
+    (``value_dim``), with ``qk_norm`` (``{"eps"}``, tensors ``q_norm``, ``k_norm`` of [head_dim]) every head of q and of k is
+    divided by its root mean square and multiplied by the weight before any rotation, and the
+    concatenated heads are multiplied by sigmoid(W_g x) before the output projection (``gate``: True, a number per
+    element, or ``"head"``, one number per head).  The position
     encoding, the scale and an optional window are parameters as for ``attention``.
 
     The columns of its input product are [q | k | v | gate]; a request's state is the convolution's last
@@ -423,11 +427,21 @@ class ConvAttention(BranchMixer):
             raise ValueError("conv_attention: heads must be a multiple of kv heads")
         self.scale = float(p["scale"])
         self.window = p.get("window")
-        self.taps = int(p["conv_taps"])
-        if self.taps < 1:
-            raise ValueError("conv_attention: conv_taps must be at least 1")
-        self.gate = bool(p.get("gate", False))
+        self.taps = int(p.get("conv_taps") or 0)
+        if self.taps < 0:
+            raise ValueError("conv_attention: conv_taps must not be negative")
+        gate = p.get("gate", False)
+        if gate not in (True, False, None, "head"):
+            raise ValueError(f"conv_attention: gate {gate!r} unknown (known: True, head)")
+        self.gate = bool(gate)
+        #: columns that share a gate
+        self.gate_per = self.value_dim if gate == "head" else 1
+        self.qk_norm = p.get("qk_norm")
         self.position = build_part("position", p["position"], hidden_size, dtype, device)
+        if self.position.rotary() is None and type(self.position).__name__ != "NoPosition":
+            raise ValueError("conv_attention: the position part must rotate or be none")
+        #: one kernel takes the float32 rows to q and the cache: norm per head, rotation, cache write
+        self.rows_path = self.qk_norm is not None or self.taps == 0
         self.q_dim = self.num_heads * self.head_dim
         self.k_dim = self.num_kv_heads * self.head_dim
         self.v_dim = self.num_kv_heads * self.value_dim
@@ -437,29 +451,34 @@ class ConvAttention(BranchMixer):
         # behind their own elements up to the values' size (no score changes; the key pages are that much wider),
         # so that those kernels serve; every other pair of sizes runs the general kernel
         self.key_dim = self.head_dim
-        if dtype == torch.bfloat16 and self.head_dim < self.value_dim <= 128 and self.value_dim % 32 == 0 and self.head_dim % 2 == 0:
+        if self.rows_path:
+            pair = ops.fast_pair(self.head_dim, self.value_dim) if dtype == torch.bfloat16 and self.head_dim % 2 == 0 else None
+            self.key_dim = pair[0] if pair is not None else self.head_dim
+        elif dtype == torch.bfloat16 and self.head_dim < self.value_dim <= 128 and self.value_dim % 32 == 0 and self.head_dim % 2 == 0:
             self.key_dim = self.value_dim
-        self.conv_w = None
+        self.conv_w = self.norms = None
 
     @classmethod
     def expected_weights(cls, spec, hidden_size):
         p, w = spec.params, spec.weights
         vd = int(p.get("value_dim") or p["head_dim"])
         q_dim, k_dim, v_dim = p["num_heads"] * p["head_dim"], p["num_kv_heads"] * p["head_dim"], p["num_kv_heads"] * vd
-        taps = int(p["conv_taps"])
+        taps = int(p.get("conv_taps") or 0)
         out = {
             w["q"]: WeightInfo((q_dim, hidden_size)), w["k"]: WeightInfo((k_dim, hidden_size)), w["v"]: WeightInfo((v_dim, hidden_size)),
-            w["q_conv"]: WeightInfo((q_dim, taps)), w["k_conv"]: WeightInfo((k_dim, taps)),
-            w["v_conv"]: WeightInfo((v_dim, taps)),
             w["o"]: WeightInfo((hidden_size, p["num_heads"] * vd)),
         }
+        if taps:
+            out.update({w["q_conv"]: WeightInfo((q_dim, taps)), w["k_conv"]: WeightInfo((k_dim, taps)), w["v_conv"]: WeightInfo((v_dim, taps))})
+        if p.get("qk_norm") is not None:
+            out.update({w["q_norm"]: WeightInfo((p["head_dim"],), "ones"), w["k_norm"]: WeightInfo((p["head_dim"],), "ones")})
         if p.get("gate", False):
-            out[w["gate"]] = WeightInfo((p["num_heads"] * vd, hidden_size))
+            out[w["gate"]] = WeightInfo((p["num_heads"] * (1 if p["gate"] == "head" else vd), hidden_size))
         out.update(part_class("position", p["position"].kind).expected_weights(p["position"], hidden_size))
         return out
 
     def state_floats(self) -> int:
-        return (self.taps - 1) * self.channels
+        return max(0, self.taps - 1) * self.channels
 
     def cache_spec(self):
         kind = "window" if self.window is not None else "full"
@@ -468,7 +487,7 @@ class ConvAttention(BranchMixer):
         return SizedValueCacheSpec(kind, self.num_kv_heads, self.key_dim, self.window, self.value_dim)
 
     def _paired(self, t: torch.Tensor) -> torch.Tensor:
-        """Rows of a q or k tensor (projection or convolution) with every head's rotary elements in paired order
+        """Rows of a q or k tensor (projection, convolution or a norm's weight) with every head's rotary elements in paired order
         (see ``PagedAttention._paired``: the rotation kernels take neighbours as pairs)."""
         rot = self.position.rotary()
         if rot is None or rot[1] == 0:
@@ -484,30 +503,43 @@ class ConvAttention(BranchMixer):
         rows = [self._paired(get(w["q"])), self._paired(get(w["k"])), get(w["v"])]
         if self.gate:
             rows.append(get(w["gate"]))
-        conv = torch.cat([self._paired(get(w["q_conv"])), self._paired(get(w["k_conv"])), get(w["v_conv"])], dim=0)
-        self.conv_w = self._to_device(conv, torch.float32).t().contiguous()      # tap-major for the kernel
+        if self.taps:
+            conv = torch.cat([self._paired(get(w["q_conv"])), self._paired(get(w["k_conv"])), get(w["v_conv"])], dim=0)
+            self.conv_w = self._to_device(conv, torch.float32).t().contiguous()      # tap-major for the kernel
+        if self.qk_norm is not None:
+            self.norms = tuple(self._to_device(self._paired(get(w[name])), torch.float32) for name in ("q_norm", "k_norm"))
         self.position.load_weights(get)
         return torch.cat([self._to_device(t) for t in rows], dim=0).contiguous(), self._to_device(get(w["o"]))
 
     def run(self, proj, col0, ctx, cache, out, out_col0, scale):
         if not cache.writes:
             raise ValueError("conv_attention: a call that reads another call's cache is not supported")
-        qkv = ops.causal_conv(proj, col0, self.channels, self.conv_w, None, cache.state, ctx.cu_seqlens, ctx.token_req,
-                              ctx.state_slots, ctx.num_requests, state_off=self.state_off, act=False)
+        qkv, qkv_col0 = proj, col0
+        if self.taps:
+            qkv_col0 = 0
+            qkv = ops.causal_conv(proj, col0, self.channels, self.conv_w, None, cache.state, ctx.cu_seqlens, ctx.token_req,
+                                  ctx.state_slots, ctx.num_requests, state_off=self.state_off, act=False)
         rot = self.position.rotary()
         inv_freq, rotary_dim, factor, table = None, 0, 1.0, None
         if rot is not None:
             inv_freq, rotary_dim, factor = rot
             table = self.position.table(ctx) if hasattr(self.position, "table") else None
-        q = ops.rope_kv_write(qkv, ctx.positions, ctx.slot_mapping[cache.group], inv_freq, rotary_dim, factor, self.num_heads,
-                              self.num_kv_heads, self.head_dim, cache.k, cache.v, self.dtype, table, value_dim=self.value_dim,
-                              pad_dim=self.key_dim)
+        if self.rows_path:
+            q = ops.qkv_rows(qkv, ctx.positions, ctx.slot_mapping[cache.group], self.num_heads, self.num_kv_heads, self.head_dim,
+                             self.value_dim, cache.k, cache.v, inv_freq, rotary_dim, factor, table, norms=self.norms,
+                             eps=float(self.qk_norm["eps"]) if self.qk_norm is not None else 0.0, pad_dim=self.key_dim, col0=qkv_col0,
+                             norm_over="head")
+        else:
+            q = ops.rope_kv_write(qkv, ctx.positions, ctx.slot_mapping[cache.group], inv_freq, rotary_dim, factor, self.num_heads,
+                                  self.num_kv_heads, self.head_dim, cache.k, cache.v, self.dtype, table, value_dim=self.value_dim,
+                                  pad_dim=self.key_dim)
         a = ops.paged_attention(q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.cu_seqlens, ctx.context_lens,
                                 ctx.token_req, self.scale, int(self.window or 0), ctx.max_q_len, ctx.max_context_len, ctx.num_single)
-        ops.sigmoid_gate(a, proj if self.gate else None, col0 + self.channels, scale, out, out_col0)
+        ops.sigmoid_gate(a, proj if self.gate else None, col0 + self.channels, scale, out, out_col0, self.gate_per if self.gate else 1)
 
 
 register_part("mixer", "conv_attention", ConvAttention)
+register_part("mixer", "branch_attention", ConvAttention)
 
 
 class LatentAttention(BranchMixer):

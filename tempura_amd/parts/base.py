@@ -78,6 +78,8 @@ class Part:
     #: True when ``forward`` only launches kernels that read the step's data from device memory
     #: (no host-side values of the batch, no host loops): decode steps may then replay a captured graph.
     graph_safe = False
+    #: the type in which the part reads its normed rows (None: the compute dtype), for blocks that ask
+    input_dtype: Optional[torch.dtype] = None
 
     def __init__(self, spec: PartSpec, hidden_size: int, dtype: torch.dtype, device):
         self.spec = spec

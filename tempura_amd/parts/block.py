@@ -279,6 +279,11 @@ class SandwichBlock(ArrangedBlock):
 
     def __init__(self, layer_spec, hidden_size, dtype, device):
         super().__init__(layer_spec, hidden_size, dtype, device)
+        self._check_parts()
+        self.hidden_size = hidden_size
+        self.dtype = dtype
+
+    def _check_parts(self):
         if len({self.ffn is None, self.ffn_norm is None, self.ffn_post_norm is None}) != 1:
             raise ValueError("block 'sandwich': a feed-forward and its two norms come together")
         if self.ffn is None and (self.ffn_gate is not None or self.ffn_scale is not None):
@@ -286,18 +291,26 @@ class SandwichBlock(ArrangedBlock):
         for post in (self.mixer_post_norm, self.ffn_post_norm):
             if post is not None and (type(post).__name__ != "RMSNorm" or getattr(post, "groups", 1) != 1):
                 raise ValueError("block 'sandwich': the norm behind a sublayer must be an RMS norm")
-        self.hidden_size = hidden_size
-        self.dtype = dtype
 
-    @staticmethod
-    def _rms(norm):
-        """(weight, eps) of an RMS norm that the closing kernel can apply, else None."""
+    def _post(self, name):
+        """The norm behind sublayer ``name``, or None where the arrangement has none."""
+        return getattr(self, name + "_post_norm")
+
+    def _input_dtype(self, part):
+        """The type in which ``part`` reads its normed rows (``Part.input_dtype``, by default the compute dtype)."""
+        return getattr(part, "input_dtype", None) or self.dtype
+
+    def _rms(self, norm, part):
+        """(weight, eps, type of the rows) of an RMS norm in front of ``part`` that the closing kernel can apply, else None."""
         if type(norm).__name__ == "RMSNorm" and getattr(norm, "groups", 1) == 1:
-            return norm.weight, norm.eps
+            return norm.weight, norm.eps, self._input_dtype(part)
         return None
 
+    def _normed(self, h, norm, part):
+        return norm.forward(h) if self._input_dtype(part) == self.dtype else norm.forward(h, out_dtype=self._input_dtype(part))
+
     def entry_norm(self, m):
-        return self._rms(self.mixer_norm)
+        return self._rms(self.mixer_norm, self.mixer)
 
     def _run(self, part, x, ctx, cache, n, device):
         """A sublayer's output as a tensor of its own, float32 [tokens, hidden]."""
@@ -314,18 +327,24 @@ class SandwichBlock(ArrangedBlock):
             if gate is not None:
                 gate.load_for(getattr(self, name), get)
         super().load_weights(get)
-        #: what multiplies a sublayer's normed result, by sublayer: the norm's weight times the layer scale
+        #: what multiplies a sublayer's (normed) result, by sublayer: the norm's weight times the layer scale
         self.closing = {}
         for name in ("mixer", "ffn"):
-            post, scale = getattr(self, name + "_post_norm"), getattr(self, name + "_scale")
-            if post is not None:
+            post, scale = self._post(name), getattr(self, name + "_scale")
+            if post is None and scale is not None:
+                self.closing[name] = scale.weight
+            elif post is not None:
                 self.closing[name] = post.weight if scale is None else (post.weight.double() * scale.weight.double()).to(torch.float32)
 
     def _close(self, h, x, result, name, opening):
         """Gate and norm the result of sublayer ``name`` (``x`` its input), add it into the stream; with ``opening``
-        (weight, eps) also return the stream normed for the next sublayer."""
-        gate, weight, eps = getattr(self, name + "_gate"), self.closing[name], getattr(self, name + "_post_norm").eps
-        after = (None, 0.0, None) if opening is None else (opening[0], opening[1], self.dtype)
+        (weight, eps, type) also return the stream normed for the next sublayer."""
+        gate, weight, post = getattr(self, name + "_gate"), self.closing[name], self._post(name)
+        after = (None, 0.0, None) if opening is None else opening
+        if post is None:
+            y, rows, col0, bias = (result, None, 0, None) if gate is None else gate.split(x, result) + (gate.bias,)
+            return ops.scale_add(h, y, weight, *after, gate=rows, gate_col0=col0, gate_bias=bias)
+        eps = post.eps
         if gate is not None:
             y, rows, col0 = gate.split(x, result)
             return ops.norm_add(h, y, weight, eps, *after, gate=rows, gate_col0=col0, gate_bias=gate.bias)
@@ -334,19 +353,38 @@ class SandwichBlock(ArrangedBlock):
     def forward(self, h, ctx, cache, x=None, next_norm=None):
         n = h.shape[0]
         if x is None:
-            x = self.mixer_norm.forward(h)
+            x = self._normed(h, self.mixer_norm, self.mixer)
         y = self._run(self.mixer, x, ctx, cache, n, h.device)
         after = next_norm if isinstance(next_norm, tuple) else None
         if self.ffn is None:
             return self._close(h, x, y, "mixer", after)
-        x2 = self._close(h, x, y, "mixer", self._rms(self.ffn_norm))
+        x2 = self._close(h, x, y, "mixer", self._rms(self.ffn_norm, self.ffn))
         if x2 is None:
-            x2 = self.ffn_norm.forward(h)
+            x2 = self._normed(h, self.ffn_norm, self.ffn)
         y2 = self._run(self.ffn, x2, ctx, None, n, h.device)
         return self._close(h, x2, y2, "ffn", after)
 
 
 register_part("block", "sandwich", SandwichBlock)
+
+
+class ScaledPreNormBlock(SandwichBlock):
+    """The sandwich arrangement without the norms behind the sublayers: ``h += scale * mixer(norm(h))``, then, when the
+    layer has a feed-forward, ``h += scale * ffn(norm(h))``, ``scale`` a vector per sublayer (each may have a gate as
+    well).  One kernel scales a sublayer's output, adds it into the stream and norms the stream for the next sublayer."""
+    ROLES = {"mixer_norm": "norm", "mixer": "mixer", "mixer_gate": "gate", "mixer_scale": "scale",
+             "ffn_norm": "norm", "ffn": "ffn", "ffn_gate": "gate", "ffn_scale": "scale"}
+    OPTIONAL = frozenset({"ffn_norm", "ffn", "mixer_gate", "ffn_gate", "ffn_scale"})
+
+    def _check_parts(self):
+        if len({self.ffn is None, self.ffn_norm is None, self.ffn_scale is None}) != 1 or (self.ffn is None and self.ffn_gate is not None):
+            raise ValueError("block 'scaled_prenorm': a feed-forward, its norm and its scale come together")
+
+    def _post(self, name):
+        return None
+
+
+register_part("block", "scaled_prenorm", ScaledPreNormBlock)
 
 
 class SharedNormBlock(ArrangedBlock):

@@ -177,9 +177,9 @@ class RoutedExperts(FeedForward):
 
     ``expert`` (default ``"gated"``): ``"plain"`` experts are ``down(act(up(x)))`` without a gate, ``activation`` naming the
     function (``ops.ACTIVATIONS``; it reads the float32 sums of the up product).
-    ``shared`` (``{"intermediate_size", "activation"}``, tensor roles ``shared_up``, ``shared_down``, ``shared_gate`` [1,
-    hidden]): one more plain expert that every token uses, its output times sigmoid(w_gate . x), one number a token, added
-    to the routed sum.  The gate row rides along in the shared up product, and the gate multiplies the activations in
+    ``shared`` (``{"intermediate_size", "activation"}``, tensor roles ``shared_up``, ``shared_down`` and, optionally,
+    ``shared_gate`` [1, hidden]): one more plain expert that every token uses, its output, with a gate times
+    sigmoid(w_gate . x), one number a token, added to the routed sum.  The gate row rides along in the shared up product, and the gate multiplies the activations in
     front of the down product (which is linear), not its result."""
     graph_safe = True
     returns_output = True
@@ -216,6 +216,7 @@ class RoutedExperts(FeedForward):
         self.shared = p.get("shared")
         if self.shared is not None and str(self.shared.get("activation", "silu")) not in ops.ACTIVATIONS:
             raise ValueError(f"moe: shared activation {self.shared.get('activation')!r} unknown")
+        self.shared_gated = "shared_gate" in spec.weights
         self.has_router_bias = "router_bias" in spec.weights
         self.plain_router = (self.score, self.group_best, self.normalize, self.weight_scale) == ("softmax", 1, False, 1.0) \
             and not self.has_router_bias
@@ -242,7 +243,8 @@ class RoutedExperts(FeedForward):
             si = int(p["shared"]["intermediate_size"])
             out[w["shared_up"]] = WeightInfo((si, hidden_size))
             out[w["shared_down"]] = WeightInfo((hidden_size, si))
-            out[w["shared_gate"]] = WeightInfo((1, hidden_size))
+            if "shared_gate" in w:
+                out[w["shared_gate"]] = WeightInfo((1, hidden_size))
         return out
 
     def load_weights(self, get):
@@ -254,11 +256,17 @@ class RoutedExperts(FeedForward):
         if self.shared is not None:
             # the gate's row behind the up rows: one product gives the activations' sums and the gate's
             self.shared_size = int(self.shared["intermediate_size"])
-            self.w_shared_up = ops.tile_weight(pad_rows(torch.cat([self._to_device(get(w["shared_up"])),
-                                                                   self._to_device(get(w["shared_gate"])).reshape(1, -1)], dim=0), 16))
+            rows = [self._to_device(get(w["shared_up"]))]
+            if self.shared_gated:
+                rows.append(self._to_device(get(w["shared_gate"])).reshape(1, -1))
+            self.w_shared_up = ops.tile_weight(pad_rows(torch.cat(rows, dim=0), 16))
+            self.shared_relu2 = not self.shared_gated and self.shared.get("activation") == "relu2" and \
+                ops.linear_relu2_ok(self.shared_size, self.hidden_size, self.dtype)
             self.w_shared_down = ops.tile_weight(self._to_device(get(w["shared_down"])))
         gated = self.expert_kind == "gated"
         self.fused = gated and self.dtype == torch.bfloat16 and ops.gated_layout_ok(self.intermediate_size, self.hidden_size)
+        # (plain experts with the squared ReLU: in the up product's own epilogue)
+        self.fused_relu2 = not gated and self.activation == "relu2" and ops.linear_relu2_ok(self.intermediate_size, self.hidden_size, self.dtype)
         stack, self.w2 = [], []
         for n in range(self.experts):
             up = self._to_device(get(w["up"].format(n)))
@@ -276,6 +284,8 @@ class RoutedExperts(FeedForward):
         self.w13 = [ops.weight_rows(self.w13_all, n * rows, (n + 1) * rows) for n in range(self.experts)]
 
     def _expert(self, n, rows):
+        if self.fused_relu2:
+            return ops.linear_relu2(rows, self.w13[n], self.intermediate_size)[0]
         if self.expert_kind == "plain":
             return ops.activation(ops.linear(rows, self.w13[n], torch.float32), self.activation, self.dtype)
         if self.fused:
@@ -283,9 +293,14 @@ class RoutedExperts(FeedForward):
         return ops.swiglu(ops.linear(rows, self.w13[n], torch.float32), self.dtype)
 
     def _add_shared(self, x, y):
-        """y += down_s(act(up_s x) * sigmoid(w_gate . x)): the expert every token uses."""
+        """y += down_s(act(up_s x) * sigmoid(w_gate . x)): the expert every token uses (without a gate: no sigmoid)."""
+        if self.shared_relu2:
+            a = ops.linear_relu2(x, self.w_shared_up, self.shared_size, blocked_out=True)[0]
+            ops.linear(a, self.w_shared_down, torch.float32, residual=y)
+            return
         u = ops.linear(x, self.w_shared_up, torch.float32)
-        a = ops.activation(u, str(self.shared.get("activation", "silu")), self.dtype, 0, self.shared_size, self.shared_size)
+        a = ops.activation(u, str(self.shared.get("activation", "silu")), self.dtype, 0, self.shared_size,
+                           self.shared_size if self.shared_gated else None)
         ops.linear(a, self.w_shared_down, torch.float32, residual=y)
 
     def forward(self, x, ctx, residual=None):
@@ -308,7 +323,9 @@ class RoutedExperts(FeedForward):
                                                 group_best=self.group_best, normalize=self.normalize, sum_eps=self.sum_eps,
                                                 scale=self.weight_scale)
         if getattr(ctx, "max_q_len", 1) <= 1:
-            if self.expert_kind == "plain":
+            if self.fused_relu2:
+                a = ops.linear_relu2(x, self.w13_all, self.experts * self.intermediate_size)[0]
+            elif self.expert_kind == "plain":
                 a = ops.activation(ops.linear(x, self.w13_all, torch.float32), self.activation, self.dtype)
             elif self.fused:
                 a = ops.linear_swiglu(x, self.w13_all)

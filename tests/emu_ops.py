@@ -348,11 +348,13 @@ class EmuOps:
         return v.to(a.dtype)
 
     def qkv_rows(self, rows, positions, slots, num_heads, num_kv_heads, head_dim, value_dim, k_cache, v_cache, inv_freq, rotary_dim,
-                 factor, biases, norms, eps, value_inv_freq, pad_dim):
+                 factor, biases, norms, eps, value_inv_freq, pad_dim, col0=0, norm_over="projection"):
         n = rows.shape[0]
         widths = [num_heads * head_dim, num_kv_heads * head_dim, num_kv_heads * value_dim]
-        q, k, v = rows.double()[:, : sum(widths)].split(widths, dim=1)
+        q, k, v = rows.double()[:, col0: col0 + sum(widths)].split(widths, dim=1)
         q, k, v = (x if b is None else x + b.double() for x, b in zip((q, k, v), biases))
+        if norms is not None and norm_over == "head":
+            q, k = (x.reshape(n, -1, head_dim) for x in (q, k))
         if norms is not None:
             q, k = (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w.double() for x, w in zip((q, k), norms))
         q = q.reshape(n, num_heads, head_dim)
@@ -409,6 +411,46 @@ class EmuOps:
         if next_weight is None:
             return None
         return self.rmsnorm(h, next_weight, next_eps, out_dtype)
+
+    def scale_add(self, h, y, weight, next_weight=None, next_eps=0.0, out_dtype=None, gate=None, gate_col0=0, gate_bias=None):
+        yd = y.double()
+        if gate is not None:
+            z = gate.double()[:, gate_col0: gate_col0 + y.shape[1]]
+            yd = yd * torch.sigmoid(z if gate_bias is None else z + gate_bias.double())
+        h.copy_((h.double() + yd * weight.double()).to(torch.float32))
+        return None if next_weight is None else self.rmsnorm(h, next_weight, next_eps, out_dtype)
+
+    def token_shift(self, x, mu, state, state_off, cu_seqlens, token_req, state_slots, num_requests, out_dtype):
+        width = x.shape[1]
+        before = torch.zeros_like(x, dtype=torch.float64)
+        cu = cu_seqlens.tolist()
+        for r in range(num_requests):
+            a, e = cu[r], cu[r + 1]
+            if e > a:
+                carried = state[int(state_slots[r]), state_off: state_off + width]
+                before[a:e] = torch.cat([carried[None], x[a: e - 1]]).double()
+                carried.copy_(x[e - 1])
+        return [(x.double() + (before - x.double()) * m.double()).to(out_dtype) for m in mu]
+
+    def linear_scan(self, q, k, v, decay, state, state_off, cu_seqlens, state_slots, num_requests, heads, dim, vdim, bonus=None, q_scale=1.0):
+        n, size = decay.shape[0], heads * dim * vdim
+        part = lambda rows, d: rows[0].double()[:, rows[1]: rows[1] + heads * d].reshape(n, heads, d)
+        q, k, v, w = part(q, dim) * q_scale, part(k, dim), part(v, vdim), decay.double().reshape(n, heads, dim)
+        y = torch.zeros(n, heads, vdim, dtype=torch.float64)
+        cu = cu_seqlens.tolist()
+        for r in range(num_requests):
+            if cu[r + 1] <= cu[r]:
+                continue
+            row = state[int(state_slots[r]), state_off: state_off + size]
+            S = row.double().reshape(heads, vdim, dim)      # (kept column by column)
+            for t in range(cu[r], cu[r + 1]):
+                own = v[t][:, :, None] * k[t][:, None, :]
+                new = w[t][:, None, :] * S + own
+                seen = new if bonus is None else S + own * bonus.double().reshape(heads, 1, dim)
+                y[t] = (seen * q[t][:, None, :]).sum(-1)
+                S = new
+            row.copy_(S.reshape(-1).to(torch.float32))
+        return y.reshape(n, heads * vdim).to(torch.float32)
 
     def activation(self, u, kind, out_dtype, col0=0, width=None, gate_col=None):
         z = u.double() if width is None else u.double()[:, col0: col0 + width]
@@ -526,6 +568,10 @@ class EmuOps:
         r = weight_t.shape[0]
         xin = x.double()[:, col0: col0 + r]
         v = (torch.tanh(xin) if in_act == "tanh" else xin) @ weight_t.double()
+        if mode == "exp_exp":
+            v = torch.exp(-torch.exp(v + bias.double()))
+        if mode == "root_sigmoid":
+            v = torch.sigmoid(v + bias.double()) ** rate
         if mode == "rate_sigmoid":
             v = torch.exp(-rate * torch.sigmoid(v + bias.double()))
         if mode == "sigmoid":
@@ -564,7 +610,7 @@ class EmuOps:
             state[slot, state_off: state_off + size] = S.transpose(1, 2).reshape(-1).to(torch.float32)
         return y.reshape(n, heads * vdim).to(torch.float32)
 
-    def head_norm_gate(self, o, weight, gate, eps, scale, heads, out, out_col0, gate_rows=None, gate_col0=0):
+    def head_norm_gate(self, o, weight, gate, eps, scale, heads, out, out_col0, gate_rows=None, gate_col0=0, gate_act="sigmoid"):
         n, vdim = o.shape[0], o.shape[1] // heads
         x = o.double().reshape(n, heads, vdim)
         w = weight.double().reshape(-1, vdim)      # [1, vdim] shared or [heads, vdim]
@@ -572,7 +618,8 @@ class EmuOps:
         if gate is not None:
             x = x * gate.double()
         if gate_rows is not None:
-            x = x * torch.sigmoid(gate_rows.double()[:, gate_col0: gate_col0 + heads * vdim])
+            z = gate_rows.double()[:, gate_col0: gate_col0 + heads * vdim]
+            x = x * torch.sigmoid(z) * (z if gate_act == "silu" else 1.0)
         out[:, out_col0: out_col0 + heads * vdim] = (x * scale).to(out.dtype)
 
     def swiglu(self, gu, out_dtype):
