@@ -58,7 +58,7 @@ def parse_args():
     ap.add_argument("--mixed-chunk", type=int, default=512)
     ap.add_argument("--mixed-temperature", type=float, default=0.0, help="0: greedy; above: seeded sampling with top-k 50")
     ap.add_argument("--decode-target-blocks", type=int, default=None, help="tuning: blocks the split decode attention aims at")
-    ap.add_argument("--design", default=None, choices=["mifutar", "bomotar", "golavik", "zemarax", "tokatar"],
+    ap.add_argument("--design", default=None, choices=["mifutar", "bomotar", "golavik", "zemarax", "tokatar", "makisun"],
                     help="instead of the headline: prefill and decode throughput of this design at layer sizes of real models, "
                          "beside Llama layers of equal size, with the time of every kernel entry point")
     ap.add_argument("--design-sizes", default="2048,4096", help="model widths of --design (comma separated)")
@@ -95,10 +95,15 @@ def design_bench(args) -> int:
     denominator, a latent attention of the Llama layer's heads (a latent of four heads beside a rotated part of half a head) and
     the first kind again, each with a gate on both sublayers and an ungated feed-forward of the Llama layer's width; it
     stands beside the Zemarax model (the closest: norms around every sublayer, attention over cached latents) and the
+    Llama layers.  A Makisun model here has, in turn, layers of a token-shifted recurrence (width / 64 heads of 64, a decay
+    of rank 64) and of two mixers side by side: an attention of the Llama layer's heads (a norm per head, window 1,024,
+    gated heads) and a gated linear attention of width / 128 heads of 64 x 128 (a decay of rank 64); feed-forwards
+    alternate between an ungated dense one and eight ungated experts of a quarter of its width, two a token, with a shared
+    expert; it stands beside the Bomotar model (the closest: an attention beside a recurrence, routed experts) and the
     Llama layers.
     Prints one JSON line."""
     import torch
-    from tempura_amd.config import BomotarConfig, GolavikConfig, LlamaConfig, MifutarConfig, TokatarConfig, ZemaraxConfig
+    from tempura_amd.config import BomotarConfig, GolavikConfig, LlamaConfig, MakisunConfig, MifutarConfig, TokatarConfig, ZemaraxConfig
     from tempura_amd.engine import Engine
     from tempura_amd.engine.loading import random_model
     from tempura_amd.engine.runner import StepEntry
@@ -174,6 +179,19 @@ def design_bench(args) -> int:
         return TokatarConfig.from_dict({"architecture": "Tokatar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
                                         "embedding": {"scale": 1.0}, "layers": ls, "max_positions": 8192})
 
+    def makisun_config(width, ff, heads, dim, kv, layers):
+        wkv = {"heads": width // 64, "dim": 64, "decay_rank": 64}
+        left = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": window},
+                "rot": {"dims": dim, "base": 500000.0}}
+        right = {"heads": width // 128, "dim": 64, "vdim": 128, "tau": 16.0, "decay_rank": 64}
+        parallel = {"left": left, "right": right, "left_scale": 0.75, "right_scale": 1.1}
+        dense = {"kind": "dense", "ff": ff}
+        moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 4}}
+        kinds = [("wkv", wkv, dense), ("parallel", parallel, moe), ("wkv", wkv, moe), ("parallel", parallel, dense)]
+        ls = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": kinds[i % 4][2]} for i in range(layers)]
+        return MakisunConfig.from_dict({"architecture": "Makisun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+                                        "embedding": {"scale": 1.0}, "layers": ls, "max_positions": 8192})
+
     def llama_config(width, ff, heads, dim, kv, layers):
         return LlamaConfig(width, ff, layers, heads, kv, dim, vocab, 8192, 1e-5, 500000.0, None, False,
                            sliding_window=window if design == "mifutar" else None)
@@ -239,6 +257,9 @@ def design_bench(args) -> int:
         if design == "tokatar":
             models = [("tokatar", tokatar_config(width, ff, heads, dim, kv, args.design_layers)),
                       ("zemarax", zemarax_config(width, ff, heads, dim, kv, args.design_layers)), models[1]]
+        if design == "makisun":
+            models = [("makisun", makisun_config(width, ff, heads, dim, kv, args.design_layers)),
+                      ("bomotar", bomotar_config(width, ff, heads, dim, kv, args.design_layers)), models[1]]
         chosen = [m for m in args.design_models.split(",") if m]
         for name, cfg in [m for m in models if not chosen or m[0] in chosen]:
             say(f"{name} width {width}: building")
@@ -256,7 +277,8 @@ def design_bench(args) -> int:
                                             "bomotar": "Bomotar beside Mifutar and Llama layers of equal size",
                                             "golavik": "Golavik beside Bomotar and Llama layers of equal size",
                                             "zemarax": "Zemarax beside Bomotar and Llama layers of equal size",
-                                            "tokatar": "Tokatar beside Zemarax and Llama layers of equal size"}[design],
+                                            "tokatar": "Tokatar beside Zemarax and Llama layers of equal size",
+                                            "makisun": "Makisun beside Bomotar and Llama layers of equal size"}[design],
                                  "layers": args.design_layers, "prompt": T, "decode_batch": batch,
                                  "window": window if design == "mifutar" else None}, "points": points}))
     return 0

@@ -148,15 +148,14 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(QkvRows a, T* __restrict_
   }
 }
 
-// The same with a norm over every head by itself (weights q_norm and k_norm [dim], shared by the heads; nullptr: no norm): a
-// wave takes one head of one token.  units: tokens times per_token, the heads of a token that this launch takes (q, k and,
-// in short steps, v).
+// The same with a norm over every head by itself (weights q_norm and k_norm [dim], shared by the heads; nullptr: no norm):
+// `group` neighbouring lanes (a power of two) take one head of one token.  units: tokens times per_token, the heads of a
+// token that this launch takes (q, k and, in short steps, v).
 template <typename T, int V>
-__global__ __launch_bounds__(256) void qkv_heads_kernel(QkvRows a, long units, int per_token, T* __restrict__ q_out, T* __restrict__ k_cache,
+__global__ __launch_bounds__(256) void qkv_heads_kernel(QkvRows a, long units, int per_token, int group, T* __restrict__ q_out, T* __restrict__ k_cache,
                                                         T* __restrict__ v_cache) {
-  const long unit = (long)blockIdx.x * 4 + threadIdx.x / TP_WAVE;
-  const int lane = threadIdx.x % TP_WAVE;
-  if (unit >= units) return;
+  const long mine = ((long)blockIdx.x * 256 + threadIdx.x) / group, unit = min(mine, units - 1);   // (every lane takes part in the sums)
+  const int lane = threadIdx.x % group;
   const int t = (int)(unit / per_token), hh = (int)(unit % per_token);
   const int sec = hh < a.heads ? 0 : hh < a.heads + a.kv ? 1 : 2;
   const int h = sec == 0 ? hh : sec == 1 ? hh - a.heads : hh - a.heads - a.kv;
@@ -176,21 +175,22 @@ __global__ __launch_bounds__(256) void qkv_heads_kernel(QkvRows a, long units, i
     return x;
   };
   float rstd = 1.f;
-  if (w != nullptr) {   // (uniform over the wave)
+  if (a.q_norm != nullptr) {   // (uniform over the wave; a value head's sum is not used)
     float ss = 0.f;
-    for (int i = lane * V; i < hdim; i += TP_WAVE * V) {
+    for (int i = lane * V; i < hdim; i += group * V) {
       const Elems<V> x = load(i);
 #pragma unroll
       for (int e = 0; e < V; ++e) ss = fmaf(x.x[e], x.x[e], ss);
     }
-    ss = wave_sum(ss);
+    ss = lanes_sum_of(ss, group);
     rstd = 1.0f / sqrtf(ss / (float)hdim + a.eps);
   }
+  if (mine >= units) return;
   const int pos = a.positions[t], slot = a.slots[t];
   const size_t page = (size_t)(slot / a.page_size), off = (size_t)(slot % a.page_size);
   if (sec == 2) {
     T* o = v_cache + ((page * a.kv + h) * a.vdim) * a.page_size + off;
-    for (int i = lane * V; i < hdim; i += TP_WAVE * V) {
+    for (int i = lane * V; i < hdim; i += group * V) {
       Elems<V> x = load(i);
       if (a.v_inv_freq != nullptr) turn_pairs<V>(x, i, a.vdim / 2, t, pos, a.v_inv_freq, a.v_table, 1.0f, 1.0f);
 #pragma unroll
@@ -199,7 +199,7 @@ __global__ __launch_bounds__(256) void qkv_heads_kernel(QkvRows a, long units, i
     return;
   }
   T* o = sec == 0 ? q_out + ((size_t)t * a.heads + h) * a.out_dim : k_cache + ((page * a.kv + h) * a.page_size + off) * a.out_dim;
-  for (int i = lane * V; i < a.out_dim; i += TP_WAVE * V) {
+  for (int i = lane * V; i < a.out_dim; i += group * V) {
     Elems<V> x;
     if (i < hdim) {
       x = load(i);
@@ -310,14 +310,16 @@ extern "C" int tp_qkv_rows(const float* rows, size_t stride, size_t width, const
   if (per_head) {
     const int per_token = heads + kv + (lng ? 0 : kv);
     const long units = (long)n * per_token;
-    TP_REQUIRE((units + 3) / 4 < 0x7fffffffL, "qkv_rows: too many rows");
-    const dim3 grid((unsigned)((units + 3) / 4));
+    int group = 1;
+    while (group < TP_WAVE && group * V < out_dim) group *= 2;
+    TP_REQUIRE(units * group / 256 + 1 < 0x7fffffffL, "qkv_rows: too many rows");
+    const dim3 grid((unsigned)((units * group + 255) / 256));
 #define QKV_HEADS(T)                                                                                                                 \
   do {                                                                                                                               \
     if (four)                                                                                                                        \
-      hipLaunchKernelGGL((qkv_heads_kernel<T, 4>), grid, dim3(256), 0, s, a, units, per_token, (T*)q_out, (T*)k_cache, (T*)v_cache); \
+      hipLaunchKernelGGL((qkv_heads_kernel<T, 4>), grid, dim3(256), 0, s, a, units, per_token, group, (T*)q_out, (T*)k_cache, (T*)v_cache); \
     else                                                                                                                             \
-      hipLaunchKernelGGL((qkv_heads_kernel<T, 2>), grid, dim3(256), 0, s, a, units, per_token, (T*)q_out, (T*)k_cache, (T*)v_cache); \
+      hipLaunchKernelGGL((qkv_heads_kernel<T, 2>), grid, dim3(256), 0, s, a, units, per_token, group, (T*)q_out, (T*)k_cache, (T*)v_cache); \
     if (lng)                                                                                                                         \
       hipLaunchKernelGGL(qkv_values_kernel<T>, dim3((n + 15) / 16, kv), dim3((vdim + 63) / 64 * 64), 0, s, a, n, (T*)v_cache);       \
   } while (0)

@@ -119,6 +119,12 @@ __device__ inline float wave_sum(float v) {
   return v;
 }
 
+// Sum over `lanes` (a power of two) neighbouring lanes, from a multiple of `lanes` on; every lane gets it.
+__device__ inline float lanes_sum_of(float v, int lanes) {
+  for (int o = lanes / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, TP_WAVE);
+  return v;
+}
+
 __device__ inline float wave_max(float v) {
 #pragma unroll
   for (int o = TP_WAVE / 2; o > 0; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, TP_WAVE));

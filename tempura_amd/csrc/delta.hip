@@ -296,12 +296,21 @@ extern "C" int tp_delta_scan(float* qkv, int row_stride, const float* decay, con
 // A block takes eight rows and 256 columns; a row's sum has the same order of additions wherever the row stands.
 #define LR_ROWS 8
 
+__device__ inline float lowrank_f(float v, int mode, float rate, float b) {
+  if (mode == 1) return d_sigmoid(v);
+  if (mode == 2) return expf(-rate * d_softplus(v + b));
+  if (mode == 3) return expf(-rate * d_sigmoid(v + b));
+  if (mode == 4) return expf(-expf(v + b));
+  if (mode == 5) return expf(-rate * d_softplus(-(v + b)));
+  return v;
+}
+
 __global__ __launch_bounds__(256) void lowrank_up_kernel(const float* __restrict__ x, int x_stride, int col0, int rank,
                                                          const float* __restrict__ wt, float* __restrict__ out, int n,
                                                          int n_out, int mode, const float* __restrict__ a_log,
                                                          const float* __restrict__ bias, int per_head, int in_act,
                                                          float rate_const) {
-  // (blocks of 64 or 256 threads: a thread owns one column)
+  // (a thread owns one column)
   extern __shared__ __attribute__((aligned(16))) float xs[];   // [LR_ROWS][rank4]: rows padded with zeros to four
   const int rank4 = (rank + 3) & ~3;
   const int t0 = blockIdx.x * LR_ROWS, c = blockIdx.y * blockDim.x + threadIdx.x;
@@ -341,14 +350,54 @@ __global__ __launch_bounds__(256) void lowrank_up_kernel(const float* __restrict
 #pragma unroll
   for (int t = 0; t < LR_ROWS; ++t) {
     if (t0 + t >= n) break;
-    float v = acc[t];
-    if (mode == 1) v = d_sigmoid(v);
-    if (mode == 2) v = expf(-rate * d_softplus(v + b));
-    if (mode == 3) v = expf(-rate * d_sigmoid(v + b));
-    if (mode == 4) v = expf(-expf(v + b));
-    if (mode == 5) v = expf(-rate * d_softplus(-(v + b)));
-    out[(size_t)(t0 + t) * n_out + c] = v;
+    out[(size_t)(t0 + t) * n_out + c] = lowrank_f(acc[t], mode, rate, b);
   }
+}
+
+// the same for a few rows: a block takes eight rows and 64 columns, its eight waves split the inner size (interleaved runs
+// of four, so that a wave has many weights in flight) and their sums meet through LDS in the order of the waves
+__global__ __launch_bounds__(512) void lowrank_up_few_kernel(const float* __restrict__ x, int x_stride, int col0, int rank,
+                                                             const float* __restrict__ wt, float* __restrict__ out, int n,
+                                                             int n_out, int mode, const float* __restrict__ a_log,
+                                                             const float* __restrict__ bias, int per_head, int in_act,
+                                                             float rate_const) {
+  extern __shared__ __attribute__((aligned(16))) float xs[];   // [LR_ROWS][rank4], then [8][LR_ROWS][64]
+  const int rank4 = (rank + 3) & ~3;
+  float* red = xs + LR_ROWS * rank4;
+  const int t0 = blockIdx.x * LR_ROWS, lane = threadIdx.x % TP_WAVE, wave = threadIdx.x / TP_WAVE;
+  const int c = blockIdx.y * TP_WAVE + lane, cc = min(c, n_out - 1);
+  for (int idx = threadIdx.x; idx < LR_ROWS * rank4; idx += 512) {
+    const int t = idx / rank4, i = idx % rank4;
+    const float v = (t0 + t < n && i < rank) ? x[(size_t)(t0 + t) * x_stride + col0 + i] : 0.f;
+    xs[idx] = in_act == 1 ? tanhf(v) : v;
+  }
+  __syncthreads();
+  float acc[LR_ROWS];
+#pragma unroll
+  for (int t = 0; t < LR_ROWS; ++t) acc[t] = 0.f;
+  for (int i = wave * 4; i < rank4; i += 32) {
+    float w[4];
+#pragma unroll
+    for (int d = 0; d < 4; ++d) w[d] = i + d < rank ? wt[(size_t)(i + d) * n_out + cc] : 0.f;
+#pragma unroll
+    for (int t = 0; t < LR_ROWS; ++t) {
+      const float4 v = *(const float4*)(xs + t * rank4 + i);
+      acc[t] = fmaf(v.x, w[0], acc[t]);
+      acc[t] = fmaf(v.y, w[1], acc[t]);
+      acc[t] = fmaf(v.z, w[2], acc[t]);
+      acc[t] = fmaf(v.w, w[3], acc[t]);
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < LR_ROWS; ++t) red[(wave * LR_ROWS + t) * TP_WAVE + lane] = acc[t];
+  __syncthreads();
+  // wave t finishes row t
+  if (c >= n_out || t0 + wave >= n) return;
+  float v = 0.f;
+#pragma unroll
+  for (int p = 0; p < 8; ++p) v += red[(p * LR_ROWS + wave) * TP_WAVE + lane];
+  const float rate = mode == 2 ? expf(a_log[c / per_head]) : rate_const, b = mode >= 2 ? bias[c] : 0.f;
+  out[(size_t)(t0 + wave) * n_out + c] = lowrank_f(v, mode, rate, b);
 }
 
 extern "C" int tp_lowrank_up(const float* x, int x_stride, int col0, int rank, const float* wt, float* out, int n, int n_out,
@@ -359,11 +408,19 @@ extern "C" int tp_lowrank_up(const float* x, int x_stride, int col0, int rank, c
   TP_REQUIRE(mode < 3 || bias, "lowrank_up: the decay needs its biases");
   TP_REQUIRE(mode != 2 || (a_log && bias && per_head > 0), "lowrank_up: the decay needs its rates and biases");
   if (n == 0) return 0;
-  // (a few rows: blocks of one wave, so that the columns are spread over many CUs)
-  const int threads = n <= 64 ? 64 : 256;
+  const size_t rows_lds = sizeof(float) * LR_ROWS * ((rank + 3) & ~3);
+  if (n <= 64) {
+    const dim3 few((n + LR_ROWS - 1) / LR_ROWS, (n_out + 63) / 64);
+    TP_REQUIRE(few.y <= 65535, "lowrank_up: too many columns");
+    hipLaunchKernelGGL(lowrank_up_few_kernel, few, dim3(512), rows_lds + sizeof(float) * 8 * LR_ROWS * 64, s, x, x_stride, col0, rank, wt, out,
+                       n, n_out, mode, a_log, bias, per_head, in_act, rate);
+    TP_CHECK_LAUNCH("lowrank_up");
+    return 0;
+  }
+  const int threads = 256;
   const dim3 grid((n + LR_ROWS - 1) / LR_ROWS, (n_out + threads - 1) / threads);
   TP_REQUIRE(grid.y <= 65535, "lowrank_up: too many columns");
-  hipLaunchKernelGGL(lowrank_up_kernel, grid, dim3(threads), sizeof(float) * LR_ROWS * ((rank + 3) & ~3), s, x, x_stride, col0, rank, wt, out, n,
+  hipLaunchKernelGGL(lowrank_up_kernel, grid, dim3(threads), rows_lds, s, x, x_stride, col0, rank, wt, out, n,
                      n_out, mode, a_log, bias, per_head, in_act, rate);
   TP_CHECK_LAUNCH("lowrank_up");
   return 0;
@@ -400,6 +457,50 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
+// the same, four neighbouring elements a lane and `group` lanes (a power of two) a head, so that heads of up to 128 elements
+// share a wave (vdim, strides and first columns multiples of four).  units: tokens times heads.
+template <typename TO>
+__global__ __launch_bounds__(256) void head_norm_gate4_kernel(const float* __restrict__ o, const float* __restrict__ w,
+                                                              const float* __restrict__ gate, float eps, float scale,
+                                                              TO* __restrict__ out, int out_stride, int out_col0, long pairs,
+                                                              int heads, int vdim, int w_stride, size_t gate_stride, int gate_raw,
+                                                              int group) {
+  const long p0 = ((long)blockIdx.x * 256 + threadIdx.x) / group;
+  const int gl = threadIdx.x % group;
+  const bool live = p0 < pairs;      // (every lane takes part in the sums)
+  const long p = live ? p0 : pairs - 1;
+  const long t = p / heads;
+  const int h = (int)(p % heads);
+  const float* row = o + (size_t)p * vdim;
+  float ss = 0.f;
+  for (int d = gl * 4; d < vdim; d += group * 4) {
+    const float4 x = *(const float4*)(row + d);
+    ss = fmaf(x.x, x.x, ss);
+    ss = fmaf(x.y, x.y, ss);
+    ss = fmaf(x.z, x.z, ss);
+    ss = fmaf(x.w, x.w, ss);
+  }
+  ss = lanes_sum_of(ss, group);
+  const float rstd = 1.0f / sqrtf(ss / (float)vdim + eps);
+  if (!live) return;
+  TO* dst = out + (size_t)t * out_stride + out_col0 + (size_t)h * vdim;
+  const float* wh = w + (size_t)h * w_stride;
+  const float* gr = gate != nullptr ? gate + (size_t)t * gate_stride + (size_t)h * vdim : nullptr;
+  auto gated = [&](float v, float g) { return v * (gate_raw == 2 ? g * d_sigmoid(g) : gate_raw ? d_sigmoid(g) : g); };
+  for (int d = gl * 4; d < vdim; d += group * 4) {
+    const float4 x = *(const float4*)(row + d), wv = *(const float4*)(wh + d);
+    float v[4] = {x.x * rstd * wv.x, x.y * rstd * wv.y, x.z * rstd * wv.z, x.w * rstd * wv.w};
+    if (gr != nullptr) {
+      const float4 g = *(const float4*)(gr + d);
+      v[0] = gated(v[0], g.x);
+      v[1] = gated(v[1], g.y);
+      v[2] = gated(v[2], g.z);
+      v[3] = gated(v[3], g.w);
+    }
+    from_float4(dst + d, v[0] * scale, v[1] * scale, v[2] * scale, v[3] * scale);
+  }
+}
+
 extern "C" int tp_head_norm_gate(const float* o, const float* w, const float* gate, float eps, float scale, void* out, int out_dt,
                                  int out_stride, int out_col0, int n, int heads, int vdim, int w_per_head, size_t gate_stride,
                                  int gate_raw, hipStream_t s) {
@@ -408,6 +509,23 @@ extern "C" int tp_head_norm_gate(const float* o, const float* w, const float* ga
   const long pairs = (long)n * heads;
   const long blocks = (pairs + 3) / 4;
   TP_REQUIRE(blocks < 0x7fffffffL, "head_norm_gate: too many rows");
+  TP_REQUIRE(out_dt == TP_F32 || out_dt == TP_BF16, "head_norm_gate: unknown dtype %d", out_dt);
+  if (vdim % 4 == 0 && out_stride % 4 == 0 && out_col0 % 4 == 0 && gate_stride % 4 == 0 &&
+      (((uintptr_t)o | (uintptr_t)w | (uintptr_t)gate | (uintptr_t)out) & 15) == 0) {
+    int group = 1;
+    while (group < 64 && group * 4 < vdim) group *= 2;
+    const dim3 grid((unsigned)((pairs * group + 255) / 256));
+#define HNG4(T)                                                                                                                          \
+  hipLaunchKernelGGL(head_norm_gate4_kernel<T>, grid, dim3(256), 0, s, o, w, gate, eps, scale, (T*)out, out_stride, out_col0, pairs, heads, \
+                     vdim, w_per_head ? vdim : 0, gate_stride, gate_raw, group)
+    if (out_dt == TP_F32)
+      HNG4(float);
+    else
+      HNG4(bf16_t);
+#undef HNG4
+    TP_CHECK_LAUNCH("head_norm_gate");
+    return 0;
+  }
   if (out_dt == TP_F32)
     hipLaunchKernelGGL(head_norm_gate_kernel<float>, dim3((unsigned)blocks), dim3(256), 0, s, o, w, gate, eps, scale, (float*)out,
                        out_stride, out_col0, pairs, heads, vdim, w_per_head ? vdim : 0, gate_stride, gate_raw);

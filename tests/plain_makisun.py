@@ -53,11 +53,11 @@ def wkv_decay(rows, w1, w2, w0):
 
 
 def wkv_chain(r, k, v, w, bonus):
-    """r, k, v, w [T, H, D]; bonus [H, D].  Per head, with S [key, value] from zero, a token reads the state as the token
-    before left it plus its own k v^T with every key channel times the bonus; then S <- diag(w) S + k v^T."""
+    """r, k, w [T, H, D]; v [T, H, E] (here E = D); bonus [H, D].  Per head, with S [key, value] from zero, a token reads the
+    state as the token before left it plus its own k v^T with every key channel times the bonus; then S <- diag(w) S + k v^T."""
     T, H, D = r.shape
-    S = torch.zeros(H, D, D, dtype=F64)
-    out = torch.zeros(T, H, D, dtype=F64)
+    S = torch.zeros(H, D, v.shape[2], dtype=F64)
+    out = torch.zeros(T, H, v.shape[2], dtype=F64)
     for t in range(T):
         own = k[t][:, :, None] * v[t][:, None, :]
         out[t] = ((S + bonus[:, :, None] * own) * r[t][:, :, None]).sum(1)
