@@ -5,6 +5,7 @@
 #include <math.h>
 
 #include "common.h"
+#include "activations.h"
 
 __device__ inline float l_sigmoid(float v) { return 1.0f / (1.0f + expf(-v)); }
 
@@ -153,6 +154,7 @@ extern "C" int tp_sigmoid_gate(const void* a, int dt, const float* proj, int pro
 // h[t] += y[t] / sqrt(mean(y[t]^2) + eps) * w; then, with w_next, the next sublayer's input
 // x[t] = h[t] / sqrt(mean(h[t]^2) + eps_next) * w_next as TO.  One block per row.
 // With gate rows, y stands for y[t, c] * sigmoid(gate.rows[t, gate.col0 + c] + gate.bias[c]).  Not normed: h[t] += y[t] * w.
+// blocked: the rows x leave as [width / 8, n, 8], what products of a few rows read best.
 struct InputGate {
   const float* rows;   // float32 [n, stride], or nullptr: no gate
   const float* bias;   // [width], or nullptr
@@ -164,7 +166,7 @@ template <typename TO>
 __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ h, const float* __restrict__ y,
                                                        const float* __restrict__ w, float eps,
                                                        const float* __restrict__ w_next, float eps_next,
-                                                       TO* __restrict__ x, int width, InputGate gate, int normed) {
+                                                       TO* __restrict__ x, int width, InputGate gate, int normed, int blocked) {
   __shared__ float scratch[32];
   const size_t base = (size_t)blockIdx.x * width;
   const float* gr = gate.rows != nullptr ? gate.rows + (size_t)blockIdx.x * gate.stride + gate.col0 : nullptr;
@@ -192,7 +194,8 @@ __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ h, co
   ss2 = block_sum(ss2, scratch);
   const float rstd2 = 1.0f / sqrtf(ss2 / (float)width + eps_next);
   // (each thread reads back what it wrote itself)
-  for (int c = threadIdx.x; c < width; c += blockDim.x) from_float(x + base + c, h[base + c] * rstd2 * w_next[c]);
+  for (int c = threadIdx.x; c < width; c += blockDim.x)
+    from_float(x + (blocked ? ((size_t)(c >> 3) * gridDim.x + blockIdx.x) * 8 + (c & 7) : base + c), h[base + c] * rstd2 * w_next[c]);
 }
 
 // The same with the row in registers: every value is read once, sixteen bytes a load, all loads of a pass in flight
@@ -202,7 +205,7 @@ template <typename TO, int NV, bool GATE>
 __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h, const float* __restrict__ y,
                                                            const float* __restrict__ w, float eps,
                                                            const float* __restrict__ w_next, float eps_next,
-                                                           TO* __restrict__ x, int width, InputGate gate, int normed) {
+                                                           TO* __restrict__ x, int width, InputGate gate, int normed, int blocked) {
   __shared__ float scratch[32];
   const size_t base = (size_t)blockIdx.x * width;
   const int w4 = width / 4;
@@ -277,26 +280,27 @@ __global__ __launch_bounds__(256) void norm_add_reg_kernel(float* __restrict__ h
 #pragma unroll
   for (int k = 0; k < NV; ++k) {
     const int c = k * 256 + threadIdx.x;
-    if (c < w4) from_float4(x + base + 4 * c, hv[k].x * rstd2 * wv[k].x, hv[k].y * rstd2 * wv[k].y, hv[k].z * rstd2 * wv[k].z, hv[k].w * rstd2 * wv[k].w);
+    if (c < w4) from_float4(x + (blocked ? ((size_t)(c >> 1) * gridDim.x + blockIdx.x) * 8 + (c & 1) * 4 : base + 4 * c), hv[k].x * rstd2 * wv[k].x, hv[k].y * rstd2 * wv[k].y, hv[k].z * rstd2 * wv[k].z, hv[k].w * rstd2 * wv[k].w);
   }
 }
 
 extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, const float* w_next, float eps_next, void* x,
                            int x_dt, int n, int width, const float* gate_rows, size_t gate_stride, int gate_col0,
-                           const float* gate_bias, int normed, hipStream_t s) {
+                           const float* gate_bias, int normed, int blocked, hipStream_t s) {
   TP_REQUIRE(n >= 0 && width > 0, "norm_add: bad sizes");
   TP_REQUIRE(gate_rows == nullptr || (gate_col0 >= 0 && gate_stride >= (size_t)gate_col0 + width), "norm_add: gate rows too short");
   const InputGate gate{gate_rows, gate_bias, gate_stride, gate_col0};
   TP_REQUIRE(w_next == nullptr || x != nullptr, "norm_add: no place for the next rows");
   if (n == 0) return 0;
   TP_REQUIRE(w_next == nullptr || x_dt == TP_F32 || x_dt == TP_BF16, "norm_add: unknown dtype %d", x_dt);
+  TP_REQUIRE(!blocked || width % 8 == 0, "norm_add: k-blocked rows need a width that is a multiple of eight");
   const bool aligned = ((uintptr_t)h % 16) == 0 && ((uintptr_t)y % 16) == 0 && ((uintptr_t)w % 16) == 0 && ((uintptr_t)w_next % 16) == 0 &&
                        ((uintptr_t)x % 16) == 0 &&
                        (gate_rows == nullptr || (((uintptr_t)gate_rows | (uintptr_t)gate_bias) % 16 == 0 && gate_stride % 4 == 0 && gate_col0 % 4 == 0));
   if (width % 4 == 0 && width >= 1024 && width <= 256 * 4 * 8 && aligned) {
     const bool bf = w_next != nullptr && x_dt == TP_BF16;
 #define NA1(TO, NV, G) \
-  hipLaunchKernelGGL((norm_add_reg_kernel<TO, NV, G>), dim3(n), dim3(256), 0, s, h, y, w, eps, w_next, eps_next, (TO*)x, width, gate, normed)
+  hipLaunchKernelGGL((norm_add_reg_kernel<TO, NV, G>), dim3(n), dim3(256), 0, s, h, y, w, eps, w_next, eps_next, (TO*)x, width, gate, normed, blocked)
 #define NA(NV)                                    \
   do {                                            \
     if (gate_rows != nullptr) {                   \
@@ -317,9 +321,9 @@ extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, 
   }
   const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
   if (w_next == nullptr || x_dt == TP_F32)
-    hipLaunchKernelGGL(norm_add_kernel<float>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (float*)x, width, gate, normed);
+    hipLaunchKernelGGL(norm_add_kernel<float>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (float*)x, width, gate, normed, blocked);
   else if (x_dt == TP_BF16)
-    hipLaunchKernelGGL(norm_add_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (bf16_t*)x, width, gate, normed);
+    hipLaunchKernelGGL(norm_add_kernel<bf16_t>, dim3(n), dim3(threads), 0, s, h, y, w, eps, w_next, eps_next, (bf16_t*)x, width, gate, normed, blocked);
   else
     TP_REQUIRE(false, "norm_add: unknown dtype %d", x_dt);
   TP_CHECK_LAUNCH("norm_add");
@@ -327,18 +331,7 @@ extern "C" int tp_norm_add(float* h, const float* y, const float* w, float eps, 
 }
 
 // ---- a plain activation -----------------------------------------------------------------------
-// kind 0: the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))); kind 1: SiLU; kind 2: the exact
-// GELU, 0.5 z (1 + erf(z / sqrt(2))); kind 3: the square of ReLU, max(z, 0)^2.
-__device__ inline float act_f(float z, int kind) {
-  if (kind == 0) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-  if (kind == 2) return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
-  if (kind == 3) {
-    const float r = fmaxf(z, 0.f);
-    return r * r;
-  }
-  return z * l_sigmoid(z);
-}
-
+// (the kinds: activations.h)
 // Rows of a wider float32 tensor: out[t, c] = act(in[t, col0 + c]) for c < width, times sigmoid(in[t, gate_col]) when
 // gate_col >= 0 (one gate a row: what a product behind it would be multiplied by, folded into its input).
 template <typename TO>
@@ -408,6 +401,29 @@ __global__ void activation4_kernel(const float* __restrict__ in, TO* __restrict_
   if (i >= total4) return;
   const float4 z = *(const float4*)(in + 4 * i);
   from_float4(out + 4 * i, act_f(z.x, kind), act_f(z.y, kind), act_f(z.z, kind), act_f(z.w, kind));
+}
+
+// float32 rows [m, width] -> [width / 8, m, 8]
+template <typename TO>
+__global__ void activation_blocked_kernel(const float* __restrict__ in, TO* __restrict__ out, int m, int width, int kind) {
+  const int i = blockIdx.x * blockDim.x + threadIdx.x, quads = width / 4;
+  if (i >= m * quads) return;
+  const int t = i / quads, c = i % quads * 4;
+  const float4 z = *(const float4*)(in + (size_t)t * width + c);
+  from_float4(out + ((size_t)(c >> 3) * m + t) * 8 + (c & 7), act_f(z.x, kind), act_f(z.y, kind), act_f(z.z, kind), act_f(z.w, kind));
+}
+
+extern "C" int tp_activation_blocked(const float* in, void* out, int out_dt, int m, int width, int kind, hipStream_t s) {
+  TP_REQUIRE(kind >= 0 && kind <= 3, "activation: unknown kind %d", kind);
+  TP_REQUIRE(m > 0 && width > 0 && width % 8 == 0 && (long)m * width < 0x7fffffffL && (((uintptr_t)in | (uintptr_t)out) & 15) == 0, "activation: bad rows");
+  TP_REQUIRE(out_dt == TP_F32 || out_dt == TP_BF16, "activation: unknown dtype %d", out_dt);
+  const dim3 grid((m * (width / 4) + 255) / 256);
+  if (out_dt == TP_F32)
+    hipLaunchKernelGGL(activation_blocked_kernel<float>, grid, dim3(256), 0, s, in, (float*)out, m, width, kind);
+  else
+    hipLaunchKernelGGL(activation_blocked_kernel<bf16_t>, grid, dim3(256), 0, s, in, (bf16_t*)out, m, width, kind);
+  TP_CHECK_LAUNCH("activation_blocked");
+  return 0;
 }
 
 extern "C" int tp_activation(const void* in, int in_dt, void* out, int out_dt, size_t total, int kind, hipStream_t s) {

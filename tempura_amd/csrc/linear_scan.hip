@@ -20,7 +20,7 @@ template <typename TO, int V>
 __global__ void token_shift_kernel(const float* __restrict__ x, const float* __restrict__ mu, float* __restrict__ state, size_t state_stride,
                                    size_t state_off, const int* __restrict__ cu_seqlens, const int* __restrict__ token_req,
                                    const int* __restrict__ state_slots, TO* __restrict__ out, size_t out_stride_mix, int width, int mixes,
-                                   int channel_blocks, int single) {
+                                   int channel_blocks, int single, int blocked) {
   const int t = blockIdx.x / channel_blocks;
   const int c = ((blockIdx.x % channel_blocks) * blockDim.x + threadIdx.x) * V;
   if (c >= width) return;
@@ -44,7 +44,7 @@ __global__ void token_shift_kernel(const float* __restrict__ x, const float* __r
   }
   for (int s = 0; s < mixes; ++s) {
     const float* m = mu + (size_t)s * width + c;
-    TO* o = out + (size_t)s * out_stride_mix + (size_t)t * width + c;
+    TO* o = out + (size_t)s * out_stride_mix + (blocked ? ((size_t)(c >> 3) * (gridDim.x / channel_blocks) + t) * 8 + (c & 7) : (size_t)t * width + c);
     if constexpr (V == 4) {
       const float4 mv = *(const float4*)m;
       from_float4(o, fmaf(gap[0], mv.x, cur[0]), fmaf(gap[1], mv.y, cur[1]), fmaf(gap[2], mv.z, cur[2]), fmaf(gap[3], mv.w, cur[3]));
@@ -63,13 +63,14 @@ __global__ void last_row_kernel(const float* __restrict__ x, float* __restrict__
   state[(size_t)state_slots[r] * state_stride + state_off + c] = x[(size_t)(end - 1) * width + c];
 }
 
-// single: every run of the step is one token long
+// single: every run of the step is one token long; blocked: every mix leaves as [width / 8, n, 8] (see decode_groups.hip)
 extern "C" int tp_token_shift(const float* x, const float* mu, float* state, size_t state_stride, size_t state_off, const int* cu_seqlens,
                               const int* token_req, const int* state_slots, void* out, int out_dt, int n, int n_req, int width, int mixes,
-                              int single, hipStream_t s) {
+                              int single, int blocked, hipStream_t s) {
   TP_REQUIRE(n >= 0 && n_req >= 0 && width > 0 && mixes > 0, "token_shift: bad sizes");
   TP_REQUIRE(state_stride >= state_off + (size_t)width, "token_shift: state rows too short");
   TP_REQUIRE(out_dt == TP_F32 || out_dt == TP_BF16, "token_shift: unknown dtype %d", out_dt);
+  TP_REQUIRE(!blocked || width % 8 == 0, "token_shift: k-blocked rows need a width that is a multiple of eight");
   TP_REQUIRE(!single || n <= n_req, "token_shift: %d tokens are not %d runs of one", n, n_req);
   if (n == 0 || n_req == 0) return 0;
   const bool four = width % 4 == 0 && (((uintptr_t)x | (uintptr_t)mu | (uintptr_t)out) & 15) == 0;
@@ -80,7 +81,7 @@ extern "C" int tp_token_shift(const float* x, const float* mu, float* state, siz
   const dim3 grid((unsigned)((long)n * cb));
 #define SHIFT(T, V)                                                                                                                        \
   hipLaunchKernelGGL((token_shift_kernel<T, V>), grid, dim3(threads), 0, s, x, mu, state, state_stride, state_off, cu_seqlens, token_req, \
-                     state_slots, (T*)out, (size_t)n * width, width, mixes, cb, single)
+                     state_slots, (T*)out, (size_t)n * width, width, mixes, cb, single, blocked)
   if (out_dt == TP_F32) {
     if (four) SHIFT(float, 4);
     else SHIFT(float, 1);

@@ -603,11 +603,15 @@ def linear_relu2(x: torch.Tensor, w, act_cols: int, blocked_out: bool = False):
     if _backend is not None:
         return _backend.linear_relu2(x, w, act_cols, blocked_out)
     wd, wl = _w_args(w)
+    shape, xl = tuple(x.shape), 0
+    if isinstance(x, KBlocked):
+        _need(x.rows <= 16 and tuple(x.data.shape) == (x.width // 8, x.rows, 8), "linear_relu2: malformed k-blocked rows")
+        x, xl = x.data, 1
     _dev_ok(x, wd)
-    _need(x.dim() == 2 and w.dim() == 2 and x.shape[1] == w.shape[1], f"linear_relu2: shapes {tuple(x.shape)} x {tuple(w.shape)}")
-    _need(x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and linear_relu2_ok(act_cols, x.shape[1], x.dtype)
+    _need(len(shape) == 2 and w.dim() == 2 and shape[1] == w.shape[1], f"linear_relu2: shapes {shape} x {tuple(w.shape)}")
+    _need(x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and linear_relu2_ok(act_cols, shape[1], x.dtype)
           and 0 < act_cols <= w.shape[0], "linear_relu2: needs bfloat16 operands, k % 64 == 0 and a multiple of 128 activated columns")
-    (m, k), n = x.shape, w.shape[0]
+    (m, k), n = shape, w.shape[0]
     blocked_out = blocked_out and 0 < m <= 16
     if blocked_out:
         out = KBlocked(torch.empty((act_cols // 8, m, 8), dtype=torch.bfloat16, device=x.device), m, act_cols)
@@ -616,7 +620,7 @@ def linear_relu2(x: torch.Tensor, w, act_cols: int, blocked_out: bool = False):
     side = torch.empty((m, n - act_cols), dtype=torch.float32, device=x.device)
     scratch, nscratch = _splitk_scratch(x, m, n)
     _call("tp_linear_fused", _ptr(x), _ptr(wd), _BF16, _ptr(out.data if blocked_out else out), _BF16, 3, m, n, k, 1, _ptr(scratch),
-          ctypes.c_size_t(nscratch), _ptr(None), 0, ctypes.c_float(0.0), _ptr(None), _ptr(None), _ptr(None), (2 if blocked_out else 0) | wl,
+          ctypes.c_size_t(nscratch), _ptr(None), 0, ctypes.c_float(0.0), _ptr(None), _ptr(None), _ptr(None), (2 if blocked_out else 0) | wl | xl,
           0, _ptr(None), ctypes.c_float(1.0), ctypes.c_float(0.0), ctypes.c_float(0.0), int(act_cols), _ptr(side), _stream(), tag=(m, n, k))
     return out, side
 
@@ -1477,10 +1481,11 @@ def head_linear(x: torch.Tensor, x_col0: int, x_head: int, w: torch.Tensor, out:
 
 def norm_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, next_weight: Optional[torch.Tensor] = None,
              next_eps: float = 0.0, out_dtype: Optional[torch.dtype] = None, gate: Optional[torch.Tensor] = None, gate_col0: int = 0,
-             gate_bias: Optional[torch.Tensor] = None, normed: bool = True) -> Optional[torch.Tensor]:
+             gate_bias: Optional[torch.Tensor] = None, normed: bool = True, blocked: bool = False):
     """h += y / sqrt(mean(y^2) + eps) * weight (not ``normed``: h += y * weight), per row, in place (float32 [n, width]).  With ``next_weight`` the
     rows of the new h normed with it (and ``next_eps``) come back as ``out_dtype``.  With ``gate`` (float32 rows [n,
-    wider]) y is first multiplied by sigmoid(gate[:, gate_col0 + c] + gate_bias[c])."""
+    wider]) y is first multiplied by sigmoid(gate[:, gate_col0 + c] + gate_bias[c]).  ``blocked``: the rows come back as
+    ``KBlocked`` (see ``few_rows_ok``)."""
     if _backend is not None:
         if gate is not None:
             return _backend.norm_add(h, y, weight, eps, next_weight, next_eps, out_dtype, gate, gate_col0, gate_bias)
@@ -1497,32 +1502,33 @@ def norm_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float,
     x = None
     if next_weight is not None:
         _need(next_weight.dtype == torch.float32 and next_weight.numel() == width and out_dtype is not None, "norm_add: bad next norm")
-        x = torch.empty((n, width), dtype=out_dtype, device=h.device)
+        x = torch.empty((width // 8, n, 8) if blocked else (n, width), dtype=out_dtype, device=h.device)
     _call("tp_norm_add", _ptr(h), _ptr(y), _ptr(weight), ctypes.c_float(eps), _ptr(next_weight), ctypes.c_float(next_eps), _ptr(x),
           _dtcode(out_dtype) if x is not None else _F32, n, width, _ptr(gate), ctypes.c_size_t(0 if gate is None else gate.shape[1]),
-          int(gate_col0), _ptr(gate_bias), int(normed), _stream())
-    return x
+          int(gate_col0), _ptr(gate_bias), int(normed), int(blocked), _stream())
+    return KBlocked(x, n, width) if blocked and x is not None else x
 
 
 def scale_add(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, next_weight: Optional[torch.Tensor] = None, next_eps: float = 0.0,
               out_dtype: Optional[torch.dtype] = None, gate: Optional[torch.Tensor] = None, gate_col0: int = 0,
-              gate_bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+              gate_bias: Optional[torch.Tensor] = None, blocked: bool = False):
     """``norm_add`` without the norm on y: h += y * weight, per row, in place (``weight`` a vector of scales), and with
     ``next_weight`` the rows of the new h normed with it come back."""
     if _backend is not None:
         return _backend.scale_add(h, y, weight, next_weight, next_eps, out_dtype, gate, gate_col0, gate_bias)
-    return norm_add(h, y, weight, 0.0, next_weight, next_eps, out_dtype, gate, gate_col0, gate_bias, normed=False)
+    return norm_add(h, y, weight, 0.0, next_weight, next_eps, out_dtype, gate, gate_col0, gate_bias, normed=False, blocked=blocked)
 
 
 ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "gelu_erf": 2, "relu2": 3}
 
 
 def activation(u: torch.Tensor, kind: str, out_dtype: torch.dtype, col0: int = 0, width: Optional[int] = None,
-               gate_col: Optional[int] = None) -> torch.Tensor:
+               gate_col: Optional[int] = None, blocked: bool = False):
     """Element by element: ``gelu_tanh`` (0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))), ``gelu_erf``
     (0.5 z (1 + erf(z / sqrt(2)))), ``relu2`` (max(z, 0)^2) or ``silu``, formed in float32, as ``out_dtype``.
     With ``width`` (``u`` float32 rows [n, wider]): the columns col0 .. col0 + width of every row, and with ``gate_col``
-    each row's results times the sigmoid of that column of the row."""
+    each row's results times the sigmoid of that column of the row.  ``blocked`` (whole float32 rows, see ``few_rows_ok``):
+    the result comes as ``KBlocked``."""
     _need(kind in ACTIVATIONS, f"activation: {kind!r} unknown (known: {sorted(ACTIVATIONS)})")
     if _backend is not None:
         if width is not None:
@@ -1537,6 +1543,12 @@ def activation(u: torch.Tensor, kind: str, out_dtype: torch.dtype, col0: int = 0
         _call("tp_activation_rows", _ptr(u), ctypes.c_size_t(u.shape[1]), int(col0), int(width), -1 if gate_col is None else int(gate_col),
               _ptr(out), _dtcode(out_dtype), u.shape[0], ACTIVATIONS[kind], _stream())
         return out
+    if blocked:
+        _need(u.dim() == 2 and u.dtype == torch.float32 and u.shape[1] % 8 == 0, "activation: k-blocked results need whole float32 rows")
+        m, n = u.shape
+        out = torch.empty((n // 8, m, 8), dtype=out_dtype, device=u.device)
+        _call("tp_activation_blocked", _ptr(u), _ptr(out), _dtcode(out_dtype), m, n, ACTIVATIONS[kind], _stream())
+        return KBlocked(out, m, n)
     out = torch.empty(u.shape, dtype=out_dtype, device=u.device)
     _call("tp_activation", _ptr(u), _dt(u), _ptr(out), _dtcode(out_dtype), ctypes.c_size_t(u.numel()), ACTIVATIONS[kind], _stream())
     return out
@@ -1906,11 +1918,13 @@ def mlstm_scan(proj: torch.Tensor, col0: int, i_bias: torch.Tensor, f_bias: torc
 # Operations of mixers around a linear recurrence: mixes of a row and the row before it, and the recurrence.
 
 def token_shift(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, state_off: int, cu_seqlens: torch.Tensor, token_req: torch.Tensor,
-                state_slots: torch.Tensor, num_requests: int, out_dtype: torch.dtype, max_run: Optional[int] = None):
+                state_slots: torch.Tensor, num_requests: int, out_dtype: torch.dtype, max_run: Optional[int] = None,
+                blocked: bool = False):
     """Mixes of float32 rows ``x`` [n, width] with the rows before them in their requests: for each of the ``mu`` [mixes,
     width] x + (x' - x) * mu, as ``out_dtype``; a list of tensors [n, width].  x' of a run's first token is what the request's
     state holds (``state`` float32 [slots, row], ``width`` numbers from ``state_off`` on); the run's last row is left there.
-    ``max_run``: the longest run of the step (None: unknown)."""
+    ``max_run``: the longest run of the step (None: unknown).  ``blocked``: one tensor [mixes, width / 8, n, 8] instead (what
+    ``group_linear`` takes)."""
     if _backend is not None:
         return _backend.token_shift(x, mu, state, state_off, cu_seqlens, token_req, state_slots, num_requests, out_dtype)
     _dev_ok(x, mu, state, cu_seqlens, token_req, state_slots)
@@ -1922,10 +1936,10 @@ def token_shift(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, state_of
     _i32(state_slots, num_requests, "state_slots")
     _i32(token_req, n, "token_req") if n else None
     mixes = mu.shape[0]
-    out = torch.empty((mixes, n, width), dtype=out_dtype, device=x.device)
+    out = torch.empty((mixes, width // 8, n, 8) if blocked else (mixes, n, width), dtype=out_dtype, device=x.device)
     _call("tp_token_shift", _ptr(x), _ptr(mu), _ptr(state), ctypes.c_size_t(state.shape[1]), ctypes.c_size_t(state_off), _ptr(cu_seqlens),
-          _ptr(token_req), _ptr(state_slots), _ptr(out), _dtcode(out_dtype), n, int(num_requests), width, mixes, int(max_run == 1), _stream())
-    return list(out.unbind(0))
+          _ptr(token_req), _ptr(state_slots), _ptr(out), _dtcode(out_dtype), n, int(num_requests), width, mixes, int(max_run == 1), int(blocked), _stream())
+    return out if blocked else list(out.unbind(0))
 
 
 #: runs longer than a piece are cut into pieces that run side by side; a piece has at least this many tokens
@@ -1975,4 +1989,68 @@ def linear_scan(q, k, v, decay: torch.Tensor, state: torch.Tensor, state_off: in
     _call("tp_linear_scan", at(q), q[0].shape[1], at(k), k[0].shape[1], at(v), v[0].shape[1], _ptr(decay), _ptr(bonus), ctypes.c_float(q_scale),
           _ptr(state), ctypes.c_size_t(state.shape[1]), ctypes.c_size_t(state_off), _ptr(cu_seqlens), _ptr(state_slots), _ptr(y), n,
           int(num_requests), int(heads), int(dim), int(vdim), max_run, piece, pieces, _ptr(scratch), _stream())
+    return y
+
+
+# ---------------------------------------------------------------------------------
+# Products of decode steps that come in groups.
+
+def few_rows_ok(m: int, width: int, dtype: torch.dtype) -> bool:
+    """Whether ``m`` rows of that width are few enough for the products that read them k-blocked."""
+    return _backend is None and allow_mfma and dtype == torch.bfloat16 and 0 < m <= 16 and width % 64 == 0
+
+
+def block_rows(x: torch.Tensor) -> KBlocked:
+    """bfloat16 rows [m, k] as ``KBlocked``."""
+    _dev_ok(x)
+    _need(x.dtype == torch.bfloat16 and x.dim() == 2 and x.shape[1] % 8 == 0, "block_rows: rows must be bfloat16 [m, a multiple of eight]")
+    m, k = x.shape
+    out = torch.empty((k // 8, m, 8), dtype=x.dtype, device=x.device)
+    _call("tp_block_rows", _ptr(x), _ptr(out), m, k, _stream())
+    return KBlocked(out, m, k)
+
+
+def group_linear_ok(m: int, w) -> bool:
+    """Whether ``group_linear`` takes ``m`` rows and the stacked weight."""
+    return isinstance(w, TiledWeight) and few_rows_ok(m, w.shape[1], w.dtype)
+
+
+def group_linear(x: torch.Tensor, w, ends) -> torch.Tensor:
+    """Several products of at most 16 bfloat16 rows in one launch: ``x`` [groups, k / 8, m, 8] (k-blocked), ``w`` the tiled
+    weights [n, k] of all groups stacked, group g's rows ending at ``ends[g]`` (multiples of 16).  Float32 [m, n]."""
+    _need(isinstance(w, TiledWeight) and x.dim() == 4 and x.dtype == torch.bfloat16 and x.shape[3] == 8, "group_linear: k-blocked rows and tiled weights")
+    groups, k8, m, _ = x.shape
+    n, k = w.shape
+    _dev_ok(x, w.data)
+    _need(k == 8 * k8 and len(ends) == groups and ends[-1] == n, "group_linear: groups and weight disagree")
+    out = torch.empty((m, n), dtype=torch.float32, device=x.device)
+    _call("tp_group_linear", _ptr(x), _ptr(w.data), _ptr(out), (ctypes.c_int * groups)(*ends), groups, m, n, k, _stream(), tag=(m, n, k))
+    return out
+
+
+def moe_few_ok(m: int, experts: int, ff: int, w_up, w_down) -> bool:
+    """Whether ``moe_few`` takes ``m`` rows and these stacked experts."""
+    return (isinstance(w_up, TiledWeight) and isinstance(w_down, TiledWeight) and experts <= 512 and ff % 64 == 0
+            and few_rows_ok(m, w_up.shape[1], w_up.dtype))
+
+
+def moe_few(x: KBlocked, w_up, w_down, dense: torch.Tensor, ff: int, activation: Optional[str], y: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The routed experts of at most 16 rows: y (+)= sum_e down_e(f(up_e x) * dense[:, e]), skipping the weights of experts
+    whose column of ``dense`` (float32 [m, experts]) is zero.  ``w_up``: the experts' tiled up weights stacked
+    ([experts * ff, k]; ``activation`` None: gate and up rows interleaved by eights, [2 experts * ff, k], f = silu(gate) * up);
+    ``w_down``: their tiled [n, ff] one behind the other, as a ``TiledWeight`` of [experts * n, ff].  ``y`` float32 [m, n] or None."""
+    m, k = x.shape
+    experts = dense.shape[1]
+    n = w_down.shape[0] // experts
+    _dev_ok(x.data, w_up.data, w_down.data, dense, y)
+    rows = ff if activation is not None else 2 * ff
+    _need(tuple(w_up.shape) == (experts * rows, k) and tuple(w_down.shape) == (experts * n, ff), "moe_few: weights disagree with the sizes")
+    _need(dense.dtype == torch.float32 and tuple(dense.shape) == (m, experts), "moe_few: dense must be float32 [m, experts]")
+    _need(y is None or (y.dtype == torch.float32 and tuple(y.shape) == (m, n)), "moe_few: y must be float32 [m, n]")
+    acc = y is not None
+    if not acc:
+        y = torch.empty((m, n), dtype=torch.float32, device=dense.device)
+    a = torch.empty((experts * ff // 8, m, 8), dtype=torch.bfloat16, device=dense.device)
+    _call("tp_moe_few", _ptr(x.data), _ptr(w_up.data), _ptr(w_down.data), _ptr(dense), _ptr(a), _ptr(y), m, experts, int(ff), k, n,
+          int(activation is None), 0 if activation is None else ACTIVATIONS[activation], int(acc), _stream(), tag=(m, experts, ff, k))
     return y

@@ -80,6 +80,8 @@ class Part:
     graph_safe = False
     #: the type in which the part reads its normed rows (None: the compute dtype), for blocks that ask
     input_dtype: Optional[torch.dtype] = None
+    #: True: in a step of a few single tokens the rows may come k-blocked (``ops.KBlocked``), for blocks that ask
+    takes_blocked_rows = False
 
     def __init__(self, spec: PartSpec, hidden_size: int, dtype: torch.dtype, device):
         self.spec = spec

@@ -301,9 +301,10 @@ class SandwichBlock(ArrangedBlock):
         return getattr(part, "input_dtype", None) or self.dtype
 
     def _rms(self, norm, part):
-        """(weight, eps, type of the rows) of an RMS norm in front of ``part`` that the closing kernel can apply, else None."""
+        """(weight, eps, type of the rows, whether a few rows may come k-blocked) of an RMS norm in front of ``part`` that the
+        closing kernel can apply, else None."""
         if type(norm).__name__ == "RMSNorm" and getattr(norm, "groups", 1) == 1:
-            return norm.weight, norm.eps, self._input_dtype(part)
+            return norm.weight, norm.eps, self._input_dtype(part), bool(getattr(part, "takes_blocked_rows", False))
         return None
 
     def _normed(self, h, norm, part):
@@ -336,19 +337,22 @@ class SandwichBlock(ArrangedBlock):
             elif post is not None:
                 self.closing[name] = post.weight if scale is None else (post.weight.double() * scale.weight.double()).to(torch.float32)
 
-    def _close(self, h, x, result, name, opening):
+    def _close(self, h, x, result, name, opening, ctx=None):
         """Gate and norm the result of sublayer ``name`` (``x`` its input), add it into the stream; with ``opening``
-        (weight, eps, type) also return the stream normed for the next sublayer."""
+        (weight, eps, type, k-blocked) also return the stream normed for the next sublayer."""
         gate, weight, post = getattr(self, name + "_gate"), self.closing[name], self._post(name)
-        after = (None, 0.0, None) if opening is None else opening
+        after = (None, 0.0, None) if opening is None else opening[:3]
+        more = {}
+        if opening is not None and opening[3] and getattr(ctx, "max_q_len", 0) == 1 and ops.few_rows_ok(h.shape[0], h.shape[1], opening[2]):
+            more["blocked"] = True
         if post is None:
             y, rows, col0, bias = (result, None, 0, None) if gate is None else gate.split(x, result) + (gate.bias,)
-            return ops.scale_add(h, y, weight, *after, gate=rows, gate_col0=col0, gate_bias=bias)
+            return ops.scale_add(h, y, weight, *after, gate=rows, gate_col0=col0, gate_bias=bias, **more)
         eps = post.eps
         if gate is not None:
             y, rows, col0 = gate.split(x, result)
-            return ops.norm_add(h, y, weight, eps, *after, gate=rows, gate_col0=col0, gate_bias=gate.bias)
-        return ops.norm_add(h, result, weight, eps, *after)
+            return ops.norm_add(h, y, weight, eps, *after, gate=rows, gate_col0=col0, gate_bias=gate.bias, **more)
+        return ops.norm_add(h, result, weight, eps, *after, **more)
 
     def forward(self, h, ctx, cache, x=None, next_norm=None):
         n = h.shape[0]
@@ -357,12 +361,12 @@ class SandwichBlock(ArrangedBlock):
         y = self._run(self.mixer, x, ctx, cache, n, h.device)
         after = next_norm if isinstance(next_norm, tuple) else None
         if self.ffn is None:
-            return self._close(h, x, y, "mixer", after)
-        x2 = self._close(h, x, y, "mixer", self._rms(self.ffn_norm, self.ffn))
+            return self._close(h, x, y, "mixer", after, ctx)
+        x2 = self._close(h, x, y, "mixer", self._rms(self.ffn_norm, self.ffn), ctx)
         if x2 is None:
             x2 = self._normed(h, self.ffn_norm, self.ffn)
         y2 = self._run(self.ffn, x2, ctx, None, n, h.device)
-        return self._close(h, x2, y2, "ffn", after)
+        return self._close(h, x2, y2, "ffn", after, ctx)
 
 
 register_part("block", "sandwich", SandwichBlock)

@@ -111,6 +111,7 @@ class DenseMLP(FeedForward):
     (sizes ``ops.linear_relu2_ok``), else as a kernel of its own."""
     graph_safe = True
     takes_side_rows = True     # (behind the up product's own columns)
+    takes_blocked_rows = True
     returns_output = True      # with ``residual`` None the output comes back instead of being added
 
     def __init__(self, spec, hidden_size, dtype, device):
@@ -146,7 +147,9 @@ class DenseMLP(FeedForward):
         if self.side_rows is not None:
             a = ops.activation(u, self.activation, self.dtype, 0, self.intermediate_size)
             return ops.linear(a, self.w_down, torch.float32, residual=residual), (u, self.intermediate_size)
-        a = ops.activation(u, self.activation, self.dtype)
+        # (a few rows go to the down product k-blocked: it reads them straight from global memory)
+        few = {"blocked": True} if ops.few_rows_ok(u.shape[0], u.shape[1], self.dtype) else {}
+        a = ops.activation(u, self.activation, self.dtype, **few)
         return ops.linear(a, self.w_down, torch.float32, residual=residual)
 
 
@@ -158,7 +161,9 @@ class RoutedExperts(FeedForward):
     ``keep``), only looks at the experts of the ``keep`` groups whose best choice score is largest; the weights are
     the chosen experts' s, not renormalised.  The output is the weighted sum of the chosen experts' outputs.
 
-    Two ways through the experts.  A step of single tokens (decoding; it may be captured): ONE gate/up product
+    Three ways through the experts.  A step of at most 16 single tokens in bfloat16 (sizes ``ops.moe_few_ok``): one product
+    over the up weights of all experts and one over their down weights, each leaving out the weights of experts that no
+    row has chosen (``ops.moe_few``).  Any other step of single tokens (decoding; it may be captured): ONE gate/up product
     over the stacked weights of all experts, then every expert's activations times the row's weight for it (zero
     where the expert was not chosen; ``ops.moe_spread``), then the experts' down products one after the other into
     one sum, ascending; nothing of the batch is read on the host, and at a few rows with several experts each
@@ -166,7 +171,7 @@ class RoutedExperts(FeedForward):
     chosen (token, expert) pairs are brought into the order of the experts, the host reads how many rows each expert
     has (the one wait of the layer), every expert with rows is one pair of products over its rows, and a token's
     sum adds its experts' rows in the order of its choice.  Either way a row's result does not depend on what else
-    is in the batch; the two ways differ in rounding only.  Tensor roles: ``router``,
+    is in the batch; the ways differ in rounding only.  Tensor roles: ``router``,
     ``correction``, and ``gate`` / ``up`` / ``down`` as name patterns with ``{}`` for the expert's number.
 
     Parameters of the router beyond that: ``score`` (``"softmax"`` or ``"sigmoid"``: s = sigmoid(logit), each expert by
@@ -279,6 +284,13 @@ class RoutedExperts(FeedForward):
         # the gate/up weights of all experts are one matrix (decoding runs them as one product); an expert's own
         # are rows of it, without a copy (tiled weights are cut at multiples of sixteen rows)
         rows = (2 if gated else 1) * self.intermediate_size
+        # (the tiled down weights lie one behind the other)
+        self.w2_all = None
+        if all(isinstance(t, ops.TiledWeight) for t in self.w2):
+            n_out, ff = self.w2[0].shape
+            data = torch.stack([t.data for t in self.w2])
+            self.w2_all = ops.TiledWeight(data.view((-1,) + tuple(data.shape[2:])), self.experts * n_out, ff)
+            self.w2 = [self.w2_all.rows(n * n_out, (n + 1) * n_out) for n in range(self.experts)]
         stacked = torch.cat(stack, dim=0).contiguous()
         self.w13_all = ops.tile_weight(stacked) if rows % 16 == 0 else stacked
         self.w13 = [ops.weight_rows(self.w13_all, n * rows, (n + 1) * rows) for n in range(self.experts)]
@@ -310,6 +322,13 @@ class RoutedExperts(FeedForward):
         self._add_shared(x, residual if residual is not None else y)
         return y
 
+    @property
+    def takes_blocked_rows(self):
+        return self._few_ok(1)
+
+    def _few_ok(self, m):
+        return (self.fused or self.expert_kind == "plain") and ops.moe_few_ok(m, self.experts, self.intermediate_size, self.w13_all, self.w2_all)
+
     def _routed(self, x, ctx, residual=None):
         logits = ops.linear(x, self.w_router, torch.float32)
         if self.router_bias is not None:
@@ -322,6 +341,11 @@ class RoutedExperts(FeedForward):
             dense, ids, weights = ops.moe_route(logits, self.correction, self.experts, self.top, self.groups, self.keep, score=self.score,
                                                 group_best=self.group_best, normalize=self.normalize, sum_eps=self.sum_eps,
                                                 scale=self.weight_scale)
+        if getattr(ctx, "max_q_len", 1) <= 1 and self._few_ok(x.shape[0]):
+            rows = x if isinstance(x, ops.KBlocked) else ops.block_rows(x)
+            y = ops.moe_few(rows, self.w13_all, self.w2_all, dense, self.intermediate_size,
+                            self.activation if self.expert_kind == "plain" else None, residual)
+            return y if residual is None else None
         if getattr(ctx, "max_q_len", 1) <= 1:
             if self.fused_relu2:
                 a = ops.linear_relu2(x, self.w13_all, self.experts * self.intermediate_size)[0]

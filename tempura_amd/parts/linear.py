@@ -63,20 +63,30 @@ class WkvMixer(Mixer):
         self.w2_t = w2.t().contiguous()      # [rank, columns]: lanes read neighbours
         self.w0, self.norm_w = f32("w0"), f32("norm")
         self.bonus = f32("u").reshape(-1)
-        # one weight per mix, in the order of the mixes
-        self.w_in = [ops.tile_weight(pad_rows(self._to_device(get(w[name])), 16)) for name in ("r", "k", "v", "gate")]
-        self.w_w1 = ops.tile_weight(pad_rows(self._to_device(w1), 16))
+        # one weight per mix, in the order of the mixes: rows of one stacked weight, which a step of a few rows takes in one launch
+        rows = [pad_rows(self._to_device(t), 16) for t in [get(w[name]) for name in ("r", "k", "v", "gate")] + [w1]]
+        self.ends, self.cols = [], []
+        for t in rows:
+            self.cols.append(self.ends[-1] if self.ends else 0)
+            self.ends.append(self.cols[-1] + t.shape[0])
+        self.w_all = ops.tile_weight(torch.cat(rows, dim=0).contiguous())
+        self.w_in = [ops.weight_rows(self.w_all, lo, hi) for lo, hi in zip(self.cols, self.ends)]
         self.w_out = ops.tile_weight(self._to_device(get(w["o"])))
 
     def forward(self, x, ctx, cache, residual=None):
+        few = {"blocked": True} if ctx.max_q_len == 1 and ops.group_linear_ok(x.shape[0], self.w_all) else {}
         mixes = ops.token_shift(x, self.mu, cache.state, self.row_off, ctx.cu_seqlens, ctx.token_req, ctx.state_slots,
-                                ctx.num_requests, self.dtype, max_run=ctx.max_q_len)
-        r, k, v, g = (ops.linear(m, wt, torch.float32) for m, wt in zip(mixes, self.w_in))
-        decay = ops.lowrank_up(ops.linear(mixes[4], self.w_w1, torch.float32), 0, self.w2_t, "exp_exp", bias=self.w0, in_act="tanh")
-        o = ops.linear_scan((r, 0), (k, 0), (v, 0), decay, cache.state, 0, ctx.cu_seqlens, ctx.state_slots, ctx.num_requests,
+                                ctx.num_requests, self.dtype, max_run=ctx.max_q_len, **few)
+        if few:
+            proj = ops.group_linear(mixes, self.w_all, self.ends)
+            r, k, v, (g, g_col), (w, w_col) = ((proj, col) for col in self.cols)
+        else:
+            r, k, v, (g, g_col), (w, w_col) = ((ops.linear(m, wt, torch.float32), 0) for m, wt in zip(mixes, self.w_in))
+        decay = ops.lowrank_up(w, w_col, self.w2_t, "exp_exp", bias=self.w0, in_act="tanh")
+        o = ops.linear_scan(r, k, v, decay, cache.state, 0, ctx.cu_seqlens, ctx.state_slots, ctx.num_requests,
                             self.num_heads, self.head_dim, self.head_dim, bonus=self.bonus, max_run=ctx.max_q_len)
         act = torch.empty((o.shape[0], self.inner), dtype=self.dtype, device=o.device)
-        ops.head_norm_gate(o, self.norm_w, None, self.norm_eps, 1.0, self.num_heads, act, 0, gate_rows=g, gate_act="silu")
+        ops.head_norm_gate(o, self.norm_w, None, self.norm_eps, 1.0, self.num_heads, act, 0, gate_rows=g, gate_col0=g_col, gate_act="silu")
         return ops.linear(act, self.w_out, torch.float32, residual=residual)
 
 

@@ -18,6 +18,7 @@ from .base import Mixer, StateSpec, build_part, pad_rows, part_class, register_p
 class ParallelMixer(Mixer):
     graph_safe = True
     returns_output = True      # with ``residual`` None the output comes back instead of being added
+    takes_blocked_rows = True
 
     def __init__(self, spec, hidden_size, dtype, device):
         super().__init__(spec, hidden_size, dtype, device)

@@ -260,6 +260,91 @@ def test_rows_into_queries_and_cache_with_a_norm_per_head(H, G, D, E, rot, pad, 
             assert float(got[..., D:].abs().max()) == 0.0
 
 
+@pytest.mark.parametrize("m", [1, 3, 8, 16])
+@pytest.mark.parametrize("k,sizes", [(64, (16, 32, 16)), (128, (48,)), (256, (16, 16, 32, 64, 16)), (1088, (64, 128, 16, 16)), (4096, (256, 256, 64)),
+                                     (192, (16,) * 8)])
+def test_products_in_groups(m, k, sizes):
+    """Every group's rows times its own weight, in one launch; a row's result does not depend on the other rows."""
+    ops = _ops()
+    g = torch.Generator().manual_seed(m * 10 + k)
+    n = sum(sizes)
+    w = (torch.randn(n, k, generator=g) * k ** -0.5).to(torch.bfloat16).to(DEV)
+    x = torch.randn(len(sizes), m, k, generator=g).to(torch.bfloat16).to(DEV)
+    blocked = x.reshape(len(sizes), m, k // 8, 8).transpose(1, 2).contiguous()
+    ends = torch.tensor(sizes).cumsum(0).tolist()
+    tiled = ops.tile_weight(w)
+    assert ops.group_linear_ok(m, tiled)
+    got = ops.group_linear(blocked, tiled, ends)
+    want = torch.cat([x[i].float() @ w[e - c: e].float().T for i, (c, e) in enumerate(zip(sizes, ends))], dim=1)
+    _close(got, want, 2e-5)
+    alone = ops.group_linear(blocked[:, :, :1].contiguous(), tiled, ends)
+    assert torch.equal(alone, got[:1])
+
+
+@pytest.mark.parametrize("m", [1, 2, 8, 16])
+@pytest.mark.parametrize("E,top,ff,k,n", [(4, 1, 64, 64, 32), (8, 2, 128, 128, 48), (16, 3, 192, 64, 64), (100, 4, 64, 128, 16), (3, 3, 640, 256, 128), (8, 2, 1088, 512, 256),
+                                          (1, 1, 64, 64, 16)])
+@pytest.mark.parametrize("activation", ["relu2", "gelu_erf", "gelu_tanh", "silu", None])
+def test_routed_experts_of_a_few_rows(m, E, top, ff, k, n, activation):
+    """Ungated and gated experts, some used by no row, into a new tensor and added to another; a row's result has the
+    same bits alone and beside rows that use other experts."""
+    ops = _ops()
+    g = torch.Generator().manual_seed(E * 100 + m + ff)
+    bf = lambda *s, std=1.0: (torch.randn(*s, generator=g) * std).to(torch.bfloat16).to(DEV)
+    up, down = bf(E, ff, k, std=k ** -0.5), bf(E, n, ff, std=ff ** -0.5)
+    gate = bf(E, ff, k, std=k ** -0.5)
+    x = bf(m, k)
+    dense = torch.zeros(m, E)
+    for t in range(m):
+        dense[t, torch.randperm(E, generator=g)[:top]] = torch.rand(top, generator=g) + 0.1
+    dense = dense.to(DEV)
+    rows = up if activation is not None else torch.stack([ops.interleave_gate_up(gate[e], up[e]) for e in range(E)])
+    w_up = ops.tile_weight(rows.reshape(-1, k).contiguous())
+    w_down = ops.tile_weight(down.reshape(-1, ff).contiguous())
+    assert ops.moe_few_ok(m, E, ff, w_up, w_down)
+    xd, want = x.double(), torch.zeros(m, n, dtype=torch.float64, device=DEV)
+    for e in range(E):
+        u = xd @ up[e].double().T
+        a = u * torch.nn.functional.silu(xd @ gate[e].double().T) if activation is None else emu.activation(u.cpu(), activation, torch.float64).to(DEV)
+        want += ((a * dense[:, e:e + 1].double()).to(torch.bfloat16).double()) @ down[e].double().T
+    got = ops.moe_few(ops.block_rows(x), w_up, w_down, dense, ff, activation)
+    _close(got, want, 6e-3)
+    y = torch.randn(m, n, generator=g).to(DEV)
+    more = ops.moe_few(ops.block_rows(x), w_up, w_down, dense, ff, activation, y.clone())
+    _close(more, want + y.double(), 6e-3)
+    alone = ops.moe_few(ops.block_rows(x[-1:].contiguous()), w_up, w_down, dense[-1:].contiguous(), ff, activation)
+    assert torch.equal(alone, got[-1:])
+
+
+@pytest.mark.parametrize("m", [1, 7, 16])
+def test_rows_that_leave_k_blocked(m):
+    """The closing kernel, the mixes, activations and the up product with the squared ReLU: k-blocked rows hold the bits of
+    the plain ones, in and out."""
+    ops = _ops()
+    g = torch.Generator().manual_seed(m)
+    for width in (64, 128, 1024, 4096):
+        h, y = torch.randn(m, width, generator=g).to(DEV), torch.randn(m, width, generator=g).to(DEV)
+        w, nw = torch.rand(width, generator=g).to(DEV), torch.rand(width, generator=g).to(DEV)
+        for op in (lambda h, **kw: ops.scale_add(h, y, w, nw, 1e-5, torch.bfloat16, **kw), lambda h, **kw: ops.norm_add(h, y, w, 1e-5, nw, 1e-5, torch.bfloat16, **kw)):
+            plain_rows, blocked = op(h.clone()), op(h.clone(), blocked=True)
+            assert isinstance(blocked, ops.KBlocked) and torch.equal(blocked.row_major(), plain_rows)
+        assert torch.equal(ops.block_rows(plain_rows).row_major(), plain_rows)
+        for kind in ("gelu_erf", "relu2"):
+            assert torch.equal(ops.activation(h, kind, torch.bfloat16, blocked=True).row_major(), ops.activation(h, kind, torch.bfloat16))
+        wt = ops.tile_weight((torch.randn(256, width, generator=g) * width ** -0.5).to(torch.bfloat16).to(DEV))
+        a, side = ops.linear_relu2(plain_rows, wt, 128)
+        b, side2 = ops.linear_relu2(blocked, wt, 128)
+        _close(b, a.float(), 8e-3)
+        _close(side2, side, 2e-5)
+        cu, tr = _dev(*_batch([1] * m))
+        slots = torch.arange(m, dtype=torch.int32, device=DEV)
+        mu, state = torch.rand(5, width, generator=g).to(DEV), torch.randn(m, width, generator=g).to(DEV)
+        shift = lambda **kw: ops.token_shift(h, mu, state.clone(), 0, cu, tr, slots, m, torch.bfloat16, 1, **kw)
+        rows, stacked = shift(), shift(blocked=True)
+        for i in range(5):
+            assert torch.equal(ops.KBlocked(stacked[i], m, width).row_major(), rows[i])
+
+
 def test_sizes_the_kernels_do_not_take_are_refused():
     ops = _ops()
     z = lambda *s: torch.zeros(*s, device=DEV)
@@ -274,6 +359,14 @@ def test_sizes_the_kernels_do_not_take_are_refused():
         ops.token_shift(z(2, 8), z(5, 8), z(1, 8), 0, i32(0, 2), i32(0, 0), i32(0), 1, torch.float32, 1)
     with pytest.raises(ops.KernelError, match="q norm must be"):
         ops.qkv_rows(z(1, 48), i32(0), i32(0), 1, 1, 16, 16, z(1, 1, 16, 16), z(1, 1, 16, 16), norms=(z(8), z(8)), norm_over="head")
+    w = ops.tile_weight(torch.zeros(32, 64, dtype=torch.bfloat16, device=DEV))
+    with pytest.raises(ops.KernelError, match="disagree"):
+        ops.group_linear(torch.zeros(2, 8, 1, 8, dtype=torch.bfloat16, device=DEV), w, [16, 48])
+    with pytest.raises(ops.KernelError, match="group borders"):
+        ops.group_linear(torch.zeros(2, 8, 1, 8, dtype=torch.bfloat16, device=DEV), w, [8, 32])
+    assert not ops.group_linear_ok(17, w)
+    with pytest.raises(ops.KernelError, match="disagree"):
+        ops.moe_few(ops.block_rows(torch.zeros(1, 64, dtype=torch.bfloat16, device=DEV)), w, w, z(1, 2), 64, "relu2")
     with pytest.raises(ops.KernelError, match="decay biases"):
         ops.lowrank_up(z(1, 4), 0, z(4, 8), "exp_exp")
 
