@@ -98,7 +98,7 @@ extern "C" int tp_token_shift(const float* x, const float* mu, float* state, siz
 }
 
 // ---- the recurrence ---------------------------------------------------------------------------
-// A block owns one request (or one piece of its run), one head and CB = TP * 256 / KS value columns; a thread holds PER
+// A block owns one request (or one piece of its run), one head and CB = WAVES * TP * 64 / KS value columns; a thread holds PER
 // consecutive key channels of TP neighbouring columns in registers, and the KS neighbouring lanes that share those columns
 // split the key channels among them (their partial read-outs meet by row permutes).  Several columns a thread share
 // what a token's q, k and w cost in LDS reads.  Tokens are taken TC at a time through LDS (rows padded to KS * PER channels
@@ -108,14 +108,16 @@ extern "C" int tp_token_shift(const float* x, const float* mu, float* state, siz
 // With the bonus the read-out of column j is sum_i q_i S_ij + (sum_i q_i u_i k_i) v_j: the second sum is the same for all
 // columns, so a lane adds its share of it times v_j to its partial read-out.
 //
-// Long runs are cut into pieces of `piece` tokens that run side by side.  Three launches:
-//   SCAN_LOCAL   every piece from a zero state: its end state and, per key channel, the product of its decays, to scratch
-//                (a run of one piece runs as in SCAN_DIRECT and is left out of the other two);
+// Long runs (keys of at most 128) are cut into pieces of `piece` tokens that run side by side.  Three launches:
+//   ends         every piece's end state from a zero state and, per key channel, the product of its decays, to scratch.  The end
+//                state is sum_j (k_j times the decays of the piece's tokens behind j) v_j^T: a float32 product on the matrix
+//                cores, the tokens walked backwards so that every factor is a product of decays (nothing is divided);
 //   carry        per state entry, piece by piece: the state a piece starts from is decay(piece before) * (the state the piece
 //                before started from) + (its end state from zero); what the last piece leaves is the request's state;
-//   SCAN_OUTPUT  every piece again from the state it starts from, now writing o.
+//   SCAN_PIECES  every piece from the state it starts from, writing o (a run of one piece runs as in SCAN_DIRECT and is left
+//                out of the other two).
 // Short runs take SCAN_DIRECT: one launch, from the request's state to its new state.
-enum { SCAN_DIRECT = 0, SCAN_LOCAL = 1, SCAN_OUTPUT = 2 };
+enum { SCAN_DIRECT = 0, SCAN_PIECES = 1 };
 
 struct LinearScan {
   const float *q, *k, *v;      // first column of each, rows of their own strides
@@ -134,11 +136,12 @@ struct LinearScan {
   float* piece_decay;          // [pieces, heads, dim]
 };
 
-template <int PER, int KS, int TP, bool BONUS>
-__global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
-  constexpr int DP = PER * KS, CW = TP_WAVE / KS * TP, CB = 4 * CW;
+template <int PER, int KS, int TP, int WAVES, bool BONUS>
+__global__ __launch_bounds__(WAVES * 64) void linear_scan_kernel(LinearScan a) {
+  constexpr int THREADS = WAVES * 64;
+  constexpr int DP = PER * KS, CW = TP_WAVE / KS * TP, CB = WAVES * CW;
   constexpr int TC = DP <= 128 ? 16 : 2048 / DP;
-  constexpr int NI = (TC * DP + 255) / 256, NV = (TC * CB + 255) / 256;
+  constexpr int NI = (TC * DP + THREADS - 1) / THREADS, NV = (TC * CB + THREADS - 1) / THREADS;
   __shared__ __attribute__((aligned(16))) float qs[TC * DP];
   __shared__ __attribute__((aligned(16))) float ks_[TC * DP];
   __shared__ __attribute__((aligned(16))) float ws[TC * DP];
@@ -150,11 +153,8 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
   if (run_len <= 0) return;
   int mode = a.mode;
   if (mode != SCAN_DIRECT) {
-    if (run_len <= a.piece) {
-      if (mode == SCAN_OUTPUT) return;
-      mode = SCAN_DIRECT;
-    }
     if ((long)pc * a.piece >= run_len) return;
+    if (run_len <= a.piece) mode = SCAN_DIRECT;
   }
   const int start = run0 + (mode == SCAN_DIRECT ? 0 : pc * a.piece);
   const int len = mode == SCAN_DIRECT ? run_len : min(a.piece, run_len - pc * a.piece);
@@ -169,7 +169,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
   float S[TP][PER];
 #pragma unroll
   for (int j = 0; j < TP; ++j) {
-    const bool have = mode != SCAN_LOCAL && j0 + j < a.vdim;
+    const bool have = j0 + j < a.vdim;
     const float* col = S_mem + (size_t)(have ? j0 + j : 0) * a.dim;
 #pragma unroll
     for (int e4 = 0; e4 < PER / 4; ++e4) {
@@ -183,12 +183,11 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
       }
     }
   }
-  float u[PER], W[PER];
+  float u[PER];
 #pragma unroll
   for (int e = 0; e < PER; ++e) {
     const int i = ks * PER + e;
     u[e] = (BONUS && i < a.dim) ? a.bonus[(size_t)h * a.dim + i] : 0.f;
-    W[e] = 1.f;
   }
   const size_t hd = (size_t)a.heads * a.dim, out_width = (size_t)a.heads * a.vdim;
   const float *q0 = a.q + (size_t)h * a.dim, *k0 = a.k + (size_t)h * a.dim, *v0 = a.v + (size_t)h * a.vdim, *w0 = a.decay + (size_t)h * a.dim;
@@ -197,17 +196,17 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
   auto fetch = [&](int t0) {
 #pragma unroll
     for (int it = 0; it < NI; ++it) {
-      const int idx = it * 256 + tid;
+      const int idx = it * THREADS + tid;
       const int t = idx / DP, i = idx % DP;
       const bool in = idx < TC * DP && t0 + t < len && i < a.dim;
       const size_t row = (size_t)(start + t0 + t);
-      fq[it] = in && mode != SCAN_LOCAL ? q0[row * a.q_stride + i] * a.q_scale : 0.f;
+      fq[it] = in ? q0[row * a.q_stride + i] * a.q_scale : 0.f;
       fk[it] = in ? k0[row * a.k_stride + i] : 0.f;
       fw[it] = in ? w0[row * hd + i] : 1.f;
     }
 #pragma unroll
     for (int it = 0; it < NV; ++it) {
-      const int idx = it * 256 + tid;
+      const int idx = it * THREADS + tid;
       const int t = idx / CB, col = slice * CB + idx % CB;
       fv[it] = (idx < TC * CB && t0 + t < len && col < a.vdim) ? v0[(size_t)(start + t0 + t) * a.v_stride + col] : 0.f;
     }
@@ -220,7 +219,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
     const int off = t * DP + ks * PER;
 #pragma unroll
     for (int e4 = 0; e4 < PER / 4; ++e4) {
-      if (mode != SCAN_LOCAL) x.q[e4] = ((const float4*)(qs + off))[e4];
+      x.q[e4] = ((const float4*)(qs + off))[e4];
       x.k[e4] = ((const float4*)(ks_ + off))[e4];
       x.w[e4] = ((const float4*)(ws + off))[e4];
     }
@@ -233,21 +232,6 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
       x.v[0] = f.x; x.v[1] = f.y;
     } else {
       x.v[0] = vr[0];
-    }
-  };
-  // the update alone (a piece from zero: nothing is read)
-  auto update = [&](const Tok& x) {
-#pragma unroll
-    for (int e4 = 0; e4 < PER / 4; ++e4) {
-      const float ka[4] = {x.k[e4].x, x.k[e4].y, x.k[e4].z, x.k[e4].w}, wa[4] = {x.w[e4].x, x.w[e4].y, x.w[e4].z, x.w[e4].w};
-#pragma unroll
-      for (int c = 0; c < 4; ++c)
-#pragma unroll
-        for (int j = 0; j < TP; ++j) S[j][e4 * 4 + c] = fmaf(wa[c], S[j][e4 * 4 + c], ka[c] * x.v[j]);
-      if (wave == 0) {
-#pragma unroll
-        for (int c = 0; c < 4; ++c) W[e4 * 4 + c] *= wa[c];
-      }
     }
   };
   auto step = [&](const Tok& x, int t_run) {
@@ -287,7 +271,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
     __syncthreads();   // the chunk before has been consumed
 #pragma unroll
     for (int it = 0; it < NI; ++it) {
-      const int idx = it * 256 + tid;
+      const int idx = it * THREADS + tid;
       if (idx < TC * DP) {
         qs[idx] = fq[it];
         ks_[idx] = fk[it];
@@ -296,7 +280,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
     }
 #pragma unroll
     for (int it = 0; it < NV; ++it) {
-      const int idx = it * 256 + tid;
+      const int idx = it * THREADS + tid;
       if (idx < TC * CB) vs[idx] = fv[it];
     }
     __syncthreads();
@@ -304,27 +288,16 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
     // two tokens a turn, each token's LDS reads issued before the token ahead of it is worked on
     Tok A, B;
     take(A, 0);
-    if (mode == SCAN_LOCAL) {
-      for (int t = 0; t < tc; t += 2) {
-        if (t + 1 < tc) take(B, t + 1);
-        update(A);
-        if (t + 1 < tc) {
-          if (t + 2 < tc) take(A, t + 2);
-          update(B);
-        }
-      }
-    } else {
-      for (int t = 0; t < tc; t += 2) {
-        if (t + 1 < tc) take(B, t + 1);
-        step(A, t0 + t);
-        if (t + 1 < tc) {
-          if (t + 2 < tc) take(A, t + 2);
-          step(B, t0 + t + 1);
-        }
+    for (int t = 0; t < tc; t += 2) {
+      if (t + 1 < tc) take(B, t + 1);
+      step(A, t0 + t);
+      if (t + 1 < tc) {
+        if (t + 2 < tc) take(A, t + 2);
+        step(B, t0 + t + 1);
       }
     }
   }
-  if (mode == SCAN_OUTPUT) return;   // (the carry has left the state after the run)
+  if (mode == SCAN_PIECES) return;   // (the carry has left the state after the run)
 #pragma unroll
   for (int j = 0; j < TP; ++j) {
     const bool have = j0 + j < a.vdim;
@@ -341,11 +314,107 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(LinearScan a) {
       }
     }
   }
-  if (mode == SCAN_LOCAL && slice == 0 && wave == 0 && lane < KS) {
+}
+
+// The end state of every piece from zero, and the products of its decays.  DT: 16-row tiles of key channels (16 DT >= dim).
+// grid: (requests, heads, pieces times slices of 64 value columns); a wave owns 16 columns.  Chunks of sixteen tokens, the
+// last first: 256 / (16 DT) groups of threads each take a run of the chunk's tokens, a thread one key channel; what decays a
+// group's keys beyond its own tokens is the product of the later groups' decays and of the chunks behind.
+// Operands of the 16x16x4 product: lane l holds row (column) l % 16 at k = l / 16; result rows (l / 16) * 4 + r of column l % 16.
+typedef float f32x4_t __attribute__((ext_vector_type(4)));
+
+template <int DT>
+__global__ __launch_bounds__(256) void linear_ends_kernel(LinearScan a) {
+  constexpr int DP = DT * 16, G = 256 / DP, TG = 16 / G;   // groups, tokens of a group
+  __shared__ float ks[16][DP + 1];
+  __shared__ float vs[16][64 + 1];
+  __shared__ float gp[G][DP];
+  const int r = blockIdx.x, h = blockIdx.y;
+  const int slices = (a.vdim + 63) / 64;
+  const int slice = blockIdx.z % slices, pc = blockIdx.z / slices;
+  const int run0 = a.cu_seqlens[r], run_len = a.cu_seqlens[r + 1] - run0;
+  if (run_len <= a.piece || (long)pc * a.piece >= run_len) return;
+  const int start = run0 + pc * a.piece, len = min(a.piece, run_len - pc * a.piece);
+  const size_t place = (size_t)(run0 / a.piece + r + pc) * a.heads + h;
+  const int tid = threadIdx.x, wave = tid / TP_WAVE, lane = tid % TP_WAVE;
+  const int d = tid % DP, g = tid / DP;
+  const bool d_ok = d < a.dim;
+  const size_t hd = (size_t)a.heads * a.dim;
+  const float *k0 = a.k + (size_t)h * a.dim + (d_ok ? d : 0), *w0 = a.decay + (size_t)h * a.dim + (d_ok ? d : 0);
+  const float* v0 = a.v + (size_t)h * a.vdim;
+  const int col = slice * 64 + tid % 64;   // (of the value that this thread fetches)
+
+  float fk[TG], fw[TG], fv[4];
+  auto fetch = [&](int t0) {
 #pragma unroll
-    for (int e = 0; e < PER; ++e)
-      if (ks * PER + e < a.dim) a.piece_decay[place * a.dim + ks * PER + e] = W[e];
+    for (int i = 0; i < TG; ++i) {
+      const int t = t0 + g * TG + i;
+      const bool in = d_ok && t < len;
+      const size_t row = (size_t)(start + (in ? t : 0));
+      fk[i] = in ? k0[row * a.k_stride] : 0.f;
+      fw[i] = in ? w0[row * hd] : 1.f;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = t0 + i * 4 + tid / 64;
+      const bool in = t < len && col < a.vdim;
+      fv[i] = in ? v0[(size_t)(start + t) * a.v_stride + col] : 0.f;
+    }
+  };
+  f32x4_t acc[DT];
+#pragma unroll
+  for (int i = 0; i < DT; ++i) acc[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+  float behind = 1.f;   // the decays of the chunks behind this one, of key channel d
+  const int chunks = (len + 15) / 16;
+  fetch((chunks - 1) * 16);
+  for (int ch = chunks - 1; ch >= 0; --ch) {
+    float own = 1.f;
+#pragma unroll
+    for (int i = 0; i < TG; ++i) own *= fw[i];
+    __syncthreads();   // (the chunk before has been consumed)
+    gp[g][d] = own;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) vs[i * 4 + tid / 64][tid % 64] = fv[i];
+    __syncthreads();
+    float later = behind, all = 1.f;
+#pragma unroll
+    for (int j = 0; j < G; ++j) {
+      const float p = gp[j][d];
+      all *= p;
+      if (j > g) later *= p;
+    }
+#pragma unroll
+    for (int i = TG - 1; i >= 0; --i) {
+      ks[g * TG + i][d] = fk[i] * later;
+      later *= fw[i];
+    }
+    behind *= all;
+    if (ch > 0) fetch((ch - 1) * 16);   // on its way while this chunk is multiplied
+    __syncthreads();
+#pragma unroll
+    for (int kk = 0; kk < 4; ++kk) {
+      const int t = kk * 4 + (lane >> 4);
+      const float b = vs[t][wave * 16 + (lane & 15)];
+#pragma unroll
+      for (int i = 0; i < DT; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(ks[t][i * 16 + (lane & 15)], b, acc[i], 0, 0, 0);
+    }
   }
+  const int j = slice * 64 + wave * 16 + (lane & 15);
+  if (j < a.vdim) {
+    float* out = a.piece_state + (place * a.vdim + j) * a.dim;
+#pragma unroll
+    for (int i = 0; i < DT; ++i) {
+      const int row = i * 16 + (lane >> 4) * 4;
+      if (a.dim % 4 == 0 && row < a.dim) {
+        *(float4*)(out + row) = make_float4(acc[i][0], acc[i][1], acc[i][2], acc[i][3]);
+      } else {
+#pragma unroll
+        for (int c = 0; c < 4; ++c)
+          if (row + c < a.dim) out[row + c] = acc[i][c];
+      }
+    }
+  }
+  if (slice == 0 && g == 0 && d_ok) a.piece_decay[place * a.dim + d] = behind;
 }
 
 // grid: (requests, heads, blocks of 256 state entries); the state each piece starts from, in place of what it ended with from
@@ -387,6 +456,7 @@ extern "C" int tp_linear_scan(const float* q, int q_stride, const float* k, int 
   TP_REQUIRE(q_stride >= heads * dim && k_stride >= heads * dim && v_stride >= heads * vdim, "linear_scan: rows too short");
   TP_REQUIRE(state_stride >= state_off + (size_t)heads * dim * vdim, "linear_scan: state rows too short");
   TP_REQUIRE(heads <= 65535, "linear_scan: too many heads");
+  TP_REQUIRE(piece == 0 || dim <= 128, "linear_scan: runs of keys of %d are not cut", dim);
   TP_REQUIRE(piece == 0 || (piece > 0 && scratch != nullptr && pieces >= n / piece + n_req), "linear_scan: no room for the pieces");
   if (n == 0 || n_req == 0) return 0;
   LinearScan a;
@@ -400,46 +470,52 @@ extern "C" int tp_linear_scan(const float* q, int q_stride, const float* k, int 
   a.piece_state = scratch;
   a.piece_decay = piece ? scratch + (size_t)pieces * heads * dim * vdim : nullptr;
   // PER key channels a lane (8 up to a key size of 128, then 16, then 32), KS lanes a column (a power of two), TP columns a
-  // lane: as many as fill the block without columns to spare; single tokens take one (more blocks, nothing to share)
+  // lane and WAVES waves a block: as many columns a lane as fill a wave without columns to spare, as many waves as the
+  // columns need (at most four); single tokens take one column a lane (more blocks, nothing to share)
   const int per = dim <= 128 ? 8 : (dim <= 256 ? 16 : 32);
   int ks = 1;
   while (ks * per < dim) ks *= 2;
   if (per == 32 && ks < 16) ks = 16;
   int tp = 1;
   const int most = per == 32 ? 1 : (per == 16 ? 2 : (ks >= 8 ? 4 : (ks == 4 ? 2 : 1)));
-  while (tp < most && max_run > 4 && 256 / ks * tp * 2 <= vdim) tp *= 2;
-  const int cb = 256 / ks * tp;
-  const int slices = (vdim + cb - 1) / cb;
+  while (tp < most && max_run > 4 && 64 / ks * tp * 2 <= vdim) tp *= 2;
+  const int cw = 64 / ks * tp;
+  const int waves = tp == 4 && vdim <= 2 * cw ? 2 : 4;
+  const int cb = cw * waves;
+  const int slices = (vdim + cb - 1) / cb, end_slices = (vdim + 63) / 64;
   const int most_pieces = piece ? (max_run + piece - 1) / piece : 1;
-  TP_REQUIRE((long)slices * most_pieces <= 65535 && ((long)dim * vdim + 255) / 256 <= 65535, "linear_scan: too many value columns or pieces");
-#define SCAN_(P, K, T, B) hipLaunchKernelGGL((linear_scan_kernel<P, K, T, B>), grid, dim3(256), 0, s, a)
-#define SCAN(P, K, T)            \
+  TP_REQUIRE((long)(slices > end_slices ? slices : end_slices) * most_pieces <= 65535 && ((long)dim * vdim + 255) / 256 <= 65535,
+             "linear_scan: too many value columns or pieces");
+#define SCAN_(P, K, T, W, B) hipLaunchKernelGGL((linear_scan_kernel<P, K, T, W, B>), grid, dim3(W * 64), 0, s, a)
+#define SCAN(P, K, T, W)         \
   do {                           \
     if (bonus != nullptr)        \
-      SCAN_(P, K, T, true);      \
+      SCAN_(P, K, T, W, true);   \
     else                         \
-      SCAN_(P, K, T, false);     \
+      SCAN_(P, K, T, W, false);  \
   } while (0)
   auto launch = [&](int mode, int across) {
     a.mode = mode;
     const dim3 grid(n_req, heads, slices * across);
     if (per == 8) {
-      if (ks == 1) SCAN(8, 1, 1);
-      else if (ks == 2) SCAN(8, 2, 1);
-      else if (ks == 4 && tp == 1) SCAN(8, 4, 1);
-      else if (ks == 4) SCAN(8, 4, 2);
-      else if (ks == 8 && tp == 1) SCAN(8, 8, 1);
-      else if (ks == 8 && tp == 2) SCAN(8, 8, 2);
-      else if (ks == 8) SCAN(8, 8, 4);
-      else if (tp == 1) SCAN(8, 16, 1);
-      else if (tp == 2) SCAN(8, 16, 2);
-      else SCAN(8, 16, 4);
+      if (ks == 1) SCAN(8, 1, 1, 4);
+      else if (ks == 2) SCAN(8, 2, 1, 4);
+      else if (ks == 4 && tp == 1) SCAN(8, 4, 1, 4);
+      else if (ks == 4) SCAN(8, 4, 2, 4);
+      else if (ks == 8 && tp == 1) SCAN(8, 8, 1, 4);
+      else if (ks == 8 && tp == 2) SCAN(8, 8, 2, 4);
+      else if (ks == 8 && waves == 2) SCAN(8, 8, 4, 2);
+      else if (ks == 8) SCAN(8, 8, 4, 4);
+      else if (tp == 1) SCAN(8, 16, 1, 4);
+      else if (tp == 2) SCAN(8, 16, 2, 4);
+      else if (waves == 2) SCAN(8, 16, 4, 2);
+      else SCAN(8, 16, 4, 4);
     } else if (per == 16) {
-      if (tp == 1) SCAN(16, 16, 1);
-      else SCAN(16, 16, 2);
+      if (tp == 1) SCAN(16, 16, 1, 4);
+      else SCAN(16, 16, 2, 4);
     } else {
-      if (ks <= 16) SCAN(32, 16, 1);
-      else SCAN(32, 32, 1);
+      if (ks <= 16) SCAN(32, 16, 1, 4);
+      else SCAN(32, 32, 1, 4);
     }
   };
 #undef SCAN
@@ -447,9 +523,13 @@ extern "C" int tp_linear_scan(const float* q, int q_stride, const float* k, int 
   if (piece == 0 || max_run <= piece) {
     launch(SCAN_DIRECT, 1);
   } else {
-    launch(SCAN_LOCAL, most_pieces);
+    const dim3 grid(n_req, heads, end_slices * most_pieces);
+    if (dim <= 16) hipLaunchKernelGGL(linear_ends_kernel<1>, grid, dim3(256), 0, s, a);
+    else if (dim <= 32) hipLaunchKernelGGL(linear_ends_kernel<2>, grid, dim3(256), 0, s, a);
+    else if (dim <= 64) hipLaunchKernelGGL(linear_ends_kernel<4>, grid, dim3(256), 0, s, a);
+    else hipLaunchKernelGGL(linear_ends_kernel<8>, grid, dim3(256), 0, s, a);
     hipLaunchKernelGGL(linear_carry_kernel, dim3(n_req, heads, (dim * vdim + 255) / 256), dim3(256), 0, s, a);
-    launch(SCAN_OUTPUT, most_pieces);
+    launch(SCAN_PIECES, most_pieces);
   }
   TP_CHECK_LAUNCH("linear_scan");
   return 0;

@@ -1950,6 +1950,8 @@ scan_target_blocks = 1024
 
 def scan_piece(n: int, max_run: int, heads: int, dim: int, vdim: int) -> int:
     """Tokens of a piece of ``linear_scan`` (0: runs are not cut)."""
+    if dim > 128:
+        return 0
     blocks = heads * max(1, vdim // 64)
     piece = max(scan_min_piece, -(-n * blocks // scan_target_blocks))
     piece = -(-piece // 16) * 16
