@@ -401,6 +401,22 @@ def test_engine_generates_what_plain_greedy_generates(dirs, name):
         assert o == plain.greedy(cfg, W, p, 6)
 
 
+@pytest.mark.parametrize("kind", ["wkv", "parallel"])
+def test_models_of_one_mixer_alone(tmp_path, kind):
+    """Recurrences alone (a model that has no paged cache) and branches alone, through the scheduler."""
+    from tempura_amd.engine import Engine
+    from tempura_amd.sampling import SamplingParams
+    cfg = cases.config_json("mix")
+    cfg["layers"] = [layer for layer in cfg["layers"] if layer["type"] == kind]
+    W = cases.make_weights("mix", 3, cfg=cfg)
+    eng = Engine(cases.write_model("mix", str(tmp_path / kind), weights=W, config=cfg), dtype="float32", page_size=16, kv_pages=12, max_batch_size=2,
+                 max_num_batched_tokens=16, prefill_chunk_size=7, device="cpu", use_graph=False)
+    assert (len(eng.runner.model.cache_groups) == 0) == (kind == "wkv")
+    prompts = [cases.tokens("mix", n, 40 + i) for i, n in enumerate((19, 2, 8))]
+    for p, o in zip(prompts, eng.generate(prompts, SamplingParams(temperature=0.0, max_new_tokens=5))):
+        assert o == plain.greedy(cfg, W, p, 5)
+
+
 def test_command_line_inspects_and_writes_random_folders(dirs, tmp_path, capsys):
     """`tempura inspect` on a folder of the design, and `tempura random-model --config-json` for it (which needs the ranks
     that a checkpoint would say)."""

@@ -545,6 +545,22 @@ def test_engine_generates_what_plain_greedy_generates(dirs, name, use_graph):
         assert eng.runner.graph_steps > 0
 
 
+@pytest.mark.parametrize("kind", ["wkv", "parallel"])
+def test_models_of_one_mixer_alone(tmp_path, kind):
+    """Recurrences alone (a model that has no paged cache) and branches alone, captured steps included."""
+    from tempura_amd.engine import Engine
+    from tempura_amd.sampling import SamplingParams
+    cfg = cases.config_json("wide")
+    cfg["layers"] = [layer for layer in cfg["layers"] if layer["type"] == kind]
+    W = cases.make_weights("wide", 3, cfg=cfg)
+    eng = Engine(cases.write_model("wide", str(tmp_path / kind), weights=W, config=cfg), dtype="float32", page_size=16, kv_pages=40, max_batch_size=3,
+                 max_num_batched_tokens=128, prefill_chunk_size=70, device=DEV, use_graph=True)
+    prompts = [cases.tokens("wide", n, 40 + i) for i, n in enumerate((90, 2, 33, 8))]
+    for p, o in zip(prompts, eng.generate(prompts, SamplingParams(temperature=0.0, max_new_tokens=8))):
+        assert o == plain.greedy(cfg, W, p, 8)
+    assert eng.runner.graph_steps > 0
+
+
 def test_replay_program_on_a_model_folder(dirs, tmp_path):
     """bin/trace_run on a small folder: steps on standard input, logits files out, against the plain result."""
     import os
